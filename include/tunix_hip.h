@@ -69,9 +69,10 @@ const char* tnx_last_error(void);
  * adds tnx_attn_desc.segment_ids, reads top_k == V in tnx_sample_topk as a real top-k, and moves
  * the measurement probe tnx_stream_read out of the library; 3.0 adds tnx_qw_expand /
  * tnx_qw_expanded_bytes, tnx_dense_expand and the w_expanded field of tnx_qlinear_desc and
- * tnx_lmhead_desc; 3.1 adds tnx_sample_topk_head / tnx_sample_topk_head_ok. */
+ * tnx_lmhead_desc; 3.1 adds tnx_sample_topk_head / tnx_sample_topk_head_ok; 3.2 adds the entry
+ * points of decoders with dense weights (tnx_dense_linear to tnx_logits_stats). */
 #define TNX_ABI_VERSION_MAJOR 3
-#define TNX_ABI_VERSION_MINOR 1
+#define TNX_ABI_VERSION_MINOR 2
 #define TNX_ABI_VERSION ((TNX_ABI_VERSION_MAJOR << 16) | TNX_ABI_VERSION_MINOR)
 int tnx_version(void);
 
@@ -536,6 +537,184 @@ int tnx_logp_drift_static(void* stream, const float* rollout_logp, const float* 
 
 /* Fill n 32-bit words with `value` (graph-capturable replacement for hipMemsetAsync). */
 int tnx_fill_u32(void* stream, uint32_t* p, int64_t n, uint32_t value);
+
+/* ---------------------------------------------------------------------------------------
+ * Decoders with dense weights and an fp32 residual stream.  They have no counterpart in the
+ * reference tree; each entry point is one mechanism with its constants as arguments.
+ *
+ * dtype: the model's: TNX_BF16 (matrix operands bf16, fp32 accumulation) or TNX_F32 (everything
+ * fp32).  The residual, norms, angles, scores, softmax and recurrent states are fp32 in both.
+ * A sequence of batch row b occupies the columns starts[b], starts[b] + 1, ... of its row (left
+ * padding in front of it); its position counts from 0 at starts[b].  *col_ptr is the column of the
+ * call's first token.
+ * Fragment order (x_frag / y_frag / out_frag = 1, bf16): activations in blocks of 32 rows x 16
+ * columns, inside a block [column / 8][row][column % 8]; what tnx_dense_linear reads fastest at few
+ * rows.  Buffers hold whole blocks of 128 rows.
+ */
+#define TNX_BF16 0
+#define TNX_F32 1
+
+/* Rows of a linear's output: y (model dtype), or with split_k > 1 the fp32 partial planes
+ * ws[z * plane + row * ld + col] to be summed in z order. */
+typedef struct {
+  const void* y;
+  const float* ws;
+  int split_k;
+  int64_t plane;
+  int64_t ld;
+} tnx_rows_src;
+
+/* y[M, N] = x[M, K] . w^T.  bf16: w is the fragment-order copy of tnx_dense_expand, K % 128 == 0
+ * (zero-padded), N % 16 == 0 for bf16 outputs.  fp32: w row-major [N, K], K % 16 == 0.
+ * epilogue: TNX_EPI_STORE (model dtype), TNX_EPI_F32, or (bf16) TNX_EPI_GELU_MUL: w's rows come in
+ * alternating blocks of 16 gate and 16 up rows and y[M, N/2] = gelu_tanh(gate) * up, formed in fp32
+ * and rounded once.  split_k > 1 (bf16, few rows): fp32 planes to ws [split_k][M][ldy] instead. */
+typedef struct {
+  int64_t M, K, N;
+  int dtype;
+  const void* x;
+  int64_t ldx;
+  int x_frag;
+  const void* w;
+  int epilogue;
+  void* y;
+  int64_t ldy;
+  int y_frag;
+  int split_k;
+  float* ws;
+} tnx_dense_desc;
+int tnx_dense_linear(void* stream, const tnx_dense_desc* d);
+
+/* x[row] (fp32) = table[ids[b, col + t]]; optionally also cat[row, cat_off ..] = the same row in the
+ * model's dtype.  Ids outside [0, V) read row 0. */
+int tnx_embed_rows(void* stream, int dtype, const void* table, int64_t V, int64_t D, const int32_t* ids,
+                   int64_t ids_ld, const int32_t* col_ptr, int64_t B, int64_t T, float* x, void* cat,
+                   int64_t cat_ld, int64_t cat_off, int cat_frag);
+
+/* The residual step between two sublayers, in fp32:
+ *   mode 1: x += norm(y) * (w_offset + w_post);  mode 2: x = y;  mode 0: x stays;
+ *   out (model dtype) = norm(x) * (w_offset + w_next), or x itself when w_next is null,
+ * with norm(v) = v / sqrt(mean(v^2) + eps).  y.ws with split_k >= 1: fp32 planes. */
+typedef struct {
+  int64_t M, D;
+  int dtype;
+  float eps, w_offset;
+  int mode;
+  tnx_rows_src y;
+  const float* w_post;
+  float* x;
+  const float* w_next;
+  void* out;
+  int64_t out_ld;
+  int out_frag;
+} tnx_residual_norm_desc;
+int tnx_residual_norm(void* stream, const tnx_residual_norm_desc* d);
+
+/* Rotation of the first rot_dims dimensions of every query and key head (pairs (i, i + rot_dims/2),
+ * angle position * inv_freq[i] in fp32) and the cache write.  y: q heads from column 0, k from k_off,
+ * v from v_off.  q_out [B*T, H, dkp]; kcache [B, G, S, dkp], vcache [B, G, S, dvp] at slot col + t;
+ * dimensions past dk / dv are written as zeros. */
+typedef struct {
+  int64_t B, T, S;
+  int H, G, dk, dv, dkp, dvp, rot_dims;
+  int dtype;
+  const float* inv_freq;
+  tnx_rows_src y;
+  int64_t k_off, v_off;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  void* q_out;
+  void* kcache;
+  void* vcache;
+} tnx_part_rope_desc;
+int tnx_part_rope_kvwrite(void* stream, const tnx_part_rope_desc* d);
+
+/* Causal attention over keys starts[b] .. col + t with softmax(scale * q.k) whose denominator also
+ * holds exp(sinks[head]) (sinks null: none).  out[row, head * dv ..].  kv_chunk > 0 splits the key range (few
+ * query rows, workspace of tnx_sink_attn_ws_bytes).  tnx_sink_attn_pad: the padded head size the
+ * MFMA kernels take (other sizes, and fp32, run a plain kernel). */
+typedef struct {
+  int64_t B, T, S;
+  int H, G, dk, dv, dkp, dvp;
+  float scale;
+  int dtype;
+  const void* q;
+  const void* kcache;
+  const void* vcache;
+  const float* sinks;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  int kv_chunk;
+  float* ws;
+  void* out;
+  int64_t out_ld;
+  int out_frag;
+} tnx_sink_attn_desc;
+int tnx_sink_attn_pad(int dim, int is_value);
+size_t tnx_sink_attn_ws_bytes(int64_t B, int64_t T, int64_t S, int H, int dvp, int kv_chunk);
+int tnx_sink_attn(void* stream, const tnx_sink_attn_desc* d);
+
+/* Lightning attention: S <- decay[h] S + k v^T, o = S^T q per head, with q, k, v = silu of y's columns
+ * (q from 0, k from k_off, v from v_off; head by head).  state fp32 [B, H, dk, dv] is read unless
+ * col <= starts[b] and written back; o fp32 [B*T, o_ld]. */
+typedef struct {
+  int64_t B, T;
+  int H, dk, dv;
+  int dtype;
+  const float* decay;
+  tnx_rows_src y;
+  int64_t k_off, v_off;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  float* state;
+  float* o;
+  int64_t o_ld;
+  float* ws;
+} tnx_lightning_desc;
+size_t tnx_lightning_ws_bytes(int64_t B, int64_t T, int H, int dk, int dv);
+int tnx_lightning(void* stream, const tnx_lightning_desc* d);
+
+/* out = norm(o) * (w_offset + w) * sigmoid(g[:, g_off ..]) over whole rows of W values. */
+typedef struct {
+  int64_t M, W;
+  int dtype;
+  float eps, w_offset;
+  const float* o;
+  int64_t o_ld;
+  tnx_rows_src g;
+  int64_t g_off;
+  const float* w;
+  void* out;
+  int64_t out_ld;
+  int out_frag;
+} tnx_gated_norm_desc;
+int tnx_gated_norm(void* stream, const tnx_gated_norm_desc* d);
+
+/* out[M, F] = gelu_tanh(y[:, :F]) * y[:, up_off : up_off + F]. */
+int tnx_gelu_mul(void* stream, int dtype, const void* y, int64_t ld, int64_t up_off, int64_t M, int64_t F,
+                 void* out, int64_t out_ld);
+
+/* Statistics and the whole-vocabulary draw of tnx_lmhead_logp over finished fp32 logits [M, V]
+ * (any V); the fields mean what they mean there. */
+typedef struct {
+  int64_t M, V;
+  const float* logits;
+  float temperature;
+  const int32_t* forbidden;
+  int n_forbidden;
+  const int32_t* targets;
+  int32_t* best_id;
+  float* best_logp;
+  float* target_logp;
+  float* lse;
+  float* entropy;
+  uint32_t draw_key0, draw_key1;
+  int draw_rng_variant;
+  const int32_t* draw_step_ptr;
+  int32_t* draw_id;
+  float* draw_logp;
+} tnx_logits_desc;
+int tnx_logits_stats(void* stream, const tnx_logits_desc* d);
 
 #ifdef __cplusplus
 }

@@ -12,12 +12,14 @@ _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libtunix_hip.so")
 
 # the ABI this binding was written against (TNX_ABI_VERSION_MAJOR / _MINOR of include/tunix_hip.h)
-ABI_VERSION = (3, 1)
+ABI_VERSION = (3, 2)
 
 TNX_Q_INT4, TNX_Q_NF4 = 0, 1
 TNX_NORM_LLAMA, TNX_NORM_QWEN3, TNX_NORM_GEMMA3 = 0, 1, 2
 TNX_ROPE_LLAMA, TNX_ROPE_QWEN3, TNX_ROPE_GEMMA3 = 0, 1, 2
 TNX_EPI_STORE, TNX_EPI_RESIDUAL, TNX_EPI_SILU_MUL, TNX_EPI_GELU_MUL, TNX_EPI_F32 = 0, 1, 2, 3, 4
+
+TNX_BF16, TNX_F32 = 0, 1
 
 _p = C.c_void_p
 _i64 = C.c_int64
@@ -91,6 +93,68 @@ class MoeGmmDesc(C.Structure):
   ]
 
 
+class RowsSrc(C.Structure):
+  _fields_ = [("y", _p), ("ws", _p), ("split_k", _i32), ("plane", _i64), ("ld", _i64)]
+
+
+class DenseDesc(C.Structure):
+  _fields_ = [
+      ("M", _i64), ("K", _i64), ("N", _i64), ("dtype", _i32),
+      ("x", _p), ("ldx", _i64), ("x_frag", _i32), ("w", _p), ("epilogue", _i32),
+      ("y", _p), ("ldy", _i64), ("y_frag", _i32), ("split_k", _i32), ("ws", _p),
+  ]
+
+
+class ResidualNormDesc(C.Structure):
+  _fields_ = [
+      ("M", _i64), ("D", _i64), ("dtype", _i32), ("eps", _f32), ("w_offset", _f32), ("mode", _i32),
+      ("y", RowsSrc), ("w_post", _p), ("x", _p), ("w_next", _p), ("out", _p), ("out_ld", _i64), ("out_frag", _i32),
+  ]
+
+
+class PartRopeDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("S", _i64),
+      ("H", _i32), ("G", _i32), ("dk", _i32), ("dv", _i32), ("dkp", _i32), ("dvp", _i32), ("rot_dims", _i32),
+      ("dtype", _i32), ("inv_freq", _p), ("y", RowsSrc), ("k_off", _i64), ("v_off", _i64),
+      ("starts", _p), ("col_ptr", _p), ("q_out", _p), ("kcache", _p), ("vcache", _p),
+  ]
+
+
+class SinkAttnDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("S", _i64),
+      ("H", _i32), ("G", _i32), ("dk", _i32), ("dv", _i32), ("dkp", _i32), ("dvp", _i32),
+      ("scale", _f32), ("dtype", _i32), ("q", _p), ("kcache", _p), ("vcache", _p), ("sinks", _p),
+      ("starts", _p), ("col_ptr", _p), ("kv_chunk", _i32), ("ws", _p), ("out", _p), ("out_ld", _i64), ("out_frag", _i32),
+  ]
+
+
+class LightningDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("H", _i32), ("dk", _i32), ("dv", _i32), ("dtype", _i32),
+      ("decay", _p), ("y", RowsSrc), ("k_off", _i64), ("v_off", _i64), ("starts", _p), ("col_ptr", _p),
+      ("state", _p), ("o", _p), ("o_ld", _i64), ("ws", _p),
+  ]
+
+
+class GatedNormDesc(C.Structure):
+  _fields_ = [
+      ("M", _i64), ("W", _i64), ("dtype", _i32), ("eps", _f32), ("w_offset", _f32),
+      ("o", _p), ("o_ld", _i64), ("g", RowsSrc), ("g_off", _i64), ("w", _p),
+      ("out", _p), ("out_ld", _i64), ("out_frag", _i32),
+  ]
+
+
+class LogitsDesc(C.Structure):
+  _fields_ = [
+      ("M", _i64), ("V", _i64), ("logits", _p), ("temperature", _f32), ("forbidden", _p), ("n_forbidden", _i32),
+      ("targets", _p), ("best_id", _p), ("best_logp", _p), ("target_logp", _p), ("lse", _p), ("entropy", _p),
+      ("draw_key0", C.c_uint32), ("draw_key1", C.c_uint32), ("draw_rng_variant", _i32), ("draw_step_ptr", _p),
+      ("draw_id", _p), ("draw_logp", _p),
+  ]
+
+
 # name -> (restype, argtypes); every symbol include/tunix_hip.h declares.
 SIGNATURES = {
     "tnx_last_error": (C.c_char_p, []),
@@ -137,6 +201,18 @@ SIGNATURES = {
     "tnx_logp_drift": (_i32, [_p, _p, _p, _p, _i64, _i64, _p, _p]),
     "tnx_logp_drift_static_max_rows": (_i64, []),
     "tnx_logp_drift_static": (_i32, [_p, _p, _p, _p, _i64, _i64, _p]),
+    "tnx_dense_linear": (_i32, [_p, C.POINTER(DenseDesc)]),
+    "tnx_embed_rows": (_i32, [_p, _i32, _p, _i64, _i64, _p, _i64, _p, _i64, _i64, _p, _p, _i64, _i64, _i32]),
+    "tnx_residual_norm": (_i32, [_p, C.POINTER(ResidualNormDesc)]),
+    "tnx_part_rope_kvwrite": (_i32, [_p, C.POINTER(PartRopeDesc)]),
+    "tnx_sink_attn_pad": (_i32, [_i32, _i32]),
+    "tnx_sink_attn_ws_bytes": (C.c_size_t, [_i64, _i64, _i64, _i32, _i32, _i32]),
+    "tnx_sink_attn": (_i32, [_p, C.POINTER(SinkAttnDesc)]),
+    "tnx_lightning_ws_bytes": (C.c_size_t, [_i64, _i64, _i32, _i32, _i32]),
+    "tnx_lightning": (_i32, [_p, C.POINTER(LightningDesc)]),
+    "tnx_gated_norm": (_i32, [_p, C.POINTER(GatedNormDesc)]),
+    "tnx_gelu_mul": (_i32, [_p, _i32, _p, _i64, _i64, _i64, _i64, _p, _i64]),
+    "tnx_logits_stats": (_i32, [_p, C.POINTER(LogitsDesc)]),
     "tnx_fill_u32": (_i32, [_p, _p, _i64, C.c_uint32]),
 }
 

@@ -1,0 +1,104 @@
+"""What a batch of sequences carries from one forward pass to the next: one entry per layer run,
+either a key / value slab (attention) or a recurrent state.  A layer that runs several times has
+one entry per run.
+
+Slabs are [B, heads, S, size] in the model's dtype, states [B, heads, dim, vdim] in fp32.  Rows of
+a batch are slots: a slot whose sequence has ended may be given to another one.  Nothing has to be
+cleared for that: attention reads no slot in front of the new sequence's first column or behind
+its last token, and a recurrence starts from zero at a sequence's first column.
+"""
+from __future__ import annotations
+
+import dataclasses
+
+import torch
+
+
+@dataclasses.dataclass(frozen=True)
+class KVSpec:
+  """Keys and values of one attention layer run."""
+  heads: int
+  k_dim: int
+  v_dim: int
+  dtype: torch.dtype = torch.bfloat16
+
+  def allocate(self, B: int, S: int, device) -> "KVEntry":
+    z = lambda d: torch.zeros(B, self.heads, S, d, dtype=self.dtype, device=device)
+    return KVEntry(z(self.k_dim), z(self.v_dim))
+
+
+@dataclasses.dataclass(frozen=True)
+class StateSpec:
+  """Matrix state of one recurrent layer run (always fp32)."""
+  heads: int
+  dim: int
+  vdim: int
+
+  def allocate(self, B: int, S: int, device) -> "StateEntry":
+    return StateEntry(torch.zeros(B, self.heads, self.dim, self.vdim, dtype=torch.float32, device=device))
+
+
+@dataclasses.dataclass
+class KVEntry:
+  k: torch.Tensor
+  v: torch.Tensor
+
+  def rows(self, b0: int, n: int) -> "KVEntry":
+    return KVEntry(self.k[b0:b0 + n], self.v[b0:b0 + n])
+
+  def grow(self, S: int):
+    for name in ("k", "v"):
+      old = getattr(self, name)
+      new = torch.zeros(*old.shape[:2], S, old.shape[3], dtype=old.dtype, device=old.device)
+      new[:, :, :old.shape[2]].copy_(old)
+      setattr(self, name, new)
+
+
+@dataclasses.dataclass
+class StateEntry:
+  s: torch.Tensor
+
+  def rows(self, b0: int, n: int) -> "StateEntry":
+    return StateEntry(self.s[b0:b0 + n])
+
+  def grow(self, S: int):
+    pass   # a state does not depend on the number of columns
+
+
+class SequenceCache:
+  """The entries of one batch.  shared=True: layer runs with equal specs use one buffer (a scratch
+  cache for passes that never come back to it)."""
+
+  def __init__(self, specs: list, B: int, S: int, device, shared: bool = False):
+    self.B, self.S = B, S
+    made: dict = {}
+    self.entries = []
+    for spec in specs:
+      if shared and spec in made:
+        self.entries.append(made[spec])
+        continue
+      entry = spec.allocate(B, S, device)
+      made[spec] = entry
+      self.entries.append(entry)
+
+  @property
+  def kcache(self) -> list:
+    return [e.k for e in self.entries if isinstance(e, KVEntry)]
+
+  @property
+  def vcache(self) -> list:
+    return [e.v for e in self.entries if isinstance(e, KVEntry)]
+
+  def rows(self, b0: int, n: int) -> "SequenceCache":
+    """A view of the slots b0 .. b0 + n - 1."""
+    view = object.__new__(SequenceCache)
+    view.B, view.S = n, self.S
+    view.entries = [e.rows(b0, n) for e in self.entries]
+    return view
+
+  def grow(self, S: int):
+    """More columns, the ones in use kept."""
+    if S > self.S:
+      for e in self.entries:
+        e.grow(S)
+      self.S = S

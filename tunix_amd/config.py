@@ -107,6 +107,139 @@ class ModelConfig:
     return self.num_kv_heads * self.head_dim
 
 
+# ---- decoders described as a list of layers (dense weights, fp32 residual stream) --------------
+@dataclasses.dataclass(frozen=True)
+class AttentionMixer:
+  """Causal grouped-query attention: separate key and value head sizes, rotation of the first
+  rot_dims dimensions of q and k, any score scale, optionally a learned sink per query head."""
+  heads: int
+  kv_heads: int
+  dim: int
+  vdim: int
+  rot_dims: int
+  rot_base: float
+  scale: float
+  sink: bool = True
+
+  def __post_init__(self):
+    if self.heads % self.kv_heads:
+      raise ValueError("heads must be a multiple of kv_heads")
+    if self.rot_dims % 2 or not 0 <= self.rot_dims <= self.dim:
+      raise ValueError(f"rot_dims={self.rot_dims} must be even and at most the head size {self.dim}")
+
+
+@dataclasses.dataclass(frozen=True)
+class LightningMixer:
+  """Linear attention with one constant decay per head and a matrix state per head; the heads'
+  outputs are normed together, gated and projected."""
+  heads: int
+  dim: int
+  vdim: int
+  decay: tuple
+
+  def __post_init__(self):
+    if len(self.decay) != self.heads:
+      raise ValueError(f"{len(self.decay)} decays for {self.heads} heads")
+
+
+@dataclasses.dataclass(frozen=True)
+class GatedMlp:
+  """down(gelu_tanh(gate h) * (up h))."""
+  ff: int
+
+
+@dataclasses.dataclass(frozen=True)
+class LayerSpec:
+  mixer: AttentionMixer | LightningMixer
+  mlp: GatedMlp | None
+
+
+@dataclasses.dataclass(frozen=True)
+class LayerLoop:
+  """Layers start .. stop - 1 run `times` times; before each pass x <- W [x; embedding output]."""
+  start: int
+  stop: int
+  times: int
+
+
+@dataclasses.dataclass(frozen=True)
+class StackConfig:
+  """A decoder given layer by layer.  Every sublayer is x += norm(f(norm(x))) with norm weights
+  stored as an offset from `norm_offset`; the head is the embedding table."""
+  family: str
+  vocab_size: int
+  embed_dim: int
+  layers: tuple
+  norm_eps: float
+  loop: LayerLoop | None = None
+  norm_offset: float = 1.0
+
+  def __post_init__(self):
+    n, lp = len(self.layers), self.loop
+    if lp is not None and not (0 <= lp.start < lp.stop <= n and lp.times >= 1):
+      raise ValueError(f"the loop {lp} does not fit {n} layers")
+
+  @property
+  def num_layers(self) -> int:
+    return len(self.layers)
+
+  @property
+  def layer_runs(self) -> list[tuple[int, bool]]:
+    """(layer, whether a pass of the loop begins with it) in running order: one cache entry each."""
+    n, lp = self.num_layers, self.loop
+    if lp is None:
+      return [(i, False) for i in range(n)]
+    one = [(i, i == lp.start) for i in range(lp.start, lp.stop)]
+    return [(i, False) for i in range(lp.start)] + one * lp.times + [(i, False) for i in range(lp.stop, n)]
+
+  def weight_shapes(self) -> dict[str, tuple]:
+    """Name -> shape of every tensor; linear weights are [out, in]."""
+    D = self.embed_dim
+    out = {"embed": (self.vocab_size, D), "final.norm": (D,)}
+    if self.loop is not None:
+      out["loop.in"] = (D, 2 * D)
+    for i, ly in enumerate(self.layers):
+      p, m = f"l{i}.", ly.mixer
+      out[p + "norm1"] = out[p + "norm1b"] = (D,)
+      attn = isinstance(m, AttentionMixer)
+      kv = m.kv_heads if attn else m.heads
+      out[p + "mix.q"], out[p + "mix.k"] = (m.heads * m.dim, D), (kv * m.dim, D)
+      out[p + "mix.v"], out[p + "mix.o"] = (kv * m.vdim, D), (D, m.heads * m.vdim)
+      if not attn:
+        out[p + "mix.g"], out[p + "mix.norm"] = (m.heads * m.vdim, D), (m.heads * m.vdim,)
+      elif m.sink:
+        out[p + "mix.sink"] = (m.heads,)
+      if ly.mlp is not None:
+        out[p + "norm2"] = out[p + "norm2b"] = (D,)
+        out[p + "mlp.gate"] = out[p + "mlp.up"] = (ly.mlp.ff, D)
+        out[p + "mlp.down"] = (D, ly.mlp.ff)
+    return out
+
+
+def nunezen_from_dict(d: dict) -> StackConfig:
+  """Reads a Nunezen config.json."""
+  layers = []
+  for i, ly in enumerate(d["layers"]):
+    m = ly["mixer"]
+    if ly["type"] == "attention":
+      rot = m["rot"]
+      mixer = AttentionMixer(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                             rot_dims=int(rot["dims"]), rot_base=float(rot["base"]), scale=float(m["scale"]))
+    elif ly["type"] == "lightning":
+      mixer = LightningMixer(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                             decay=tuple(float(x) for x in m["decay"]))
+    else:
+      raise ValueError(f"layer {i}: unknown mixer type {ly['type']!r}")
+    mlp = ly.get("mlp")
+    if mlp is not None and mlp["kind"] != "dense":
+      raise ValueError(f"layer {i}: unknown feed-forward kind {mlp['kind']!r}")
+    layers.append(LayerSpec(mixer, None if mlp is None else GatedMlp(int(mlp["ff"]))))
+  lp = d.get("loop")
+  return StackConfig(family="nunezen", vocab_size=int(d["vocab"]), embed_dim=int(d["width"]), layers=tuple(layers),
+                     norm_eps=float(d["norm"]["eps"]),
+                     loop=None if lp is None else LayerLoop(int(lp["start"]), int(lp["stop"]), int(lp["times"])))
+
+
 # ---- the shapes the headline metric and the parity cases are quoted on ------------------------
 def tiny_qwen3(**kw) -> ModelConfig:
   """2-layer Qwen3-style decoder: D512, 8q/2kv, dh64, MLP 1536, V32000, int4 g64, LoRA r8."""

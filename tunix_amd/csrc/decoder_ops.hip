@@ -1,0 +1,560 @@
+// The small operations of decoders with dense weights and an fp32 residual stream: embedding,
+// post-norm + residual + next pre-norm, partial rotation + cache write, gated norm, gated unit,
+// and the statistics / sampling of finished logits.  Norms, angles and the residual are 32-bit;
+// matrix operands leave in the model's dtype (bf16 or fp32).
+#include <string.h>
+
+#include "decoder.h"
+#include "rng.h"
+
+namespace {
+
+__device__ __forceinline__ float block_sum(float v, float* red) {
+  v = wave_sum(v);
+  const int wave = threadIdx.x >> 6, nw = (blockDim.x + 63) >> 6;
+  __syncthreads();
+  if ((threadIdx.x & 63) == 0) red[wave] = v;
+  __syncthreads();
+  float s = 0.f;
+  for (int w = 0; w < nw; ++w) s += red[w];
+  return s;
+}
+
+// ---- embedding ---------------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void embed_rows_kernel(const T* table, int64_t V, int64_t D, const int32_t* ids,
+                                                         int64_t ids_ld, const int32_t* col_ptr, int64_t Tn, float* x,
+                                                         T* cat, int64_t cat_ld, int64_t cat_off, int cat_frag) {
+  const int64_t row = blockIdx.x, b = row / Tn, t = row % Tn;
+  const int col = col_ptr ? *col_ptr : 0;
+  int64_t id = ids[b * ids_ld + col + t];
+  if (id < 0 || id >= V) id = 0;   // padding columns: never read by a later token
+  for (int64_t i = threadIdx.x; i < D; i += 256) {
+    const T v = table[id * D + i];
+    x[row * D + i] = ld_elem(&v, 0);
+    if (cat) cat[cat_frag ? frag_index(row, cat_off + i, cat_ld) : row * cat_ld + cat_off + i] = v;
+  }
+}
+
+// ---- residual + norms --------------------------------------------------------------------------
+struct ResNormArgs {
+  int64_t M, D;
+  float eps, w_offset;
+  const void* y;
+  const float* ws;
+  int split;
+  int64_t plane, y_ld;
+  int mode;               // 0: nothing arrives, 1: x += norm(y) . w_post, 2: x = y
+  const float* w_post;
+  float* x;
+  const float* w_next;    // null: out = x in the model's dtype
+  void* out;
+  int64_t out_ld;
+  int out_frag;
+};
+
+// any D that fits LDS
+template <typename T>
+__global__ __launch_bounds__(256) void resnorm_kernel(const ResNormArgs a) {
+  extern __shared__ __align__(16) float hrow[];
+  __shared__ float red[4];
+  const int64_t row = blockIdx.x;
+  const RowSrc<T> src{reinterpret_cast<const T*>(a.y), a.ws, a.ws ? max(a.split, 2) : 1, a.plane, a.y_ld};
+  auto incoming = [&](int64_t i) {
+    if (!a.ws) return src.get(row, i);
+    float v = 0.f;
+    for (int z = 0; z < a.split; ++z) v += a.ws[z * a.plane + row * a.y_ld + i];
+    return v;
+  };
+  float ss = 0.f;
+  if (a.mode != 0)
+    for (int64_t i = threadIdx.x; i < a.D; i += 256) {
+      const float v = incoming(i);
+      hrow[i] = v;
+      ss += v * v;
+    }
+  float r = 1.f;
+  if (a.mode == 1) r = 1.0f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
+  ss = 0.f;
+  for (int64_t i = threadIdx.x; i < a.D; i += 256) {
+    float h;
+    if (a.mode == 1) h = a.x[row * a.D + i] + hrow[i] * r * (a.w_offset + a.w_post[i]);
+    else if (a.mode == 2) h = hrow[i];
+    else h = a.x[row * a.D + i];
+    if (a.mode != 0) a.x[row * a.D + i] = h;
+    hrow[i] = h;
+    ss += h * h;
+  }
+  float rn = 1.f;
+  if (a.w_next) rn = 1.0f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
+  T* out = reinterpret_cast<T*>(a.out);
+  for (int64_t i = threadIdx.x; i < a.D; i += 256) {
+    const float v = a.w_next ? hrow[i] * rn * (a.w_offset + a.w_next[i]) : hrow[i];
+    st_elem(out, a.out_frag ? frag_index(row, i, a.out_ld) : row * a.out_ld + i, v);
+  }
+}
+
+// D % 8 == 0: eight elements per thread and turn, the row stays in registers
+template <int MAXC, typename T>
+__global__ __launch_bounds__(256) void resnorm_vec_kernel(const ResNormArgs a) {
+  __shared__ float red[4];
+  const int64_t row = blockIdx.x;
+  const int nch = (int)(a.D / 8);
+  float h[MAXC][8], xo[MAXC][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = c * 256 + threadIdx.x;
+    const bool ok = ch < nch;
+    const int64_t col = (int64_t)min(ch, nch - 1) * 8;
+    if (a.mode != 2) {
+      const f32x4 x0 = *reinterpret_cast<const f32x4*>(a.x + row * a.D + col);
+      const f32x4 x1 = *reinterpret_cast<const f32x4*>(a.x + row * a.D + col + 4);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        xo[c][j] = x0[j];
+        xo[c][4 + j] = x1[j];
+      }
+    }
+    if (a.mode != 0) {
+      if (a.ws) {
+        const float* p = a.ws + row * a.y_ld + col;
+        f32x4 s0 = *reinterpret_cast<const f32x4*>(p), s1 = *reinterpret_cast<const f32x4*>(p + 4);
+        for (int z0 = 1; z0 < a.split; z0 += 4) {   // four planes in flight, added in plane order
+          f32x4 q0[4], q1[4];
+#pragma unroll
+          for (int u = 0; u < 4; ++u) {
+            const float* q = p + (int64_t)min(z0 + u, a.split - 1) * a.plane;
+            q0[u] = *reinterpret_cast<const f32x4*>(q);
+            q1[u] = *reinterpret_cast<const f32x4*>(q + 4);
+          }
+#pragma unroll
+          for (int u = 0; u < 4; ++u)
+            if (z0 + u < a.split) {
+              s0 += q0[u];
+              s1 += q1[u];
+            }
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          h[c][j] = s0[j];
+          h[c][4 + j] = s1[j];
+        }
+      } else if constexpr (sizeof(T) == 2) {
+        const u32x4 v = *reinterpret_cast<const u32x4*>(reinterpret_cast<const T*>(a.y) + row * a.y_ld + col);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          h[c][2 * j] = bflo(v[j]);
+          h[c][2 * j + 1] = bfhi(v[j]);
+        }
+      } else {
+        const T* p = reinterpret_cast<const T*>(a.y) + row * a.y_ld + col;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) h[c][j] = ld_elem(p, j);
+      }
+      if (ok)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) ss += h[c][j] * h[c][j];
+    }
+  }
+  float r = 1.f;
+  if (a.mode == 1) r = 1.0f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
+  ss = 0.f;
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = c * 256 + threadIdx.x;
+    const int64_t col = (int64_t)min(ch, nch - 1) * 8;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      if (a.mode == 1) h[c][j] = xo[c][j] + h[c][j] * r * (a.w_offset + a.w_post[col + j]);
+      else if (a.mode == 0) h[c][j] = xo[c][j];
+    }
+    if (ch < nch) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss += h[c][j] * h[c][j];
+      if (a.mode != 0) {
+        *reinterpret_cast<f32x4*>(a.x + row * a.D + col) = f32x4{h[c][0], h[c][1], h[c][2], h[c][3]};
+        *reinterpret_cast<f32x4*>(a.x + row * a.D + col + 4) = f32x4{h[c][4], h[c][5], h[c][6], h[c][7]};
+      }
+    }
+  }
+  float rn = 1.f;
+  if (a.w_next) rn = 1.0f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
+  T* out = reinterpret_cast<T*>(a.out);
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = c * 256 + threadIdx.x;
+    if (ch >= nch) continue;
+    const int64_t col = (int64_t)ch * 8;
+    float v[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] = a.w_next ? h[c][j] * rn * (a.w_offset + a.w_next[col + j]) : h[c][j];
+    T* o = out + (a.out_frag ? frag_index(row, col, a.out_ld) : row * a.out_ld + col);
+    if constexpr (sizeof(T) == 2) {
+      *reinterpret_cast<u32x4*>(o) = u32x4{pack2bf(v[0], v[1]), pack2bf(v[2], v[3]), pack2bf(v[4], v[5]), pack2bf(v[6], v[7])};
+    } else {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) st_elem(o, j, v[j]);
+    }
+  }
+}
+
+template <typename T>
+void launch_resnorm(hipStream_t st, const ResNormArgs& a) {
+  const bool vec = a.D % 8 == 0 && a.D <= 16384 && a.y_ld % 8 == 0 && a.out_ld % 8 == 0 && a.plane % 4 == 0;
+  const dim3 grid((unsigned)a.M);
+  if (!vec) hipLaunchKernelGGL((resnorm_kernel<T>), grid, dim3(256), (size_t)a.D * 4, st, a);
+  else if (a.D <= 2048) hipLaunchKernelGGL((resnorm_vec_kernel<1, T>), grid, dim3(256), 0, st, a);
+  else if (a.D <= 4096) hipLaunchKernelGGL((resnorm_vec_kernel<2, T>), grid, dim3(256), 0, st, a);
+  else if (a.D <= 8192) hipLaunchKernelGGL((resnorm_vec_kernel<4, T>), grid, dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((resnorm_vec_kernel<8, T>), grid, dim3(256), 0, st, a);
+}
+
+// ---- rotation of the first rot_dims dimensions of q and k, cache write --------------------------
+struct PartRopeArgs {
+  int64_t T, S;
+  int H, G, dk, dv, dkp, dvp, half;
+  const float* inv_freq;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  int64_t k_off, v_off;
+};
+constexpr int kMaxHalf = 256;
+
+template <typename T>
+__global__ __launch_bounds__(256) void part_rope_kernel(const PartRopeArgs a, const RowSrc<T> src, T* q_out, T* kc, T* vc) {
+  __shared__ float sn[kMaxHalf], cs[kMaxHalf];
+  const int64_t row = blockIdx.x, b = row / a.T, t = row % a.T;
+  const int slot = *a.col_ptr + (int)t;
+  if (slot >= a.S) return;                                    // (uniform; the host sizes the cache)
+  const float pos = (float)max(slot - a.starts[b], 0);
+  for (int i = threadIdx.x; i < a.half; i += 256) sincosf(pos * a.inv_freq[i], &sn[i], &cs[i]);
+  __syncthreads();
+  const int heads = a.H + a.G, hpt = a.dkp - a.half;           // one item per pair or lone dimension
+  for (int it = threadIdx.x; it < heads * hpt; it += 256) {
+    const int hd = it / hpt, i = it % hpt;
+    const bool is_k = hd >= a.H;
+    const int64_t base = is_k ? a.k_off + (int64_t)(hd - a.H) * a.dk : (int64_t)hd * a.dk;
+    T* dst = is_k ? kc + ((b * a.G + (hd - a.H)) * a.S + slot) * a.dkp : q_out + (row * a.H + hd) * a.dkp;
+    if (i < a.half) {
+      const float u = src.get(row, base + i), v = src.get(row, base + i + a.half);
+      st_elem(dst, i, u * cs[i] - v * sn[i]);
+      st_elem(dst, i + a.half, v * cs[i] + u * sn[i]);
+    } else {
+      const int d = i + a.half;
+      st_elem(dst, d, d < a.dk ? src.get(row, base + d) : 0.f);
+    }
+  }
+  for (int it = threadIdx.x; it < a.G * a.dvp; it += 256) {
+    const int g = it / a.dvp, d = it % a.dvp;
+    st_elem(vc, ((b * a.G + g) * a.S + slot) * a.dvp + d, d < a.dv ? src.get(row, a.v_off + (int64_t)g * a.dv + d) : 0.f);
+  }
+}
+
+// Finished bf16 rows whose heads, offsets and rotated halves come in whole runs of eight: 16 bytes
+// per access (prefill).
+__global__ __launch_bounds__(256) void part_rope_vec_kernel(const PartRopeArgs a, const uint16_t* y, int64_t ld, uint16_t* q_out,
+                                                            uint16_t* kc, uint16_t* vc) {
+  __shared__ __align__(16) float sn[kMaxHalf], cs[kMaxHalf];
+  const int64_t row = blockIdx.x, b = row / a.T, t = row % a.T;
+  const int slot = *a.col_ptr + (int)t;
+  if (slot >= a.S) return;
+  const float pos = (float)max(slot - a.starts[b], 0);
+  for (int i = threadIdx.x; i < a.half; i += 256) sincosf(pos * a.inv_freq[i], &sn[i], &cs[i]);
+  __syncthreads();
+  const uint16_t* yr = y + row * ld;
+  const int heads = a.H + a.G, hpt = (a.dkp - a.half) / 8, half8 = a.half / 8;
+  for (int it = threadIdx.x; it < heads * hpt; it += 256) {
+    const int hd = it / hpt, c = it % hpt;
+    const bool is_k = hd >= a.H;
+    const uint16_t* s = yr + (is_k ? a.k_off + (int64_t)(hd - a.H) * a.dk : (int64_t)hd * a.dk);
+    uint16_t* dst = is_k ? kc + ((b * a.G + (hd - a.H)) * a.S + slot) * a.dkp : q_out + (row * a.H + hd) * a.dkp;
+    if (c < half8) {
+      const u32x4 u = *reinterpret_cast<const u32x4*>(s + c * 8), v = *reinterpret_cast<const u32x4*>(s + a.half + c * 8);
+      u32x4 o1, o2;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const float c0 = cs[c * 8 + 2 * j], c1 = cs[c * 8 + 2 * j + 1], s0 = sn[c * 8 + 2 * j], s1 = sn[c * 8 + 2 * j + 1];
+        const float u0 = bflo(u[j]), u1 = bfhi(u[j]), v0 = bflo(v[j]), v1 = bfhi(v[j]);
+        o1[j] = pack2bf(u0 * c0 - v0 * s0, u1 * c1 - v1 * s1);
+        o2[j] = pack2bf(v0 * c0 + u0 * s0, v1 * c1 + u1 * s1);
+      }
+      *reinterpret_cast<u32x4*>(dst + c * 8) = o1;
+      *reinterpret_cast<u32x4*>(dst + a.half + c * 8) = o2;
+    } else {
+      const int d = a.half + c * 8;
+      *reinterpret_cast<u32x4*>(dst + d) = d < a.dk ? *reinterpret_cast<const u32x4*>(s + d) : u32x4{0, 0, 0, 0};
+    }
+  }
+  const int vch = a.dvp / 8;
+  for (int it = threadIdx.x; it < a.G * vch; it += 256) {
+    const int g = it / vch, d = (it % vch) * 8;
+    *reinterpret_cast<u32x4*>(vc + ((b * a.G + g) * a.S + slot) * a.dvp + d) =
+        d < a.dv ? *reinterpret_cast<const u32x4*>(yr + a.v_off + (int64_t)g * a.dv + d) : u32x4{0, 0, 0, 0};
+  }
+}
+
+// ---- RMS norm over the whole row times sigmoid(gate) --------------------------------------------
+struct GatedNormArgs {
+  int64_t W, o_ld, out_ld, g_off;
+  float eps, w_offset;
+  const float* w;
+  const float* o;
+  int out_frag;
+};
+template <typename T>
+__global__ __launch_bounds__(256) void gated_norm_kernel(const GatedNormArgs a, const RowSrc<T> g, T* out) {
+  __shared__ float red[4];
+  const int64_t row = blockIdx.x;
+  const float* o = a.o + row * a.o_ld;
+  float ss = 0.f;
+  if (a.W % 4 == 0 && a.o_ld % 4 == 0) {
+    for (int64_t i = (int64_t)threadIdx.x * 4; i < a.W; i += 1024) {
+      const f32x4 v = *reinterpret_cast<const f32x4*>(o + i);
+      ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+    }
+  } else {
+    for (int64_t i = threadIdx.x; i < a.W; i += 256) ss += o[i] * o[i];
+  }
+  const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)a.W + a.eps);
+  if (sizeof(T) == 2 && g.split <= 1 && a.W % 8 == 0 && a.o_ld % 8 == 0 && g.ld % 8 == 0 && a.g_off % 8 == 0 && a.out_ld % 8 == 0) {
+    for (int64_t i = (int64_t)threadIdx.x * 8; i < a.W; i += 2048) {
+      const f32x4 v0 = *reinterpret_cast<const f32x4*>(o + i), v1 = *reinterpret_cast<const f32x4*>(o + i + 4);
+      const f32x4 w0 = *reinterpret_cast<const f32x4*>(a.w + i), w1 = *reinterpret_cast<const f32x4*>(a.w + i + 4);
+      const u32x4 gv = *reinterpret_cast<const u32x4*>(reinterpret_cast<const uint16_t*>(g.y) + row * g.ld + a.g_off + i);
+      u32x4 p;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const float e0 = j < 2 ? v0[2 * j] : v1[2 * j - 4], e1 = j < 2 ? v0[2 * j + 1] : v1[2 * j - 3];
+        const float f0 = j < 2 ? w0[2 * j] : w1[2 * j - 4], f1 = j < 2 ? w0[2 * j + 1] : w1[2 * j - 3];
+        p[j] = pack2bf(e0 * r * (a.w_offset + f0) * sigmoid_f32(bflo(gv[j])), e1 * r * (a.w_offset + f1) * sigmoid_f32(bfhi(gv[j])));
+      }
+      *reinterpret_cast<u32x4*>(reinterpret_cast<uint16_t*>(out) + (a.out_frag ? frag_index(row, i, a.out_ld) : row * a.out_ld + i)) = p;
+    }
+    return;
+  }
+  for (int64_t i = threadIdx.x; i < a.W; i += 256)
+    st_elem(out, a.out_frag ? frag_index(row, i, a.out_ld) : row * a.out_ld + i,
+            o[i] * r * (a.w_offset + a.w[i]) * sigmoid_f32(g.get(row, a.g_off + i)));
+}
+
+// ---- gated unit on finished projections: out = gelu_tanh(y[:, :F]) * y[:, u_off : u_off + F] -----
+template <typename T>
+__global__ __launch_bounds__(256) void gelu_mul_kernel(const T* y, int64_t ld, int64_t u_off, int64_t F, T* out, int64_t out_ld) {
+  const int64_t row = blockIdx.y, i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (i < F) st_elem(out, row * out_ld + i, gelu_tanh_f32(ld_elem(y, row * ld + i)) * ld_elem(y, row * ld + u_off + i));
+}
+
+// ---- statistics and the whole-vocabulary draw over finished fp32 logits -------------------------
+struct LogitsArgs {
+  int64_t M, V;
+  const float* logits;
+  float temperature;
+  const int32_t* forbidden;
+  int n_forbidden;
+  const int32_t* targets;
+  int32_t* best_id;
+  float *best_logp, *target_logp, *lse, *entropy;
+  uint32_t key0, key1;
+  int variant;
+  const int32_t* step_ptr;
+  int32_t* draw_id;
+  float* draw_logp;
+};
+struct Best {
+  float v;
+  int i;
+};
+__device__ __forceinline__ Best better(Best a, Best b) {   // larger value, then lower index
+  return (b.v > a.v || (b.v == a.v && b.i < a.i)) ? b : a;
+}
+__device__ __forceinline__ Best block_best(Best v, Best* red) {
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) v = better(v, Best{__shfl_xor(v.v, o, 64), __shfl_xor(v.i, o, 64)});
+  __syncthreads();
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  Best r = red[0];
+  for (int w = 1; w < (int)(blockDim.x >> 6); ++w) r = better(r, red[w]);
+  return r;
+}
+__global__ __launch_bounds__(256) void logits_stats_kernel(const LogitsArgs a) {
+  __shared__ float red[4];
+  __shared__ Best bred[4];
+  const int64_t row = blockIdx.x;
+  const float* l = a.logits + row * a.V;
+  const float ninf = -__builtin_inff();
+  auto value = [&](int64_t i) {
+    for (int f = 0; f < a.n_forbidden; ++f)
+      if (a.forbidden[f] == i) return ninf;
+    return __fdiv_rn(l[i], a.temperature);
+  };
+  uint32_t ks0 = 0u, ks1 = 0u;
+  if (a.draw_id) {
+    ks1 = (uint32_t)(*a.step_ptr);
+    threefry2x32(a.key0, a.key1, ks0, ks1);
+  }
+  Best top{ninf, 0x7fffffff}, drawn{ninf, 0x7fffffff};
+  for (int64_t i = threadIdx.x; i < a.V; i += 256) {
+    const float v = value(i);
+    top = better(top, Best{v, (int)i});
+    if (a.draw_id && v != ninf)
+      drawn = better(drawn, Best{v + gumbel_from_bits(random_bits(ks0, ks1, (uint64_t)row * (uint64_t)a.V + (uint64_t)i,
+                                                                   (uint64_t)a.M * (uint64_t)a.V, a.variant)), (int)i});
+  }
+  top = block_best(top, bred);
+  if (a.draw_id) drawn = block_best(drawn, bred);
+  float se = 0.f, we = 0.f;
+  for (int64_t i = threadIdx.x; i < a.V; i += 256) {
+    const float v = value(i);
+    if (v == ninf) continue;
+    const float e = expf(v - top.v);
+    se += e;
+    we += e * v;
+  }
+  se = block_sum(se, red);
+  we = block_sum(we, red);
+  if (threadIdx.x == 0) {
+    const float lse = top.v + logf(se);
+    if (a.best_id) a.best_id[row] = top.i;
+    if (a.best_logp) a.best_logp[row] = top.v - lse;
+    if (a.target_logp) {
+      const int t = a.targets[row];
+      a.target_logp[row] = (t >= 0 && t < a.V ? value(t) : ninf) - lse;
+    }
+    if (a.lse) a.lse[row] = lse;
+    if (a.entropy) a.entropy[row] = lse - we / se;
+    if (a.draw_id) {
+      a.draw_id[row] = drawn.i;
+      if (a.draw_logp) a.draw_logp[row] = (drawn.i < a.V ? value(drawn.i) : ninf) - lse;
+    }
+  }
+}
+
+template <typename T>
+RowSrc<T> row_src(const tnx_rows_src& s) {
+  return RowSrc<T>{reinterpret_cast<const T*>(s.y), s.ws, s.split_k, s.plane, s.ld};
+}
+
+}  // namespace
+
+extern "C" int tnx_embed_rows(void* stream, int dtype, const void* table, int64_t V, int64_t D, const int32_t* ids,
+                              int64_t ids_ld, const int32_t* col_ptr, int64_t B, int64_t T, float* x, void* cat,
+                              int64_t cat_ld, int64_t cat_off, int cat_frag) {
+  TNX_REQUIRE(table && ids && x, "embed_rows: null pointer");
+  TNX_REQUIRE(V > 0 && D > 0 && B > 0 && T > 0, "embed_rows: bad shape");
+  TNX_REQUIRE(!cat || cat_ld >= cat_off + D, "embed_rows: the second copy does not fit its rows");
+  TNX_REQUIRE(dtype == TNX_BF16 || dtype == TNX_F32, "embed_rows: bad dtype %d", dtype);
+  if (dtype == TNX_BF16)
+    hipLaunchKernelGGL(embed_rows_kernel<uint16_t>, dim3((unsigned)(B * T)), dim3(256), 0, as_stream(stream), (const uint16_t*)table,
+                       V, D, ids, ids_ld, col_ptr, T, x, (uint16_t*)cat, cat_ld, cat_off, cat_frag);
+  else
+    hipLaunchKernelGGL(embed_rows_kernel<float>, dim3((unsigned)(B * T)), dim3(256), 0, as_stream(stream), (const float*)table, V, D,
+                       ids, ids_ld, col_ptr, T, x, (float*)cat, cat_ld, cat_off, cat_frag);
+  TNX_CHECK_LAUNCH("embed_rows");
+  return TNX_OK;
+}
+
+extern "C" int tnx_residual_norm(void* stream, const tnx_residual_norm_desc* d) {
+  TNX_REQUIRE(d, "residual_norm: null descriptor");
+  TNX_REQUIRE(d->M > 0 && d->D > 0 && d->D <= 16384, "residual_norm: D=%lld out of range (1..16384)", (long long)d->D);
+  TNX_REQUIRE(d->x && d->out && d->out_ld >= d->D, "residual_norm: null pointer or short output rows");
+  TNX_REQUIRE(d->mode >= 0 && d->mode <= 2, "residual_norm: bad mode %d", d->mode);
+  TNX_REQUIRE(d->mode == 0 || d->y.y || d->y.ws, "residual_norm: no incoming rows");
+  TNX_REQUIRE(d->mode != 1 || d->w_post, "residual_norm: null post-norm weight");
+  TNX_REQUIRE(d->dtype == TNX_BF16 || d->dtype == TNX_F32, "residual_norm: bad dtype %d", d->dtype);
+  ResNormArgs a;
+  a.M = d->M; a.D = d->D; a.eps = d->eps; a.w_offset = d->w_offset; a.y = d->y.y; a.ws = d->y.ws;
+  a.split = d->y.split_k < 1 ? 1 : d->y.split_k; a.plane = d->y.plane; a.y_ld = d->mode ? d->y.ld : 8; a.mode = d->mode;
+  a.w_post = d->w_post; a.x = d->x; a.w_next = d->w_next; a.out = d->out; a.out_ld = d->out_ld; a.out_frag = d->out_frag;
+  if (d->mode == 0) a.plane = 0;
+  if (d->dtype == TNX_BF16) launch_resnorm<uint16_t>(as_stream(stream), a);
+  else launch_resnorm<float>(as_stream(stream), a);
+  TNX_CHECK_LAUNCH("residual_norm");
+  return TNX_OK;
+}
+
+extern "C" int tnx_part_rope_kvwrite(void* stream, const tnx_part_rope_desc* d) {
+  TNX_REQUIRE(d, "part_rope: null descriptor");
+  TNX_REQUIRE(d->B > 0 && d->T > 0 && d->S > 0 && d->H > 0 && d->G > 0 && d->H % d->G == 0, "part_rope: bad shape");
+  TNX_REQUIRE(d->dk > 0 && d->dv > 0 && d->dkp >= d->dk && d->dvp >= d->dv, "part_rope: bad head sizes");
+  TNX_REQUIRE(d->rot_dims >= 0 && d->rot_dims % 2 == 0 && d->rot_dims <= d->dk && d->rot_dims / 2 <= kMaxHalf,
+              "part_rope: rot_dims=%d must be even, at most the head size and at most 512", d->rot_dims);
+  TNX_REQUIRE(src_given(d->y) && d->starts && d->col_ptr && d->q_out && d->kcache && d->vcache && (d->rot_dims == 0 || d->inv_freq),
+              "part_rope: null pointer");
+  TNX_REQUIRE(d->dtype == TNX_BF16 || d->dtype == TNX_F32, "part_rope: bad dtype %d", d->dtype);
+  PartRopeArgs a;
+  a.T = d->T; a.S = d->S; a.H = d->H; a.G = d->G; a.dk = d->dk; a.dv = d->dv; a.dkp = d->dkp; a.dvp = d->dvp;
+  a.half = d->rot_dims / 2; a.inv_freq = d->inv_freq; a.starts = d->starts; a.col_ptr = d->col_ptr;
+  a.k_off = d->k_off; a.v_off = d->v_off;
+  const dim3 grid((unsigned)(d->B * d->T));
+  hipStream_t st = as_stream(stream);
+  const bool vec = d->dtype == TNX_BF16 && d->y.split_k <= 1 && d->dk % 8 == 0 && d->dv % 8 == 0 && d->dkp % 8 == 0 &&
+                   d->dvp % 8 == 0 && a.half % 8 == 0 && d->k_off % 8 == 0 && d->v_off % 8 == 0 && d->y.ld % 8 == 0;
+  if (vec)
+    hipLaunchKernelGGL(part_rope_vec_kernel, grid, dim3(256), 0, st, a, (const uint16_t*)d->y.y, d->y.ld, (uint16_t*)d->q_out,
+                       (uint16_t*)d->kcache, (uint16_t*)d->vcache);
+  else if (d->dtype == TNX_BF16)
+    hipLaunchKernelGGL(part_rope_kernel<uint16_t>, grid, dim3(256), 0, st, a, row_src<uint16_t>(d->y), (uint16_t*)d->q_out,
+                       (uint16_t*)d->kcache, (uint16_t*)d->vcache);
+  else
+    hipLaunchKernelGGL(part_rope_kernel<float>, grid, dim3(256), 0, st, a, row_src<float>(d->y), (float*)d->q_out, (float*)d->kcache,
+                       (float*)d->vcache);
+  TNX_CHECK_LAUNCH("part_rope");
+  return TNX_OK;
+}
+
+extern "C" int tnx_gated_norm(void* stream, const tnx_gated_norm_desc* d) {
+  TNX_REQUIRE(d, "gated_norm: null descriptor");
+  TNX_REQUIRE(d->M > 0 && d->W > 0 && d->o && d->o_ld >= d->W && src_given(d->g) && d->w && d->out && d->out_ld >= d->W,
+              "gated_norm: null pointer or bad shape");
+  TNX_REQUIRE(d->dtype == TNX_BF16 || d->dtype == TNX_F32, "gated_norm: bad dtype %d", d->dtype);
+  GatedNormArgs a;
+  a.W = d->W; a.o_ld = d->o_ld; a.out_ld = d->out_ld; a.g_off = d->g_off; a.eps = d->eps; a.w_offset = d->w_offset;
+  a.w = d->w; a.o = d->o; a.out_frag = d->out_frag;
+  if (d->dtype == TNX_BF16)
+    hipLaunchKernelGGL(gated_norm_kernel<uint16_t>, dim3((unsigned)d->M), dim3(256), 0, as_stream(stream), a, row_src<uint16_t>(d->g),
+                       (uint16_t*)d->out);
+  else
+    hipLaunchKernelGGL(gated_norm_kernel<float>, dim3((unsigned)d->M), dim3(256), 0, as_stream(stream), a, row_src<float>(d->g),
+                       (float*)d->out);
+  TNX_CHECK_LAUNCH("gated_norm");
+  return TNX_OK;
+}
+
+extern "C" int tnx_gelu_mul(void* stream, int dtype, const void* y, int64_t ld, int64_t up_off, int64_t M, int64_t F, void* out,
+                            int64_t out_ld) {
+  TNX_REQUIRE(y && out && M > 0 && F > 0 && ld >= up_off + F && out_ld >= F, "gelu_mul: null pointer or bad shape");
+  TNX_REQUIRE(dtype == TNX_BF16 || dtype == TNX_F32, "gelu_mul: bad dtype %d", dtype);
+  for (int64_t r0 = 0; r0 < M; r0 += 65535) {
+    const int64_t n = M - r0 < 65535 ? M - r0 : 65535;
+    const dim3 grid((unsigned)cdiv(F, 256), (unsigned)n);
+    if (dtype == TNX_BF16)
+      hipLaunchKernelGGL(gelu_mul_kernel<uint16_t>, grid, dim3(256), 0, as_stream(stream), (const uint16_t*)y + r0 * ld, ld, up_off, F,
+                         (uint16_t*)out + r0 * out_ld, out_ld);
+    else
+      hipLaunchKernelGGL(gelu_mul_kernel<float>, grid, dim3(256), 0, as_stream(stream), (const float*)y + r0 * ld, ld, up_off, F,
+                         (float*)out + r0 * out_ld, out_ld);
+  }
+  TNX_CHECK_LAUNCH("gelu_mul");
+  return TNX_OK;
+}
+
+extern "C" int tnx_logits_stats(void* stream, const tnx_logits_desc* d) {
+  TNX_REQUIRE(d && d->logits && d->M > 0 && d->V > 0 && d->V < (1LL << 31), "logits_stats: null pointer or bad shape");
+  TNX_REQUIRE(!d->target_logp || d->targets, "logits_stats: target log-probabilities need targets");
+  LogitsArgs a;
+  memset(&a, 0, sizeof(a));
+  a.M = d->M; a.V = d->V; a.logits = d->logits; a.temperature = d->temperature == 0.f ? 1.0f : d->temperature;
+  a.forbidden = d->forbidden; a.n_forbidden = d->forbidden ? d->n_forbidden : 0; a.targets = d->targets;
+  a.best_id = d->best_id; a.best_logp = d->best_logp; a.target_logp = d->target_logp; a.lse = d->lse; a.entropy = d->entropy;
+  if (d->draw_id) {
+    TNX_REQUIRE(d->draw_step_ptr && (d->draw_rng_variant == 0 || d->draw_rng_variant == 1) && d->temperature > 0.f,
+                "logits_stats: the draw needs a step pointer, a known rng_variant and a positive temperature");
+    a.key0 = d->draw_key0; a.key1 = d->draw_key1; a.variant = d->draw_rng_variant; a.step_ptr = d->draw_step_ptr;
+    a.draw_id = d->draw_id; a.draw_logp = d->draw_logp;
+  }
+  hipLaunchKernelGGL(logits_stats_kernel, dim3((unsigned)d->M), dim3(256), 0, as_stream(stream), a);
+  TNX_CHECK_LAUNCH("logits_stats");
+  return TNX_OK;
+}

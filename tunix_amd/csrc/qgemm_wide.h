@@ -543,7 +543,26 @@ void qgemm_wide_kernel(const QLArgs a, const WideHead h) {
   // The bf16 tile goes through LDS (row stride cols + 8 elements) and leaves as 16-byte chunks
   // of whole rows.  A lane holds, for row rt * 32 + l % 32 and group cg, the columns
   // 8 b + 4 (l / 32) + e of the group in register 4 b + e.
-  const bool mul = a.epilogue == TNX_EPI_SILU_MUL || a.epilogue == TNX_EPI_GELU_MUL;
+  const bool mul = a.epilogue == TNX_EPI_SILU_MUL || a.epilogue == TNX_EPI_GELU_MUL || a.epilogue == kEpiGeluMulF32;
+  if constexpr (PRE) {
+    if (a.epilogue == TNX_EPI_F32) {   // fp32 results leave from the accumulators, 16 bytes per lane
+      float* y = reinterpret_cast<float*>(a.y);
+#pragma unroll
+      for (int cg = 0; cg < CG; ++cg)
+#pragma unroll
+        for (int rt = 0; rt < RT; ++rt)
+#pragma unroll
+          for (int b = 0; b < 4; ++b) {
+            const int64_t col = (int64_t)ntile * kWideCols + wn * 64 + cg * 32 + 8 * b + 4 * lh;
+            float* o = y + (m0 + rt * 32 + l32) * a.ldy + col;
+            if (rt * 32 + l32 < rows_here)
+#pragma unroll
+              for (int e = 0; e < 4; ++e)
+                if (col + e < a.N) o[e] = acc[rt][cg][4 * b + e];
+          }
+      return;
+    }
+  }
   const int cols = mul ? kWideCols / 2 : kWideCols;      // output columns of the work-group
   const int sld = cols + 8;
   const uint32_t stage = 0;   // 128 rows x (256 + 8) columns: over both tiles and into the table, all dead now
@@ -558,6 +577,12 @@ void qgemm_wide_kernel(const QLArgs a, const WideHead h) {
           float v[4];
 #pragma unroll
           for (int e = 0; e < 4; ++e) {
+            if (PRE && a.epilogue == kEpiGeluMulF32) {
+              const float z = acc[rt][cg][4 * b + e];
+              v[e] = 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))) *
+                     acc[rt][cg][4 * (b + 2) + e];
+              continue;
+            }
             const float g = rbf(acc[rt][cg][4 * b + e]);
             const float u = rbf(acc[rt][cg][4 * (b + 2) + e]);
             const float act = a.epilogue == TNX_EPI_SILU_MUL ? silu_bf16(g) : gelu_tanh_bf16(g);
@@ -735,12 +760,12 @@ void qgemm_wide_kernel(const QLArgs a, const WideHead h) {
     return;
   }
   {
-    const int64_t ldy = mul ? a.N / 2 : a.N;
+    const int64_t width = mul ? a.N / 2 : a.N, ldy = a.ldy > 0 ? a.ldy : width;
     const int64_t col0 = (int64_t)ntile * cols;
     const int chunks = cols / 8;                       // 16-byte chunks per row: 16 | 32
     const int ch = tid % chunks, r0 = tid / chunks, rstep = 256 / chunks;
     uint16_t* y = reinterpret_cast<uint16_t*>(a.y);
-    const bool col_ok = col0 + ch * 8 + 8 <= ldy;
+    const bool col_ok = col0 + ch * 8 + 8 <= width;
     for (int row = r0; row < kWideRows; row += rstep) {
       if (row >= rows_here || !col_ok) continue;
       u32x4 v = lds_ld128(stage + (uint32_t)((row * sld + ch * 8) * 2));

@@ -41,7 +41,12 @@ struct QLArgs {
   float* next_tpart;
   // optional: the weights converted once into the many-row kernel's fragments (tnx_qw_expand)
   const uint16_t* w_pre;
+  // row stride of the stored output in elements, 0: the output's width (many-row kernel only)
+  int64_t ldy;
 };
+// gate | up with the activation and the product in fp32 and one rounding (dense-weight decoders;
+// many-row kernel only)
+constexpr int kEpiGeluMulF32 = 16;
 // Second argument of the 128 x 256 kernel: with `part` set it reduces its tile to lm_head
 // statistics instead of storing it.
 struct WideHead {
@@ -525,6 +530,7 @@ QLArgs to_args(const tnx_qlinear_desc* d) {
   a.offsets = nullptr; a.sorted_route = nullptr; a.x_div = 1; a.codes_stride = 0; a.scales_stride = 0;
   a.next_a_t = d->next_a_t; a.next_rank = d->next_rank; a.next_tpart = d->next_tpart;
   a.w_pre = d->w_expanded;
+  a.ldy = 0;
   return a;
 }
 
@@ -993,6 +999,18 @@ int tnx_internal_wide_head(hipStream_t st, const tnx_lmhead_desc* d, float tempe
     h.step_ptr = d->draw_step_ptr;
   }
   return scales_per_tile(a.group) == 2 ? launch_qgemm_wide<2>(st, a, h) : launch_qgemm_wide<4>(st, a, h);
+}
+
+// A dense linear over many rows on the 128 x 256 kernel, from its fragment-order weights
+// (tnx_dense_expand).  The caller has checked the shapes.
+int tnx_internal_wide_dense(hipStream_t st, int64_t M, int64_t K, int64_t N, const uint16_t* x, const uint16_t* w,
+                            int epilogue, void* y, int64_t ldy) {
+  QLArgs a;
+  memset(&a, 0, sizeof(a));
+  a.M = M; a.K = K; a.N = N; a.group = KTILE; a.x = x; a.w_pre = w; a.x_div = 1;
+  a.epilogue = epilogue == TNX_EPI_GELU_MUL ? kEpiGeluMulF32 : epilogue;
+  a.y = y; a.ldy = ldy; a.split_k = 1; a.ktiles_per_split = (int)(K / KTILE);
+  return launch_qgemm_wide<2>(st, a);
 }
 
 extern "C" int tnx_splitk_finish(void* stream, const tnx_qlinear_desc* d) {

@@ -3,7 +3,7 @@ with the jitted prefill / while_loop decode replaced by libtunix_hip.so kernels.
 
 Same call contract as the reference: `Sampler(transformer, tokenizer, cache_config)` and
 `sampler(input_strings, max_generation_steps, ...) -> SamplerOutput`.  `transformer` is a
-`tunix_amd.model.QLoRAModel`.  One decode step is captured into a HIP graph and replayed: the
+`tunix_amd.model.QLoRAModel` or a `tunix_amd.stack_model.StackModel`.  One decode step is captured into a HIP graph and replayed: the
 step counter, positions and token buffer live in device memory, so no host round trip happens
 inside the loop.
 """
@@ -16,7 +16,6 @@ import numpy as np
 import torch
 
 from .. import ops
-from ..model import QLoRAModel, Runner
 from . import utils
 from .base_sampler import SamplerOutput
 
@@ -26,9 +25,9 @@ class CacheConfig:
   """Configuration for the KV cache (tunix/common/configs.py:60-67)."""
 
   cache_size: int
-  num_layers: int
-  num_kv_heads: int
-  head_dim: int
+  num_layers: int = 0       # (the model itself says what its layers keep: `cache_specs`)
+  num_kv_heads: int = 0
+  head_dim: int = 0
 
 
 def _threefry_seed(seed: int) -> tuple[int, int]:
@@ -62,10 +61,14 @@ def sampling_plan(top_k: int | None, top_p: float, vocab_size: int) -> tuple[int
 class _SamplingState:
   """Device-resident counterpart of _SamplingState (tunix/generate/sampler.py:49-102)."""
 
-  def __init__(self, model: QLoRAModel, all_input_ids: np.ndarray, total_sampling_steps: int,
-               cache_size: int, pad_id: int, include_logits: bool, include_logprobs: bool):
+  def __init__(self, model, all_input_ids: np.ndarray, total_sampling_steps: int,
+               cache_size: int, pad_id: int, include_logits: bool, include_logprobs: bool,
+               lengths: Sequence[int] | None = None):
+    """lengths: tokens of each left-padded prompt (default: what follows the leading pad ids)."""
     cfg, dev = model.cfg, model.device
     B, P = all_input_ids.shape
+    if lengths is None:
+      lengths = [P - int(np.argmax(np.append(r != pad_id, True))) for r in all_input_ids]
     L = total_sampling_steps
     tb = np.full((B, L), pad_id, dtype=np.int32)
     tb[:, :P] = all_input_ids
@@ -78,19 +81,27 @@ class _SamplingState:
     self.done = torch.zeros(B, dtype=torch.int32, device=dev)
     # decoding_step: column of the last committed token
     self.step = torch.full((1,), P - 1, dtype=torch.int32, device=dev)
-    shape = (B, cfg.num_kv_heads, cache_size, cfg.head_dim)
-    self.kcache = [torch.zeros(shape, dtype=torch.bfloat16, device=dev) for _ in range(cfg.num_layers)]
-    self.vcache = [torch.zeros(shape, dtype=torch.bfloat16, device=dev) for _ in range(cfg.num_layers)]
+    # column of each row's first token
+    self.starts = torch.tensor([P - n for n in lengths], dtype=torch.int32, device=dev)
+    self.cache = model.new_cache(B, cache_size)
     self.logits_buffer = (torch.zeros(B, L, cfg.vocab_size, dtype=torch.float32, device=dev)
                           if include_logits else None)
     self.logprobs_buffer = (torch.zeros(B, L, dtype=torch.float32, device=dev)
                             if include_logprobs else None)
 
+  @property
+  def kcache(self) -> list:
+    return self.cache.kcache
+
+  @property
+  def vcache(self) -> list:
+    return self.cache.vcache
+
 
 class Sampler:
   """Sampler for transformer model."""
 
-  def __init__(self, transformer: QLoRAModel, tokenizer, cache_config: CacheConfig,
+  def __init__(self, transformer, tokenizer, cache_config: CacheConfig,
                use_graph: bool = True, prefill_rows: int = 16384):
     self._transformer = transformer
     self.tokenizer = tokenizer
@@ -101,7 +112,7 @@ class Sampler:
     self.last_stats: dict = {}
 
   @property
-  def transformer(self) -> QLoRAModel:
+  def transformer(self):
     return self._transformer
 
   @property
@@ -118,7 +129,7 @@ class Sampler:
 
   @property
   def dtype(self):
-    return torch.bfloat16
+    return self._transformer.dtype
 
   def tokenize(self, input_string) -> np.ndarray:
     """BOS + ids of one prompt (sampler.py:465-472); id sequences pass through unchanged."""
@@ -133,7 +144,7 @@ class Sampler:
     return np.asarray(ids, dtype=np.int32)
 
   # ---- one sampling step on the device -------------------------------------------------------
-  def _sample(self, runner: Runner, x, st: _SamplingState, mode: dict):
+  def _sample(self, runner, x, st: _SamplingState, mode: dict):
     """lm_head + sampling + bookkeeping for the B rows in x (sampler.py:474-552)."""
     want_lp = st.logprobs_buffer is not None
     if mode["name"] == "greedy":
@@ -165,22 +176,29 @@ class Sampler:
       ids, lp = mode["ids"], (mode["logp"] if want_lp else None)
     ops.sample_commit(ids, lp, st.token_buffer, st.logprobs_buffer, st.done, mode["eos"], st.step)
 
-  def _prefill(self, st: _SamplingState, runner_dec: Runner, mode: dict, return_logits: bool):
-    """sampler.py:554-673: forward over the padded prompts, fill the cache, sample one token."""
-    model = self._transformer
+  def forward_prompt(self, st: _SamplingState, on_rows):
+    """Forward over the padded prompts (sampler.py:554-616), filling the cache, in groups of rows:
+    on_rows(b0, nb, runner, xn) gets the final hidden states [nb * P, width] of rows b0 .. b0 + nb - 1."""
     B, P = st.token_buffer.shape[0], st.num_input_tokens
-    S = self.cache_config.cache_size
     rows = max(1, min(B, self.prefill_rows // max(P, 1)))
-    pad = self.tokenizer.pad_id()
-    runner = Runner(model, rows, P, S, pad, kv_chunk=0)
-    D = model.cfg.embed_dim
+    runner = self._transformer.new_runner(rows, P, st.cache.S, self.tokenizer.pad_id(), kv_chunk=0)
     for b0 in range(0, B, rows):
       nb = min(rows, B - b0)
-      kc = [k[b0:b0 + nb] for k in st.kcache]
-      vc = [v[b0:b0 + nb] for v in st.vcache]
-      xn = runner.forward_hidden(st.token_buffer[b0:b0 + nb], st.positions[b0:b0 + nb],
-                                 runner.zero, kc, vc, B=nb, T=P)
-      runner_dec.xlast[b0:b0 + nb].copy_(xn[: nb * P].view(nb, P, D)[:, P - 1])
+      xn = runner.forward_hidden(st.token_buffer[b0:b0 + nb], st.positions[b0:b0 + nb], runner.zero,
+                                 st.cache.rows(b0, nb), B=nb, T=P, starts=st.starts[b0:b0 + nb])
+      on_rows(b0, nb, runner, xn)
+
+  def forward_step(self, runner, st: _SamplingState):
+    """Forward over the one token per row in column `st.step`, from the cached state."""
+    return runner.forward_hidden(st.token_buffer, st.positions, st.step, st.cache, starts=st.starts)
+
+  def _prefill(self, st: _SamplingState, runner_dec, mode: dict, return_logits: bool):
+    """sampler.py:554-673: forward over the padded prompts, fill the cache, sample one token."""
+    model = self._transformer
+    P = st.num_input_tokens
+
+    def on_rows(b0, nb, runner, xn):
+      runner_dec.xlast[b0:b0 + nb].copy_(xn[: nb * P].view(nb, P, -1)[:, P - 1])
       if return_logits:
         # logits of every prompt position go to logits_buffer[:, 1:P+1] (sampler.py:617-625)
         part = torch.empty(nb * P * runner.nvb * 4, dtype=torch.float32, device=model.device)
@@ -191,13 +209,13 @@ class Sampler:
         L = st.total_sampling_steps
         n_fit = min(P, L - 1)
         st.logits_buffer[b0:b0 + nb, 1:1 + n_fit].copy_(lg[:, :n_fit])
-    del runner
+
+    self.forward_prompt(st, on_rows)
     self._sample(runner_dec, runner_dec.xlast, st, mode)
 
-  def _decode_step(self, runner: Runner, st: _SamplingState, mode: dict):
+  def _decode_step(self, runner, st: _SamplingState, mode: dict):
     """sampler.py:692-736: one token per row from the cached state."""
-    xn = runner.forward_hidden(st.token_buffer, st.positions, st.step, st.kcache, st.vcache)
-    self._sample(runner, xn, st, mode)
+    self._sample(runner, self.forward_step(runner, st), st, mode)
 
   # ---- public entry --------------------------------------------------------------------------
   def __call__(
@@ -250,7 +268,7 @@ class Sampler:
     B = all_input_ids.shape[0]
     S = self.cache_config.cache_size
     st = _SamplingState(model, all_input_ids, total_sampling_steps, S, pad, return_logits,
-                        return_logprobs)
+                        return_logprobs, lengths=[len(x) for x in tokens])
     mode = {"name": "greedy", "forbidden": None,
             "eos": torch.tensor(eos_ids, dtype=torch.int32, device=dev)}
     if forbidden:
@@ -266,14 +284,14 @@ class Sampler:
                   ws=torch.empty(max(ws_bytes // 4, 1), dtype=torch.float32, device=dev),
                   ids=torch.empty(B, dtype=torch.int32, device=dev),
                   logp=torch.empty(B, dtype=torch.float32, device=dev))
-      if path == "topk" and ops.sample_topk_head_ok(cfg.vocab_size, k):
+      if path == "topk" and getattr(model, "block_head", True) and ops.sample_topk_head_ok(cfg.vocab_size, k):
         mode["head_lse"] = torch.empty(B, dtype=torch.float32, device=dev)
       if k == 0 and top_p >= 1.0:
         mode["part_draw"] = torch.empty(B * ops.lmhead_nblocks(cfg.vocab_size) * 3, dtype=torch.float32,
                                         device=dev)
     in_head_draw = mode["name"] == "top_p" and mode["top_k"] == 0 and mode["top_p"] >= 1.0
     need_logits = return_logits or (mode["name"] == "top_p" and not in_head_draw)
-    runner = Runner(model, B, 1, S, pad, want_logits=need_logits)
+    runner = model.new_runner(B, 1, S, pad, want_logits=need_logits)
 
     ev = [torch.cuda.Event(enable_timing=True) for _ in range(3)]
     ev[0].record()

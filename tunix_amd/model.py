@@ -15,6 +15,7 @@ import torch
 
 from . import _lib as L
 from . import ops
+from .cache import KVSpec, SequenceCache
 from .config import ModelConfig
 
 _NORM = {"llama3": L.TNX_NORM_LLAMA, "qwen3": L.TNX_NORM_QWEN3, "gemma3": L.TNX_NORM_GEMMA3}
@@ -261,6 +262,19 @@ class QLoRAModel:
         self.head_expanded = ops.dense_expand(dense_head)
       torch.cuda.synchronize(dev)
 
+  # ---- what the sampler asks of a model ------------------------------------------------------
+  dtype = torch.bfloat16
+
+  def cache_specs(self) -> list:
+    cfg = self.cfg
+    return [KVSpec(cfg.num_kv_heads, cfg.head_dim, cfg.head_dim)] * cfg.num_layers
+
+  def new_cache(self, B: int, S: int, shared: bool = False) -> SequenceCache:
+    return SequenceCache(self.cache_specs(), B, S, self.device, shared=shared)
+
+  def new_runner(self, B: int, T: int, S: int, pad_id: int, **kw) -> "Runner":
+    return Runner(self, B, T, S, pad_id, **kw)
+
   # weight sync: LoRA-only replacement (tunix/generate/sampler.py:333-352)
   def update_lora(self, new_lora: dict):
     expected = set()
@@ -390,7 +404,70 @@ class QLoRAModel:
     return {"quantized": q, "lora": lora, "head": head}
 
 
-class Runner:
+class HeadRunner:
+  """The lm_head half of a runner: statistics, sampling inputs and logits of finished hidden rows."""
+
+  def _init_head(self, B: int, width: int, dtype, want_logits: bool):
+    cfg, dev = self.model.cfg, self.model.device
+    self.nvb = ops.lmhead_nblocks(cfg.vocab_size)
+    self.head_rows = B
+    self.head_width = width
+    self.xlast = torch.empty(B, width, dtype=dtype, device=dev)
+    self.part = torch.empty(B * self.nvb * 4, dtype=torch.float32, device=dev)
+    self.best_id = torch.empty(B, dtype=torch.int32, device=dev)
+    self.best_logp = torch.empty(B, dtype=torch.float32, device=dev)
+    self.logits = (torch.empty(B, cfg.vocab_size, dtype=torch.float32, device=dev)
+                   if want_logits else None)
+
+  # whether run_head leaves the per-block statistics that tnx_sample_topk_head reads
+  block_stats = True
+
+  def head_desc(self, x, rows, part, temperature=1.0, targets=None, best_id=None, best_logp=None,
+                target_logp=None, lse=None, logits_out=None, forbidden=None, entropy=None,
+                part_entropy=None, draw=None, logits_fp32=False) -> L.LmHeadDesc:
+    cfg, m = self.cfg, self.model
+    d = L.LmHeadDesc()
+    d.M, d.D, d.V = rows, self.head_width, cfg.vocab_size
+    d.x = x.data_ptr()
+    if m.head is not None:
+      f = m.head
+      d.codes, d.scales, d.group, d.qtype = f.codes.data_ptr(), f.scales.data_ptr(), f.group, f.qtype
+      if f.expanded is not None:
+        d.w_expanded = f.expanded.data_ptr()
+      if f.has_lora:
+        d.lora_rank, d.t, d.t_ld = f.rp, self.t.data_ptr(), self.t.shape[1]
+        d.lora_b, d.lora_scale = f.b_t.data_ptr(), f.lora_scale
+    else:
+      d.w_bf16 = (m.head_w if m.head_w is not None else m.embed).data_ptr()
+      if m.head_expanded is not None:
+        d.w_expanded = m.head_expanded.data_ptr()
+    d.temperature = float(temperature)
+    d.logits_fp32 = 1 if logits_fp32 else 0
+    if forbidden is not None:
+      d.forbidden, d.n_forbidden = forbidden.data_ptr(), forbidden.numel()
+    for name, tns in (("targets", targets), ("best_id", best_id), ("best_logp", best_logp),
+                      ("target_logp", target_logp), ("lse", lse), ("logits_out", logits_out),
+                      ("entropy", entropy), ("part_entropy", part_entropy)):
+      if tns is not None:
+        setattr(d, name, tns.data_ptr())
+    d.part = part.data_ptr()
+    if draw is not None:  # whole-vocabulary categorical draw inside the head
+      d.part_draw = draw["part"].data_ptr()
+      d.draw_key0, d.draw_key1 = int(draw["key"][0]), int(draw["key"][1])
+      d.draw_rng_variant, d.draw_step_ptr = int(draw["variant"]), draw["step"].data_ptr()
+      d.draw_id = draw["ids"].data_ptr()
+      if draw.get("logp") is not None:
+        d.draw_logp = draw["logp"].data_ptr()
+    return d
+
+  def run_head(self, x, rows, **kw):
+    m = self.model
+    if m.head is not None and m.head.has_lora:
+      ops.lora_down(x, m.head.a_t, self.t, M=rows)
+    ops.lmhead(self.head_desc(x, rows, self.part, **kw))
+
+
+class Runner(HeadRunner):
   """Workspaces + the kernel sequence for up to `max_rows` = B*T token rows.
 
   State tensors (token buffer, positions, KV cache, step counter) are owned by the caller and
@@ -460,15 +537,7 @@ class Runner:
     nb = ops.attn_ws_bytes(B, T, S, cfg.num_heads, cfg.head_dim, kv_chunk)
     self.attn_ws = torch.empty(max(nb // 4, 1), dtype=torch.float32, device=dev)
     self.zero = torch.zeros(1, dtype=torch.int32, device=dev)
-    # head
-    self.nvb = ops.lmhead_nblocks(cfg.vocab_size)
-    self.head_rows = B
-    self.xlast = torch.empty(B, D, dtype=bf, device=dev)
-    self.part = torch.empty(B * self.nvb * 4, dtype=torch.float32, device=dev)
-    self.best_id = torch.empty(B, dtype=torch.int32, device=dev)
-    self.best_logp = torch.empty(B, dtype=torch.float32, device=dev)
-    self.logits = (torch.empty(B, cfg.vocab_size, dtype=torch.float32, device=dev)
-                   if want_logits else None)
+    self._init_head(B, D, bf, want_logits)
 
   # ---- building blocks -----------------------------------------------------------------------
   def _split_k(self, f: FusedLinear, M: int) -> int:
@@ -547,10 +616,11 @@ class Runner:
     ops.rmsnorm_pair(w, self.h, w2, self.xn, cfg.norm_eps, _NORM[cfg.family], M, cfg.embed_dim,
                      res_post=self.h, **kw)
 
-  def forward_hidden(self, tokens, positions, col_ptr, kcache, vcache, B=None, T=None, segment_ids=None):
+  def forward_hidden(self, tokens, positions, col_ptr, cache, B=None, T=None, segment_ids=None, starts=None):
     """Runs all layers for tokens[b, col .. col+T) of each row; leaves the final-normed hidden
-    state in self.xn[:B*T].  kcache/vcache: lists of [B,Hkv,S,dh] tensors.  segment_ids (int32,
-    the shape of `tokens`): a packed batch, attention stays inside a token's own segment."""
+    state in self.xn[:B*T].  cache: a SequenceCache of [B,Hkv,S,dh] slabs.  segment_ids (int32,
+    the shape of `tokens`): a packed batch, attention stays inside a token's own segment.
+    starts: not read here, padding is told by its token id."""
     if segment_ids is not None and (tuple(segment_ids.shape) != tuple(tokens.shape)
                                     or segment_ids.dtype != torch.int32 or not segment_ids.is_contiguous()):
       raise ValueError("segment_ids must be a contiguous int32 tensor of the token buffer's shape")
@@ -568,6 +638,7 @@ class Runner:
       ops.rope_table(positions, col_ptr, B, m.layers[0]["timescale"], cfg.head_dim, self.rope_sin, self.rope_cos)
     xn_ready = False   # gemma3: the block before has already normed the residual stream into self.xn
     for i, ly in enumerate(m.layers):
+      kv = cache.entries[i]
       if not xn_ready:
         self.norm_after(pending, ly["attn_norm"], M)
       pending, xn_ready = 1, False
@@ -593,7 +664,7 @@ class Runner:
         if qkv_split > 1:  # the rope kernel sums the partial planes itself
           rd.qkv_ws, rd.split_k = self.splitk_ws.data_ptr(), qkv_split
         rd.col_ptr = col_ptr.data_ptr()
-        rd.q_out, rd.kcache, rd.vcache = self.q.data_ptr(), kcache[i].data_ptr(), vcache[i].data_ptr()
+        rd.q_out, rd.kcache, rd.vcache = self.q.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr()
         ops.rope_kvwrite(rd)
       ad = L.AttnDesc()
       ad.B, ad.T, ad.S = B, T, self.S
@@ -601,7 +672,7 @@ class Runner:
       ad.scale = 0.0 if cfg.family == "gemma3" else cfg.head_dim ** -0.5
       ad.window = cfg.sliding_window if cfg.is_local_layer(i) else 0
       ad.pad_id = self.pad_id
-      ad.q, ad.kcache, ad.vcache = self.q.data_ptr(), kcache[i].data_ptr(), vcache[i].data_ptr()
+      ad.q, ad.kcache, ad.vcache = self.q.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr()
       ad.tokens, ad.tok_ld, ad.col_ptr = tokens.data_ptr(), tokens.shape[1], col_ptr.data_ptr()
       ad.kv_chunk = self.kv_chunk if T == 1 else 0
       if segment_ids is not None:
@@ -668,47 +739,3 @@ class Runner:
       return _MOE_PENDING
     ops.moe_combine(self.y_route, self.topk_w, M, k, cfg.embed_dim, self.h, self.h)
     return 1
-
-  def head_desc(self, x, rows, part, temperature=1.0, targets=None, best_id=None, best_logp=None,
-                target_logp=None, lse=None, logits_out=None, forbidden=None, entropy=None,
-                part_entropy=None, draw=None, logits_fp32=False) -> L.LmHeadDesc:
-    cfg, m = self.cfg, self.model
-    d = L.LmHeadDesc()
-    d.M, d.D, d.V = rows, cfg.embed_dim, cfg.vocab_size
-    d.x = x.data_ptr()
-    if m.head is not None:
-      f = m.head
-      d.codes, d.scales, d.group, d.qtype = f.codes.data_ptr(), f.scales.data_ptr(), f.group, f.qtype
-      if f.expanded is not None:
-        d.w_expanded = f.expanded.data_ptr()
-      if f.has_lora:
-        d.lora_rank, d.t, d.t_ld = f.rp, self.t.data_ptr(), self.t.shape[1]
-        d.lora_b, d.lora_scale = f.b_t.data_ptr(), f.lora_scale
-    else:
-      d.w_bf16 = (m.head_w if m.head_w is not None else m.embed).data_ptr()
-      if m.head_expanded is not None:
-        d.w_expanded = m.head_expanded.data_ptr()
-    d.temperature = float(temperature)
-    d.logits_fp32 = 1 if logits_fp32 else 0
-    if forbidden is not None:
-      d.forbidden, d.n_forbidden = forbidden.data_ptr(), forbidden.numel()
-    for name, tns in (("targets", targets), ("best_id", best_id), ("best_logp", best_logp),
-                      ("target_logp", target_logp), ("lse", lse), ("logits_out", logits_out),
-                      ("entropy", entropy), ("part_entropy", part_entropy)):
-      if tns is not None:
-        setattr(d, name, tns.data_ptr())
-    d.part = part.data_ptr()
-    if draw is not None:  # whole-vocabulary categorical draw inside the head
-      d.part_draw = draw["part"].data_ptr()
-      d.draw_key0, d.draw_key1 = int(draw["key"][0]), int(draw["key"][1])
-      d.draw_rng_variant, d.draw_step_ptr = int(draw["variant"]), draw["step"].data_ptr()
-      d.draw_id = draw["ids"].data_ptr()
-      if draw.get("logp") is not None:
-        d.draw_logp = draw["logp"].data_ptr()
-    return d
-
-  def run_head(self, x, rows, **kw):
-    m = self.model
-    if m.head is not None and m.head.has_lora:
-      ops.lora_down(x, m.head.a_t, self.t, M=rows)
-    ops.lmhead(self.head_desc(x, rows, self.part, **kw))

@@ -301,3 +301,67 @@ def logp_drift_static(rollout_logp, trainer_logp, mask, out5):
 def fill_u32(t: torch.Tensor, value: int = 0):
   assert t.element_size() == 4
   L.check(L.lib().tnx_fill_u32(_stream(), _ptr(t), t.numel(), value), "tnx_fill_u32")
+
+
+# ---- decoders with dense weights ----------------------------------------------------------------
+DTYPES = {torch.bfloat16: L.TNX_BF16, torch.float32: L.TNX_F32}
+
+
+def dense_linear(desc: L.DenseDesc):
+  L.check(L.lib().tnx_dense_linear(_stream(), C.byref(desc)), "tnx_dense_linear")
+
+
+def embed_rows(table, ids, col_ptr, B, T, V, D, x, cat=None, cat_off=0, cat_frag=False):
+  """x fp32 [B*T, D] = rows of `table` [V, D]; cat: a second copy in the table's dtype."""
+  L.check(L.lib().tnx_embed_rows(_stream(), DTYPES[table.dtype], _ptr(table), V, D, _ptr(ids), ids.shape[1],
+                                 _ptr(col_ptr), B, T, _ptr(x), _ptr(cat), 0 if cat is None else cat.shape[1], cat_off,
+                                 1 if cat_frag else 0), "tnx_embed_rows")
+
+
+def rows_src(y=None, ws=None, split_k=1, plane=0, ld=0) -> L.RowsSrc:
+  """A linear's output for its reader: finished rows y, or fp32 partial planes in ws."""
+  s = L.RowsSrc()
+  s.y, s.ws, s.split_k, s.plane, s.ld = _ptr(y), _ptr(ws), split_k, plane, ld
+  return s
+
+
+def residual_norm(desc: L.ResidualNormDesc):
+  L.check(L.lib().tnx_residual_norm(_stream(), C.byref(desc)), "tnx_residual_norm")
+
+
+def part_rope_kvwrite(desc: L.PartRopeDesc):
+  L.check(L.lib().tnx_part_rope_kvwrite(_stream(), C.byref(desc)), "tnx_part_rope_kvwrite")
+
+
+def sink_attn_pad(dim: int, value: bool, dtype) -> int:
+  """Row length of a key (value) cache for heads of this size: what the MFMA kernels take."""
+  return int(L.lib().tnx_sink_attn_pad(dim, 1 if value else 0)) if dtype == torch.bfloat16 else dim
+
+
+def sink_attn_ws_bytes(B, T, S, H, dvp, kv_chunk) -> int:
+  return int(L.lib().tnx_sink_attn_ws_bytes(B, T, S, H, dvp, kv_chunk))
+
+
+def sink_attn(desc: L.SinkAttnDesc):
+  L.check(L.lib().tnx_sink_attn(_stream(), C.byref(desc)), "tnx_sink_attn")
+
+
+def lightning_ws_bytes(B, T, H, dk, dv) -> int:
+  return int(L.lib().tnx_lightning_ws_bytes(B, T, H, dk, dv))
+
+
+def lightning(desc: L.LightningDesc):
+  L.check(L.lib().tnx_lightning(_stream(), C.byref(desc)), "tnx_lightning")
+
+
+def gated_norm(desc: L.GatedNormDesc):
+  L.check(L.lib().tnx_gated_norm(_stream(), C.byref(desc)), "tnx_gated_norm")
+
+
+def gelu_mul(y, up_off, M, F, out):
+  L.check(L.lib().tnx_gelu_mul(_stream(), DTYPES[y.dtype], _ptr(y), y.shape[1], up_off, M, F, _ptr(out), out.shape[1]),
+          "tnx_gelu_mul")
+
+
+def logits_stats(desc: L.LogitsDesc):
+  L.check(L.lib().tnx_logits_stats(_stream(), C.byref(desc)), "tnx_logits_stats")

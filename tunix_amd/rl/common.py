@@ -18,7 +18,7 @@ import numpy as np
 import torch
 
 from .. import ops
-from ..model import QLoRAModel, Runner
+from ..model import QLoRAModel
 
 
 def selective_log_softmax(logits: torch.Tensor, input_ids: torch.Tensor) -> torch.Tensor:
@@ -100,24 +100,25 @@ def compute_per_token_logps(model: QLoRAModel, prompt_tokens, completion_tokens,
   cfg = model.cfg
   temp = 1.0 if temperature in (0.0, 1.0) else float(temperature)
   rows_b = max(1, min(B, max_rows // Ltot))
-  runner = Runner(model, rows_b, Ltot, Ltot, pad_id, kv_chunk=0)
-  # the cache is scratch here: every layer writes its keys / values and reads them back
-  # within the same pass, so one pair of buffers serves all layers
-  kc = torch.empty(rows_b, cfg.num_kv_heads, Ltot, cfg.head_dim, dtype=torch.bfloat16, device=dev)
-  vc = torch.empty_like(kc)
+  runner = model.new_runner(rows_b, Ltot, Ltot, pad_id, kv_chunk=0)
+  # the cache is scratch here: every layer writes what it keeps and reads it back within the same
+  # pass, so layers of one kind share their buffers
+  cache = model.new_cache(rows_b, Ltot, shared=True)
+  # column of each row's first token: behind the prompt's leading padding
+  starts = torch.cumprod((ids == pad_id).to(torch.int32), dim=1).sum(dim=1).to(torch.int32)
   head_rows = rows_b * T if chunk_size <= 0 else rows_b * min(T, chunk_size)
   head_rows = min(head_rows, 8192)
   part = torch.empty(head_rows * runner.nvb * 4, dtype=torch.float32, device=dev)
   runner.part = part
-  xsel = torch.empty(rows_b * T, cfg.embed_dim, dtype=torch.bfloat16, device=dev)
+  xsel = torch.empty(rows_b * T, runner.xn.shape[1], dtype=runner.xn.dtype, device=dev)
   out = torch.empty(B, T, dtype=torch.float32, device=dev)
   ent = torch.empty(B, T, dtype=torch.float32, device=dev) if return_entropy else None
   part_ent = torch.empty(head_rows * runner.nvb, dtype=torch.float32, device=dev) if return_entropy else None
   for b0 in range(0, B, rows_b):
     nb = min(rows_b, B - b0)
     xn = runner.forward_hidden(ids[b0:b0 + nb], positions[b0:b0 + nb], runner.zero,
-                               [kc[:nb]] * cfg.num_layers, [vc[:nb]] * cfg.num_layers, B=nb, T=Ltot,
-                               segment_ids=None if seg is None else seg[b0:b0 + nb])
+                               cache.rows(0, nb), B=nb, T=Ltot,
+                               segment_ids=None if seg is None else seg[b0:b0 + nb], starts=starts[b0:b0 + nb])
     # logits[:, -T-1:-1] predict the completion tokens (:462-467)
     xs = xsel[: nb * T]
     xs.view(nb, T, -1).copy_(xn[: nb * Ltot].view(nb, Ltot, -1)[:, Ltot - T - 1: Ltot - 1])

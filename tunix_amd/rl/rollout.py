@@ -46,7 +46,8 @@ class HipRollout:
     cfg = model.cfg
     if isinstance(cache_config_or_size, int):
       cache_config_or_size = CacheConfig(cache_size=cache_config_or_size, num_layers=cfg.num_layers,
-                                         num_kv_heads=cfg.num_kv_heads, head_dim=cfg.head_dim)
+                                         num_kv_heads=getattr(cfg, "num_kv_heads", 0),
+                                         head_dim=getattr(cfg, "head_dim", 0))
     self._sampler = Sampler(model, tokenizer, cache_config_or_size)
 
   def generate(self, prompts: list[str], rollout_config: RolloutConfig, **kwargs) -> RolloutOutput:
