@@ -585,6 +585,212 @@ def config_workload(name, steps):
       "hbm_roofline_frac_step": round(step_bytes / (ms * 1e-3) / 1e9 / HBM_PEAK_GBS, 4), "step_bytes": int(step_bytes)}
 
 
+STACK_SIZES = {   # (width, query heads, kv heads, feed-forward, decode batch)
+    "2048": (2048, 16, 4, 8192, 32),
+    "4096": (4096, 32, 8, 14336, 128),
+}
+
+
+def roof_row(us, nbytes, flops):
+  """A kernel's time against the slower of its two roofs (HBM for its algorithmic bytes, the dense
+  bf16 MFMA peak for its flops)."""
+  hbm, mfma = nbytes / (HBM_PEAK_GBS * 1e3), flops / (MFMA_BF16_PEAK_TFLOPS * 1e6)
+  return {"us": round(us, 2), "bound": "hbm" if hbm >= mfma else "mfma", "times_roof": round(us / max(hbm, mfma, 1e-9), 2)}
+
+
+def in_turn(fns, iters):
+  """Mean microseconds of one launch when the launches of `fns` (the same kernel over different
+  layers' weights and caches) follow each other, so that none finds its operands in a cache."""
+  def one():
+    for fn in fns:
+      fn()
+  return time_loop(one, iters, per_graph=max(1, 8 // len(fns))) * 1e3 / len(fns)
+
+
+def stack_kernels(model, runner, st, ctx, iters):
+  """Per-kernel times of a layer-list model's pass: T = runner.T tokens per row, the last of them at
+  context `ctx`."""
+  import torch
+
+  from tunix_amd.config import AttentionMixer
+  B, T, M = runner.B, runner.T, runner.M
+  col = torch.tensor([ctx - T], dtype=torch.int32, device=model.device)
+  D = model.cfg.embed_dim
+  attn = [i for i, ly in enumerate(model.layers) if isinstance(ly["spec"].mixer, AttentionMixer)]
+  light = [i for i, ly in enumerate(model.layers) if i not in attn]
+  first = {}
+  for (i, _), e in zip(model.cfg.layer_runs, st.cache.entries):
+    first.setdefault(i, e)
+  out = {}
+
+  def lin(name, idx, key, x, paired=False):
+    f = model.layers[idx[0]][key]
+    us = in_turn([(lambda g=model.layers[i][key], ly=model.layers[i]:
+                   runner.gate_up(ly, x, M) if paired else runner.linear(g, x, M)) for i in idx], iters)
+    n_out = f.N // (2 if paired else 1)
+    out[name] = roof_row(us, f.nbytes() + M * (f.K + n_out) * 2, 2.0 * M * f.K * f.N)
+
+  h = runner._buf("h", model.Dp)
+  ly0 = model.layers[attn[0]]
+  m = ly0["spec"].mixer
+  lin("linear qkv", attn, "in", h)
+  lin("linear o", attn, "out", runner._buf("attn", ly0["out"].Kp))
+  lin("linear gate_up", attn, "gu", h, paired=True)
+  lin("linear down", attn, "down", runner._buf("act", ly0["down"].Kp))
+  lin("linear lightning in", light, "in", h)
+  if model.loop_in is not None:
+    f, cat = model.loop_in, runner._buf("cat", model.loop_in.Kp)
+    us = in_turn([lambda: runner.linear(f, cat, M, fp32_out=True)], iters)
+    out["linear loop in"] = roof_row(us, f.nbytes() + M * (f.K * 2 + D * 4), 2.0 * M * f.K * f.N)
+  src = runner.linear(ly0["in"], h, M)
+  us = in_turn([(lambda i=i: runner.rotate(model.layers[i], src, first[i], col, st.starts, B, T)) for i in attn], iters)
+  row = (m.heads * m.dim + m.kv_heads * (m.dim + m.vdim)) * 2
+  out["rotation + cache write"] = roof_row(us, 2 * M * row, 0)
+  q = runner._buf("q", m.heads * first[attn[0]].k.shape[3])
+  us = in_turn([(lambda i=i: runner.attend(model.layers[i], q, first[i], col, st.starts, B, T)) for i in attn], iters)
+  pairs = T * ctx - T * (T - 1) / 2
+  out["attention"] = roof_row(us, B * m.kv_heads * ctx * (m.dim + m.vdim) * 2 + 2 * M * m.heads * m.dim * 2,
+                              2.0 * B * m.heads * pairs * (m.dim + m.vdim))
+  ll, w = model.layers[light[0]], model.layers[light[0]]["spec"].mixer
+  lsrc = runner.linear(ll["in"], h, M)
+  us = in_turn([(lambda i=i: runner.recur(model.layers[i], lsrc, first[i], col, st.starts, B, T)) for i in light], iters)
+  out["lightning"] = roof_row(us, M * w.heads * (2 * w.dim + w.vdim) * 2 + M * w.heads * w.vdim * 4 + B * w.heads * w.dim * w.vdim * 8,
+                              2.0 * M * w.heads * (2 * w.dim * w.vdim) if T == 1 else 2.0 * M * w.heads * (2 * w.dim * w.vdim + 32 * (w.dim + w.vdim)))
+  o = runner.recur(ll, lsrc, first[light[0]], col, st.starts, B, T)
+  us = in_turn([lambda: runner.gate(ll, o, lsrc, M)], iters)
+  out["gated norm"] = roof_row(us, M * o.shape[1] * 8, 0)
+  osrc = runner.linear(ly0["out"], runner._buf("attn", ly0["out"].Kp), M)
+  us = in_turn([lambda: runner.residual_norm(("add", osrc, ly0["norm1b"]), ly0["norm2"], h, M, runner.frag)], iters)
+  out["post-norm + residual + norm"] = roof_row(us, M * D * (2 + 8 + 2), 0)
+  return out
+
+
+def family_kernels(model, runner, st, ctx, iters):
+  """The same kernels of a gemma3-family model of the same size."""
+  import torch
+
+  from tunix_amd import _lib as L
+  from tunix_amd import ops
+  cfg = model.cfg
+  B, T, M, S = runner.B, runner.T, runner.M, runner.S
+  col = torch.tensor([ctx - T], dtype=torch.int32, device=model.device)
+  out = {}
+
+  def lin(name, key, x, y, epi=L.TNX_EPI_STORE):
+    f = model.layers[0][key]
+    us = in_turn([(lambda g=ly[key]: runner.linear(g, x, y, M, epilogue=epi, defer=True)) for ly in model.layers], iters)
+    nbytes = f.codes.numel() * 4 + f.scales.numel() * 2 + M * (f.K + f.N // (2 if f.interleave2 else 1)) * 2
+    out[name] = roof_row(us, nbytes, 2.0 * M * f.K * f.N)
+
+  lin("linear qkv", "qkv", runner.xn, runner.qkv)
+  lin("linear o", "o", runner.attn, runner.tmp)
+  lin("linear gate_up", "gu", runner.xn, runner.act, L.TNX_EPI_GELU_MUL)
+  lin("linear down", "down", runner.act, runner.tmp)
+
+  def rope(i):
+    ly, kv = model.layers[i], st.cache.entries[i]
+    rd = L.RopeDesc()
+    rd.B, rd.T, rd.S, rd.Hq, rd.Hkv, rd.dh = B, T, S, cfg.num_heads, cfg.num_kv_heads, cfg.head_dim
+    rd.rope_flavor, rd.rope_scale, rd.timescale = L.TNX_ROPE_GEMMA3, ly["rope_scale"], ly["timescale"].data_ptr()
+    rd.qk_norm, rd.norm_eps = L.TNX_NORM_GEMMA3, 1e-6
+    rd.q_norm_w, rd.k_norm_w, rd.q_prescale = ly["q_norm"].data_ptr(), ly["k_norm"].data_ptr(), cfg.query_pre_attn_scalar
+    rd.qkv, rd.positions, rd.pos_ld = runner.qkv.data_ptr(), st.positions.data_ptr(), st.positions.shape[1]
+    rd.col_ptr, rd.q_out, rd.kcache, rd.vcache = col.data_ptr(), runner.q.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr()
+    ops.rope_kvwrite(rd)
+
+  def attend(i):
+    kv = st.cache.entries[i]
+    ad = L.AttnDesc()
+    ad.B, ad.T, ad.S, ad.Hq, ad.Hkv, ad.dh = B, T, S, cfg.num_heads, cfg.num_kv_heads, cfg.head_dim
+    ad.scale, ad.window, ad.pad_id = 0.0, 0, runner.pad_id
+    ad.q, ad.kcache, ad.vcache = runner.q.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr()
+    ad.tokens, ad.tok_ld, ad.col_ptr = st.token_buffer.data_ptr(), st.token_buffer.shape[1], col.data_ptr()
+    ad.kv_chunk, ad.ws, ad.out = runner.kv_chunk if T == 1 else 0, runner.attn_ws.data_ptr(), runner.attn.data_ptr()
+    ops.gqa_attn(ad)
+
+  layers = range(len(model.layers))
+  us = in_turn([(lambda i=i: rope(i)) for i in layers], iters)
+  out["rotation + cache write"] = roof_row(us, 2 * M * (cfg.q_dim + 2 * cfg.kv_dim) * 2, 0)
+  us = in_turn([(lambda i=i: attend(i)) for i in layers], iters)
+  pairs = T * ctx - T * (T - 1) / 2
+  out["attention"] = roof_row(us, B * 2 * cfg.kv_dim * ctx * 2 + 2 * M * cfg.q_dim * 2,
+                              4.0 * B * cfg.q_dim * pairs)
+  ly = model.layers[0]
+  us = in_turn([lambda: runner.norm_pair(1, ly["post_attn_norm"], ly["mlp_norm"], M)], iters)
+  out["post-norm + residual + norm"] = roof_row(us, M * cfg.embed_dim * 8, 0)
+  return out
+
+
+def stack_workload(size, iters, steps, kernels=True):
+  """Prefill and decode of a Nunezen decoder with layers of a real model's size (random weights),
+  beside a gemma3-family model (pre- and post-norms, gated GELU, int4 linears) with the same width,
+  heads, feed-forward and number of attention layers, and the time of every kernel of the two
+  against its roof."""
+  import numpy as np
+  import torch
+
+  from tunix_amd import config, dummy_model
+  from tunix_amd.generate import CacheConfig, Sampler
+  from tunix_amd.generate.sampler import _SamplingState
+  from tunix_amd.generate.utils import IdTokenizer
+  from tunix_amd.model import QLoRAModel
+  from tunix_amd.stack_model import StackModel
+  dev = torch.device("cuda:0")
+  width, H, G, ff, B = STACK_SIZES[size]
+  new_cfg = config.nunezen_shape(width, H, G, ff)
+  runs = new_cfg.layer_runs
+  n_attn = sum(isinstance(new_cfg.layers[i].mixer, config.AttentionMixer) for i, _ in runs)
+  like_cfg = config.gemma3_1b(num_layers=n_attn, vocab_size=new_cfg.vocab_size, embed_dim=width, hidden_dim=ff, num_heads=H,
+                              num_kv_heads=G, head_dim=128, lora_rank=0, lora_alpha=0.0, sliding_window=0)
+  P, T = 1024, 256
+  S = P + T
+  ids = np.random.Generator(np.random.PCG64(5)).integers(1, new_cfg.vocab_size, size=(B, P)).astype(np.int32)
+  result = {"size": {"width": width, "heads": H, "kv_heads": G, "head_dim": 128, "feed_forward": ff, "batch": B, "prompt": P,
+                     "layer_runs": len(runs), "attention_layer_runs": n_attn}}
+  models = (("nunezen", lambda: StackModel(new_cfg, dummy_model.create_stack_weights(new_cfg, 1, dev), dev)),
+            ("gemma3-family", lambda: QLoRAModel(like_cfg, dummy_model.create_dummy_weights(like_cfg, 1, dev), dev)))
+  for name, build in models:
+    model = build()
+    sampler = Sampler(model, IdTokenizer(new_cfg.vocab_size, pad_id=0, eos_id=1), CacheConfig(S))
+    prompts, ms, pre = [r for r in ids], [], []
+    for n in (4, 4, 4 + steps):
+      sampler(prompts, n, max_prompt_length=P, eos_tokens=[-1])
+      ms.append(sampler.last_stats["decode_ms"])
+      pre.append(sampler.last_stats["prefill_ms"])
+    d_ms = (ms[2] - ms[1]) / steps
+    r = {"prefill_tokens_per_s": round(B * P / (min(pre[1:]) * 1e-3)), "prefill_ms": round(min(pre[1:]), 2),
+         "decode_tokens_per_s": round(B / (d_ms * 1e-3)), "decode_ms_per_step": round(d_ms, 4)}
+    log(size, name, r)
+    if kernels:
+      measure = stack_kernels if name == "nunezen" else family_kernels
+      st = _SamplingState(model, ids, S, S, 0, False, False)
+      st.token_buffer.fill_(5)
+      st.starts.zero_()
+      for kc, vc in zip(st.kcache, st.vcache):
+        kc.normal_()
+        vc.normal_()
+      r["decode_kernels"] = measure(model, model.new_runner(B, 1, S, 0), st, P + T // 2, iters)
+      pb = 8      # rows of a prefill group: 8 x 1024 tokens
+      stp = _SamplingState(model, ids[:pb], S, S, 0, False, False)
+      stp.token_buffer.fill_(5)
+      stp.starts.zero_()
+      r["prefill_kernels"] = measure(model, model.new_runner(pb, P, S, 0, kv_chunk=0), stp, P, max(2, iters // 4))
+      del st, stp
+    result[name] = r
+    del model, sampler
+    torch.cuda.empty_cache()
+  if kernels:
+    for phase in ("decode_kernels", "prefill_kernels"):
+      a, b = result["nunezen"][phase], result["gemma3-family"][phase]
+      for k, v in a.items():
+        like = {"lightning": "attention", "gated norm": "post-norm + residual + norm", "linear lightning in": "linear qkv",
+                "linear loop in": "linear qkv"}.get(k, k)
+        v["vs_like"] = round(v["times_roof"] / b[like]["times_roof"], 2)
+        log(f"  {size} {phase:16s} {k:28s} {v['us']:9.1f} us  {v['times_roof']:6.2f} x roof ({v['bound']})   like: "
+            f"{b[like]['us']:9.1f} us  {b[like]['times_roof']:6.2f} x ({b[like]['bound']})   ratio {v['vs_like']}")
+  return result
+
+
 def main():
   ap = argparse.ArgumentParser()
   ap.add_argument("--gpus", type=int, default=1)
@@ -610,6 +816,11 @@ def main():
                        "instead of reading the head's expanded copy")
   ap.add_argument("--no-fused-logps", action="store_true",
                   help="leave the standalone log-probability workload out of the default run's line")
+  ap.add_argument("--stack", choices=sorted(STACK_SIZES) + ["all"], default=None,
+                  help="instead of the decode benchmark: a Nunezen decoder with layers of a real model's size (model "
+                       "width 2048 or 4096), prefill, decode and every kernel against its roof, beside a gemma3-family "
+                       "model of the same size; its own JSON line")
+  ap.add_argument("--stack-no-kernels", action="store_true", help="with --stack: throughput only")
   ap.add_argument("--config", choices=["c1", "c2", "c3", "c4"], default="c3",
                   help="c3 (default): the headline workload; c1 / c2 / c4: the other rollout workloads through "
                        "the public Sampler call, their own JSON line")
@@ -650,6 +861,14 @@ def main():
     print("bench.py measures one GPU: this build has no multi-GPU path (the decode path shards "
           "by batch rows with no exchange); run with --gpus 1", file=sys.stderr)
     sys.exit(2)
+
+  if args.stack:
+    sizes = sorted(STACK_SIZES) if args.stack == "all" else [args.stack]
+    print(json.dumps({"metric": "Nunezen prefill and decode tokens/sec @1 MI355X", "unit": "tokens/s", "n_gpus": 1,
+                      "dtype": "bf16", "data": "synthetic",
+                      "sizes": {z: stack_workload(z, args.kernel_iters, 64, not args.stack_no_kernels) for z in sizes}}),
+          flush=True)
+    return
 
   if args.config != "c3":
     print(json.dumps(config_workload(args.config, args.steps if args.steps != 508 else 200)), flush=True)

@@ -35,6 +35,9 @@ def read_safetensors(path: str) -> dict[str, torch.Tensor]:
     count = int(np.prod(shape, dtype=np.int64)) * torch.empty(0, dtype=dtype).element_size()
     if not 0 <= a <= b <= size - 8 - n or b - a != count:
       raise ValueError(f"{path}: tensor {name} does not fit the file")
+    if count == 0:
+      out[name] = torch.empty(shape, dtype=dtype)
+      continue
     out[name] = torch.from_numpy(np.array(raw[8 + n + a: 8 + n + b])).view(dtype).reshape(shape)
   return out
 

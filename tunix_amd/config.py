@@ -277,3 +277,15 @@ def qwen3_30b_a3b(**kw) -> ModelConfig:
            num_experts_per_tok=8)
   d.update(kw)
   return ModelConfig(**d)
+
+
+def nunezen_shape(width: int, heads: int, kv_heads: int, ff: int, vocab: int = 32768, dim: int = 128,
+                  layers: int = 4) -> StackConfig:
+  """A Nunezen decoder with layers of a real model's size: attention (+ feed-forward) and lightning
+  layers in turn, the middle layers run twice."""
+  attn = LayerSpec(AttentionMixer(heads, kv_heads, dim, dim, dim // 2, 500_000.0, dim ** -0.5), GatedMlp(ff))
+  decay = tuple(1.0 - 2.0 ** (-1.0 - 8.0 * h / max(heads - 1, 1)) for h in range(heads))
+  light = LayerSpec(LightningMixer(heads, dim, dim, decay), None)
+  return StackConfig(family="nunezen", vocab_size=vocab, embed_dim=width, norm_eps=1e-6,
+                     layers=tuple(attn if i % 2 == 0 else light for i in range(layers)),
+                     loop=LayerLoop(1, layers - 1, 2) if layers > 2 else None)

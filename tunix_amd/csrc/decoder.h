@@ -41,4 +41,54 @@ struct RowSrc {
   }
 };
 
+// Eight consecutive values of a row (col, ld and planes on 8-element boundaries); partial planes are
+// requested together, four at a time, and added in plane order.
+template <typename T>
+__device__ __forceinline__ void get8(const RowSrc<T>& s, int64_t row, int64_t col, float (&f)[8]) {
+  const int64_t o = row * s.ld + col;
+  if (s.split > 1) {
+    const float* p = s.ws + o;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) f[j] = 0.f;
+    for (int z0 = 0; z0 < s.split; z0 += 4) {
+      f32x4 a[4], b[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const float* q = p + (int64_t)min(z0 + u, s.split - 1) * s.plane;
+        a[u] = *reinterpret_cast<const f32x4*>(q);
+        b[u] = *reinterpret_cast<const f32x4*>(q + 4);
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+        if (z0 + u < s.split)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            f[j] += a[u][j];
+            f[4 + j] += b[u][j];
+          }
+    }
+  } else if constexpr (sizeof(T) == 2) {
+    const u32x4 v = *reinterpret_cast<const u32x4*>(s.y + o);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      f[2 * j] = bflo(v[j]);
+      f[2 * j + 1] = bfhi(v[j]);
+    }
+  } else {
+    const f32x4 a = *reinterpret_cast<const f32x4*>(s.y + o), b = *reinterpret_cast<const f32x4*>(s.y + o + 4);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      f[j] = a[j];
+      f[4 + j] = b[j];
+    }
+  }
+}
+__device__ __forceinline__ void put8(uint16_t* p, const float (&f)[8]) {
+  *reinterpret_cast<u32x4*>(p) = u32x4{pack2bf(f[0], f[1]), pack2bf(f[2], f[3]), pack2bf(f[4], f[5]), pack2bf(f[6], f[7])};
+}
+__device__ __forceinline__ void put8(float* p, const float (&f)[8]) {
+  *reinterpret_cast<f32x4*>(p) = f32x4{f[0], f[1], f[2], f[3]};
+  *reinterpret_cast<f32x4*>(p + 4) = f32x4{f[4], f[5], f[6], f[7]};
+}
+
 static inline bool src_given(const tnx_rows_src& s) { return s.ld > 0 && (s.split_k > 1 ? s.ws != nullptr : s.y != nullptr); }

@@ -94,88 +94,59 @@ __global__ __launch_bounds__(256) void resnorm_kernel(const ResNormArgs a) {
   }
 }
 
-// D % 8 == 0: eight elements per thread and turn, the row stays in registers
+// D % 8 == 0: eight elements per thread and turn, the row stays in registers.  Everything the row needs
+// -- residual, incoming values, both weights -- is requested before the first sum: the kernel is one
+// memory round trip and two block reductions long.
 template <int MAXC, typename T>
 __global__ __launch_bounds__(256) void resnorm_vec_kernel(const ResNormArgs a) {
   __shared__ float red[4];
   const int64_t row = blockIdx.x;
   const int nch = (int)(a.D / 8);
-  float h[MAXC][8], xo[MAXC][8];
-  float ss = 0.f;
+  // (mode and w_next are the same for the whole grid: uniform branches)
+  const RowSrc<T> src{reinterpret_cast<const T*>(a.y), a.ws, a.split, a.plane, a.y_ld};
+  float h[MAXC][8], xo[MAXC][8], wp[MAXC][8], wn[MAXC][8];
+  auto load8f = [](const float* p, float (&f)[8]) {
+    const f32x4 u = *reinterpret_cast<const f32x4*>(p), v = *reinterpret_cast<const f32x4*>(p + 4);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      f[j] = u[j];
+      f[4 + j] = v[j];
+    }
+  };
 #pragma unroll
   for (int c = 0; c < MAXC; ++c) {
-    const int ch = c * 256 + threadIdx.x;
-    const bool ok = ch < nch;
-    const int64_t col = (int64_t)min(ch, nch - 1) * 8;
-    if (a.mode != 2) {
-      const f32x4 x0 = *reinterpret_cast<const f32x4*>(a.x + row * a.D + col);
-      const f32x4 x1 = *reinterpret_cast<const f32x4*>(a.x + row * a.D + col + 4);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        xo[c][j] = x0[j];
-        xo[c][4 + j] = x1[j];
-      }
-    }
+    const int64_t col = (int64_t)min(c * 256 + (int)threadIdx.x, nch - 1) * 8;
+    if (a.mode != 2) load8f(a.x + row * a.D + col, xo[c]);
+    if (a.mode == 1) load8f(a.w_post + col, wp[c]);
+    if (a.w_next) load8f(a.w_next + col, wn[c]);
     if (a.mode != 0) {
-      if (a.ws) {
-        const float* p = a.ws + row * a.y_ld + col;
-        f32x4 s0 = *reinterpret_cast<const f32x4*>(p), s1 = *reinterpret_cast<const f32x4*>(p + 4);
-        for (int z0 = 1; z0 < a.split; z0 += 4) {   // four planes in flight, added in plane order
-          f32x4 q0[4], q1[4];
-#pragma unroll
-          for (int u = 0; u < 4; ++u) {
-            const float* q = p + (int64_t)min(z0 + u, a.split - 1) * a.plane;
-            q0[u] = *reinterpret_cast<const f32x4*>(q);
-            q1[u] = *reinterpret_cast<const f32x4*>(q + 4);
-          }
-#pragma unroll
-          for (int u = 0; u < 4; ++u)
-            if (z0 + u < a.split) {
-              s0 += q0[u];
-              s1 += q1[u];
-            }
-        }
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          h[c][j] = s0[j];
-          h[c][4 + j] = s1[j];
-        }
-      } else if constexpr (sizeof(T) == 2) {
-        const u32x4 v = *reinterpret_cast<const u32x4*>(reinterpret_cast<const T*>(a.y) + row * a.y_ld + col);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          h[c][2 * j] = bflo(v[j]);
-          h[c][2 * j + 1] = bfhi(v[j]);
-        }
-      } else {
-        const T* p = reinterpret_cast<const T*>(a.y) + row * a.y_ld + col;
-#pragma unroll
-        for (int j = 0; j < 8; ++j) h[c][j] = ld_elem(p, j);
-      }
-      if (ok)
-#pragma unroll
-        for (int j = 0; j < 8; ++j) ss += h[c][j] * h[c][j];
+      if (a.ws && a.split == 1) load8f(a.ws + row * a.y_ld + col, h[c]);
+      else get8(src, row, col, h[c]);
     }
   }
+  float ss = 0.f;
   float r = 1.f;
-  if (a.mode == 1) r = 1.0f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
+  if (a.mode == 1) {
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c)
+      if (c * 256 + (int)threadIdx.x < nch)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) ss += h[c][j] * h[c][j];
+    r = 1.0f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
+  }
   ss = 0.f;
 #pragma unroll
   for (int c = 0; c < MAXC; ++c) {
     const int ch = c * 256 + threadIdx.x;
-    const int64_t col = (int64_t)min(ch, nch - 1) * 8;
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-      if (a.mode == 1) h[c][j] = xo[c][j] + h[c][j] * r * (a.w_offset + a.w_post[col + j]);
+      if (a.mode == 1) h[c][j] = xo[c][j] + h[c][j] * r * (a.w_offset + wp[c][j]);
       else if (a.mode == 0) h[c][j] = xo[c][j];
     }
     if (ch < nch) {
 #pragma unroll
       for (int j = 0; j < 8; ++j) ss += h[c][j] * h[c][j];
-      if (a.mode != 0) {
-        *reinterpret_cast<f32x4*>(a.x + row * a.D + col) = f32x4{h[c][0], h[c][1], h[c][2], h[c][3]};
-        *reinterpret_cast<f32x4*>(a.x + row * a.D + col + 4) = f32x4{h[c][4], h[c][5], h[c][6], h[c][7]};
-      }
+      if (a.mode != 0) put8(a.x + row * a.D + (int64_t)ch * 8, h[c]);
     }
   }
   float rn = 1.f;
@@ -186,22 +157,16 @@ __global__ __launch_bounds__(256) void resnorm_vec_kernel(const ResNormArgs a) {
     const int ch = c * 256 + threadIdx.x;
     if (ch >= nch) continue;
     const int64_t col = (int64_t)ch * 8;
-    float v[8];
+    if (a.w_next)
 #pragma unroll
-    for (int j = 0; j < 8; ++j) v[j] = a.w_next ? h[c][j] * rn * (a.w_offset + a.w_next[col + j]) : h[c][j];
-    T* o = out + (a.out_frag ? frag_index(row, col, a.out_ld) : row * a.out_ld + col);
-    if constexpr (sizeof(T) == 2) {
-      *reinterpret_cast<u32x4*>(o) = u32x4{pack2bf(v[0], v[1]), pack2bf(v[2], v[3]), pack2bf(v[4], v[5]), pack2bf(v[6], v[7])};
-    } else {
-#pragma unroll
-      for (int j = 0; j < 8; ++j) st_elem(o, j, v[j]);
-    }
+      for (int j = 0; j < 8; ++j) h[c][j] = h[c][j] * rn * (a.w_offset + wn[c][j]);
+    put8(out + (a.out_frag ? frag_index(row, col, a.out_ld) : row * a.out_ld + col), h[c]);
   }
 }
 
 template <typename T>
 void launch_resnorm(hipStream_t st, const ResNormArgs& a) {
-  const bool vec = a.D % 8 == 0 && a.D <= 16384 && a.y_ld % 8 == 0 && a.out_ld % 8 == 0 && a.plane % 4 == 0;
+  const bool vec = a.D % 8 == 0 && a.y_ld % 8 == 0 && a.out_ld % 8 == 0 && a.plane % 8 == 0;
   const dim3 grid((unsigned)a.M);
   if (!vec) hipLaunchKernelGGL((resnorm_kernel<T>), grid, dim3(256), (size_t)a.D * 4, st, a);
   else if (a.D <= 2048) hipLaunchKernelGGL((resnorm_vec_kernel<1, T>), grid, dim3(256), 0, st, a);
@@ -251,46 +216,54 @@ __global__ __launch_bounds__(256) void part_rope_kernel(const PartRopeArgs a, co
   }
 }
 
-// Finished bf16 rows whose heads, offsets and rotated halves come in whole runs of eight: 16 bytes
-// per access (prefill).
-__global__ __launch_bounds__(256) void part_rope_vec_kernel(const PartRopeArgs a, const uint16_t* y, int64_t ld, uint16_t* q_out,
-                                                            uint16_t* kc, uint16_t* vc) {
+// Heads, offsets and rotated halves in whole runs of eight: an item is eight dimensions (with their
+// partners, where rotated) of one head; the items of a row are spread over gridDim.y work-groups.
+template <typename T>
+__global__ __launch_bounds__(256) void part_rope_vec_kernel(const PartRopeArgs a, const RowSrc<T> src, T* q_out, T* kc, T* vc) {
   __shared__ __align__(16) float sn[kMaxHalf], cs[kMaxHalf];
   const int64_t row = blockIdx.x, b = row / a.T, t = row % a.T;
+  const int heads = a.H + a.G, hpt = (a.dkp - a.half) / 8, half8 = a.half / 8, vch = a.dvp / 8;
+  const int n_rot = heads * hpt, n = n_rot + a.G * vch;
+  const int first = blockIdx.y * 256 + threadIdx.x;
   const int slot = *a.col_ptr + (int)t;
-  if (slot >= a.S) return;
+  if (slot >= a.S) return;                                    // (uniform)
   const float pos = (float)max(slot - a.starts[b], 0);
   for (int i = threadIdx.x; i < a.half; i += 256) sincosf(pos * a.inv_freq[i], &sn[i], &cs[i]);
   __syncthreads();
-  const uint16_t* yr = y + row * ld;
-  const int heads = a.H + a.G, hpt = (a.dkp - a.half) / 8, half8 = a.half / 8;
-  for (int it = threadIdx.x; it < heads * hpt; it += 256) {
+  for (int it = first; it < n; it += 256 * gridDim.y) {
+    float u[8];
+    if (it >= n_rot) {
+      const int g = (it - n_rot) / vch, d = ((it - n_rot) % vch) * 8;
+      T* dst = vc + ((b * a.G + g) * a.S + slot) * a.dvp + d;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) u[j] = 0.f;
+      if (d < a.dv) get8(src, row, a.v_off + (int64_t)g * a.dv + d, u);
+      put8(dst, u);
+      continue;
+    }
     const int hd = it / hpt, c = it % hpt;
     const bool is_k = hd >= a.H;
-    const uint16_t* s = yr + (is_k ? a.k_off + (int64_t)(hd - a.H) * a.dk : (int64_t)hd * a.dk);
-    uint16_t* dst = is_k ? kc + ((b * a.G + (hd - a.H)) * a.S + slot) * a.dkp : q_out + (row * a.H + hd) * a.dkp;
+    const int64_t base = is_k ? a.k_off + (int64_t)(hd - a.H) * a.dk : (int64_t)hd * a.dk;
+    T* dst = is_k ? kc + ((b * a.G + (hd - a.H)) * a.S + slot) * a.dkp : q_out + (row * a.H + hd) * a.dkp;
     if (c < half8) {
-      const u32x4 u = *reinterpret_cast<const u32x4*>(s + c * 8), v = *reinterpret_cast<const u32x4*>(s + a.half + c * 8);
-      u32x4 o1, o2;
+      float v[8], o1[8], o2[8];
+      get8(src, row, base + c * 8, u);
+      get8(src, row, base + a.half + c * 8, v);
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const float c0 = cs[c * 8 + 2 * j], c1 = cs[c * 8 + 2 * j + 1], s0 = sn[c * 8 + 2 * j], s1 = sn[c * 8 + 2 * j + 1];
-        const float u0 = bflo(u[j]), u1 = bfhi(u[j]), v0 = bflo(v[j]), v1 = bfhi(v[j]);
-        o1[j] = pack2bf(u0 * c0 - v0 * s0, u1 * c1 - v1 * s1);
-        o2[j] = pack2bf(v0 * c0 + u0 * s0, v1 * c1 + u1 * s1);
+      for (int j = 0; j < 8; ++j) {
+        const float co = cs[c * 8 + j], si = sn[c * 8 + j];
+        o1[j] = u[j] * co - v[j] * si;
+        o2[j] = v[j] * co + u[j] * si;
       }
-      *reinterpret_cast<u32x4*>(dst + c * 8) = o1;
-      *reinterpret_cast<u32x4*>(dst + a.half + c * 8) = o2;
+      put8(dst + c * 8, o1);
+      put8(dst + a.half + c * 8, o2);
     } else {
       const int d = a.half + c * 8;
-      *reinterpret_cast<u32x4*>(dst + d) = d < a.dk ? *reinterpret_cast<const u32x4*>(s + d) : u32x4{0, 0, 0, 0};
+#pragma unroll
+      for (int j = 0; j < 8; ++j) u[j] = 0.f;
+      if (d < a.dk) get8(src, row, base + d, u);
+      put8(dst + d, u);
     }
-  }
-  const int vch = a.dvp / 8;
-  for (int it = threadIdx.x; it < a.G * vch; it += 256) {
-    const int g = it / vch, d = (it % vch) * 8;
-    *reinterpret_cast<u32x4*>(vc + ((b * a.G + g) * a.S + slot) * a.dvp + d) =
-        d < a.dv ? *reinterpret_cast<const u32x4*>(yr + a.v_off + (int64_t)g * a.dv + d) : u32x4{0, 0, 0, 0};
   }
 }
 
@@ -308,34 +281,52 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(const GatedNormArgs a, 
   const int64_t row = blockIdx.x;
   const float* o = a.o + row * a.o_ld;
   float ss = 0.f;
-  if (a.W % 4 == 0 && a.o_ld % 4 == 0) {
-    for (int64_t i = (int64_t)threadIdx.x * 4; i < a.W; i += 1024) {
-      const f32x4 v = *reinterpret_cast<const f32x4*>(o + i);
-      ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
-    }
-  } else {
-    for (int64_t i = threadIdx.x; i < a.W; i += 256) ss += o[i] * o[i];
-  }
+  for (int64_t i = threadIdx.x; i < a.W; i += 256) ss += o[i] * o[i];
   const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)a.W + a.eps);
-  if (sizeof(T) == 2 && g.split <= 1 && a.W % 8 == 0 && a.o_ld % 8 == 0 && g.ld % 8 == 0 && a.g_off % 8 == 0 && a.out_ld % 8 == 0) {
-    for (int64_t i = (int64_t)threadIdx.x * 8; i < a.W; i += 2048) {
-      const f32x4 v0 = *reinterpret_cast<const f32x4*>(o + i), v1 = *reinterpret_cast<const f32x4*>(o + i + 4);
-      const f32x4 w0 = *reinterpret_cast<const f32x4*>(a.w + i), w1 = *reinterpret_cast<const f32x4*>(a.w + i + 4);
-      const u32x4 gv = *reinterpret_cast<const u32x4*>(reinterpret_cast<const uint16_t*>(g.y) + row * g.ld + a.g_off + i);
-      u32x4 p;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const float e0 = j < 2 ? v0[2 * j] : v1[2 * j - 4], e1 = j < 2 ? v0[2 * j + 1] : v1[2 * j - 3];
-        const float f0 = j < 2 ? w0[2 * j] : w1[2 * j - 4], f1 = j < 2 ? w0[2 * j + 1] : w1[2 * j - 3];
-        p[j] = pack2bf(e0 * r * (a.w_offset + f0) * sigmoid_f32(bflo(gv[j])), e1 * r * (a.w_offset + f1) * sigmoid_f32(bfhi(gv[j])));
-      }
-      *reinterpret_cast<u32x4*>(reinterpret_cast<uint16_t*>(out) + (a.out_frag ? frag_index(row, i, a.out_ld) : row * a.out_ld + i)) = p;
-    }
-    return;
-  }
   for (int64_t i = threadIdx.x; i < a.W; i += 256)
     st_elem(out, a.out_frag ? frag_index(row, i, a.out_ld) : row * a.out_ld + i,
             o[i] * r * (a.w_offset + a.w[i]) * sigmoid_f32(g.get(row, a.g_off + i)));
+}
+// eight elements per thread and turn, everything requested ahead of the sum
+template <int MAXC, typename T>
+__global__ __launch_bounds__(256) void gated_norm_vec_kernel(const GatedNormArgs a, const RowSrc<T> g, T* out) {
+  __shared__ float red[4];
+  const int64_t row = blockIdx.x;
+  const int nch = (int)(a.W / 8);
+  float o[MAXC][8], w[MAXC][8], gv[MAXC][8];
+  const RowSrc<float> os{a.o, nullptr, 1, 0, a.o_ld}, wsrc{a.w, nullptr, 1, 0, 0};
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int64_t col = (int64_t)min(c * 256 + (int)threadIdx.x, nch - 1) * 8;
+    get8(os, row, col, o[c]);
+    get8(wsrc, 0, col, w[c]);
+    get8(g, row, a.g_off + col, gv[c]);
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c)
+    if (c * 256 + (int)threadIdx.x < nch)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss += o[c][j] * o[c][j];
+  const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)a.W + a.eps);
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = c * 256 + threadIdx.x;
+    if (ch >= nch) continue;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o[c][j] = o[c][j] * r * (a.w_offset + w[c][j]) * sigmoid_f32(gv[c][j]);
+    put8(out + (a.out_frag ? frag_index(row, (int64_t)ch * 8, a.out_ld) : row * a.out_ld + (int64_t)ch * 8), o[c]);
+  }
+}
+template <typename T>
+void launch_gated_norm(hipStream_t st, int64_t M, const GatedNormArgs& a, const RowSrc<T>& g, T* out) {
+  const dim3 grid((unsigned)M);
+  const bool vec = a.W % 8 == 0 && a.W <= 16384 && a.o_ld % 8 == 0 && g.ld % 8 == 0 && g.plane % 8 == 0 && a.g_off % 8 == 0 && a.out_ld % 8 == 0;
+  if (!vec) hipLaunchKernelGGL((gated_norm_kernel<T>), grid, dim3(256), 0, st, a, g, out);
+  else if (a.W <= 2048) hipLaunchKernelGGL((gated_norm_vec_kernel<1, T>), grid, dim3(256), 0, st, a, g, out);
+  else if (a.W <= 4096) hipLaunchKernelGGL((gated_norm_vec_kernel<2, T>), grid, dim3(256), 0, st, a, g, out);
+  else if (a.W <= 8192) hipLaunchKernelGGL((gated_norm_vec_kernel<4, T>), grid, dim3(256), 0, st, a, g, out);
+  else hipLaunchKernelGGL((gated_norm_vec_kernel<8, T>), grid, dim3(256), 0, st, a, g, out);
 }
 
 // ---- gated unit on finished projections: out = gelu_tanh(y[:, :F]) * y[:, u_off : u_off + F] -----
@@ -489,17 +480,23 @@ extern "C" int tnx_part_rope_kvwrite(void* stream, const tnx_part_rope_desc* d) 
   a.k_off = d->k_off; a.v_off = d->v_off;
   const dim3 grid((unsigned)(d->B * d->T));
   hipStream_t st = as_stream(stream);
-  const bool vec = d->dtype == TNX_BF16 && d->y.split_k <= 1 && d->dk % 8 == 0 && d->dv % 8 == 0 && d->dkp % 8 == 0 &&
-                   d->dvp % 8 == 0 && a.half % 8 == 0 && d->k_off % 8 == 0 && d->v_off % 8 == 0 && d->y.ld % 8 == 0;
-  if (vec)
-    hipLaunchKernelGGL(part_rope_vec_kernel, grid, dim3(256), 0, st, a, (const uint16_t*)d->y.y, d->y.ld, (uint16_t*)d->q_out,
-                       (uint16_t*)d->kcache, (uint16_t*)d->vcache);
-  else if (d->dtype == TNX_BF16)
-    hipLaunchKernelGGL(part_rope_kernel<uint16_t>, grid, dim3(256), 0, st, a, row_src<uint16_t>(d->y), (uint16_t*)d->q_out,
-                       (uint16_t*)d->kcache, (uint16_t*)d->vcache);
-  else
-    hipLaunchKernelGGL(part_rope_kernel<float>, grid, dim3(256), 0, st, a, row_src<float>(d->y), (float*)d->q_out, (float*)d->kcache,
-                       (float*)d->vcache);
+  const bool vec = d->dk % 8 == 0 && d->dv % 8 == 0 && d->dkp % 8 == 0 && d->dvp % 8 == 0 && a.half % 8 == 0 && d->k_off % 8 == 0 &&
+                   d->v_off % 8 == 0 && d->y.ld % 8 == 0 && d->y.plane % 8 == 0;
+  const bool bf = d->dtype == TNX_BF16;
+  uint16_t *q16 = (uint16_t*)d->q_out, *k16 = (uint16_t*)d->kcache, *v16 = (uint16_t*)d->vcache;
+  float *q32 = (float*)d->q_out, *k32 = (float*)d->kcache, *v32 = (float*)d->vcache;
+  if (vec) {
+    // few rows: one item per thread; many rows fill the device by themselves
+    const int items = (d->H + d->G) * ((d->dkp - a.half) / 8) + d->G * (d->dvp / 8);
+    const unsigned ny = d->B * d->T >= 1024 ? 1 : (unsigned)cdiv(items, 256);
+    const dim3 g2((unsigned)(d->B * d->T), ny);
+    if (bf) hipLaunchKernelGGL(part_rope_vec_kernel<uint16_t>, g2, dim3(256), 0, st, a, row_src<uint16_t>(d->y), q16, k16, v16);
+    else hipLaunchKernelGGL(part_rope_vec_kernel<float>, g2, dim3(256), 0, st, a, row_src<float>(d->y), q32, k32, v32);
+  } else if (bf) {
+    hipLaunchKernelGGL(part_rope_kernel<uint16_t>, grid, dim3(256), 0, st, a, row_src<uint16_t>(d->y), q16, k16, v16);
+  } else {
+    hipLaunchKernelGGL(part_rope_kernel<float>, grid, dim3(256), 0, st, a, row_src<float>(d->y), q32, k32, v32);
+  }
   TNX_CHECK_LAUNCH("part_rope");
   return TNX_OK;
 }
@@ -512,12 +509,8 @@ extern "C" int tnx_gated_norm(void* stream, const tnx_gated_norm_desc* d) {
   GatedNormArgs a;
   a.W = d->W; a.o_ld = d->o_ld; a.out_ld = d->out_ld; a.g_off = d->g_off; a.eps = d->eps; a.w_offset = d->w_offset;
   a.w = d->w; a.o = d->o; a.out_frag = d->out_frag;
-  if (d->dtype == TNX_BF16)
-    hipLaunchKernelGGL(gated_norm_kernel<uint16_t>, dim3((unsigned)d->M), dim3(256), 0, as_stream(stream), a, row_src<uint16_t>(d->g),
-                       (uint16_t*)d->out);
-  else
-    hipLaunchKernelGGL(gated_norm_kernel<float>, dim3((unsigned)d->M), dim3(256), 0, as_stream(stream), a, row_src<float>(d->g),
-                       (float*)d->out);
+  if (d->dtype == TNX_BF16) launch_gated_norm(as_stream(stream), d->M, a, row_src<uint16_t>(d->g), (uint16_t*)d->out);
+  else launch_gated_norm(as_stream(stream), d->M, a, row_src<float>(d->g), (float*)d->out);
   TNX_CHECK_LAUNCH("gated_norm");
   return TNX_OK;
 }

@@ -39,9 +39,9 @@ constexpr int kDenseKT = 128;   // k-tile of the fragment layout: eight 16-deep 
 // Products are formed transposed (weights as the MFMA's A operand): a lane owns runs of four
 // consecutive columns of one row.
 template <int RT>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, RT == 4 ? 2 : 4)))
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, RT == 4 ? 1 : RT == 2 ? 2 : 4)))
 void dense_rows_kernel(const DenseArgs a) {
-  constexpr int CG = 2;
+  constexpr int CG = 2, XD = 4;   // column groups; slabs of activations in flight
   __shared__ __align__(16) float red[4][CG * 16 * 64];
   const int tid = threadIdx.x, lane = tid & 63, l32 = lane & 31, lh = lane >> 5;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -79,20 +79,22 @@ void dense_rows_kernel(const DenseArgs a) {
   if (kt < kt1) {
 #pragma unroll
     for (int u = 0; u < 8; ++u) load_w(kt, u);
-    u32x4 xr[2][RT];
+    u32x4 xr[XD][RT];
 #pragma unroll
-    for (int rt = 0; rt < RT; ++rt) xr[0][rt] = load_x(kt * 8, rt);
+    for (int u = 0; u < XD - 1; ++u)
+#pragma unroll
+      for (int rt = 0; rt < RT; ++rt) xr[u][rt] = load_x(kt * 8 + u, rt);
     for (; kt < kt1; kt += 4) {
       const int ktn = min(kt + 4, kt1 - 1);   // (past the end: a valid tile, loaded and not used)
 #pragma unroll
       for (int u = 0; u < 8; ++u) {
-        const int nslab = u < 7 ? kt * 8 + u + 1 : ktn * 8;
+        const int n = u + XD - 1, nslab = n < 8 ? kt * 8 + n : ktn * 8 + n - 8;
 #pragma unroll
-        for (int rt = 0; rt < RT; ++rt) xr[(u + 1) & 1][rt] = load_x(nslab, rt);
+        for (int rt = 0; rt < RT; ++rt) xr[n % XD][rt] = load_x(nslab, rt);
 #pragma unroll
         for (int cg = 0; cg < CG; ++cg)
 #pragma unroll
-          for (int rt = 0; rt < RT; ++rt) acc[rt][cg] = mfma32(wr[u][cg], xr[u & 1][rt], acc[rt][cg]);
+          for (int rt = 0; rt < RT; ++rt) acc[rt][cg] = mfma32(wr[u][cg], xr[u % XD][rt], acc[rt][cg]);
         load_w(ktn, u);
       }
     }

@@ -90,7 +90,7 @@ __global__ __launch_bounds__(256) void lightning_step_kernel(const LightArgs a, 
   for (int u = 0; u < PF; ++u) {
     const int i = grp + u * ng;
     s[u] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (mine && i < a.dk && !fresh) s[u] = S[(int64_t)i * nc + c];
+    if (mine && i < a.dk && !fresh) s[u] = __builtin_nontemporal_load(&S[(int64_t)i * nc + c]);
   }
   for (int i = tid; i < a.dk; i += 256) {
     sm[i] = silu_f32(src.get(b, (int64_t)h * a.dk + i));
@@ -108,14 +108,14 @@ __global__ __launch_bounds__(256) void lightning_step_kernel(const LightArgs a, 
       for (int u = 0; u < PF; ++u) {
         const int i = i0 + (PF + u) * ng;
         nx[u] = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (i < a.dk && !fresh) nx[u] = S[(int64_t)i * nc + c];
+        if (i < a.dk && !fresh) nx[u] = __builtin_nontemporal_load(&S[(int64_t)i * nc + c]);
       }
 #pragma unroll
       for (int u = 0; u < PF; ++u) {
         const int i = i0 + u * ng;
         if (i < a.dk) {
           const f32x4 w = lam * s[u] + sm[a.dk + i] * v;
-          S[(int64_t)i * nc + c] = w;
+          __builtin_nontemporal_store(w, &S[(int64_t)i * nc + c]);
           acc += sm[i] * w;
         }
         s[u] = nx[u];

@@ -555,10 +555,14 @@ void qgemm_wide_kernel(const QLArgs a, const WideHead h) {
           for (int b = 0; b < 4; ++b) {
             const int64_t col = (int64_t)ntile * kWideCols + wn * 64 + cg * 32 + 8 * b + 4 * lh;
             float* o = y + (m0 + rt * 32 + l32) * a.ldy + col;
-            if (rt * 32 + l32 < rows_here)
+            if (rt * 32 + l32 >= rows_here) continue;
+            if (col + 4 <= a.N && (a.ldy & 3) == 0) {
+              *reinterpret_cast<f32x4*>(o) = f32x4{acc[rt][cg][4 * b], acc[rt][cg][4 * b + 1], acc[rt][cg][4 * b + 2], acc[rt][cg][4 * b + 3]};
+            } else {
 #pragma unroll
               for (int e = 0; e < 4; ++e)
                 if (col + e < a.N) o[e] = acc[rt][cg][4 * b + e];
+            }
           }
       return;
     }

@@ -15,7 +15,7 @@ from __future__ import annotations
 import numpy as np
 import torch
 
-from .config import ModelConfig
+from .config import ModelConfig, StackConfig
 
 
 def create_dummy_weights(cfg: ModelConfig, seed: int = 0, device="cpu", scale: float = 0.02,
@@ -63,6 +63,27 @@ def create_dummy_weights(cfg: ModelConfig, seed: int = 0, device="cpu", scale: f
     w[name + ".lora_a"] = normal(K, cfg.lora_rank, s=0.02)
     w[name + ".lora_b"] = normal(cfg.lora_rank, N, s=lora_b_scale)
   return w
+
+
+def create_stack_weights(cfg: StackConfig, seed: int = 0, device="cpu", scale: float | None = None) -> dict:
+  """Random weights of a layer-list decoder, by file name: linears ~ N(0, 1) / sqrt(inputs) (or
+  `scale`), norm weights near zero (around one for the plain norm of a lightning layer), sinks ~ N(0, 1)."""
+  dev = torch.device(device)
+  gen = torch.Generator(device=dev)
+  gen.manual_seed(seed)
+  out = {}
+  for name, shape in cfg.weight_shapes().items():
+    t = torch.randn(*shape, generator=gen, device=dev, dtype=torch.float32)
+    if name.endswith("mix.sink"):
+      pass
+    elif name.endswith("mix.norm"):
+      t = 1.0 + 0.1 * t
+    elif len(shape) == 1:
+      t = 0.1 * t
+    else:
+      t = t * (shape[1] ** -0.5 if scale is None else scale)
+    out[name] = t.to(torch.bfloat16)
+  return out
 
 
 def from_reference_tree(cfg: ModelConfig, tree: dict) -> dict:

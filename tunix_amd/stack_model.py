@@ -279,7 +279,7 @@ class StackRunner(HeadRunner):
     if not self.frag or f.paired:
       return 1
     groups = math.ceil(f.N / 64) * math.ceil(self.M / 128)
-    return int(max(1, min(8, 512 // groups, f.Kp // 512)))
+    return int(max(1, min(8, (256 if self.M > 32 else 512) // groups, f.Kp // 512)))
 
   def linear(self, f: DenseLinear, x, M: int, fp32_out: bool = False) -> L.RowsSrc:
     """Runs one projection of x [M, f.Kp]; returns its output as the reading kernel wants it."""
@@ -315,51 +315,70 @@ class StackRunner(HeadRunner):
     d.out, d.out_ld, d.out_frag = out.data_ptr(), out.shape[1], 1 if frag else 0
     ops.residual_norm(d)
 
-  def _attention(self, ly, m: AttentionMixer, src, entry, col_ptr, starts, B, T) -> torch.Tensor:
-    f = ly["in"]
+  def rotate(self, ly, src, entry, col_ptr, starts, B, T):
+    """Rotates q and k of an attention layer's projection and writes the cache; returns q."""
+    m, f = ly["spec"].mixer, ly["in"]
     dkp, dvp = entry.k.shape[3], entry.v.shape[3]
     q = self._buf("q", m.heads * dkp)
+    d = L.PartRopeDesc()
+    d.B, d.T, d.S, d.H, d.G = B, T, entry.k.shape[2], m.heads, m.kv_heads
+    d.dk, d.dv, d.dkp, d.dvp, d.rot_dims, d.dtype = m.dim, m.vdim, dkp, dvp, m.rot_dims, self.code
+    d.inv_freq, d.y, d.k_off, d.v_off = ly["inv_freq"].data_ptr(), src, f.offsets[1], f.offsets[2]
+    d.starts, d.col_ptr = starts.data_ptr(), col_ptr.data_ptr()
+    d.q_out, d.kcache, d.vcache = q.data_ptr(), entry.k.data_ptr(), entry.v.data_ptr()
+    ops.part_rope_kvwrite(d)
+    return q
+
+  def attend(self, ly, q, entry, col_ptr, starts, B, T) -> torch.Tensor:
+    m = ly["spec"].mixer
     out = self._buf("attn", ly["out"].Kp)
-    rd = L.PartRopeDesc()
-    rd.B, rd.T, rd.S, rd.H, rd.G = B, T, entry.k.shape[2], m.heads, m.kv_heads
-    rd.dk, rd.dv, rd.dkp, rd.dvp, rd.rot_dims, rd.dtype = m.dim, m.vdim, dkp, dvp, m.rot_dims, self.code
-    rd.inv_freq, rd.y, rd.k_off, rd.v_off = ly["inv_freq"].data_ptr(), src, f.offsets[1], f.offsets[2]
-    rd.starts, rd.col_ptr = starts.data_ptr(), col_ptr.data_ptr()
-    rd.q_out, rd.kcache, rd.vcache = q.data_ptr(), entry.k.data_ptr(), entry.v.data_ptr()
-    ops.part_rope_kvwrite(rd)
-    ad = L.SinkAttnDesc()
-    ad.B, ad.T, ad.S, ad.H, ad.G = rd.B, rd.T, rd.S, rd.H, rd.G
-    ad.dk, ad.dv, ad.dkp, ad.dvp, ad.scale, ad.dtype = m.dim, m.vdim, dkp, dvp, m.scale, self.code
-    ad.q, ad.kcache, ad.vcache = rd.q_out, rd.kcache, rd.vcache
-    ad.sinks = None if ly["sink"] is None else ly["sink"].data_ptr()
-    ad.starts, ad.col_ptr = rd.starts, rd.col_ptr
-    ad.kv_chunk = self._kv_chunk(m, self.kv_chunk_arg) if T == 1 else 0
-    ad.ws, ad.out, ad.out_ld, ad.out_frag = self.attn_ws.data_ptr(), out.data_ptr(), out.shape[1], 1 if self.frag else 0
-    ops.sink_attn(ad)
+    d = L.SinkAttnDesc()
+    d.B, d.T, d.S, d.H, d.G = B, T, entry.k.shape[2], m.heads, m.kv_heads
+    d.dk, d.dv, d.dkp, d.dvp, d.scale, d.dtype = m.dim, m.vdim, entry.k.shape[3], entry.v.shape[3], m.scale, self.code
+    d.q, d.kcache, d.vcache = q.data_ptr(), entry.k.data_ptr(), entry.v.data_ptr()
+    d.sinks = None if ly["sink"] is None else ly["sink"].data_ptr()
+    d.starts, d.col_ptr = starts.data_ptr(), col_ptr.data_ptr()
+    d.kv_chunk = self._kv_chunk(m, self.kv_chunk_arg) if T == 1 else 0
+    d.ws, d.out, d.out_ld, d.out_frag = self.attn_ws.data_ptr(), out.data_ptr(), out.shape[1], 1 if self.frag else 0
+    ops.sink_attn(d)
     return out
 
-  def _lightning(self, ly, m: LightningMixer, src, entry, col_ptr, starts, B, T) -> torch.Tensor:
-    f, W = ly["in"], m.heads * m.vdim
-    o = self._buf("state_out", W, torch.float32)
-    out = self._buf("gated", ly["out"].Kp)
+  def recur(self, ly, src, entry, col_ptr, starts, B, T) -> torch.Tensor:
+    """The lightning recurrence of a projection's rows: fp32 [rows, heads * vdim]."""
+    m, f = ly["spec"].mixer, ly["in"]
+    o = self._buf("state_out", m.heads * m.vdim, torch.float32)
     d = L.LightningDesc()
     d.B, d.T, d.H, d.dk, d.dv, d.dtype = B, T, m.heads, m.dim, m.vdim, self.code
     d.decay, d.y, d.k_off, d.v_off = ly["decay"].data_ptr(), src, f.offsets[1], f.offsets[2]
     d.starts, d.col_ptr, d.state = starts.data_ptr(), col_ptr.data_ptr(), entry.s.data_ptr()
-    d.o, d.o_ld, d.ws = o.data_ptr(), W, self.light_ws.data_ptr()
+    d.o, d.o_ld, d.ws = o.data_ptr(), o.shape[1], self.light_ws.data_ptr()
     ops.lightning(d)
-    g = L.GatedNormDesc()
-    g.M, g.W, g.dtype, g.eps, g.w_offset = B * T, W, self.code, self.cfg.norm_eps, 0.0
-    g.o, g.o_ld, g.g, g.g_off, g.w = d.o, W, src, f.offsets[3], ly["norm"].data_ptr()
-    g.out, g.out_ld, g.out_frag = out.data_ptr(), out.shape[1], 1 if self.frag else 0
-    ops.gated_norm(g)
+    return o
+
+  def gate(self, ly, o, src, M: int) -> torch.Tensor:
+    """norm(o) . weight * sigmoid(gate columns of the projection)."""
+    out = self._buf("gated", ly["out"].Kp)
+    d = L.GatedNormDesc()
+    d.M, d.W, d.dtype, d.eps, d.w_offset = M, o.shape[1], self.code, self.cfg.norm_eps, 0.0
+    d.o, d.o_ld, d.g, d.g_off, d.w = o.data_ptr(), o.shape[1], src, ly["in"].offsets[3], ly["norm"].data_ptr()
+    d.out, d.out_ld, d.out_frag = out.data_ptr(), out.shape[1], 1 if self.frag else 0
+    ops.gated_norm(d)
     return out
 
-  def _mlp(self, ly, h, M: int) -> L.RowsSrc:
-    f, down = ly["gu"], ly["down"]
-    act = self._buf("act", down.Kp)
+  def _mixer(self, ly, h, entry, col_ptr, starts, B, T) -> L.RowsSrc:
+    src = self.linear(ly["in"], h, B * T)
+    if isinstance(ly["spec"].mixer, AttentionMixer):
+      q = self.rotate(ly, src, entry, col_ptr, starts, B, T)
+      out = self.attend(ly, q, entry, col_ptr, starts, B, T)
+    else:
+      out = self.gate(ly, self.recur(ly, src, entry, col_ptr, starts, B, T), src, B * T)
+    return self.linear(ly["out"], out, B * T)
+
+  def gate_up(self, ly, h, M: int) -> torch.Tensor:
+    f = ly["gu"]
+    act = self._buf("act", ly["down"].Kp)
     if self.dtype == torch.float32:
-      src = self.linear(f, h, M)
+      self.linear(f, h, M)
       ops.gelu_mul(self.y[:M * f.N].view(M, f.N), f.offsets[1], M, ly["spec"].mlp.ff, act)
     else:
       d = L.DenseDesc()
@@ -367,7 +386,7 @@ class StackRunner(HeadRunner):
       d.x, d.ldx, d.x_frag, d.w = h.data_ptr(), h.shape[1], 1 if self.frag else 0, f.w.data_ptr()
       d.epilogue, d.y, d.ldy, d.y_frag, d.split_k = L.TNX_EPI_GELU_MUL, act.data_ptr(), act.shape[1], 1 if self.frag else 0, 1
       ops.dense_linear(d)
-    return self.linear(down, act, M)
+    return act
 
   def forward_hidden(self, tokens, positions, col_ptr, cache, B=None, T=None, segment_ids=None, starts=None):
     """Runs all layers for tokens[b, col .. col+T) of each row from what `cache` holds of the columns
@@ -395,17 +414,14 @@ class StackRunner(HeadRunner):
 
     for (i, begins), entry in zip(cfg.layer_runs, cache.entries):
       ly = m.layers[i]
-      mixer = ly["spec"].mixer
       if begins:   # a pass of the loop: x <- W [x; embedding output]
         norm(None, cat, self.frag)
         pending = ("set", self.linear(m.loop_in, cat, M, fp32_out=True), None)
       norm(ly["norm1"], h, self.frag)
-      src = self.linear(ly["in"], h, M)
-      mix = self._attention if isinstance(mixer, AttentionMixer) else self._lightning
-      pending = ("add", self.linear(ly["out"], mix(ly, mixer, src, entry, col_ptr, starts, B, T), M), ly["norm1b"])
+      pending = ("add", self._mixer(ly, h, entry, col_ptr, starts, B, T), ly["norm1b"])
       if "gu" in ly:
         norm(ly["norm2"], h, self.frag)
-        pending = ("add", self._mlp(ly, h, M), ly["norm2b"])
+        pending = ("add", self.linear(ly["down"], self.gate_up(ly, h, M), M), ly["norm2b"])
       behind_layer = True
     norm(m.final_norm, self.xn, False)
     return self.xn
