@@ -156,9 +156,9 @@ def test_oracle_is_causal():
   d = C.CONFIGS["mixed"]
   w = C.random_weights(d, 3)
   toks = C.tokens(d, 20, 4)
-  a = R.forward(d, w, toks)
+  a = R.forward(d, w, toks, torch.float64)
   other = list(toks)
   other[12] = (other[12] + 1) % d["vocab"]
-  b = R.forward(d, w, other)
+  b = R.forward(d, w, other, torch.float64)
   assert torch.allclose(a[:12], b[:12], atol=1e-5) and not torch.allclose(a[12:], b[12:], atol=1e-3)
-  np.testing.assert_allclose(a[:7].numpy(), R.forward(d, w, toks[:7]).numpy(), atol=1e-4)
+  np.testing.assert_allclose(a[:7].numpy(), R.forward(d, w, toks[:7], torch.float64).numpy(), atol=1e-8)

@@ -29,6 +29,16 @@ __global__ __launch_bounds__(256) void embed_rows_kernel(const T* table, int64_t
   const int col = col_ptr ? *col_ptr : 0;
   int64_t id = ids[b * ids_ld + col + t];
   if (id < 0 || id >= V) id = 0;   // padding columns: never read by a later token
+  if (D % 8 == 0 && cat_ld % 8 == 0) {   // (cat_off is then a multiple of eight, too, where cat is given)
+    const RowSrc<T> src{table, nullptr, 1, 0, D};
+    for (int64_t i = (int64_t)threadIdx.x * 8; i < D; i += 2048) {
+      float f[8];
+      get8(src, id, i, f);
+      put8(x + row * D + i, f);
+      if (cat) put8(cat + (cat_frag ? frag_index(row, cat_off + i, cat_ld) : row * cat_ld + cat_off + i), f);
+    }
+    return;
+  }
   for (int64_t i = threadIdx.x; i < D; i += 256) {
     const T v = table[id * D + i];
     x[row * D + i] = ld_elem(&v, 0);
@@ -434,7 +444,7 @@ extern "C" int tnx_embed_rows(void* stream, int dtype, const void* table, int64_
                               int64_t cat_ld, int64_t cat_off, int cat_frag) {
   TNX_REQUIRE(table && ids && x, "embed_rows: null pointer");
   TNX_REQUIRE(V > 0 && D > 0 && B > 0 && T > 0, "embed_rows: bad shape");
-  TNX_REQUIRE(!cat || cat_ld >= cat_off + D, "embed_rows: the second copy does not fit its rows");
+  TNX_REQUIRE(!cat || (cat_ld >= cat_off + D && cat_off % D == 0), "embed_rows: the second copy does not fit its rows");
   TNX_REQUIRE(dtype == TNX_BF16 || dtype == TNX_F32, "embed_rows: bad dtype %d", dtype);
   if (dtype == TNX_BF16)
     hipLaunchKernelGGL(embed_rows_kernel<uint16_t>, dim3((unsigned)(B * T)), dim3(256), 0, as_stream(stream), (const uint16_t*)table,
