@@ -84,7 +84,10 @@ def test_struct_layouts_match_the_header(tmp_path):
   # the descriptor structs cross the C ABI by pointer: the ctypes mirrors must have the sizes and
   # the field offsets a C compiler gives the header's structs
   pairs = {"tnx_qlinear_desc": L.QLinearDesc, "tnx_rope_desc": L.RopeDesc,
-           "tnx_attn_desc": L.AttnDesc, "tnx_lmhead_desc": L.LmHeadDesc, "tnx_moe_gmm_desc": L.MoeGmmDesc}
+           "tnx_attn_desc": L.AttnDesc, "tnx_lmhead_desc": L.LmHeadDesc, "tnx_moe_gmm_desc": L.MoeGmmDesc,
+           "tnx_rows_src": L.RowsSrc, "tnx_dense_desc": L.DenseDesc, "tnx_residual_norm_desc": L.ResidualNormDesc,
+           "tnx_part_rope_desc": L.PartRopeDesc, "tnx_sink_attn_desc": L.SinkAttnDesc, "tnx_lightning_desc": L.LightningDesc,
+           "tnx_gated_norm_desc": L.GatedNormDesc, "tnx_logits_desc": L.LogitsDesc}
   lines = ['#include <stdio.h>', '#include <stddef.h>', '#include "tunix_hip.h"', 'int main(void) {']
   for cname, cls in pairs.items():
     lines.append(f'  printf("{cname} %zu\\n", sizeof({cname}));')

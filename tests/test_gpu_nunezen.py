@@ -1,7 +1,6 @@
 """Nunezen on the GPU against the plain implementation (oracle/nunezen_ref.py): every mechanism alone,
 then whole models -- prompts, token-by-token decoding, portions, unequal batches, reused slots, greedy
 generation -- in bf16 and in fp32, at sizes that reach every kernel."""
-import ctypes
 import json
 import math
 import os
@@ -15,7 +14,7 @@ import torch
 from oracle import nunezen_ref as R
 from tests import nunezen_cases as C
 from tunix_amd import _lib as L
-from tunix_amd import config, ops, registry
+from tunix_amd import config, ops
 from tunix_amd.generate import CacheConfig, Sampler
 from tunix_amd.generate.replay import Replay
 from tunix_amd.generate.utils import IdTokenizer
@@ -269,7 +268,7 @@ class Attn:
         assert float(d) < tol, (b, float(d))
 
 
-SHAPES = [(4, 1, 64, 80, 32), (6, 2, 48, 24, 48), (5, 1, 136, 200, 2), (8, 8, 32, 64, 0), (3, 3, 256, 256, 256), (10, 5, 21, 45, 6),
+SHAPES = [(6, 1, 64, 112, 48), (6, 2, 48, 24, 48), (5, 1, 136, 200, 2), (8, 8, 32, 64, 0), (3, 3, 256, 256, 256), (10, 5, 21, 45, 6),
           (16, 4, 128, 128, 64), (2, 1, 192, 128, 64), (40, 1, 64, 64, 32), (2, 1, 320, 300, 64)]
 
 
@@ -732,15 +731,4 @@ def test_descriptor_errors(gpu):
   r.B, r.T, r.S, r.H, r.G, r.dk, r.dv, r.dkp, r.dvp, r.rot_dims = 1, 1, 8, 2, 2, 16, 16, 16, 16, 18
   with pytest.raises(ValueError, match="rot_dims"):
     ops.part_rope_kvwrite(r)
-  with pytest.raises(ValueError, match="not in"):
-    registry.ARCHITECTURES["llama3"].dtypes and registry.load_model(_llama_folder(), gpu, F32)
-  assert ctypes.sizeof(L.RowsSrc) == 40
 
-
-def _llama_folder():
-  import tempfile
-  f = tempfile.mkdtemp()
-  q = {"architecture": "llama3", "num_layers": 1, "vocab_size": 64, "embed_dim": 128, "hidden_dim": 256, "num_heads": 2,
-       "num_kv_heads": 1, "head_dim": 64}
-  json.dump(q, open(os.path.join(f, "config.json"), "w"))
-  return f

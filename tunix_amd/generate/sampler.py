@@ -3,7 +3,8 @@ with the jitted prefill / while_loop decode replaced by libtunix_hip.so kernels.
 
 Same call contract as the reference: `Sampler(transformer, tokenizer, cache_config)` and
 `sampler(input_strings, max_generation_steps, ...) -> SamplerOutput`.  `transformer` is a
-`tunix_amd.model.QLoRAModel` or a `tunix_amd.stack_model.StackModel`.  One decode step is captured into a HIP graph and replayed: the
+`tunix_amd.model.QLoRAModel` or a `tunix_amd.stack_model.StackModel`.  One decode step is captured
+into a HIP graph and replayed: the
 step counter, positions and token buffer live in device memory, so no host round trip happens
 inside the loop.
 """
