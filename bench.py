@@ -660,7 +660,7 @@ def stack_kernels(model, runner, st, ctx, iters):
   us = in_turn([lambda: runner.gate(ll, o, lsrc, M)], iters)
   out["gated norm"] = roof_row(us, M * o.shape[1] * 8, 0)
   osrc = runner.linear(ly0["out"], runner._buf("attn", ly0["out"].Kp), M)
-  us = in_turn([lambda: runner.residual_norm(("add", osrc, ly0["norm1b"]), ly0["norm2"], h, M, runner.frag)], iters)
+  us = in_turn([lambda: runner.residual_norm(("add", osrc, ly0["post1"]), ly0["norm2"], h, M, runner.frag)], iters)
   out["post-norm + residual + norm"] = roof_row(us, M * D * (2 + 8 + 2), 0)
   return out
 

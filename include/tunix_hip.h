@@ -70,9 +70,12 @@ const char* tnx_last_error(void);
  * the measurement probe tnx_stream_read out of the library; 3.0 adds tnx_qw_expand /
  * tnx_qw_expanded_bytes, tnx_dense_expand and the w_expanded field of tnx_qlinear_desc and
  * tnx_lmhead_desc; 3.1 adds tnx_sample_topk_head / tnx_sample_topk_head_ok; 3.2 adds the entry
- * points of decoders with dense weights (tnx_dense_linear to tnx_logits_stats). */
-#define TNX_ABI_VERSION_MAJOR 3
-#define TNX_ABI_VERSION_MINOR 2
+ * points of decoders with dense weights (tnx_dense_linear to tnx_logits_stats); 4.0 adds batches and experts
+ * to tnx_dense_desc, parts, routed rows and the token shift to tnx_residual_norm_desc, the gate in front
+ * to tnx_gated_norm_desc, out_head to tnx_sink_attn_desc, and tnx_silu_mul, tnx_route_softmax,
+ * tnx_short_conv, tnx_ring_write, tnx_ssd, tnx_latent_* and tnx_gate_mul. */
+#define TNX_ABI_VERSION_MAJOR 4
+#define TNX_ABI_VERSION_MINOR 0
 #define TNX_ABI_VERSION ((TNX_ABI_VERSION_MAJOR << 16) | TNX_ABI_VERSION_MINOR)
 int tnx_version(void);
 
@@ -566,9 +569,13 @@ typedef struct {
 
 /* y[M, N] = x[M, K] . w^T.  bf16: w is the fragment-order copy of tnx_dense_expand, K % 128 == 0
  * (zero-padded), N % 16 == 0 for bf16 outputs.  fp32: w row-major [N, K], K % 16 == 0.
- * epilogue: TNX_EPI_STORE (model dtype), TNX_EPI_F32, or (bf16) TNX_EPI_GELU_MUL: w's rows come in
- * alternating blocks of 16 gate and 16 up rows and y[M, N/2] = gelu_tanh(gate) * up, formed in fp32
- * and rounded once.  split_k > 1 (bf16, few rows): fp32 planes to ws [split_k][M][ldy] instead. */
+ * epilogue: TNX_EPI_STORE (model dtype), TNX_EPI_F32, or (bf16) TNX_EPI_GELU_MUL / TNX_EPI_SILU_MUL: w's
+ * rows come in alternating blocks of 16 gate and 16 up rows and y[M, N/2] = act(gate) * up with act =
+ * gelu_tanh / silu, formed in fp32 and rounded once.  split_k > 1 (bf16, few rows): fp32 planes to ws
+ * [split_k][M][ldy] instead.
+ * batch > 1: the same for z = 0 .. batch - 1 with x, w and y moved on by z times their strides.
+ * n_experts > 0: M counts routes; route r of expert e (sorted_route[offsets[e] .. offsets[e + 1])) reads row
+ * r / x_div of x and weight e (w + e * w_stride) and writes row r of y. */
 typedef struct {
   int64_t M, K, N;
   int dtype;
@@ -582,6 +589,11 @@ typedef struct {
   int y_frag;
   int split_k;
   float* ws;
+  int64_t batch;
+  int64_t x_stride, w_stride, y_stride;   /* elements */
+  int n_experts, x_div;
+  const int32_t* offsets;                 /* [n_experts + 1] */
+  const int32_t* sorted_route;            /* [M] */
 } tnx_dense_desc;
 int tnx_dense_linear(void* stream, const tnx_dense_desc* d);
 
@@ -592,9 +604,16 @@ int tnx_embed_rows(void* stream, int dtype, const void* table, int64_t V, int64_
                    int64_t cat_ld, int64_t cat_off, int cat_frag);
 
 /* The residual step between two sublayers, in fp32:
- *   mode 1: x += norm(y) * (w_offset + w_post);  mode 2: x = y;  mode 0: x stays;
+ *   mode 1: x += norm(y) * (w_offset + w_post);  mode 2: x = y;  mode 3: x = norm(x) * (w_offset + w_post);
+ *   mode 0: x stays;
  *   out (model dtype) = norm(x) * (w_offset + w_next), or x itself when w_next is null,
- * with norm(v) = v / sqrt(mean(v^2) + eps).  y.ws with split_k >= 1: fp32 planes. */
+ * with norm(v) = v / sqrt(mean(v^2) + eps), over each of `groups` equal parts of the row (0: one part).  y.ws
+ * with split_k >= 1: fp32 planes.  x_out (null: x) takes the new x.
+ * route_w (null: none): y holds route_k rows per row of x, which are summed with the weights route_w[row, :].
+ * shift (null: none; instead of w_next): out = x + (x' - x) * shift with x' the x of the token before: the row in
+ * front of it, or `before` [B, D] for the first token of a call (zeros for the first token of a sequence).  The
+ * rows are T tokens for each of B sequences.  T == 1: `before` takes the new x; T > 1: x_out is another
+ * buffer than x, and the caller keeps the last rows (tnx_ring_write). */
 typedef struct {
   int64_t M, D;
   int dtype;
@@ -607,6 +626,15 @@ typedef struct {
   void* out;
   int64_t out_ld;
   int out_frag;
+  int groups;
+  float* x_out;
+  const float* route_w;
+  int route_k;
+  const float* shift;
+  float* before;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  int64_t B, T;
 } tnx_residual_norm_desc;
 int tnx_residual_norm(void* stream, const tnx_residual_norm_desc* d);
 
@@ -630,7 +658,7 @@ typedef struct {
 int tnx_part_rope_kvwrite(void* stream, const tnx_part_rope_desc* d);
 
 /* Causal attention over keys starts[b] .. col + t with softmax(scale * q.k) whose denominator also
- * holds exp(sinks[head]) (sinks null: none).  out[row, head * dv ..].  kv_chunk > 0 splits the key range (few
+ * holds exp(sinks[head]) (sinks null: none).  out[row, head * out_head ..] (out_head 0: dv).  kv_chunk > 0 splits the key range (few
  * query rows, workspace of tnx_sink_attn_ws_bytes).  tnx_sink_attn_pad: the padded head size the
  * MFMA kernels take (other sizes, and fp32, run a plain kernel). */
 typedef struct {
@@ -649,6 +677,7 @@ typedef struct {
   void* out;
   int64_t out_ld;
   int out_frag;
+  int64_t out_head;
 } tnx_sink_attn_desc;
 int tnx_sink_attn_pad(int dim, int is_value);
 size_t tnx_sink_attn_ws_bytes(int64_t B, int64_t T, int64_t S, int H, int dvp, int kv_chunk);
@@ -674,7 +703,8 @@ typedef struct {
 size_t tnx_lightning_ws_bytes(int64_t B, int64_t T, int H, int dk, int dv);
 int tnx_lightning(void* stream, const tnx_lightning_desc* d);
 
-/* out = norm(o) * (w_offset + w) * sigmoid(g[:, g_off ..]) over whole rows of W values. */
+/* out = norm(o) * (w_offset + w) * sigmoid(g[:, g_off ..]) over whole rows of W values; gate_first: out =
+ * norm(o * silu(g[:, g_off ..])) * (w_offset + w) over each of `groups` equal parts of a row (0: one). */
 typedef struct {
   int64_t M, W;
   int dtype;
@@ -687,12 +717,170 @@ typedef struct {
   void* out;
   int64_t out_ld;
   int out_frag;
+  int gate_first, groups;
 } tnx_gated_norm_desc;
 int tnx_gated_norm(void* stream, const tnx_gated_norm_desc* d);
 
 /* out[M, F] = gelu_tanh(y[:, :F]) * y[:, up_off : up_off + F]. */
 int tnx_gelu_mul(void* stream, int dtype, const void* y, int64_t ld, int64_t up_off, int64_t M, int64_t F,
                  void* out, int64_t out_ld);
+/* The same with silu. */
+int tnx_silu_mul(void* stream, int dtype, const void* y, int64_t ld, int64_t up_off, int64_t M, int64_t F,
+                 void* out, int64_t out_ld);
+
+/* Choice of experts from fp32 logits z [M, E] (z.y fp32, or planes): topk_id int32 [M, k], the k largest logits in
+ * descending order (lower id first among equals); topk_w fp32 [M, k], the softmax over these k alone. */
+int tnx_route_softmax(void* stream, const tnx_rows_src* z, int64_t M, int E, int k, float* topk_w, int32_t* topk_id);
+
+/* Causal convolution per channel and silu: out[row, c] = silu(bias[c] + sum_j w[taps - 1 - j, c] u(t - j, c)) for
+ * the channels off .. off + C - 1 of y.  Tokens before the call's first one come from the ring [B, slots, C] (model
+ * dtype, slot = column % slots, slots >= taps - 1); before starts[b] lie zeros.  The ring is not written. */
+typedef struct {
+  int64_t B, T, C;
+  int taps, slots;
+  int dtype;
+  tnx_rows_src y;
+  int64_t off;
+  const float* w;
+  const float* bias;
+  const void* ring;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  void* out;
+  int64_t out_ld;
+} tnx_short_conv_desc;
+int tnx_short_conv(void* stream, const tnx_short_conv_desc* d);
+/* ring[b, (col + t) % slots, :] = y[b * T + t, off .. off + C) for the last min(T, slots) tokens. */
+int tnx_ring_write(void* stream, int dtype, const tnx_rows_src* y, int64_t off, int64_t B, int64_t T, int64_t C, int slots,
+                   const int32_t* col_ptr, void* ring);
+
+/* State-space duality: per head h (group h / (H / G)), dt = softplus(y[:, dt_off + h] + dt_bias[h]),
+ *   S <- exp(-exp(A_log[h]) dt) S + dt B x^T,  o[row, h * P ..] = S^T C + D[h] x.
+ * u: convolved rows (model dtype): x [H, P] from column 0, B [G, N] behind it, C [G, N] behind that.  u null, T == 1 and
+ * tnx_ssd_step_ok: x, B and C are formed from y's channels c_off .. with the convolution of tnx_short_conv
+ * (slots >= taps), whose ring takes the current inputs.  state fp32 [B, H, N, P] is read unless col <= starts[b] and
+ * written back; o fp32.  ws: tnx_ssd_ws_bytes. */
+typedef struct {
+  int64_t B, T;
+  int H, G, N, P;
+  int dtype;
+  const float* A_log;
+  const float* dt_bias;
+  const float* D;
+  tnx_rows_src y;
+  int64_t dt_off;
+  const void* u;
+  int64_t u_ld;
+  int64_t c_off;
+  int taps, slots;
+  const float* conv_w;
+  const float* conv_b;
+  void* ring;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  float* state;
+  float* o;
+  int64_t o_ld;
+  float* ws;
+} tnx_ssd_desc;
+int tnx_ssd_step_ok(int N, int P);
+size_t tnx_ssd_ws_bytes(int64_t B, int64_t T, int H, int G, int N, int P);
+int tnx_ssd(void* stream, const tnx_ssd_desc* d);
+
+/* Attention through a latent.  A position's cache row (model dtype, `row` elements): its latent c [rank], zeros to
+ * rank_pad = rank rounded up to 16, the rotated key part [rot] that all heads share, zeros to row.  tnx_latent_row: the row
+ * length to use.
+ * tnx_latent_prep: q_out = norm(y[:, q_off .. + q_rank]) * w_q, c = norm(y[:, kv_off .. + rank]) * w_kv (also to c_out
+ * unless null), the rot columns behind it rotated (pairs (2i, 2i + 1), angle position * inv_freq[i]), cache row at slot
+ * col + t. */
+typedef struct {
+  int64_t B, T, S;
+  int q_rank, rank, rot, rank_pad, row;
+  int dtype;
+  float eps;
+  tnx_rows_src y;
+  int64_t q_off, kv_off;
+  const float* w_q;
+  const float* w_kv;
+  const float* inv_freq;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  void* q_out;
+  int64_t q_ld;
+  int q_frag;
+  void* c_out;
+  int64_t c_ld;
+  int c_frag;
+  void* cache;
+} tnx_latent_prep_desc;
+int tnx_latent_row(int rank, int rot, int dtype);
+int tnx_latent_prep(void* stream, const tnx_latent_prep_desc* d);
+/* Heads of y ([n unrotated, r rotated] each): un[row, head * un_ld ..] = the first n and zeros to un_pad,
+ * rot[row, head * rot_ld ..] = the last r, rotated as above, and zeros to rot_pad. */
+typedef struct {
+  int64_t B, T;
+  int H, n, r;
+  int dtype;
+  tnx_rows_src y;
+  const float* inv_freq;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  void* un;
+  int64_t un_ld;
+  int un_pad;
+  void* rot;
+  int64_t rot_ld;
+  int rot_pad;
+} tnx_latent_q_desc;
+int tnx_latent_q(void* stream, const tnx_latent_q_desc* d);
+/* Operands of tnx_sink_attn for the first T columns: k [B, H, T, dkp] = [y's n columns of the head | the cache row's
+ * rotated part], v [B, H, T, dvp] = y's vd columns of the head from v_off on; zeros behind. */
+typedef struct {
+  int64_t B, T, S;
+  int H, n, r, vd, dkp, dvp, rank_pad, row;
+  int dtype;
+  tnx_rows_src y;
+  int64_t v_off;
+  const void* cache;
+  void* k;
+  void* v;
+} tnx_latent_kv_desc;
+int tnx_latent_kv(void* stream, const tnx_latent_kv_desc* d);
+/* bf16: q [B * T, H, row] against the cache rows of columns starts[b] .. col + t, softmax(scale * q . row), out[row, head]
+ * [out_head] = the weighted sum of the rows' first `rank` elements.  kv_chunk > 0 (a multiple of 128) splits the key
+ * range (workspace of tnx_latent_attn_ws_bytes).  Rows of other lengths, and fp32: tnx_sink_attn with one kv head whose
+ * keys and values are the cache rows. */
+typedef struct {
+  int64_t B, T, S;
+  int H, rank, row;
+  float scale;
+  const void* q;
+  const void* cache;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  int kv_chunk;
+  float* ws;
+  void* out;
+  int64_t out_head;
+} tnx_latent_attn_desc;
+int tnx_latent_attn_ok(int rank, int row, int64_t S);
+size_t tnx_latent_attn_ws_bytes(int64_t B, int64_t T, int64_t S, int H, int rank, int kv_chunk);
+int tnx_latent_attn(void* stream, const tnx_latent_attn_desc* d);
+
+/* out[row, i] = y[row * y_ld + (i / head) * y_head + i % head] * sigmoid(g[row, g_off + i]), i < W. */
+typedef struct {
+  int64_t M, W;
+  int head;
+  int dtype;
+  const void* y;
+  int64_t y_ld, y_head;
+  tnx_rows_src g;
+  int64_t g_off;
+  void* out;
+  int64_t out_ld;
+  int out_frag;
+} tnx_gate_mul_desc;
+int tnx_gate_mul(void* stream, const tnx_gate_mul_desc* d);
 
 /* Statistics and the whole-vocabulary draw of tnx_lmhead_logp over finished fp32 logits [M, V]
  * (any V); the fields mean what they mean there. */

@@ -12,7 +12,7 @@ _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libtunix_hip.so")
 
 # the ABI this binding was written against (TNX_ABI_VERSION_MAJOR / _MINOR of include/tunix_hip.h)
-ABI_VERSION = (3, 2)
+ABI_VERSION = (4, 0)
 
 TNX_Q_INT4, TNX_Q_NF4 = 0, 1
 TNX_NORM_LLAMA, TNX_NORM_QWEN3, TNX_NORM_GEMMA3 = 0, 1, 2
@@ -102,6 +102,8 @@ class DenseDesc(C.Structure):
       ("M", _i64), ("K", _i64), ("N", _i64), ("dtype", _i32),
       ("x", _p), ("ldx", _i64), ("x_frag", _i32), ("w", _p), ("epilogue", _i32),
       ("y", _p), ("ldy", _i64), ("y_frag", _i32), ("split_k", _i32), ("ws", _p),
+      ("batch", _i64), ("x_stride", _i64), ("w_stride", _i64), ("y_stride", _i64),
+      ("n_experts", _i32), ("x_div", _i32), ("offsets", _p), ("sorted_route", _p),
   ]
 
 
@@ -109,6 +111,8 @@ class ResidualNormDesc(C.Structure):
   _fields_ = [
       ("M", _i64), ("D", _i64), ("dtype", _i32), ("eps", _f32), ("w_offset", _f32), ("mode", _i32),
       ("y", RowsSrc), ("w_post", _p), ("x", _p), ("w_next", _p), ("out", _p), ("out_ld", _i64), ("out_frag", _i32),
+      ("groups", _i32), ("x_out", _p), ("route_w", _p), ("route_k", _i32), ("shift", _p), ("before", _p),
+      ("starts", _p), ("col_ptr", _p), ("B", _i64), ("T", _i64),
   ]
 
 
@@ -127,6 +131,7 @@ class SinkAttnDesc(C.Structure):
       ("H", _i32), ("G", _i32), ("dk", _i32), ("dv", _i32), ("dkp", _i32), ("dvp", _i32),
       ("scale", _f32), ("dtype", _i32), ("q", _p), ("kcache", _p), ("vcache", _p), ("sinks", _p),
       ("starts", _p), ("col_ptr", _p), ("kv_chunk", _i32), ("ws", _p), ("out", _p), ("out_ld", _i64), ("out_frag", _i32),
+      ("out_head", _i64),
   ]
 
 
@@ -142,7 +147,65 @@ class GatedNormDesc(C.Structure):
   _fields_ = [
       ("M", _i64), ("W", _i64), ("dtype", _i32), ("eps", _f32), ("w_offset", _f32),
       ("o", _p), ("o_ld", _i64), ("g", RowsSrc), ("g_off", _i64), ("w", _p),
-      ("out", _p), ("out_ld", _i64), ("out_frag", _i32),
+      ("out", _p), ("out_ld", _i64), ("out_frag", _i32), ("gate_first", _i32), ("groups", _i32),
+  ]
+
+
+class ShortConvDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("C", _i64), ("taps", _i32), ("slots", _i32), ("dtype", _i32),
+      ("y", RowsSrc), ("off", _i64), ("w", _p), ("bias", _p), ("ring", _p), ("starts", _p), ("col_ptr", _p),
+      ("out", _p), ("out_ld", _i64),
+  ]
+
+
+class SsdDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("H", _i32), ("G", _i32), ("N", _i32), ("P", _i32), ("dtype", _i32),
+      ("A_log", _p), ("dt_bias", _p), ("D", _p), ("y", RowsSrc), ("dt_off", _i64), ("u", _p), ("u_ld", _i64),
+      ("c_off", _i64), ("taps", _i32), ("slots", _i32), ("conv_w", _p), ("conv_b", _p), ("ring", _p),
+      ("starts", _p), ("col_ptr", _p), ("state", _p), ("o", _p), ("o_ld", _i64), ("ws", _p),
+  ]
+
+
+class LatentPrepDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("S", _i64),
+      ("q_rank", _i32), ("rank", _i32), ("rot", _i32), ("rank_pad", _i32), ("row", _i32), ("dtype", _i32), ("eps", _f32),
+      ("y", RowsSrc), ("q_off", _i64), ("kv_off", _i64), ("w_q", _p), ("w_kv", _p), ("inv_freq", _p),
+      ("starts", _p), ("col_ptr", _p), ("q_out", _p), ("q_ld", _i64), ("q_frag", _i32),
+      ("c_out", _p), ("c_ld", _i64), ("c_frag", _i32), ("cache", _p),
+  ]
+
+
+class LatentQDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("H", _i32), ("n", _i32), ("r", _i32), ("dtype", _i32), ("y", RowsSrc),
+      ("inv_freq", _p), ("starts", _p), ("col_ptr", _p),
+      ("un", _p), ("un_ld", _i64), ("un_pad", _i32), ("rot", _p), ("rot_ld", _i64), ("rot_pad", _i32),
+  ]
+
+
+class LatentKvDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("S", _i64),
+      ("H", _i32), ("n", _i32), ("r", _i32), ("vd", _i32), ("dkp", _i32), ("dvp", _i32), ("rank_pad", _i32), ("row", _i32),
+      ("dtype", _i32), ("y", RowsSrc), ("v_off", _i64), ("cache", _p), ("k", _p), ("v", _p),
+  ]
+
+
+class LatentAttnDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("S", _i64), ("H", _i32), ("rank", _i32), ("row", _i32), ("scale", _f32),
+      ("q", _p), ("cache", _p), ("starts", _p), ("col_ptr", _p), ("kv_chunk", _i32), ("ws", _p),
+      ("out", _p), ("out_head", _i64),
+  ]
+
+
+class GateMulDesc(C.Structure):
+  _fields_ = [
+      ("M", _i64), ("W", _i64), ("head", _i32), ("dtype", _i32), ("y", _p), ("y_ld", _i64), ("y_head", _i64),
+      ("g", RowsSrc), ("g_off", _i64), ("out", _p), ("out_ld", _i64), ("out_frag", _i32),
   ]
 
 
@@ -212,6 +275,21 @@ SIGNATURES = {
     "tnx_lightning": (_i32, [_p, C.POINTER(LightningDesc)]),
     "tnx_gated_norm": (_i32, [_p, C.POINTER(GatedNormDesc)]),
     "tnx_gelu_mul": (_i32, [_p, _i32, _p, _i64, _i64, _i64, _i64, _p, _i64]),
+    "tnx_silu_mul": (_i32, [_p, _i32, _p, _i64, _i64, _i64, _i64, _p, _i64]),
+    "tnx_route_softmax": (_i32, [_p, C.POINTER(RowsSrc), _i64, _i32, _i32, _p, _p]),
+    "tnx_short_conv": (_i32, [_p, C.POINTER(ShortConvDesc)]),
+    "tnx_ring_write": (_i32, [_p, _i32, C.POINTER(RowsSrc), _i64, _i64, _i64, _i64, _i32, _p, _p]),
+    "tnx_ssd_step_ok": (_i32, [_i32, _i32]),
+    "tnx_ssd_ws_bytes": (C.c_size_t, [_i64, _i64, _i32, _i32, _i32, _i32]),
+    "tnx_ssd": (_i32, [_p, C.POINTER(SsdDesc)]),
+    "tnx_latent_row": (_i32, [_i32, _i32, _i32]),
+    "tnx_latent_prep": (_i32, [_p, C.POINTER(LatentPrepDesc)]),
+    "tnx_latent_q": (_i32, [_p, C.POINTER(LatentQDesc)]),
+    "tnx_latent_kv": (_i32, [_p, C.POINTER(LatentKvDesc)]),
+    "tnx_latent_attn_ok": (_i32, [_i32, _i32, _i64]),
+    "tnx_latent_attn_ws_bytes": (C.c_size_t, [_i64, _i64, _i64, _i32, _i32, _i32]),
+    "tnx_latent_attn": (_i32, [_p, C.POINTER(LatentAttnDesc)]),
+    "tnx_gate_mul": (_i32, [_p, C.POINTER(GateMulDesc)]),
     "tnx_logits_stats": (_i32, [_p, C.POINTER(LogitsDesc)]),
     "tnx_fill_u32": (_i32, [_p, _p, _i64, C.c_uint32]),
 }

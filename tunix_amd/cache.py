@@ -1,11 +1,13 @@
 """What a batch of sequences carries from one forward pass to the next: one entry per layer run,
-either a key / value slab (attention) or a recurrent state.  A layer that runs several times has
-one entry per run.
+a key / value slab (attention), a slab of latents, a recurrent state, a ring of the last columns' rows,
+or several of these.  A layer that runs several times has one entry per run.
 
-Slabs are [B, heads, S, size] in the model's dtype, states [B, heads, dim, vdim] in fp32.  Rows of
+Slabs are [B, heads, S, size] or [B, S, size] in the model's dtype, states [B, heads, dim, vdim] in fp32,
+rings [B, slots, width] with slot = column % slots.  Rows of
 a batch are slots: a slot whose sequence has ended may be given to another one.  Nothing has to be
 cleared for that: attention reads no slot in front of the new sequence's first column or behind
-its last token, and a recurrence starts from zero at a sequence's first column.
+its last token, a recurrence starts from zero at a sequence's first column, and no ring slot of a column in
+front of it is read.
 """
 from __future__ import annotations
 
@@ -38,6 +40,36 @@ class StateSpec:
     return StateEntry(torch.zeros(B, self.heads, self.dim, self.vdim, dtype=torch.float32, device=device))
 
 
+@dataclasses.dataclass(frozen=True)
+class LatentSpec:
+  """One row per position of a latent-attention layer run."""
+  row: int
+  dtype: torch.dtype = torch.bfloat16
+
+  def allocate(self, B: int, S: int, device) -> "LatentEntry":
+    return LatentEntry(torch.zeros(B, S, self.row, dtype=self.dtype, device=device))
+
+
+@dataclasses.dataclass(frozen=True)
+class RingSpec:
+  """Rows of the last `slots` columns: what a short convolution or a token shift looks back to."""
+  slots: int
+  width: int
+  dtype: torch.dtype = torch.bfloat16
+
+  def allocate(self, B: int, S: int, device) -> "RingEntry":
+    return RingEntry(torch.zeros(B, self.slots, self.width, dtype=self.dtype, device=device))
+
+
+@dataclasses.dataclass(frozen=True)
+class PartsSpec:
+  """Several things one layer run keeps: ((name, spec), ...)."""
+  parts: tuple
+
+  def allocate(self, B: int, S: int, device) -> "PartsEntry":
+    return PartsEntry({name: spec.allocate(B, S, device) for name, spec in self.parts})
+
+
 @dataclasses.dataclass
 class KVEntry:
   k: torch.Tensor
@@ -63,6 +95,45 @@ class StateEntry:
 
   def grow(self, S: int):
     pass   # a state does not depend on the number of columns
+
+
+@dataclasses.dataclass
+class LatentEntry:
+  c: torch.Tensor
+
+  def rows(self, b0: int, n: int) -> "LatentEntry":
+    return LatentEntry(self.c[b0:b0 + n])
+
+  def grow(self, S: int):
+    new = torch.zeros(self.c.shape[0], S, self.c.shape[2], dtype=self.c.dtype, device=self.c.device)
+    new[:, :self.c.shape[1]].copy_(self.c)
+    self.c = new
+
+
+@dataclasses.dataclass
+class RingEntry:
+  r: torch.Tensor
+
+  def rows(self, b0: int, n: int) -> "RingEntry":
+    return RingEntry(self.r[b0:b0 + n])
+
+  def grow(self, S: int):
+    pass
+
+
+@dataclasses.dataclass
+class PartsEntry:
+  parts: dict
+
+  def __getitem__(self, name: str):
+    return self.parts[name]
+
+  def rows(self, b0: int, n: int) -> "PartsEntry":
+    return PartsEntry({k: e.rows(b0, n) for k, e in self.parts.items()})
+
+  def grow(self, S: int):
+    for e in self.parts.values():
+      e.grow(S)
 
 
 class SequenceCache:

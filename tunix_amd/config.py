@@ -127,6 +127,13 @@ class AttentionMixer:
     if self.rot_dims % 2 or not 0 <= self.rot_dims <= self.dim:
       raise ValueError(f"rot_dims={self.rot_dims} must be even and at most the head size {self.dim}")
 
+  def weight_shapes(self, D: int) -> dict[str, tuple]:
+    out = {"q": (self.heads * self.dim, D), "k": (self.kv_heads * self.dim, D), "v": (self.kv_heads * self.vdim, D),
+           "o": (D, self.heads * self.vdim)}
+    if self.sink:
+      out["sink"] = (self.heads,)
+    return out
+
 
 @dataclasses.dataclass(frozen=True)
 class LightningMixer:
@@ -141,17 +148,104 @@ class LightningMixer:
     if len(self.decay) != self.heads:
       raise ValueError(f"{len(self.decay)} decays for {self.heads} heads")
 
+  def weight_shapes(self, D: int) -> dict[str, tuple]:
+    qk, v = self.heads * self.dim, self.heads * self.vdim
+    return {"q": (qk, D), "k": (qk, D), "v": (v, D), "g": (v, D), "norm": (v,), "o": (D, v)}
+
+
+@dataclasses.dataclass(frozen=True)
+class SsdMixer:
+  """State-space duality: per head a matrix state [state, vdim] whose decay depends on the token; inputs
+  behind a short causal convolution, B and C shared by the heads of a group; the heads' outputs gated,
+  then normed in norm_groups equal parts and projected."""
+  heads: int
+  vdim: int
+  state: int
+  groups: int
+  conv: int
+  norm_groups: int
+
+  def __post_init__(self):
+    if self.heads % self.groups:
+      raise ValueError("heads must be a multiple of groups")
+    if self.inner % self.norm_groups:
+      raise ValueError(f"{self.inner} values do not divide into {self.norm_groups} norm groups")
+    if self.conv < 1:
+      raise ValueError("the convolution needs a tap")
+
+  @property
+  def inner(self) -> int:
+    return self.heads * self.vdim
+
+  @property
+  def channels(self) -> int:
+    """Of the convolution: x, B and C."""
+    return self.inner + 2 * self.groups * self.state
+
+  def weight_shapes(self, D: int) -> dict[str, tuple]:
+    C, H = self.channels, self.heads
+    return {"in": (self.inner + C + H, D), "conv": (C, self.conv), "conv.b": (C,), "dt_bias": (H,), "A_log": (H,), "D": (H,),
+            "norm": (self.inner,), "o": (D, self.inner)}
+
+
+@dataclasses.dataclass(frozen=True)
+class LatentMixer:
+  """Causal attention whose keys and values are linear in a normed latent of size kv_rank (all that is
+  cached, beside one rotated key part shared by the heads); queries through a latent of size q_rank; `dim`
+  unrotated and rot_dim rotated query / key dimensions per head; output gate."""
+  heads: int
+  dim: int
+  rot_dim: int
+  vdim: int
+  q_rank: int
+  kv_rank: int
+  rot_base: float
+  scale: float
+
+  def __post_init__(self):
+    if self.rot_dim % 2 or self.rot_dim < 0:
+      raise ValueError(f"rot_dim={self.rot_dim} must be even")
+
+  def weight_shapes(self, D: int) -> dict[str, tuple]:
+    H = self.heads
+    return {"dq": (self.q_rank, D), "dq.norm": (self.q_rank,), "uq": (H * (self.dim + self.rot_dim), self.q_rank),
+            "dkv": (self.kv_rank + self.rot_dim, D), "dkv.norm": (self.kv_rank,), "uk": (H * self.dim, self.kv_rank),
+            "uv": (H * self.vdim, self.kv_rank), "g": (H * self.vdim, D), "o": (D, H * self.vdim)}
+
 
 @dataclasses.dataclass(frozen=True)
 class GatedMlp:
   """down(gelu_tanh(gate h) * (up h))."""
   ff: int
 
+  def weight_shapes(self, D: int) -> dict[str, tuple]:
+    return {"gate": (self.ff, D), "up": (self.ff, D), "down": (D, self.ff)}
+
+
+@dataclasses.dataclass(frozen=True)
+class ExpertsMlp:
+  """The weighted sum of down(silu(gate h) * (up h)) of the `top` experts with the largest router logits;
+  weights: softmax over the chosen logits."""
+  ff: int
+  experts: int
+  top: int
+
+  def __post_init__(self):
+    if not 1 <= self.top <= self.experts:
+      raise ValueError(f"{self.top} of {self.experts} experts")
+
+  def weight_shapes(self, D: int) -> dict[str, tuple]:
+    out = {"router": (self.experts, D)}
+    for e in range(self.experts):
+      out[f"e{e}.gate"] = out[f"e{e}.up"] = (self.ff, D)
+      out[f"e{e}.down"] = (D, self.ff)
+    return out
+
 
 @dataclasses.dataclass(frozen=True)
 class LayerSpec:
-  mixer: AttentionMixer | LightningMixer
-  mlp: GatedMlp | None
+  mixer: AttentionMixer | LightningMixer | SsdMixer | LatentMixer
+  mlp: GatedMlp | ExpertsMlp | None
 
 
 @dataclasses.dataclass(frozen=True)
@@ -164,8 +258,10 @@ class LayerLoop:
 
 @dataclasses.dataclass(frozen=True)
 class StackConfig:
-  """A decoder given layer by layer.  Every sublayer is x += norm(f(norm(x))) with norm weights
-  stored as an offset from `norm_offset`; the head is the embedding table."""
+  """A decoder given layer by layer.  Every sublayer is x += norm(f(norm(x))), or x += norm(f(x)) without
+  pre_norm, with norm weights stored as an offset from `norm_offset` and norms taken over norm_groups equal
+  parts of the row; the head is the embedding table.  embed_norm: the embedding is normed.  token_shift:
+  what a mixer reads is first moved towards the same of the token before, per element."""
   family: str
   vocab_size: int
   embed_dim: int
@@ -173,11 +269,23 @@ class StackConfig:
   norm_eps: float
   loop: LayerLoop | None = None
   norm_offset: float = 1.0
+  norm_groups: int = 1
+  pre_norm: bool = True
+  embed_norm: bool = False
+  token_shift: bool = False
 
   def __post_init__(self):
     n, lp = len(self.layers), self.loop
     if lp is not None and not (0 <= lp.start < lp.stop <= n and lp.times >= 1):
       raise ValueError(f"the loop {lp} does not fit {n} layers")
+    if self.embed_dim % self.norm_groups:
+      raise ValueError(f"width {self.embed_dim} does not divide into {self.norm_groups} norm groups")
+    if self.token_shift and self.pre_norm:
+      raise ValueError("a token shift goes with norms behind the sublayers only")
+
+  def post_norm(self, n: int) -> str:
+    """Name of the norm behind a layer's mixer (n = 1) or feed-forward (2)."""
+    return f"norm{n}b" if self.pre_norm else f"norm{n}"
 
   @property
   def num_layers(self) -> int:
@@ -196,24 +304,48 @@ class StackConfig:
     """Name -> shape of every tensor; linear weights are [out, in]."""
     D = self.embed_dim
     out = {"embed": (self.vocab_size, D), "final.norm": (D,)}
+    if self.embed_norm:
+      out["embed.norm"] = (D,)
     if self.loop is not None:
       out["loop.in"] = (D, 2 * D)
     for i, ly in enumerate(self.layers):
-      p, m = f"l{i}.", ly.mixer
-      out[p + "norm1"] = out[p + "norm1b"] = (D,)
-      attn = isinstance(m, AttentionMixer)
-      kv = m.kv_heads if attn else m.heads
-      out[p + "mix.q"], out[p + "mix.k"] = (m.heads * m.dim, D), (kv * m.dim, D)
-      out[p + "mix.v"], out[p + "mix.o"] = (kv * m.vdim, D), (D, m.heads * m.vdim)
-      if not attn:
-        out[p + "mix.g"], out[p + "mix.norm"] = (m.heads * m.vdim, D), (m.heads * m.vdim,)
-      elif m.sink:
-        out[p + "mix.sink"] = (m.heads,)
-      if ly.mlp is not None:
-        out[p + "norm2"] = out[p + "norm2b"] = (D,)
-        out[p + "mlp.gate"] = out[p + "mlp.up"] = (ly.mlp.ff, D)
-        out[p + "mlp.down"] = (D, ly.mlp.ff)
+      p = f"l{i}."
+      parts = [(1, "mix.", ly.mixer)] + ([(2, "mlp.", ly.mlp)] if ly.mlp is not None else [])
+      if self.token_shift:
+        out[p + "shift"] = (D,)
+      for n, at, part in parts:
+        if self.pre_norm:
+          out[p + f"norm{n}"] = (D,)
+        out[p + self.post_norm(n)] = (D,)
+        out.update({p + at + k: s for k, s in part.weight_shapes(D).items()})
     return out
+
+
+def lapevik_from_dict(d: dict) -> StackConfig:
+  """Reads a Lapevik config.json."""
+  layers = []
+  for i, ly in enumerate(d["layers"]):
+    m = ly["mixer"]
+    if ly["type"] in ("mamba2", "mamba2_2"):
+      mixer = SsdMixer(heads=int(m["heads"]), vdim=int(m["vdim"]), state=int(m["state"]), groups=int(m["groups"]),
+                       conv=int(m["conv"]), norm_groups=int(m["norm_groups"]))
+    elif ly["type"] == "latent_attention":
+      rot = m["rot"]
+      if int(rot["dims"]) != int(m["rot_dim"]):
+        raise ValueError(f"layer {i}: rotation over {rot['dims']} of {m['rot_dim']} dimensions")
+      mixer = LatentMixer(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                          q_rank=int(m["q_rank"]), kv_rank=int(m["kv_rank"]), rot_base=float(rot["base"]), scale=float(m["scale"]))
+    else:
+      raise ValueError(f"layer {i}: unknown mixer type {ly['type']!r}")
+    mlp = ly.get("mlp")
+    if mlp is not None:
+      if mlp["kind"] != "moe":
+        raise ValueError(f"layer {i}: unknown feed-forward kind {mlp['kind']!r}")
+      mlp = ExpertsMlp(ff=int(mlp["expert"]["ff"]), experts=int(mlp["router"]["experts"]), top=int(mlp["router"]["top"]))
+    layers.append(LayerSpec(mixer, mlp))
+  return StackConfig(family="lapevik", vocab_size=int(d["vocab"]), embed_dim=int(d["width"]), layers=tuple(layers),
+                     norm_eps=float(d["norm"]["eps"]), norm_offset=0.0, norm_groups=int(d["norm"]["groups"]), pre_norm=False,
+                     embed_norm=True, token_shift=True)
 
 
 def nunezen_from_dict(d: dict) -> StackConfig:

@@ -1,7 +1,20 @@
 // Device helpers shared by the dense-weight decoder kernels (dense.hip, decoder_ops.hip,
-// sink_attention.hip, lightning.hip): element access by dtype, activations, fragment order.
+// sink_attention.hip, lightning.hip, ssd.hip, latent.hip): element access by dtype, activations,
+// fragment order, MFMA.
 #pragma once
 #include "common.h"
+
+typedef float f32x16 __attribute__((ext_vector_type(16)));
+__device__ __forceinline__ f32x16 mfma32(u32x4 a, u32x4 b, f32x16 c) {
+  // D[32x32] += A[32x16] * B[16x32]; lane l holds A row l%32 / B column l%32, k = 8*(l/32)..+7;
+  // D: column l%32, rows 8*(r/4) + 4*(l/32) + r%4 for register r.
+  return __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
+}
+// bf16 pairs of (x, y) and of what that rounding left out: together 16 mantissa bits
+__device__ __forceinline__ void split2(float x, float y, uint32_t& hi, uint32_t& lo) {
+  hi = cvt_pk_bf16(x, y);
+  lo = cvt_pk_bf16(x - bflo(hi), y - bfhi(hi));
+}
 
 __device__ __forceinline__ float gelu_tanh_f32(float z) {
   const float k0 = 0.7978845608028654f, k1 = 0.044715f;

@@ -1,6 +1,6 @@
 // The small operations of decoders with dense weights and an fp32 residual stream: embedding,
-// post-norm + residual + next pre-norm, partial rotation + cache write, gated norm, gated unit,
-// and the statistics / sampling of finished logits.  Norms, angles and the residual are 32-bit;
+// post-norm + residual + next pre-norm or token shift, partial rotation + cache write, gated norms,
+// gated unit, the choice of experts, and the statistics / sampling of finished logits.  Norms, angles and the residual are 32-bit;
 // matrix operands leave in the model's dtype (bf16 or fp32).
 #include <string.h>
 
@@ -54,9 +54,20 @@ struct ResNormArgs {
   const float* ws;
   int split;
   int64_t plane, y_ld;
-  int mode;               // 0: nothing arrives, 1: x += norm(y) . w_post, 2: x = y
+  int mode;               // 0: nothing arrives, 1: x += norm(y) . w_post, 2: x = y, 3: x = norm(x) . w_post
   const float* w_post;
   float* x;
+  // rows_kernel: norms in equal parts of a row, routed rows, token shift
+  int groups;
+  float* x_out;
+  const float* route_w;   // [M, route_k]: y holds route_k rows per row of x, summed with these weights
+  int route_k;
+  const float* shift;     // [D]: out = x + (x of the token before - x) . shift
+  float* before;          // [B, D]: x of the last token of the call before
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  int64_t B, T;
+  int run;                // tokens of a work-group
   const float* w_next;    // null: out = x in the model's dtype
   void* out;
   int64_t out_ld;
@@ -174,6 +185,214 @@ __global__ __launch_bounds__(256) void resnorm_vec_kernel(const ResNormArgs a) {
   }
 }
 
+// 1 / sqrt(mean + eps) of equal parts of a row whose elements the threads own in runs: part[i] is the
+// sum of squares of run i, `per` runs (of `len / per` elements) make a part.  Two barriers; the result is in gs[part].
+__device__ __forceinline__ void part_scales(const float* part, float* gs, int groups, int per, float len, float eps) {
+  __syncthreads();
+  const int lane = threadIdx.x & 63, nw = blockDim.x >> 6;
+  for (int g = threadIdx.x >> 6; g < groups; g += nw) {
+    float s = 0.f;
+    for (int i = lane; i < per; i += 64) s += part[g * per + i];
+    s = wave_sum(s);
+    if (lane == 0) gs[g] = 1.0f / sqrtf(s / len + eps);
+  }
+  __syncthreads();
+}
+
+// The general residual step: norms over equal parts of a row, weighted sums of routed rows, token shift.
+// A work-group walks `run` tokens of one sequence; with a shift it forms the token before its first one
+// as well (x and x_out are then different buffers, unless the call brings one token per sequence).
+template <int MAXC, typename T>
+__global__ __launch_bounds__(256) void resnorm_rows_kernel(const ResNormArgs a) {
+  __shared__ float red[4], part[MAXC * 256], gs[MAXC * 256];
+  const int64_t runs = (a.T + a.run - 1) / a.run, b = blockIdx.x / runs, t0 = blockIdx.x % runs * a.run;
+  const int64_t t1 = min(a.T, t0 + a.run);
+  const int nch = (int)(a.D / 8), per = nch / a.groups, tid = threadIdx.x;
+  const int col0 = a.shift ? *a.col_ptr : 0, start = a.shift ? a.starts[b] : 0;
+  const RowSrc<T> src{reinterpret_cast<const T*>(a.y), a.ws, a.split, a.plane, a.y_ld};
+  float wp[MAXC][8], wn[MAXC][8], prev[MAXC][8], h[MAXC][8];
+  auto load8f = [](const float* p, float (&f)[8]) {
+    const f32x4 u = *reinterpret_cast<const f32x4*>(p), v = *reinterpret_cast<const f32x4*>(p + 4);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      f[j] = u[j];
+      f[4 + j] = v[j];
+    }
+  };
+  const float* wnext = a.shift ? a.shift : a.w_next;
+  auto column = [&](int c) { return (int64_t)min(c * 256 + tid, nch - 1) * 8; };
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    if (a.w_post) load8f(a.w_post + column(c), wp[c]);
+    if (wnext) load8f(wnext + column(c), wn[c]);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) prev[c][j] = 0.f;
+    if (a.shift && t0 == 0 && col0 > start) load8f(a.before + b * a.D + column(c), prev[c]);
+  }
+  float r[MAXC];
+  auto scales = [&](const float (&v)[MAXC][8]) {
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      if (c * 256 + tid >= nch) continue;
+      float q = 0.f;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) q += v[c][j] * v[c][j];
+      ss += q;
+      if (a.groups > 1) part[c * 256 + tid] = q;
+    }
+    if (a.groups == 1) {
+      const float s = 1.0f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) r[c] = s;
+      return;
+    }
+    part_scales(part, gs, a.groups, per, (float)(per * 8), a.eps);
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) r[c] = gs[min(c * 256 + tid, nch - 1) / per];
+  };
+  for (int64_t t = a.shift && t0 > 0 ? t0 - 1 : t0; t < t1; ++t) {
+    const int64_t row = b * a.T + t;
+    float xo[MAXC][8];
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      const int64_t col = column(c);
+      if (a.mode != 2) load8f(a.x + row * a.D + col, xo[c]);
+      if (a.mode == 1 || a.mode == 2) {
+        if (a.route_w) {
+#pragma unroll
+          for (int j = 0; j < 8; ++j) h[c][j] = 0.f;
+          for (int k = 0; k < a.route_k; ++k) {
+            const float w = a.route_w[row * a.route_k + k];
+            float f[8];
+            get8(src, row * a.route_k + k, col, f);
+#pragma unroll
+            for (int j = 0; j < 8; ++j) h[c][j] += w * f[j];
+          }
+        } else if (a.ws && a.split == 1) {
+          load8f(a.ws + row * a.y_ld + col, h[c]);
+        } else {
+          get8(src, row, col, h[c]);
+        }
+      } else {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) h[c][j] = xo[c][j];
+      }
+    }
+    if (a.mode == 1 || a.mode == 3) {
+      scales(h);
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          const float v = h[c][j] * r[c] * (a.w_offset + wp[c][j]);
+          h[c][j] = a.mode == 1 ? xo[c][j] + v : v;
+        }
+    }
+    if (t >= t0) {
+      if (a.w_next) scales(h);   // (uniform)
+      T* out = reinterpret_cast<T*>(a.out);
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) {
+        if (c * 256 + tid >= nch) continue;
+        const int64_t col = column(c);
+        if (a.mode != 0 || a.x_out != a.x) put8(a.x_out + row * a.D + col, h[c]);
+        float o[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          o[j] = h[c][j];
+          if (a.shift) o[j] = h[c][j] + ((col0 + t > start ? prev[c][j] : 0.f) - h[c][j]) * wn[c][j];
+          else if (a.w_next) o[j] = h[c][j] * r[c] * (a.w_offset + wn[c][j]);
+        }
+        put8(out + (a.out_frag ? frag_index(row, col, a.out_ld) : row * a.out_ld + col), o);
+      }
+    }
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) prev[c][j] = h[c][j];
+  }
+  if (a.shift && a.T == 1)
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c)
+      if (c * 256 + tid < nch) put8(a.before + b * a.D + column(c), h[c]);
+}
+
+// the same for any D that fits LDS twice: h and the token before, a thread owning the columns tid + 256 i
+template <typename T>
+__global__ __launch_bounds__(256) void resnorm_rows_any_kernel(const ResNormArgs a) {
+  extern __shared__ __align__(16) float hrow[];
+  float* prev = hrow + a.D;
+  __shared__ float gs[1024];
+  const int64_t runs = (a.T + a.run - 1) / a.run, b = blockIdx.x / runs, t0 = blockIdx.x % runs * a.run;
+  const int64_t t1 = min(a.T, t0 + a.run);
+  const int per = (int)(a.D / a.groups), tid = threadIdx.x, lane = tid & 63;
+  const int col0 = a.shift ? *a.col_ptr : 0, start = a.shift ? a.starts[b] : 0;
+  const RowSrc<T> src{reinterpret_cast<const T*>(a.y), a.ws, a.split, a.plane, a.y_ld};
+  auto scales = [&]() {
+    __syncthreads();
+    for (int g = tid >> 6; g < a.groups; g += 4) {
+      float s = 0.f;
+      for (int i = lane; i < per; i += 64) s += hrow[g * per + i] * hrow[g * per + i];
+      s = wave_sum(s);
+      if (lane == 0) gs[g] = 1.0f / sqrtf(s / (float)per + a.eps);
+    }
+    __syncthreads();
+  };
+  for (int64_t i = tid; i < a.D; i += 256) prev[i] = a.shift && t0 == 0 && col0 > start ? a.before[b * a.D + i] : 0.f;
+  for (int64_t t = a.shift && t0 > 0 ? t0 - 1 : t0; t < t1; ++t) {
+    const int64_t row = b * a.T + t;
+    for (int64_t i = tid; i < a.D; i += 256) {
+      float v = 0.f;
+      if (a.mode == 0 || a.mode == 3) v = a.x[row * a.D + i];
+      else if (a.route_w)
+        for (int k = 0; k < a.route_k; ++k) v += a.route_w[row * a.route_k + k] * src.get(row * a.route_k + k, i);
+      else if (a.ws && a.split == 1) v = a.ws[row * a.y_ld + i];
+      else v = src.get(row, i);
+      hrow[i] = v;
+    }
+    if (a.mode == 1 || a.mode == 3) {
+      scales();
+      for (int64_t i = tid; i < a.D; i += 256) {
+        const float v = hrow[i] * gs[i / per] * (a.w_offset + a.w_post[i]);
+        hrow[i] = a.mode == 1 ? a.x[row * a.D + i] + v : v;
+      }
+    }
+    if (t >= t0) {
+      if (a.w_next) scales();
+      T* out = reinterpret_cast<T*>(a.out);
+      for (int64_t i = tid; i < a.D; i += 256) {
+        const float h = hrow[i];
+        if (a.mode != 0 || a.x_out != a.x) a.x_out[row * a.D + i] = h;
+        float o = h;
+        if (a.shift) o = h + ((col0 + t > start ? prev[i] : 0.f) - h) * a.shift[i];
+        else if (a.w_next) o = h * gs[i / per] * (a.w_offset + a.w_next[i]);
+        st_elem(out, a.out_frag ? frag_index(row, i, a.out_ld) : row * a.out_ld + i, o);
+      }
+    }
+    __syncthreads();   // every group's sums have read hrow
+    for (int64_t i = tid; i < a.D; i += 256) prev[i] = hrow[i];
+  }
+  if (a.shift && a.T == 1)
+    for (int64_t i = tid; i < a.D; i += 256) a.before[b * a.D + i] = prev[i];
+}
+
+template <typename T>
+int launch_resnorm_rows(hipStream_t st, ResNormArgs a) {
+  a.run = 8;
+  while (a.run > 1 && a.B * cdiv(a.T, a.run) < 1024) a.run /= 2;
+  const dim3 grid((unsigned)(a.B * cdiv(a.T, a.run)));
+  const bool vec = a.D % 8 == 0 && a.D / a.groups % 8 == 0 && a.y_ld % 8 == 0 && a.out_ld % 8 == 0 && a.plane % 8 == 0;
+  if (!vec) {
+    TNX_REQUIRE(a.D <= 7168 && a.groups <= 1024, "residual_norm: D=%lld in %d parts needs runs of eight", (long long)a.D, a.groups);
+    hipLaunchKernelGGL((resnorm_rows_any_kernel<T>), grid, dim3(256), (size_t)a.D * 8, st, a);
+  } else if (a.D <= 2048) hipLaunchKernelGGL((resnorm_rows_kernel<1, T>), grid, dim3(256), 0, st, a);
+  else if (a.D <= 4096) hipLaunchKernelGGL((resnorm_rows_kernel<2, T>), grid, dim3(256), 0, st, a);
+  else if (a.D <= 8192) hipLaunchKernelGGL((resnorm_rows_kernel<4, T>), grid, dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((resnorm_rows_kernel<8, T>), grid, dim3(256), 0, st, a);
+  return TNX_OK;
+}
+
 template <typename T>
 void launch_resnorm(hipStream_t st, const ResNormArgs& a) {
   const bool vec = a.D % 8 == 0 && a.y_ld % 8 == 0 && a.out_ld % 8 == 0 && a.plane % 8 == 0;
@@ -277,14 +496,83 @@ __global__ __launch_bounds__(256) void part_rope_vec_kernel(const PartRopeArgs a
   }
 }
 
-// ---- RMS norm over the whole row times sigmoid(gate) --------------------------------------------
+// ---- RMS norm and a gate: norm(o) . w . sigmoid(g) over the whole row, or norm(o . silu(g)) . w in parts --
 struct GatedNormArgs {
   int64_t W, o_ld, out_ld, g_off;
   float eps, w_offset;
   const float* w;
   const float* o;
-  int out_frag;
+  int out_frag, groups;
 };
+// the gate first, then norms over equal parts: any width that fits LDS
+template <typename T>
+__global__ __launch_bounds__(256) void gate_first_kernel(const GatedNormArgs a, const RowSrc<T> g, T* out) {
+  extern __shared__ __align__(16) float v[];
+  __shared__ float gs[1024];
+  const int64_t row = blockIdx.x;
+  const int per = (int)(a.W / a.groups), lane = threadIdx.x & 63;
+  for (int64_t i = threadIdx.x; i < a.W; i += 256) v[i] = a.o[row * a.o_ld + i] * silu_f32(g.get(row, a.g_off + i));
+  __syncthreads();
+  for (int p = threadIdx.x >> 6; p < a.groups; p += 4) {
+    float s = 0.f;
+    for (int i = lane; i < per; i += 64) s += v[p * per + i] * v[p * per + i];
+    s = wave_sum(s);
+    if (lane == 0) gs[p] = 1.0f / sqrtf(s / (float)per + a.eps);
+  }
+  __syncthreads();
+  for (int64_t i = threadIdx.x; i < a.W; i += 256)
+    st_elem(out, a.out_frag ? frag_index(row, i, a.out_ld) : row * a.out_ld + i, v[i] * gs[i / per] * (a.w_offset + a.w[i]));
+}
+template <int MAXC, typename T>
+__global__ __launch_bounds__(256) void gate_first_vec_kernel(const GatedNormArgs a, const RowSrc<T> g, T* out) {
+  __shared__ float part[MAXC * 256], gs[MAXC * 256];
+  const int64_t row = blockIdx.x;
+  const int nch = (int)(a.W / 8), per = nch / a.groups;
+  float o[MAXC][8], w[MAXC][8], gv[MAXC][8];
+  const RowSrc<float> os{a.o, nullptr, 1, 0, a.o_ld}, wsrc{a.w, nullptr, 1, 0, 0};
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int64_t col = (int64_t)min(c * 256 + (int)threadIdx.x, nch - 1) * 8;
+    get8(os, row, col, o[c]);
+    get8(wsrc, 0, col, w[c]);
+    get8(g, row, a.g_off + col, gv[c]);
+  }
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    float q = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      o[c][j] *= silu_f32(gv[c][j]);
+      q += o[c][j] * o[c][j];
+    }
+    part[c * 256 + threadIdx.x] = q;
+  }
+  part_scales(part, gs, a.groups, per, (float)(per * 8), a.eps);
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = c * 256 + threadIdx.x;
+    if (ch >= nch) continue;
+    const float r = gs[ch / per];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o[c][j] = o[c][j] * r * (a.w_offset + w[c][j]);
+    put8(out + (a.out_frag ? frag_index(row, (int64_t)ch * 8, a.out_ld) : row * a.out_ld + (int64_t)ch * 8), o[c]);
+  }
+}
+template <typename T>
+int launch_gate_first(hipStream_t st, int64_t M, const GatedNormArgs& a, const RowSrc<T>& g, T* out) {
+  const dim3 grid((unsigned)M);
+  const bool vec = a.W % 8 == 0 && a.W / a.groups % 8 == 0 && a.W <= 16384 && a.o_ld % 8 == 0 && g.ld % 8 == 0 && g.plane % 8 == 0 && a.g_off % 8 == 0 &&
+                   a.out_ld % 8 == 0;
+  if (!vec) {
+    TNX_REQUIRE(a.W <= 15360 && a.groups <= 1024, "gated_norm: W=%lld in %d parts needs runs of eight", (long long)a.W, a.groups);
+    hipLaunchKernelGGL((gate_first_kernel<T>), grid, dim3(256), (size_t)a.W * 4, st, a, g, out);
+  } else if (a.W <= 2048) hipLaunchKernelGGL((gate_first_vec_kernel<1, T>), grid, dim3(256), 0, st, a, g, out);
+  else if (a.W <= 4096) hipLaunchKernelGGL((gate_first_vec_kernel<2, T>), grid, dim3(256), 0, st, a, g, out);
+  else if (a.W <= 8192) hipLaunchKernelGGL((gate_first_vec_kernel<4, T>), grid, dim3(256), 0, st, a, g, out);
+  else hipLaunchKernelGGL((gate_first_vec_kernel<8, T>), grid, dim3(256), 0, st, a, g, out);
+  TNX_CHECK_LAUNCH("gated_norm");
+  return TNX_OK;
+}
 template <typename T>
 __global__ __launch_bounds__(256) void gated_norm_kernel(const GatedNormArgs a, const RowSrc<T> g, T* out) {
   __shared__ float red[4];
@@ -339,11 +627,77 @@ void launch_gated_norm(hipStream_t st, int64_t M, const GatedNormArgs& a, const 
   else hipLaunchKernelGGL((gated_norm_vec_kernel<8, T>), grid, dim3(256), 0, st, a, g, out);
 }
 
-// ---- gated unit on finished projections: out = gelu_tanh(y[:, :F]) * y[:, u_off : u_off + F] -----
-template <typename T>
-__global__ __launch_bounds__(256) void gelu_mul_kernel(const T* y, int64_t ld, int64_t u_off, int64_t F, T* out, int64_t out_ld) {
+// ---- gated unit on finished projections: out = act(y[:, :F]) * y[:, u_off : u_off + F] -----------
+template <bool SILU, typename T>
+__global__ __launch_bounds__(256) void act_mul_kernel(const T* y, int64_t ld, int64_t u_off, int64_t F, T* out, int64_t out_ld) {
   const int64_t row = blockIdx.y, i = (int64_t)blockIdx.x * 256 + threadIdx.x;
-  if (i < F) st_elem(out, row * out_ld + i, gelu_tanh_f32(ld_elem(y, row * ld + i)) * ld_elem(y, row * ld + u_off + i));
+  if (i >= F) return;
+  const float z = ld_elem(y, row * ld + i);
+  st_elem(out, row * out_ld + i, (SILU ? silu_f32(z) : gelu_tanh_f32(z)) * ld_elem(y, row * ld + u_off + i));
+}
+template <bool SILU>
+int launch_act_mul(hipStream_t st, int dtype, const void* y, int64_t ld, int64_t up_off, int64_t M, int64_t F, void* out, int64_t out_ld) {
+  TNX_REQUIRE(y && out && M > 0 && F > 0 && ld >= up_off + F && out_ld >= F, "act_mul: null pointer or bad shape");
+  TNX_REQUIRE(dtype == TNX_BF16 || dtype == TNX_F32, "act_mul: bad dtype %d", dtype);
+  for (int64_t r0 = 0; r0 < M; r0 += 65535) {
+    const int64_t n = M - r0 < 65535 ? M - r0 : 65535;
+    const dim3 grid((unsigned)cdiv(F, 256), (unsigned)n);
+    if (dtype == TNX_BF16)
+      hipLaunchKernelGGL((act_mul_kernel<SILU, uint16_t>), grid, dim3(256), 0, st, (const uint16_t*)y + r0 * ld, ld, up_off, F,
+                         (uint16_t*)out + r0 * out_ld, out_ld);
+    else
+      hipLaunchKernelGGL((act_mul_kernel<SILU, float>), grid, dim3(256), 0, st, (const float*)y + r0 * ld, ld, up_off, F,
+                         (float*)out + r0 * out_ld, out_ld);
+  }
+  TNX_CHECK_LAUNCH("act_mul");
+  return TNX_OK;
+}
+
+// ---- choice of experts: the k largest logits (first among equals), softmax over them ---------------
+// One wave per token.  NaN logits rank below every number, so that k distinct experts are found whatever
+// the logits hold; they leave as NaN weights.
+__global__ __launch_bounds__(64) void route_softmax_kernel(const RowSrc<float> src, int E, int k, float* topk_w, int32_t* topk_id) {
+  extern __shared__ float z[];   // logits [E], chosen logits [k]
+  float* sel = z + E;
+  const int64_t m = blockIdx.x;
+  const int lane = threadIdx.x;
+  const float ninf = -__builtin_inff();
+  bool bad = false;
+  for (int e = lane; e < E; e += 64) {
+    const float v = src.get(m, e);
+    bad |= v != v;
+    z[e] = v == v ? fmaxf(v, -3.0e38f) : -3.0e38f;   // (a taken expert is -inf)
+  }
+  bad = __any(bad);
+  __syncthreads();
+  for (int j = 0; j < k; ++j) {
+    float best = ninf;
+    int bi = 0x7fffffff;
+    for (int e = lane; e < E; e += 64)
+      if (z[e] > best) {
+        best = z[e];
+        bi = e;
+      }
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const float ob = __shfl_xor(best, o, 64);
+      const int oi = __shfl_xor(bi, o, 64);
+      if (ob > best || (ob == best && oi < bi)) {
+        best = ob;
+        bi = oi;
+      }
+    }
+    if (lane == 0) {
+      sel[j] = best;
+      topk_id[m * k + j] = bi;
+      z[bi] = ninf;
+    }
+    __syncthreads();
+  }
+  float sum = 0.f;
+  for (int j = lane; j < k; j += 64) sum += expf(sel[j] - sel[0]);
+  sum = wave_sum(sum);
+  for (int j = lane; j < k; j += 64) topk_w[m * k + j] = bad ? __builtin_nanf("") : expf(sel[j] - sel[0]) / sum;
 }
 
 // ---- statistics and the whole-vocabulary draw over finished fp32 logits -------------------------
@@ -460,15 +814,30 @@ extern "C" int tnx_residual_norm(void* stream, const tnx_residual_norm_desc* d) 
   TNX_REQUIRE(d, "residual_norm: null descriptor");
   TNX_REQUIRE(d->M > 0 && d->D > 0 && d->D <= 16384, "residual_norm: D=%lld out of range (1..16384)", (long long)d->D);
   TNX_REQUIRE(d->x && d->out && d->out_ld >= d->D, "residual_norm: null pointer or short output rows");
-  TNX_REQUIRE(d->mode >= 0 && d->mode <= 2, "residual_norm: bad mode %d", d->mode);
-  TNX_REQUIRE(d->mode == 0 || d->y.y || d->y.ws, "residual_norm: no incoming rows");
-  TNX_REQUIRE(d->mode != 1 || d->w_post, "residual_norm: null post-norm weight");
+  TNX_REQUIRE(d->mode >= 0 && d->mode <= 3, "residual_norm: bad mode %d", d->mode);
+  const bool arrives = d->mode == 1 || d->mode == 2;
+  TNX_REQUIRE(!arrives || d->y.y || d->y.ws, "residual_norm: no incoming rows");
+  TNX_REQUIRE((d->mode != 1 && d->mode != 3) || d->w_post, "residual_norm: null post-norm weight");
+  const int groups = d->groups < 1 ? 1 : d->groups;
+  TNX_REQUIRE(d->D % groups == 0, "residual_norm: D=%lld does not divide into %d parts", (long long)d->D, groups);
+  TNX_REQUIRE(!d->route_w || (d->route_k > 0 && arrives), "residual_norm: routed rows need their number per row");
+  TNX_REQUIRE(!d->shift || (!d->w_next && d->before && d->starts && d->col_ptr && d->B > 0 && d->T > 0 && d->B * d->T == d->M),
+              "residual_norm: a shift needs the rows before, their columns and no next norm");
+  TNX_REQUIRE(!d->shift || d->T == 1 || (d->x_out && d->x_out != d->x), "residual_norm: a shift over several tokens needs a second buffer");
   TNX_REQUIRE(d->dtype == TNX_BF16 || d->dtype == TNX_F32, "residual_norm: bad dtype %d", d->dtype);
   ResNormArgs a;
   a.M = d->M; a.D = d->D; a.eps = d->eps; a.w_offset = d->w_offset; a.y = d->y.y; a.ws = d->y.ws;
-  a.split = d->y.split_k < 1 ? 1 : d->y.split_k; a.plane = d->y.plane; a.y_ld = d->mode ? d->y.ld : 8; a.mode = d->mode;
+  a.split = d->y.split_k < 1 ? 1 : d->y.split_k; a.plane = d->y.plane; a.y_ld = arrives ? d->y.ld : 8; a.mode = d->mode;
   a.w_post = d->w_post; a.x = d->x; a.w_next = d->w_next; a.out = d->out; a.out_ld = d->out_ld; a.out_frag = d->out_frag;
-  if (d->mode == 0) a.plane = 0;
+  if (!arrives) a.plane = 0;
+  a.groups = groups; a.x_out = d->x_out ? d->x_out : d->x; a.route_w = d->route_w; a.route_k = d->route_k; a.shift = d->shift;
+  a.before = d->before; a.starts = d->starts; a.col_ptr = d->col_ptr; a.B = d->shift ? d->B : 1; a.T = d->shift ? d->T : d->M;
+  if (groups > 1 || d->mode == 3 || d->route_w || d->shift || a.x_out != a.x) {
+    const int rc = d->dtype == TNX_BF16 ? launch_resnorm_rows<uint16_t>(as_stream(stream), a) : launch_resnorm_rows<float>(as_stream(stream), a);
+    if (rc) return rc;
+    TNX_CHECK_LAUNCH("residual_norm");
+    return TNX_OK;
+  }
   if (d->dtype == TNX_BF16) launch_resnorm<uint16_t>(as_stream(stream), a);
   else launch_resnorm<float>(as_stream(stream), a);
   TNX_CHECK_LAUNCH("residual_norm");
@@ -518,7 +887,11 @@ extern "C" int tnx_gated_norm(void* stream, const tnx_gated_norm_desc* d) {
   TNX_REQUIRE(d->dtype == TNX_BF16 || d->dtype == TNX_F32, "gated_norm: bad dtype %d", d->dtype);
   GatedNormArgs a;
   a.W = d->W; a.o_ld = d->o_ld; a.out_ld = d->out_ld; a.g_off = d->g_off; a.eps = d->eps; a.w_offset = d->w_offset;
-  a.w = d->w; a.o = d->o; a.out_frag = d->out_frag;
+  a.w = d->w; a.o = d->o; a.out_frag = d->out_frag; a.groups = d->groups < 1 ? 1 : d->groups;
+  TNX_REQUIRE(d->W % a.groups == 0 && (d->gate_first || a.groups == 1), "gated_norm: the row does not divide into %d parts", a.groups);
+  if (d->gate_first)
+    return d->dtype == TNX_BF16 ? launch_gate_first(as_stream(stream), d->M, a, row_src<uint16_t>(d->g), (uint16_t*)d->out)
+                                : launch_gate_first(as_stream(stream), d->M, a, row_src<float>(d->g), (float*)d->out);
   if (d->dtype == TNX_BF16) launch_gated_norm(as_stream(stream), d->M, a, row_src<uint16_t>(d->g), (uint16_t*)d->out);
   else launch_gated_norm(as_stream(stream), d->M, a, row_src<float>(d->g), (float*)d->out);
   TNX_CHECK_LAUNCH("gated_norm");
@@ -527,19 +900,20 @@ extern "C" int tnx_gated_norm(void* stream, const tnx_gated_norm_desc* d) {
 
 extern "C" int tnx_gelu_mul(void* stream, int dtype, const void* y, int64_t ld, int64_t up_off, int64_t M, int64_t F, void* out,
                             int64_t out_ld) {
-  TNX_REQUIRE(y && out && M > 0 && F > 0 && ld >= up_off + F && out_ld >= F, "gelu_mul: null pointer or bad shape");
-  TNX_REQUIRE(dtype == TNX_BF16 || dtype == TNX_F32, "gelu_mul: bad dtype %d", dtype);
-  for (int64_t r0 = 0; r0 < M; r0 += 65535) {
-    const int64_t n = M - r0 < 65535 ? M - r0 : 65535;
-    const dim3 grid((unsigned)cdiv(F, 256), (unsigned)n);
-    if (dtype == TNX_BF16)
-      hipLaunchKernelGGL(gelu_mul_kernel<uint16_t>, grid, dim3(256), 0, as_stream(stream), (const uint16_t*)y + r0 * ld, ld, up_off, F,
-                         (uint16_t*)out + r0 * out_ld, out_ld);
-    else
-      hipLaunchKernelGGL(gelu_mul_kernel<float>, grid, dim3(256), 0, as_stream(stream), (const float*)y + r0 * ld, ld, up_off, F,
-                         (float*)out + r0 * out_ld, out_ld);
-  }
-  TNX_CHECK_LAUNCH("gelu_mul");
+  return launch_act_mul<false>(as_stream(stream), dtype, y, ld, up_off, M, F, out, out_ld);
+}
+
+extern "C" int tnx_silu_mul(void* stream, int dtype, const void* y, int64_t ld, int64_t up_off, int64_t M, int64_t F, void* out,
+                            int64_t out_ld) {
+  return launch_act_mul<true>(as_stream(stream), dtype, y, ld, up_off, M, F, out, out_ld);
+}
+
+extern "C" int tnx_route_softmax(void* stream, const tnx_rows_src* z, int64_t M, int E, int k, float* topk_w, int32_t* topk_id) {
+  TNX_REQUIRE(z && src_given(*z) && topk_w && topk_id, "route_softmax: null pointer");
+  TNX_REQUIRE(M > 0 && M < ((int64_t)1 << 31) && E > 0 && E <= 4096 && k > 0 && k <= E && z->ld >= E, "route_softmax: bad shape E=%d k=%d", E, k);
+  hipLaunchKernelGGL(route_softmax_kernel, dim3((unsigned)M), dim3(64), (size_t)(E + k) * 4, as_stream(stream), row_src<float>(*z), E, k,
+                     topk_w, topk_id);
+  TNX_CHECK_LAUNCH("route_softmax");
   return TNX_OK;
 }
 

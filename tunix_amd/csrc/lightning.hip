@@ -132,16 +132,6 @@ __global__ __launch_bounds__(256) void lightning_step_kernel(const LightArgs a, 
   }
 }
 
-typedef float f32x16 __attribute__((ext_vector_type(16)));
-__device__ __forceinline__ f32x16 mfma32(u32x4 a, u32x4 b, f32x16 c) {
-  return __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
-}
-// bf16 pairs of (x, y) and of what that rounding left out: together 16 mantissa bits
-__device__ __forceinline__ void split2(float x, float y, uint32_t& hi, uint32_t& lo) {
-  hi = cvt_pk_bf16(x, y);
-  lo = cvt_pk_bf16(x - bflo(hi), y - bfhi(hi));
-}
-
 constexpr int kChunk = 64, kTLD = kChunk + 8;
 constexpr size_t light_smem_bytes(int kt) {
   // Q, K [64][dk + 8]; decayed K^T high and low [dk][72]; V^T [128][72] (bf16); two power tables

@@ -72,7 +72,6 @@ __global__ __launch_bounds__(256)
 __attribute__((amdgpu_waves_per_eu(MODE == kWidePre ? 2 : 1, MODE == kWidePre ? 2 : 1)))
 void qgemm_wide_kernel(const QLArgs a, const WideHead h) {
   constexpr bool INT4 = MODE == kWideInt4, PRE = MODE == kWidePre;
-  static_assert(!(PRE && GROUPED), "the grouped form reads packed codes");
   constexpr int RT = 4, CG = 2, PF = 3, AP = 8;   // 32-row tiles, 32-column groups per wave
   extern __shared__ __align__(16) unsigned char smem[];
   const int tid = threadIdx.x, lane = tid & 63;
@@ -144,8 +143,8 @@ void qgemm_wide_kernel(const QLArgs a, const WideHead h) {
   const u32x4 rx = GROUPED ? raw_rsrc(a.x, (uint64_t)(a.M / a.x_div) * a.K * 2)
                            : raw_rsrc(a.x + m0 * a.K, (uint64_t)rows_here * a.K * 2);
   const uint64_t ntk = (uint64_t)ntiles * ktiles;
-  const rsrc_t rc = make_rsrc(a.codes + (GROUPED ? (int64_t)expert * a.codes_stride : 0), ntk * 1024);
-  const rsrc_t rs = make_rsrc(a.scales + (GROUPED ? (int64_t)expert * a.scales_stride : 0), ntk * 16 * SPT * 2 + 16);
+  const rsrc_t rc = make_rsrc(a.codes + (GROUPED && !PRE ? (int64_t)expert * a.codes_stride : 0), ntk * 1024);
+  const rsrc_t rs = make_rsrc(a.scales + (GROUPED && !PRE ? (int64_t)expert * a.scales_stride : 0), ntk * 16 * SPT * 2 + 16);
   // Lane l: column l % 32 of a group = column (l % 16) of packed tile 2 cg + (l % 32) / 16.  A
   // packed tile holds, at chunk 16 q + c, the k-groups 8 q + 32 j (dword j) of its column c;
   // slab u of the MFMA wants k-group 2 u + l / 32 from this lane: chunk q = l / 32 gives the
@@ -207,7 +206,7 @@ void qgemm_wide_kernel(const QLArgs a, const WideHead h) {
   u32x4 wf[2][CG];           // weight fragments of the current / next slab
   // PRE: the fragments of the next kWidePreStages slabs, loaded as they are; stage = slab % stages
   u32x4 wr[PRE ? kWidePreStages : 1][CG];
-  const rsrc_t re = make_rsrc(PRE ? (const void*)a.w_pre : (const void*)a.x,
+  const rsrc_t re = make_rsrc(PRE ? (const void*)(a.w_pre + (GROUPED ? (int64_t)expert * tiles_n * ktiles * 32768 : 0)) : (const void*)a.x,
                               PRE ? (uint64_t)tiles_n * (uint64_t)ktiles * 65536u : 0u);
   uint32_t evoff[CG];
 #pragma unroll
@@ -543,7 +542,7 @@ void qgemm_wide_kernel(const QLArgs a, const WideHead h) {
   // The bf16 tile goes through LDS (row stride cols + 8 elements) and leaves as 16-byte chunks
   // of whole rows.  A lane holds, for row rt * 32 + l % 32 and group cg, the columns
   // 8 b + 4 (l / 32) + e of the group in register 4 b + e.
-  const bool mul = a.epilogue == TNX_EPI_SILU_MUL || a.epilogue == TNX_EPI_GELU_MUL || a.epilogue == kEpiGeluMulF32;
+  const bool mul = a.epilogue == TNX_EPI_SILU_MUL || a.epilogue == TNX_EPI_GELU_MUL || a.epilogue == kEpiGeluMulF32 || a.epilogue == kEpiSiluMulF32;
   if constexpr (PRE) {
     if (a.epilogue == TNX_EPI_F32) {   // fp32 results leave from the accumulators, 16 bytes per lane
       float* y = reinterpret_cast<float*>(a.y);
@@ -581,6 +580,11 @@ void qgemm_wide_kernel(const QLArgs a, const WideHead h) {
           float v[4];
 #pragma unroll
           for (int e = 0; e < 4; ++e) {
+            if (PRE && a.epilogue == kEpiSiluMulF32) {
+              const float z = acc[rt][cg][4 * b + e];
+              v[e] = z / (1.0f + expf(-z)) * acc[rt][cg][4 * (b + 2) + e];
+              continue;
+            }
             if (PRE && a.epilogue == kEpiGeluMulF32) {
               const float z = acc[rt][cg][4 * b + e];
               v[e] = 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))) *

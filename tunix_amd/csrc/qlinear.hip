@@ -46,7 +46,7 @@ struct QLArgs {
 };
 // gate | up with the activation and the product in fp32 and one rounding (dense-weight decoders;
 // many-row kernel only)
-constexpr int kEpiGeluMulF32 = 16;
+constexpr int kEpiGeluMulF32 = 16, kEpiSiluMulF32 = 17;
 // Second argument of the 128 x 256 kernel: with `part` set it reduces its tile to lm_head
 // statistics instead of storing it.
 struct WideHead {
@@ -761,15 +761,16 @@ int launch_qgemm_wide(hipStream_t st, const QLArgs& a, const WideHead& h = WideH
 
 // The grouped form: the grid covers an upper bound of the 128-row blocks, sum over the experts
 // of ceil(rows / 128) <= n_routes / 128 + E (work-groups past the last block exit at once).
-template <int SPT, bool INT4>
+template <int SPT, int MODE>
 int launch_qgemm_wide_grouped_as(hipStream_t st, const QLArgs& a) {
   static std::once_flag once;
   static int attr_rc = TNX_OK;
-  std::call_once(once, [] { attr_rc = prepare_qgemm128(&qgemm_wide_kernel<SPT, true, INT4 ? kWideInt4 : kWideTable>, kWideSmemBytes); });
+  constexpr size_t kSmem = MODE == kWidePre ? kWidePreSmemBytes : kWideSmemBytes;
+  std::call_once(once, [] { attr_rc = prepare_qgemm128(&qgemm_wide_kernel<SPT, true, MODE>, kSmem); });
   if (attr_rc) return attr_rc;
   const int64_t blocks = a.M / kWideRows + a.n_experts;
   const unsigned wgs = (unsigned)(blocks * cdiv(a.N, kWideCols));
-  hipLaunchKernelGGL((qgemm_wide_kernel<SPT, true, INT4 ? kWideInt4 : kWideTable>), dim3(wgs), dim3(256), kWideSmemBytes, st, a,
+  hipLaunchKernelGGL((qgemm_wide_kernel<SPT, true, MODE>), dim3(wgs), dim3(256), kSmem, st, a,
                      WideHead{nullptr, nullptr, nullptr, 0, 1.0f, nullptr});
   TNX_CHECK_LAUNCH("qgemm_wide_grouped");
   return TNX_OK;
@@ -777,7 +778,7 @@ int launch_qgemm_wide_grouped_as(hipStream_t st, const QLArgs& a) {
 
 template <int SPT>
 int launch_qgemm_wide_grouped(hipStream_t st, const QLArgs& a) {
-  return a.qtype == TNX_Q_INT4 ? launch_qgemm_wide_grouped_as<SPT, true>(st, a) : launch_qgemm_wide_grouped_as<SPT, false>(st, a);
+  return a.qtype == TNX_Q_INT4 ? launch_qgemm_wide_grouped_as<SPT, kWideInt4>(st, a) : launch_qgemm_wide_grouped_as<SPT, kWideTable>(st, a);
 }
 
 // Shapes the 128 x 256 kernel takes: enough rows to fill the device with its tiles, no k split,
@@ -1001,6 +1002,9 @@ int tnx_internal_wide_head(hipStream_t st, const tnx_lmhead_desc* d, float tempe
   return scales_per_tile(a.group) == 2 ? launch_qgemm_wide<2>(st, a, h) : launch_qgemm_wide<4>(st, a, h);
 }
 
+static int once_rounded(int epilogue) {
+  return epilogue == TNX_EPI_GELU_MUL ? kEpiGeluMulF32 : epilogue == TNX_EPI_SILU_MUL ? kEpiSiluMulF32 : epilogue;
+}
 // A dense linear over many rows on the 128 x 256 kernel, from its fragment-order weights
 // (tnx_dense_expand).  The caller has checked the shapes.
 int tnx_internal_wide_dense(hipStream_t st, int64_t M, int64_t K, int64_t N, const uint16_t* x, const uint16_t* w,
@@ -1008,9 +1012,22 @@ int tnx_internal_wide_dense(hipStream_t st, int64_t M, int64_t K, int64_t N, con
   QLArgs a;
   memset(&a, 0, sizeof(a));
   a.M = M; a.K = K; a.N = N; a.group = KTILE; a.x = x; a.w_pre = w; a.x_div = 1;
-  a.epilogue = epilogue == TNX_EPI_GELU_MUL ? kEpiGeluMulF32 : epilogue;
+  a.epilogue = once_rounded(epilogue);
   a.y = y; a.ldy = ldy; a.split_k = 1; a.ktiles_per_split = (int)(K / KTILE);
   return launch_qgemm_wide<2>(st, a);
+}
+
+// The same with one weight per expert (copies behind each other), rows gathered through the sorted routes.
+int tnx_internal_wide_dense_grouped(hipStream_t st, int64_t n_routes, int64_t K, int64_t N, const uint16_t* x, const uint16_t* w,
+                                    int epilogue, void* y, int64_t ldy, int n_experts, const int32_t* offsets,
+                                    const int32_t* sorted_route, int x_div) {
+  QLArgs a;
+  memset(&a, 0, sizeof(a));
+  a.M = n_routes; a.K = K; a.N = N; a.group = KTILE; a.x = x; a.w_pre = w; a.x_div = x_div;
+  a.epilogue = once_rounded(epilogue);
+  a.y = y; a.ldy = ldy; a.split_k = 1; a.ktiles_per_split = (int)(K / KTILE);
+  a.n_experts = n_experts; a.offsets = offsets; a.sorted_route = sorted_route;
+  return launch_qgemm_wide_grouped_as<2, kWidePre>(st, a);
 }
 
 extern "C" int tnx_splitk_finish(void* stream, const tnx_qlinear_desc* d) {

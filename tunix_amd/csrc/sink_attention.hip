@@ -29,16 +29,12 @@ struct SinkArgs {
   void* out;
   int64_t out_ld;
   int out_frag;
+  int64_t out_head;        // distance of two heads in an output row
 };
 
 constexpr float kNegBig = -1.0e30f;
 constexpr float kLog2e = 1.4426950408889634f;
 __device__ __forceinline__ float exp2_hw(float x) { return __builtin_amdgcn_exp2f(x); }
-
-typedef float f32x16 __attribute__((ext_vector_type(16)));
-__device__ __forceinline__ f32x16 mfma32(u32x4 a, u32x4 b, f32x16 c) {
-  return __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
-}
 
 // Weight of the finished sum: O * result is the output.  m is in log2 units.
 __device__ __forceinline__ float finish_scale(float m, float l, bool has_sink, float sink) {
@@ -58,7 +54,7 @@ __global__ __launch_bounds__(256) void sink_attn_any_kernel(const SinkArgs a) {
   const T* q = reinterpret_cast<const T*>(a.q) + (row * a.H + h) * a.dkp;
   const T* k = reinterpret_cast<const T*>(a.k) + (b * a.G + g) * a.S * a.dkp;
   const T* v = reinterpret_cast<const T*>(a.v) + (b * a.G + g) * a.S * a.dvp;
-  constexpr int kMaxOut = 4;   // dv <= 1024
+  constexpr int kMaxOut = 8;   // dv <= 2048
   float o[kMaxOut] = {};
   float m = kNegBig, l = 0.f;
   if (last < a.S)
@@ -106,7 +102,7 @@ __global__ __launch_bounds__(256) void sink_attn_any_kernel(const SinkArgs a) {
   for (int c = 0; c < kMaxOut; ++c) {
     const int d = c * 256 + tid;
     if (d >= a.dv) break;
-    const int64_t col = (int64_t)h * a.dv + d;
+    const int64_t col = (int64_t)h * a.out_head + d;
     st_elem(out, a.out_frag ? frag_index(row, col, a.out_ld) : row * a.out_ld + col, o[c] * w);
   }
 }
@@ -271,7 +267,7 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 2))) void
 #pragma unroll
       for (int j = 0; j < NJ; ++j)
         if (d0 + j < a.dv) {
-          const int64_t col = (int64_t)head * a.dv + d0 + j;
+          const int64_t col = (int64_t)head * a.out_head + d0 + j;
           out[a.out_frag ? frag_index(row, col, a.out_ld) : row * a.out_ld + col] = f2bf(O[h][j][i] * w);
         }
     }
@@ -304,7 +300,7 @@ __global__ __launch_bounds__(128) void sink_attn_merge_kernel(const SinkArgs a) 
   for (int d = threadIdx.x; d < a.dv; d += 128) {
     float acc = 0.f;
     for (int c = 0; c < a.n_chunks; ++c) acc += wts[c] * po[(int64_t)c * a.dvp + d];
-    const int64_t col = (int64_t)head * a.dv + d;
+    const int64_t col = (int64_t)head * a.out_head + d;
     out[a.out_frag ? frag_index(row, col, a.out_ld) : row * a.out_ld + col] = f2bf(acc * tot);
   }
 }
@@ -462,8 +458,8 @@ void sink_attn_tile_kernel(const SinkArgs a) {
   const float w = finish_scale(m_run, l_run, a.sinks != nullptr, a.sinks ? a.sinks[head] : 0.f);
   // register 4 b + e of O[j]: value column NV (8 b + 4 lh + e) + j: runs of 4 NV columns
   uint16_t* out = reinterpret_cast<uint16_t*>(a.out);
-  const int64_t orow = b * a.T + tq, cb = (int64_t)head * a.dv;
-  const bool vec = a.dv % 8 == 0 && a.out_ld % 8 == 0;
+  const int64_t orow = b * a.T + tq, cb = (int64_t)head * a.out_head;
+  const bool vec = a.dv % 8 == 0 && a.out_head % 8 == 0 && a.out_ld % 8 == 0;
 #pragma unroll
   for (int bb = 0; bb < 4; ++bb) {
     const int d0 = NV * (8 * bb + 4 * lh);
@@ -535,15 +531,17 @@ extern "C" size_t tnx_sink_attn_ws_bytes(int64_t B, int64_t T, int64_t S, int H,
 extern "C" int tnx_sink_attn(void* stream, const tnx_sink_attn_desc* d) {
   TNX_REQUIRE(d, "sink_attn: null descriptor");
   TNX_REQUIRE(d->B > 0 && d->T > 0 && d->S >= d->T && d->H > 0 && d->G > 0 && d->H % d->G == 0, "sink_attn: bad shape");
-  TNX_REQUIRE(d->dk > 0 && d->dv > 0 && d->dkp >= d->dk && d->dvp >= d->dv && d->dv <= 1024, "sink_attn: bad head sizes");
+  TNX_REQUIRE(d->dk > 0 && d->dv > 0 && d->dkp >= d->dk && d->dvp >= d->dv && d->dv <= 2048, "sink_attn: bad head sizes");
   TNX_REQUIRE(d->q && d->kcache && d->vcache && d->starts && d->col_ptr && d->out, "sink_attn: null pointer");
-  TNX_REQUIRE(d->out_ld >= (int64_t)d->H * d->dv, "sink_attn: short output rows");
+  TNX_REQUIRE(d->out_head == 0 || d->out_head >= d->dv, "sink_attn: short output heads");
+  TNX_REQUIRE(d->out_ld >= (int64_t)d->H * (d->out_head ? d->out_head : d->dv), "sink_attn: short output rows");
   TNX_REQUIRE(d->dtype == TNX_BF16 || d->dtype == TNX_F32, "sink_attn: bad dtype %d", d->dtype);
   TNX_REQUIRE(d->B <= 65535, "sink_attn: too many rows");
   SinkArgs a;
   a.B = d->B; a.T = d->T; a.S = d->S; a.H = d->H; a.G = d->G; a.R = d->H / d->G; a.dk = d->dk; a.dv = d->dv; a.dkp = d->dkp;
   a.dvp = d->dvp; a.scale = d->scale; a.q = d->q; a.k = d->kcache; a.v = d->vcache; a.sinks = d->sinks; a.starts = d->starts;
   a.col_ptr = d->col_ptr; a.ws = d->ws; a.out = d->out; a.out_ld = d->out_ld; a.out_frag = d->out_frag;
+  a.out_head = d->out_head ? d->out_head : d->dv;
   a.kv_chunk = d->kv_chunk; a.n_chunks = d->kv_chunk > 0 && d->kv_chunk < d->S ? (int)cdiv(d->S, d->kv_chunk) : 1;
   hipStream_t st = as_stream(stream);
   const bool mfma = d->dtype == TNX_BF16 && mfma_sizes(d->dkp, d->dvp) && (uint64_t)d->S * (uint64_t)(d->dkp > d->dvp ? d->dkp : d->dvp) * 2 < (1ull << 31);

@@ -67,17 +67,21 @@ def create_dummy_weights(cfg: ModelConfig, seed: int = 0, device="cpu", scale: f
 
 def create_stack_weights(cfg: StackConfig, seed: int = 0, device="cpu", scale: float | None = None) -> dict:
   """Random weights of a layer-list decoder, by file name: linears ~ N(0, 1) / sqrt(inputs) (or
-  `scale`), norm weights near zero (around one for the plain norm of a lightning layer), sinks ~ N(0, 1)."""
+  `scale`), norm weights near zero, or around one where they are not stored around zero, sinks ~ N(0, 1)."""
   dev = torch.device(device)
   gen = torch.Generator(device=dev)
   gen.manual_seed(seed)
   out = {}
   for name, shape in cfg.weight_shapes().items():
     t = torch.randn(*shape, generator=gen, device=dev, dtype=torch.float32)
-    if name.endswith("mix.sink"):
+    if name.endswith(("mix.sink", "mix.dt_bias")):
       pass
-    elif name.endswith("mix.norm"):
+    elif name.endswith("mix.A_log"):
+      t = 0.5 * t + 0.5
+    elif name.endswith(("mix.norm", "mix.D", "dq.norm", "dkv.norm")) or (not cfg.pre_norm and "norm" in name):
       t = 1.0 + 0.1 * t
+    elif name.endswith(".shift"):
+      t = 0.5 + 0.2 * t
     elif len(shape) == 1:
       t = 0.1 * t
     else:

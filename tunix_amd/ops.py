@@ -363,5 +363,68 @@ def gelu_mul(y, up_off, M, F, out):
           "tnx_gelu_mul")
 
 
+def silu_mul(y, up_off, M, F, out):
+  L.check(L.lib().tnx_silu_mul(_stream(), DTYPES[y.dtype], _ptr(y), y.shape[1], up_off, M, F, _ptr(out), out.shape[1]),
+          "tnx_silu_mul")
+
+
+def route_softmax(src: L.RowsSrc, M, E, k, topk_w, topk_id):
+  L.check(L.lib().tnx_route_softmax(_stream(), C.byref(src), M, E, k, _ptr(topk_w), _ptr(topk_id)), "tnx_route_softmax")
+
+
+def short_conv(desc: L.ShortConvDesc):
+  L.check(L.lib().tnx_short_conv(_stream(), C.byref(desc)), "tnx_short_conv")
+
+
+def ring_write(src: L.RowsSrc, off, B, T, col_ptr, ring):
+  """The last min(T, slots) rows of every sequence into ring [B, slots, width]."""
+  L.check(L.lib().tnx_ring_write(_stream(), DTYPES[ring.dtype], C.byref(src), off, B, T, ring.shape[2], ring.shape[1],
+                                 _ptr(col_ptr), _ptr(ring)), "tnx_ring_write")
+
+
+def ssd_step_ok(N, P) -> bool:
+  return bool(L.lib().tnx_ssd_step_ok(N, P))
+
+
+def ssd_ws_bytes(B, T, H, G, N, P) -> int:
+  return int(L.lib().tnx_ssd_ws_bytes(B, T, H, G, N, P))
+
+
+def ssd(desc: L.SsdDesc):
+  L.check(L.lib().tnx_ssd(_stream(), C.byref(desc)), "tnx_ssd")
+
+
+def latent_row(rank: int, rot: int, dtype) -> int:
+  return int(L.lib().tnx_latent_row(rank, rot, DTYPES[dtype]))
+
+
+def latent_prep(desc: L.LatentPrepDesc):
+  L.check(L.lib().tnx_latent_prep(_stream(), C.byref(desc)), "tnx_latent_prep")
+
+
+def latent_q(desc: L.LatentQDesc):
+  L.check(L.lib().tnx_latent_q(_stream(), C.byref(desc)), "tnx_latent_q")
+
+
+def latent_kv(desc: L.LatentKvDesc):
+  L.check(L.lib().tnx_latent_kv(_stream(), C.byref(desc)), "tnx_latent_kv")
+
+
+def latent_attn_ok(rank, row, S) -> bool:
+  return bool(L.lib().tnx_latent_attn_ok(rank, row, S))
+
+
+def latent_attn_ws_bytes(B, T, S, H, rank, kv_chunk) -> int:
+  return int(L.lib().tnx_latent_attn_ws_bytes(B, T, S, H, rank, kv_chunk))
+
+
+def latent_attn(desc: L.LatentAttnDesc):
+  L.check(L.lib().tnx_latent_attn(_stream(), C.byref(desc)), "tnx_latent_attn")
+
+
+def gate_mul(desc: L.GateMulDesc):
+  L.check(L.lib().tnx_gate_mul(_stream(), C.byref(desc)), "tnx_gate_mul")
+
+
 def logits_stats(desc: L.LogitsDesc):
   L.check(L.lib().tnx_logits_stats(_stream(), C.byref(desc)), "tnx_logits_stats")

@@ -29,13 +29,19 @@ def _qlora_config(d: dict) -> config.ModelConfig:
 
 
 _QLORA = Architecture(_qlora_config, lambda cfg, w, device, dtype: QLoRAModel(cfg, w, device))
+
+
+def _stack(reader) -> Architecture:
+  """A decoder given layer by layer."""
+  return Architecture(reader, lambda cfg, w, device, dtype: StackModel(cfg, w, device, dtype), (torch.bfloat16, torch.float32))
+
+
 ARCHITECTURES: dict[str, Architecture] = {
     "llama3": _QLORA,
     "qwen3": _QLORA,
     "gemma3": _QLORA,
-    "Nunezen": Architecture(config.nunezen_from_dict,
-                            lambda cfg, w, device, dtype: StackModel(cfg, w, device, dtype),
-                            (torch.bfloat16, torch.float32)),
+    "Nunezen": _stack(config.nunezen_from_dict),
+    "Lapevik": _stack(config.lapevik_from_dict),
 }
 
 

@@ -15,8 +15,8 @@ import torch
 
 from . import _lib as L
 from . import ops
-from .cache import KVSpec, SequenceCache, StateSpec
-from .config import AttentionMixer, LightningMixer, StackConfig
+from .cache import KVSpec, LatentSpec, PartsSpec, RingSpec, SequenceCache, StateSpec
+from .config import AttentionMixer, ExpertsMlp, LatentMixer, LightningMixer, SsdMixer, StackConfig
 from .model import HeadRunner
 
 
@@ -29,14 +29,18 @@ FRAG_ROWS = 512
 
 
 class DenseLinear:
-  """One dense projection, possibly several weights [N_i, K] that share an input.  Every member
-  starts at a multiple of 16 output columns (`offsets`), K is zero-padded to a multiple of 128.
+  """One dense projection, possibly several weights [N_i, K] that share an input.  A member is a name, or
+  (name, first row, end row) for some rows of a weight.  Every member starts at a multiple of 16 output
+  columns (`offsets`), K is zero-padded to a multiple of 128.
   paired: two members of one shape whose rows alternate in blocks of 16 (gate | up), so that the
-  kernel's epilogue finds both in one wave (bf16)."""
+  kernel's epilogue finds both in one wave (bf16).  transpose: the members' transposes."""
 
-  def __init__(self, names: list[str], weights: dict, dtype, device, paired: bool = False):
-    self.names, self.dtype, self.device, self.paired = names, dtype, device, paired
-    self.shapes = [tuple(weights[n].shape) for n in names]
+  def __init__(self, members: list, weights: dict, dtype, device, paired: bool = False, transpose: bool = False):
+    self.members = [m if isinstance(m, tuple) else (m, 0, weights[m].shape[0]) for m in members]
+    self.names, self.dtype, self.device, self.paired = [m[0] for m in self.members], dtype, device, paired
+    self.transpose = transpose
+    self.full_shapes = [tuple(weights[n].shape) for n in self.names]
+    self.shapes = [(r1 - r0, s[1])[::-1 if transpose else 1] for (_, r0, r1), s in zip(self.members, self.full_shapes)]
     self.K = self.shapes[0][1]
     self.Kp = _up(self.K, 128)
     widths = [_up(s[0], 16) for s in self.shapes]
@@ -46,7 +50,7 @@ class DenseLinear:
     self.load(weights)
 
   def check(self, weights: dict):
-    for n, s in zip(self.names, self.shapes):
+    for n, s in zip(self.names, self.full_shapes):
       if n not in weights:
         raise ValueError(f"New state must have the same structure as the old state: {n} is missing")
       if tuple(weights[n].shape) != s:
@@ -55,8 +59,9 @@ class DenseLinear:
   def load(self, weights: dict):
     self.check(weights)
     w = torch.zeros(self.N, self.Kp, dtype=self.dtype, device=self.device)
-    for n, off in zip(self.names, self.offsets):
-      src = weights[n].to(self.device, self.dtype)
+    for (n, r0, r1), off in zip(self.members, self.offsets):
+      src = weights[n][r0:r1].to(self.device, self.dtype)
+      src = src.T if self.transpose else src
       w[off:off + src.shape[0], :self.K] = src
     if self.dtype == torch.bfloat16:
       if self.paired:
@@ -69,6 +74,25 @@ class DenseLinear:
 
   def nbytes(self) -> int:
     return sum(a * b for a, b in self.shapes) * (2 if self.dtype == torch.bfloat16 else 4)
+
+
+class LinearBank:
+  """Projections of one shape behind each other in memory: experts, or one per head."""
+
+  def __init__(self, linears: list[DenseLinear]):
+    self.linears = linears
+    first = linears[0]
+    self.w = torch.stack([f.w for f in linears])
+    for f, w in zip(linears, self.w):   # (a member's load writes into the bank)
+      f.w = w
+    self.K, self.Kp, self.N, self.shapes, self.offsets = first.K, first.Kp, first.N, first.shapes, first.offsets
+    self.stride = self.w[0].numel()
+
+  def __len__(self) -> int:
+    return len(self.linears)
+
+  def nbytes(self) -> int:
+    return sum(f.nbytes() for f in self.linears)
 
 
 class StackModel:
@@ -86,25 +110,45 @@ class StackModel:
     vec = lambda name: weights[name].to(dev, torch.float32).contiguous()
     self.embed = torch.zeros(V, D, dtype=dtype, device=dev)
     self.final_norm = vec("final.norm")
-    self.linears: dict[str, DenseLinear] = {}
+    self.linears: dict[str, list[DenseLinear]] = {}    # the projections a weight takes part in
     self.vectors: dict[str, torch.Tensor] = {"final.norm": self.final_norm}
 
-    def linear(names, paired=False):
-      f = DenseLinear(names, weights, dtype, dev, paired)
-      for n in names:
-        self.linears[n] = f
+    def linear(members, paired=False, transpose=False):
+      f = DenseLinear(members, weights, dtype, dev, paired, transpose)
+      for n in dict.fromkeys(f.names):
+        self.linears.setdefault(n, []).append(f)
       return f
 
     def vector(name):
       self.vectors[name] = vec(name)
       return self.vectors[name]
 
+    self.embed_norm = vector("embed.norm") if cfg.embed_norm else None
     self.loop_in = linear(["loop.in"]) if cfg.loop is not None else None
     self.layers = []
     for i, spec in enumerate(cfg.layers):
       p, m = f"l{i}.", spec.mixer
-      ly = {"spec": spec, "norm1": vector(p + "norm1"), "norm1b": vector(p + "norm1b")}
-      if isinstance(m, AttentionMixer):
+      ly = {"spec": spec, "norm1": vector(p + "norm1") if cfg.pre_norm else None, "post1": vector(p + cfg.post_norm(1))}
+      if cfg.token_shift:
+        ly["shift"] = vector(p + "shift")
+      if isinstance(m, SsdMixer):
+        x = p + "mix."
+        ly["in"] = linear([(x + "in", 0, m.inner), (x + "in", m.inner, m.inner + m.channels),
+                           (x + "in", m.inner + m.channels, m.inner + m.channels + m.heads)])
+        self.vectors[x + "conv"] = ly["conv"] = vec(x + "conv").T.contiguous()      # [taps, channels]
+        for key, name in (("conv_b", "conv.b"), ("dt_bias", "dt_bias"), ("A_log", "A_log"), ("D", "D"), ("norm", "norm")):
+          ly[key] = vector(x + name)
+      elif isinstance(m, LatentMixer):
+        x = p + "mix."
+        ly["in"] = linear([x + "dq", x + "dkv", x + "g"])
+        ly["uq"], ly["ukv"] = linear([x + "uq"]), linear([x + "uk", x + "uv"])
+        # the key projection applied to a head's query, the value projection to its weighted latent
+        ly["absorb_k"] = LinearBank([linear([(x + "uk", h * m.dim, (h + 1) * m.dim)], transpose=True) for h in range(m.heads)])
+        ly["absorb_v"] = LinearBank([linear([(x + "uv", h * m.vdim, (h + 1) * m.vdim)]) for h in range(m.heads)])
+        ly["q_norm"], ly["kv_norm"] = vector(x + "dq.norm"), vector(x + "dkv.norm")
+        freq = np.float64(m.rot_base) ** (-2.0 * np.arange(m.rot_dim // 2) / max(m.rot_dim, 1))
+        ly["inv_freq"] = torch.from_numpy(freq.astype(np.float32)).to(dev)
+      elif isinstance(m, AttentionMixer):
         ly["in"] = linear([p + "mix.q", p + "mix.k", p + "mix.v"])
         ly["sink"] = vector(p + "mix.sink") if m.sink else None
         freq = np.float64(m.rot_base) ** (-2.0 * np.arange(m.rot_dims // 2) / max(m.rot_dims, 1))
@@ -115,7 +159,13 @@ class StackModel:
         ly["decay"] = torch.tensor(m.decay, dtype=torch.float32, device=dev)
       ly["out"] = linear([p + "mix.o"])
       if spec.mlp is not None:
-        ly["norm2"], ly["norm2b"] = vector(p + "norm2"), vector(p + "norm2b")
+        ly["norm2"], ly["post2"] = vector(p + "norm2") if cfg.pre_norm else None, vector(p + cfg.post_norm(2))
+      if isinstance(spec.mlp, ExpertsMlp):
+        e = [p + f"mlp.e{j}." for j in range(spec.mlp.experts)]
+        ly["router"] = linear([p + "mlp.router"])
+        ly["gu"] = LinearBank([linear([n + "gate", n + "up"], paired=True) for n in e])
+        ly["down"] = LinearBank([linear([n + "down"]) for n in e])
+      elif spec.mlp is not None:
         ly["gu"] = linear([p + "mlp.gate", p + "mlp.up"], paired=True)
         ly["down"] = linear([p + "mlp.down"])
       self.layers.append(ly)
@@ -154,10 +204,17 @@ class StackModel:
     for i, _ in self.cfg.layer_runs:
       m = self.cfg.layers[i].mixer
       if isinstance(m, AttentionMixer):
-        specs.append(KVSpec(m.kv_heads, ops.sink_attn_pad(m.dim, False, self.dtype),
-                            ops.sink_attn_pad(m.vdim, True, self.dtype), self.dtype))
+        spec = KVSpec(m.kv_heads, ops.sink_attn_pad(m.dim, False, self.dtype),
+                      ops.sink_attn_pad(m.vdim, True, self.dtype), self.dtype)
+      elif isinstance(m, SsdMixer):
+        spec = PartsSpec((("state", StateSpec(m.heads, m.state, m.vdim)), ("conv", RingSpec(m.conv, m.channels, self.dtype))))
+      elif isinstance(m, LatentMixer):
+        spec = LatentSpec(ops.latent_row(m.kv_rank, m.rot_dim, self.dtype), self.dtype)
       else:
-        specs.append(StateSpec(m.heads, m.dim, m.vdim))
+        spec = StateSpec(m.heads, m.dim, m.vdim)
+      if self.cfg.token_shift:
+        spec = PartsSpec((("mixer", spec), ("shift", RingSpec(1, self.cfg.embed_dim, torch.float32))))
+      specs.append(spec)
     return specs
 
   def new_cache(self, B: int, S: int, shared: bool = False) -> SequenceCache:
@@ -174,14 +231,15 @@ class StackModel:
     """Replaces parameters by name; the members of a fused projection come together.  A rejected
     state changes nothing."""
     self._check_names(new_state, complete=False)
-    owners = {id(f): f for n, f in self.linears.items() if n in new_state}
+    owners = {id(f): f for n, fs in self.linears.items() if n in new_state for f in fs}
     for f in owners.values():
       f.check(new_state)
     for f in owners.values():
       f.load(new_state)
     for n, t in new_state.items():
       if n in self.vectors:
-        self.vectors[n].copy_(t.to(self.device, torch.float32))
+        t = t.to(self.device, torch.float32)
+        self.vectors[n].copy_(t.T if t.dim() == 2 else t)
     if "embed" in new_state:
       self._load_embed(new_state["embed"])
     torch.cuda.synchronize(self.device)
@@ -191,7 +249,7 @@ class StackModel:
     n = 0
     for i, begins in self.cfg.layer_runs:
       ly = self.layers[i]
-      n += sum(ly[k].nbytes() for k in ("in", "out", "gu", "down") if k in ly)
+      n += sum(ly[k].nbytes() for k in ("in", "uq", "absorb_k", "absorb_v", "out", "router", "gu", "down") if k in ly)
       n += self.loop_in.nbytes() if begins else 0
     return {"dense": n, "head": self.embed.numel() * self.embed.element_size()}
 
@@ -215,29 +273,46 @@ class StackRunner(HeadRunner):
     self._bufs: dict = {}
     D = cfg.embed_dim
     self.x = torch.empty(M, D, dtype=torch.float32, device=dev)
+    # a token shift reads the row in front of a row: over several tokens the new rows go to a second buffer
+    self.x_next = torch.empty_like(self.x) if cfg.token_shift and T > 1 else None
     # the final-normed rows (row-major, zero columns behind the model width)
     width = D if model.block_head else model.Dp
     self.xn = torch.zeros(M, width, dtype=self.dtype, device=dev)
     self.split_k_override = dict(split_k_override or {})
-    n_y = n_ws = n_light = n_attn = 1
+    n_light = n_attn = n_routes = n_experts = 1
+    n_y, n_ws = [1, 1], [1, 1]     # a projection's output, and that of one which runs while the first is still read
     for i, begins in cfg.layer_runs:
       ly = model.layers[i]
       m = ly["spec"].mixer
-      for key in ("in", "out", "gu", "down"):
-        if key in ly:
-          f = ly[key]
-          n_y = max(n_y, M * f.N)
-          n_ws = max(n_ws, self._split(f) * M * f.N if self._split(f) > 1 else 1)
+      for key, slot in (("in", 0), ("out", 0), ("router", 0), ("gu", 0), ("down", 0), ("uq", 1), ("ukv", 1)):
+        f = ly.get(key)
+        if isinstance(f, DenseLinear):
+          n_y[slot] = max(n_y[slot], M * f.N)
+          n_ws[slot] = max(n_ws[slot], self._split(f) * M * f.N if self._split(f) > 1 or key == "router" else 1)
       if begins:
-        n_ws = max(n_ws, self._split(model.loop_in) * M * model.loop_in.N)
+        n_ws[0] = max(n_ws[0], self._split(model.loop_in) * M * model.loop_in.N)
+      if isinstance(ly["spec"].mlp, ExpertsMlp):
+        e = ly["spec"].mlp
+        n_routes, n_experts = max(n_routes, M * e.top), max(n_experts, e.experts)
+        if self.dtype == torch.float32:
+          n_y[0] = max(n_y[0], M * e.top * ly["gu"].N)
       if isinstance(m, LightningMixer):   # (a call may bring fewer rows, and cut them into more spans)
         n_light = max([n_light] + [ops.lightning_ws_bytes(b, T, m.heads, m.dim, m.vdim) // 4 for b in range(1, B + 1)])
+      elif isinstance(m, SsdMixer):
+        n_light = max([n_light] + [ops.ssd_ws_bytes(b, T, m.heads, m.groups, m.state, m.vdim) // 4 for b in range(1, B + 1)])
+      elif isinstance(m, LatentMixer):
+        if self.dtype == torch.bfloat16:
+          n_attn = max(n_attn, ops.latent_attn_ws_bytes(B, T, S, m.heads, m.kv_rank, self._latent_chunk(m)) // 4)
       else:
         n_attn = max(n_attn, ops.sink_attn_ws_bytes(B, T, S, m.heads, ops.sink_attn_pad(m.vdim, True, self.dtype),
                                                     self._kv_chunk(m, kv_chunk)) // 4)
     self.kv_chunk_arg = kv_chunk
-    self.y = torch.empty(n_y, dtype=self.dtype, device=dev)
-    self.ws = torch.empty(n_ws, dtype=torch.float32, device=dev)
+    self.y = [torch.empty(n, dtype=self.dtype, device=dev) for n in n_y]
+    self.ws = [torch.empty(n, dtype=torch.float32, device=dev) for n in n_ws]
+    if n_routes > 1 or n_experts > 1:
+      i32 = lambda n: torch.empty(n, dtype=torch.int32, device=dev)
+      self.topk_id, self.counts, self.offsets, self.sorted_route = i32(n_routes), i32(n_experts), i32(n_experts + 1), i32(n_routes)
+      self.topk_w = torch.empty(n_routes, dtype=torch.float32, device=dev)
     self.light_ws = torch.empty(n_light, dtype=torch.float32, device=dev)
     self.attn_ws = torch.empty(n_attn, dtype=torch.float32, device=dev)
     self.zero = torch.zeros(1, dtype=torch.int32, device=dev)
@@ -251,12 +326,13 @@ class StackRunner(HeadRunner):
     self.residual_sink = None   # called with the fp32 residual [M, D] behind every layer run
 
   # ---- building blocks -----------------------------------------------------------------------
-  def _buf(self, name: str, cols: int, dtype=None) -> torch.Tensor:
+  def _buf(self, name: str, cols: int, dtype=None, rows: int | None = None) -> torch.Tensor:
     """Activation buffer [rows, cols], zero where nothing is ever written (the padding columns of a
     linear's input must be zero); whole blocks of 128 rows for the fragment order."""
-    key = (name, cols)
+    key = (name, cols, rows)
     if key not in self._bufs:
-      rows = _up(self.M, 128) if self.frag else self.M
+      if rows is None:
+        rows = _up(self.M, 128) if self.frag else self.M
       self._bufs[key] = torch.zeros(rows, cols, dtype=self.dtype if dtype is None else dtype, device=self.model.device)
     return self._bufs[key]
 
@@ -271,6 +347,14 @@ class StackRunner(HeadRunner):
     chunk = max(32, _up(math.ceil(self.S / n), 32))
     return 0 if chunk >= self.S else chunk
 
+  def _latent_chunk(self, m: LatentMixer) -> int:
+    """The same for latent attention, whose work-groups have a compute unit to themselves."""
+    groups = self.B * math.ceil(self.T * m.heads / 32)
+    if self.T != 1 or groups >= 256 or self.S <= 128:
+      return 0
+    chunk = _up(math.ceil(self.S / math.ceil(256 / groups)), 128)
+    return 0 if chunk >= self.S else chunk
+
   def _split(self, f: DenseLinear) -> int:
     """k split of a few-row linear whose reader sums fp32 planes."""
     key = f.names[0].split(".")[-1]
@@ -281,8 +365,9 @@ class StackRunner(HeadRunner):
     groups = math.ceil(f.N / 64) * math.ceil(self.M / 128)
     return int(max(1, min(8, (256 if self.M > 32 else 512) // groups, f.Kp // 512)))
 
-  def linear(self, f: DenseLinear, x, M: int, fp32_out: bool = False) -> L.RowsSrc:
-    """Runs one projection of x [M, f.Kp]; returns its output as the reading kernel wants it."""
+  def linear(self, f: DenseLinear, x, M: int, fp32_out: bool = False, slot: int = 0) -> L.RowsSrc:
+    """Runs one projection of x [M, f.Kp]; returns its output as the reading kernel wants it.  It holds until
+    the next projection of the same slot."""
     d = L.DenseDesc()
     d.M, d.K, d.N, d.dtype = M, f.Kp, f.N, self.code
     d.x, d.ldx, d.x_frag, d.w = x.data_ptr(), x.shape[1], 1 if self.frag else 0, f.w.data_ptr()
@@ -290,30 +375,52 @@ class StackRunner(HeadRunner):
     src = L.RowsSrc()
     src.ld, src.plane, src.split_k = f.N, M * f.N, d.split_k
     if d.split_k > 1:
-      d.epilogue, d.ws = L.TNX_EPI_F32, self.ws.data_ptr()
+      d.epilogue, d.ws = L.TNX_EPI_F32, self.ws[slot].data_ptr()
       src.ws = d.ws
     elif fp32_out and self.dtype != torch.float32:
-      d.epilogue, d.y = L.TNX_EPI_F32, self.ws.data_ptr()
+      d.epilogue, d.y = L.TNX_EPI_F32, self.ws[slot].data_ptr()
       src.ws = d.y
     else:
-      d.epilogue, d.y = L.TNX_EPI_STORE, self.y.data_ptr()
+      d.epilogue, d.y = L.TNX_EPI_STORE, self.y[slot].data_ptr()
       src.y = d.y
     ops.dense_linear(d)
     return src
 
-  def residual_norm(self, pending, w_next, out, M: int, frag: bool):
-    """x takes what is pending (None, ("add", rows, post-norm weight) or ("set", rows, None));
-    out = norm(x) . w_next, or x itself when w_next is None."""
+  def bank(self, f: LinearBank, x, ldx: int, x_stride: int, y, ldy: int, y_stride: int, M: int):
+    """Every row of x through every projection of a bank: x + z x_stride -> y + z y_stride."""
+    d = L.DenseDesc()
+    d.M, d.K, d.N, d.dtype = M, f.Kp, f.N, self.code
+    d.x, d.ldx, d.x_stride, d.w, d.w_stride = x.data_ptr(), ldx, x_stride, f.w.data_ptr(), f.stride
+    d.epilogue, d.y, d.ldy, d.y_stride, d.split_k, d.batch = L.TNX_EPI_STORE, y.data_ptr(), ldy, y_stride, 1, len(f)
+    ops.dense_linear(d)
+
+  def residual_norm(self, pending, w_next, out, M: int, frag: bool, shift=None):
+    """x takes what is pending: None, ("add", rows, post-norm weight), ("set", rows, None), ("norm", None, weight) --
+    x itself normed -- or ("routes", rows, post-norm weight, route weights, routes per row);
+    out = norm(x) . w_next, or x itself when w_next is None, or x moved towards the token before:
+    shift = (weight, ring of the rows before, col_ptr, starts, B, T)."""
     cfg = self.cfg
     d = L.ResidualNormDesc()
-    d.M, d.D, d.dtype, d.eps, d.w_offset = M, cfg.embed_dim, self.code, cfg.norm_eps, cfg.norm_offset
+    d.M, d.D, d.dtype, d.eps, d.w_offset, d.groups = M, cfg.embed_dim, self.code, cfg.norm_eps, cfg.norm_offset, cfg.norm_groups
     if pending is not None:
-      kind, d.y, w_post = pending
-      d.mode = 1 if kind == "add" else 2
+      kind, rows, w_post = pending[:3]
+      d.mode = {"add": 1, "routes": 1, "set": 2, "norm": 3}[kind]
+      if rows is not None:
+        d.y = rows
       d.w_post = None if w_post is None else w_post.data_ptr()
+      if kind == "routes":
+        d.route_w, d.route_k = pending[3].data_ptr(), pending[4]
     d.x, d.w_next = self.x.data_ptr(), None if w_next is None else w_next.data_ptr()
     d.out, d.out_ld, d.out_frag = out.data_ptr(), out.shape[1], 1 if frag else 0
+    if shift is not None:
+      w, ring, col_ptr, starts, B, T = shift
+      d.shift, d.before, d.starts, d.col_ptr, d.B, d.T = w.data_ptr(), ring.data_ptr(), starts.data_ptr(), col_ptr.data_ptr(), B, T
+      if T > 1:
+        d.x_out = self.x_next.data_ptr()
     ops.residual_norm(d)
+    if shift is not None and T > 1:
+      self.x, self.x_next = self.x_next, self.x
+      ops.ring_write(ops.rows_src(y=self.x, ld=cfg.embed_dim), 0, B, T, col_ptr, ring)
 
   def rotate(self, ly, src, entry, col_ptr, starts, B, T):
     """Rotates q and k of an attention layer's projection and writes the cache; returns q."""
@@ -365,21 +472,201 @@ class StackRunner(HeadRunner):
     ops.gated_norm(d)
     return out
 
+  # state-space duality
+  def convolve(self, ly, src, entry, col_ptr, starts, B, T) -> torch.Tensor:
+    """silu(convolution) of x, B and C: [rows, channels]; the ring takes the last inputs."""
+    m, ring = ly["spec"].mixer, entry["conv"].r
+    u = self._buf("conv", _up(m.channels, 8), rows=self.M)
+    d = L.ShortConvDesc()
+    d.B, d.T, d.C, d.taps, d.slots, d.dtype = B, T, m.channels, m.conv, ring.shape[1], self.code
+    d.y, d.off, d.w, d.bias, d.ring = src, ly["in"].offsets[1], ly["conv"].data_ptr(), ly["conv_b"].data_ptr(), ring.data_ptr()
+    d.starts, d.col_ptr, d.out, d.out_ld = starts.data_ptr(), col_ptr.data_ptr(), u.data_ptr(), u.shape[1]
+    ops.short_conv(d)
+    ops.ring_write(src, ly["in"].offsets[1], B, T, col_ptr, ring)
+    return u
+
+  def ssd(self, ly, src, u, entry, col_ptr, starts, B, T) -> torch.Tensor:
+    """The recurrence: fp32 [rows, heads * vdim].  u None: one token, the convolution inside."""
+    m, f, ring = ly["spec"].mixer, ly["in"], entry["conv"].r
+    o = self._buf("state_out", m.inner, torch.float32)
+    d = L.SsdDesc()
+    d.B, d.T, d.H, d.G, d.N, d.P, d.dtype = B, T, m.heads, m.groups, m.state, m.vdim, self.code
+    d.A_log, d.dt_bias, d.D = ly["A_log"].data_ptr(), ly["dt_bias"].data_ptr(), ly["D"].data_ptr()
+    d.y, d.c_off, d.dt_off = src, f.offsets[1], f.offsets[2]
+    if u is not None:
+      d.u, d.u_ld = u.data_ptr(), u.shape[1]
+    d.taps, d.slots, d.conv_w, d.conv_b, d.ring = m.conv, ring.shape[1], ly["conv"].data_ptr(), ly["conv_b"].data_ptr(), ring.data_ptr()
+    d.starts, d.col_ptr, d.state = starts.data_ptr(), col_ptr.data_ptr(), entry["state"].s.data_ptr()
+    d.o, d.o_ld, d.ws = o.data_ptr(), o.shape[1], self.light_ws.data_ptr()
+    ops.ssd(d)
+    return o
+
+  def ssd_gate(self, ly, o, src, M: int) -> torch.Tensor:
+    """norm(o * silu(gate columns of the projection)) . weight, in the mixer's norm groups."""
+    m, out = ly["spec"].mixer, self._buf("gated", ly["out"].Kp)
+    d = L.GatedNormDesc()
+    d.M, d.W, d.dtype, d.eps, d.gate_first, d.groups = M, m.inner, self.code, self.cfg.norm_eps, 1, m.norm_groups
+    d.o, d.o_ld, d.g, d.g_off, d.w = o.data_ptr(), o.shape[1], src, ly["in"].offsets[0], ly["norm"].data_ptr()
+    d.out, d.out_ld, d.out_frag = out.data_ptr(), out.shape[1], 1 if self.frag else 0
+    ops.gated_norm(d)
+    return out
+
+  # latent attention
+  def latent_prep(self, ly, src, entry, col_ptr, starts, B, T, expand: bool):
+    """Norms the query latent (returned) and the key / value latent (returned with `expand`), fills the cache."""
+    m, f, c = ly["spec"].mixer, ly["in"], entry.c
+    cq = self._buf("cq", ly["uq"].Kp)
+    ckv = self._buf("ckv", ly["ukv"].Kp) if expand else None
+    d = L.LatentPrepDesc()
+    d.B, d.T, d.S = B, T, c.shape[1]
+    d.q_rank, d.rank, d.rot, d.rank_pad, d.row = m.q_rank, m.kv_rank, m.rot_dim, _up(m.kv_rank, 16), c.shape[2]
+    d.dtype, d.eps, d.y, d.q_off, d.kv_off = self.code, self.cfg.norm_eps, src, f.offsets[0], f.offsets[1]
+    d.w_q, d.w_kv, d.inv_freq = ly["q_norm"].data_ptr(), ly["kv_norm"].data_ptr(), ly["inv_freq"].data_ptr()
+    d.starts, d.col_ptr, d.cache = starts.data_ptr(), col_ptr.data_ptr(), c.data_ptr()
+    d.q_out, d.q_ld, d.q_frag = cq.data_ptr(), cq.shape[1], 1 if self.frag else 0
+    if expand:
+      d.c_out, d.c_ld, d.c_frag = ckv.data_ptr(), ckv.shape[1], 1 if self.frag else 0
+    ops.latent_prep(d)
+    return cq, ckv
+
+  def latent_q(self, ly, src, col_ptr, starts, B, T, un, un_ld, un_pad, rot, rot_at, rot_ld, rot_pad):
+    """Splits the heads of a query projection: the unrotated parts to `un`, the rotated ones to rot[rot_at ..]."""
+    m = ly["spec"].mixer
+    d = L.LatentQDesc()
+    d.B, d.T, d.H, d.n, d.r, d.dtype, d.y = B, T, m.heads, m.dim, m.rot_dim, self.code, src
+    d.inv_freq, d.starts, d.col_ptr = ly["inv_freq"].data_ptr(), starts.data_ptr(), col_ptr.data_ptr()
+    d.un, d.un_ld, d.un_pad = un.data_ptr(), un_ld, un_pad
+    d.rot, d.rot_ld, d.rot_pad = rot.data_ptr() + rot_at * rot.element_size(), rot_ld, rot_pad
+    ops.latent_q(d)
+
+  def gate_mul(self, ly, y, head: int, y_head: int, src, M: int) -> torch.Tensor:
+    m, out = ly["spec"].mixer, self._buf("gated", ly["out"].Kp)
+    d = L.GateMulDesc()
+    d.M, d.W, d.head, d.dtype, d.y, d.y_ld, d.y_head = M, m.heads * head, head, self.code, y.data_ptr(), m.heads * y_head, y_head
+    d.g, d.g_off, d.out, d.out_ld, d.out_frag = src, ly["in"].offsets[2], out.data_ptr(), out.shape[1], 1 if self.frag else 0
+    ops.gate_mul(d)
+    return out
+
+  def _sink_free_attention(self, m, q, k, v, dk, dv, starts, col_ptr, B, T, S, G, out, out_head):
+    """softmax(scale q k) v over plain keys and values (one kv head per query head, or one for all)."""
+    d = L.SinkAttnDesc()
+    d.B, d.T, d.S, d.H, d.G = B, T, S, m.heads, G
+    d.dk, d.dv, d.dkp, d.dvp, d.scale, d.dtype = dk, dv, k.shape[-1], v.shape[-1], m.scale, self.code
+    d.q, d.kcache, d.vcache, d.starts, d.col_ptr = q.data_ptr(), k.data_ptr(), v.data_ptr(), starts.data_ptr(), col_ptr.data_ptr()
+    d.ws, d.out, d.out_ld, d.out_head = self.attn_ws.data_ptr(), out.data_ptr(), m.heads * out_head, out_head
+    ops.sink_attn(d)
+
+  def latent_prompt(self, ly, cq, ckv, entry, col_ptr, starts, B, T):
+    """A prompt from its first column on: keys and values of all heads are formed for its tokens."""
+    m, M, c = ly["spec"].mixer, B * T, entry.c
+    dkp, dvp = ops.sink_attn_pad(m.dim + m.rot_dim, False, self.dtype), ops.sink_attn_pad(m.vdim, True, self.dtype)
+    q = self._buf("q", m.heads * dkp, rows=self.M)
+    self.latent_q(ly, self.linear(ly["uq"], cq, M, slot=1), col_ptr, starts, B, T, q, dkp, m.dim, q, m.dim, dkp, dkp - m.dim)
+    k, v = self._buf("k_full", dkp, rows=self.M * m.heads), self._buf("v_full", dvp, rows=self.M * m.heads)
+    d = L.LatentKvDesc()
+    d.B, d.T, d.S, d.H, d.n, d.r, d.vd = B, T, c.shape[1], m.heads, m.dim, m.rot_dim, m.vdim
+    d.dkp, d.dvp, d.rank_pad, d.row, d.dtype = dkp, dvp, _up(m.kv_rank, 16), c.shape[2], self.code
+    d.y, d.v_off, d.cache = self.linear(ly["ukv"], ckv, M, slot=1), ly["ukv"].offsets[1], c.data_ptr()
+    d.k, d.v = k.data_ptr(), v.data_ptr()
+    ops.latent_kv(d)
+    out = self._buf("heads", m.heads * m.vdim, rows=self.M)
+    self._sink_free_attention(m, q, k, v, m.dim + m.rot_dim, m.vdim, starts, col_ptr, B, T, T, m.heads, out, m.vdim)
+    return out, m.vdim
+
+  def latent_rows(self, ly, cq, entry, col_ptr, starts, B, T):
+    """Decoding and portions: the heads attend to the cache rows themselves."""
+    m, M, c = ly["spec"].mixer, B * T, entry.c
+    H, row, fk, fv = m.heads, c.shape[2], ly["absorb_k"], ly["absorb_v"]
+    un, q = self._buf("q_un", H * fk.Kp, rows=self.M), self._buf("q", H * row, rows=self.M)
+    self.latent_q(ly, self.linear(ly["uq"], cq, M, slot=1), col_ptr, starts, B, T, un, fk.Kp, fk.Kp, q, fk.N, row, row - fk.N)
+    self.bank(fk, un, H * fk.Kp, fk.Kp, q, H * row, row, M)
+    lat = self._buf("latent_out", H * fv.Kp, rows=self.M)
+    self.latent_attend(ly, q, lat, fv.Kp, entry, col_ptr, starts, B, T)
+    out = self._buf("heads", H * fv.N, rows=self.M)
+    self.bank(fv, lat, H * fv.Kp, fv.Kp, out, H * fv.N, fv.N, M)
+    return out, fv.N
+
+  def latent_attend(self, ly, q, out, out_head, entry, col_ptr, starts, B, T):
+    m, c = ly["spec"].mixer, entry.c
+    S, row = c.shape[1], c.shape[2]
+    if self.dtype != torch.bfloat16 or not ops.latent_attn_ok(m.kv_rank, row, S):
+      self._sink_free_attention(m, q, c, c, _up(m.kv_rank, 16) + m.rot_dim, m.kv_rank, starts, col_ptr, B, T, S, 1, out, out_head)
+      return
+    d = L.LatentAttnDesc()
+    d.B, d.T, d.S, d.H, d.rank, d.row, d.scale = B, T, S, m.heads, m.kv_rank, row, m.scale
+    d.q, d.cache, d.starts, d.col_ptr = q.data_ptr(), c.data_ptr(), starts.data_ptr(), col_ptr.data_ptr()
+    d.kv_chunk, d.ws, d.out, d.out_head = self._latent_chunk(m) if T == 1 else 0, self.attn_ws.data_ptr(), out.data_ptr(), out_head
+    ops.latent_attn(d)
+
   def _mixer(self, ly, h, entry, col_ptr, starts, B, T) -> L.RowsSrc:
-    src = self.linear(ly["in"], h, B * T)
-    if isinstance(ly["spec"].mixer, AttentionMixer):
-      q = self.rotate(ly, src, entry, col_ptr, starts, B, T)
-      out = self.attend(ly, q, entry, col_ptr, starts, B, T)
+    m, M = ly["spec"].mixer, B * T
+    src = self.linear(ly["in"], h, M)
+    at = (entry, col_ptr, starts, B, T)
+    if isinstance(m, AttentionMixer):
+      out = self.attend(ly, self.rotate(ly, src, *at), *at)
+    elif isinstance(m, SsdMixer):
+      u = None if T == 1 and ops.ssd_step_ok(m.state, m.vdim) else self.convolve(ly, src, *at)
+      out = self.ssd_gate(ly, self.ssd(ly, src, u, *at), src, M)
+    elif isinstance(m, LatentMixer):
+      prompt = T > 1 and col_ptr is self.zero
+      cq, ckv = self.latent_prep(ly, src, *at, expand=prompt)
+      y, y_head = self.latent_prompt(ly, cq, ckv, *at) if prompt else self.latent_rows(ly, cq, *at)
+      out = self.gate_mul(ly, y, m.vdim, y_head, src, M)
     else:
-      out = self.gate(ly, self.recur(ly, src, entry, col_ptr, starts, B, T), src, B * T)
-    return self.linear(ly["out"], out, B * T)
+      out = self.gate(ly, self.recur(ly, src, *at), src, M)
+    return self.linear(ly["out"], out, M)
+
+  # experts
+  def route(self, ly, h, M: int):
+    """Chooses every row's experts and sorts the routes by expert."""
+    e = ly["spec"].mlp
+    src = self.linear(ly["router"], h, M, fp32_out=True)
+    if src.split_k <= 1 and src.ws:
+      src.y = src.ws
+    ids = self.topk_id[:M * e.top].view(M, e.top)
+    ops.route_softmax(src, M, e.experts, e.top, self.topk_w, ids)
+    ops.moe_sort_routes(ids, e.experts, self.counts, self.offsets, self.sorted_route)
+
+  def experts_linear(self, f: LinearBank, x, x_frag: bool, x_div: int, routes: int, epilogue: int, y, ldy: int):
+    d = L.DenseDesc()
+    d.M, d.K, d.N, d.dtype = routes, f.Kp, f.N, self.code
+    d.x, d.ldx, d.x_frag, d.w, d.w_stride = x.data_ptr(), x.shape[1], 1 if x_frag else 0, f.w.data_ptr(), f.stride
+    d.epilogue, d.y, d.ldy, d.split_k = epilogue, y.data_ptr(), ldy, 1
+    d.n_experts, d.x_div, d.offsets, d.sorted_route = len(f), x_div, self.offsets.data_ptr(), self.sorted_route.data_ptr()
+    ops.dense_linear(d)
+
+  def experts_gate_up(self, ly, h, M: int) -> torch.Tensor:
+    e, f = ly["spec"].mlp, ly["gu"]
+    act = self._buf("act", ly["down"].Kp, rows=self.M * e.top)
+    if self.dtype == torch.float32:
+      y = self.y[0][:M * e.top * f.N].view(M * e.top, f.N)
+      self.experts_linear(f, h, False, e.top, M * e.top, L.TNX_EPI_STORE, y, f.N)
+      ops.silu_mul(y, f.offsets[1], M * e.top, e.ff, act)
+    else:
+      self.experts_linear(f, h, self.frag, e.top, M * e.top, L.TNX_EPI_SILU_MUL, act, act.shape[1])
+    return act
+
+  def experts_down(self, ly, act, M: int):
+    """The routes' results, to be summed with their weights by the residual step."""
+    e, f = ly["spec"].mlp, ly["down"]
+    y = self._buf("routes", f.N, rows=self.M * e.top)
+    self.experts_linear(f, act, False, 1, M * e.top, L.TNX_EPI_STORE, y, f.N)
+    return ops.rows_src(y=y, ld=f.N)
+
+  def _mlp(self, ly, h, M: int):
+    """The feed-forward of h, as `residual_norm` takes it."""
+    e = ly["spec"].mlp
+    if isinstance(e, ExpertsMlp):
+      self.route(ly, h, M)
+      return ("routes", self.experts_down(ly, self.experts_gate_up(ly, h, M), M), ly["post2"], self.topk_w, e.top)
+    return ("add", self.linear(ly["down"], self.gate_up(ly, h, M), M), ly["post2"])
 
   def gate_up(self, ly, h, M: int) -> torch.Tensor:
     f = ly["gu"]
     act = self._buf("act", ly["down"].Kp)
     if self.dtype == torch.float32:
       self.linear(f, h, M)
-      ops.gelu_mul(self.y[:M * f.N].view(M, f.N), f.offsets[1], M, ly["spec"].mlp.ff, act)
+      ops.gelu_mul(self.y[0][:M * f.N].view(M, f.N), f.offsets[1], M, ly["spec"].mlp.ff, act)
     else:
       d = L.DenseDesc()
       d.M, d.K, d.N, d.dtype = M, f.Kp, f.N, self.code
@@ -403,11 +690,11 @@ class StackRunner(HeadRunner):
     cat = None if m.loop_in is None else self._buf("cat", m.loop_in.Kp)
     ops.embed_rows(m.embed, tokens, col_ptr, B, T, cfg.vocab_size, D, self.x, cat=cat, cat_off=D, cat_frag=self.frag)
     h = self._buf("h", m.Dp)
-    pending, behind_layer = None, False
+    pending, behind_layer = None if m.embed_norm is None else ("norm", None, m.embed_norm), False
 
-    def norm(w_next, out, frag):
+    def norm(w_next, out, frag, shift=None):
       nonlocal behind_layer
-      self.residual_norm(pending, w_next, out, M, frag)
+      self.residual_norm(pending, w_next, out, M, frag, shift)
       if behind_layer and self.residual_sink is not None:
         self.residual_sink(self.x[:M])
       behind_layer = False
@@ -417,11 +704,15 @@ class StackRunner(HeadRunner):
       if begins:   # a pass of the loop: x <- W [x; embedding output]
         norm(None, cat, self.frag)
         pending = ("set", self.linear(m.loop_in, cat, M, fp32_out=True), None)
-      norm(ly["norm1"], h, self.frag)
-      pending = ("add", self._mixer(ly, h, entry, col_ptr, starts, B, T), ly["norm1b"])
+      if cfg.token_shift:
+        norm(None, h, self.frag, (ly["shift"], entry["shift"].r, col_ptr, starts, B, T))
+        entry = entry["mixer"]
+      else:
+        norm(ly["norm1"], h, self.frag)
+      pending = ("add", self._mixer(ly, h, entry, col_ptr, starts, B, T), ly["post1"])
       if "gu" in ly:
         norm(ly["norm2"], h, self.frag)
-        pending = ("add", self.linear(ly["down"], self.gate_up(ly, h, M), M), ly["norm2b"])
+        pending = self._mlp(ly, h, M)
       behind_layer = True
     norm(m.final_norm, self.xn, False)
     return self.xn
