@@ -631,6 +631,7 @@ def stack_kernels(model, runner, st, ctx, iters):
     out[name] = roof_row(us, f.nbytes() + M * (f.K + n_out) * 2, 2.0 * M * f.K * f.N)
 
   h = runner._buf("h", model.Dp)
+  h.normal_()
   ly0 = model.layers[attn[0]]
   m = ly0["spec"].mixer
   lin("linear qkv", attn, "in", h)
@@ -791,6 +792,234 @@ def stack_workload(size, iters, steps, kernels=True):
   return result
 
 
+LAPEVIK_SIZES = {   # width: (query heads, experts, experts per token, their width); batch as in STACK_SIZES
+    "2048": (16, 64, 8, 768),
+    "4096": (32, 64, 8, 1536),
+}
+# the like kernel of each: of a Nunezen decoder, or (experts) of a qwen3-family model with int4 experts
+LAPEVIK_LIKE = {
+    "linear ssd in": "linear lightning in", "linear latent in": "linear qkv", "linear ssd out": "linear o", "linear latent out": "linear o",
+    "linear uq": "linear qkv", "linear ukv": "linear qkv", "linear router": "router", "absorb k": "linear o", "absorb v": "linear o",
+    "convolution": "rotation + cache write", "recurrence": "lightning", "gate + norm": "gated norm", "latent norms + cache write": "rotation + cache write",
+    "query rotation": "rotation + cache write", "key / value layout": "rotation + cache write", "latent attention": "attention",
+    "output gate": "gated norm", "choice of experts": "choice of experts", "route sort": "route sort", "experts gate_up": "experts gate_up",
+    "experts down": "experts down", "post-norm + residual": "post-norm + residual + norm", "routes + norm + residual + shift": "post-norm + residual + norm",
+}
+
+
+def lapevik_kernels(model, runner, st, ctx, iters):
+  """Per-kernel times of a Lapevik model's pass: T = runner.T tokens per row, the last of them at context `ctx`."""
+  import torch
+
+  from tunix_amd import ops
+  from tunix_amd.config import LatentMixer
+  B, T, M, D = runner.B, runner.T, runner.M, model.cfg.embed_dim
+  prompt = T > 1
+  col = runner.zero if prompt else torch.tensor([ctx - T], dtype=torch.int32, device=model.device)
+  latent = [i for i, ly in enumerate(model.layers) if isinstance(ly["spec"].mixer, LatentMixer)]
+  ssd = [i for i in range(len(model.layers)) if i not in latent]
+  entry = lambda i: st.cache.entries[i]["mixer"]
+  at = lambda i: (entry(i), col, st.starts, B, T)
+  out = {}
+
+  def timed(name, fns, nbytes, flops=0.0):
+    out[name] = roof_row(in_turn(fns, iters), nbytes, flops)
+
+  def lin(name, idx, key, x, slot=0, **kw):
+    f = model.layers[idx[0]][key]
+    timed(name, [(lambda g=model.layers[i][key]: runner.linear(g, x, M, slot=slot, **kw)) for i in idx],
+          f.nbytes() + M * (f.K + f.N) * 2, 2.0 * M * f.K * f.N)
+
+  h = runner._buf("h", model.Dp)
+  h.normal_()
+  # state-space layers
+  ls, ms = model.layers[ssd[0]], model.layers[ssd[0]]["spec"].mixer
+  lin("linear ssd in", ssd, "in", h)
+  src = runner.linear(ls["in"], h, M)
+  u = None
+  if prompt:
+    timed("convolution", [(lambda i=i: runner.convolve(model.layers[i], src, *at(i))) for i in ssd], M * ms.channels * 4)
+    u = runner.convolve(ls, src, *at(ssd[0]))
+  timed("recurrence", [(lambda i=i: runner.ssd(model.layers[i], src, u, *at(i))) for i in ssd],
+        M * (ms.channels * 2 + ms.inner * 4) + B * ms.heads * ms.state * ms.vdim * 8 + (0 if prompt else B * ms.channels * 2 * ms.conv),
+        2.0 * M * ms.heads * (2 * ms.state * ms.vdim + (32 * (ms.state + ms.vdim) if prompt else 0)))
+  o = runner.ssd(ls, src, u, *at(ssd[0]))
+  timed("gate + norm", [lambda: runner.ssd_gate(ls, o, src, M)], M * ms.inner * 8)
+  lin("linear ssd out", ssd, "out", runner.ssd_gate(ls, o, src, M))
+  # latent attention
+  la, m = model.layers[latent[0]], model.layers[latent[0]]["spec"].mixer
+  lin("linear latent in", latent, "in", h)
+  src = runner.linear(la["in"], h, M)
+  timed("latent norms + cache write", [(lambda i=i: runner.latent_prep(model.layers[i], src, *at(i), expand=prompt)) for i in latent],
+        M * (m.q_rank + (2 if prompt else 1) * m.kv_rank + m.rot_dim) * 2 * 2)
+  cq, ckv = runner.latent_prep(la, src, *at(latent[0]), expand=prompt)
+  lin("linear uq", latent, "uq", cq, slot=1)
+  qs = runner.linear(la["uq"], cq, M, slot=1)
+  H, dk, row = m.heads, m.dim + m.rot_dim, entry(latent[0]).c.shape[2]
+  pairs = T * ctx - T * (T - 1) / 2
+  if prompt:
+    dkp = ops.sink_attn_pad(dk, False, runner.dtype)
+    q = runner._buf("q", H * dkp, rows=M)
+    timed("query rotation", [lambda: runner.latent_q(la, qs, col, st.starts, B, T, q, dkp, m.dim, q, m.dim, dkp, dkp - m.dim)], M * H * dk * 4)
+    lin("linear ukv", latent, "ukv", ckv, slot=1)
+    y, y_head = runner.latent_prompt(la, cq, ckv, *at(latent[0]))
+    k, v = runner._buf("k_full", dkp, rows=M * H), runner._buf("v_full", ops.sink_attn_pad(m.vdim, True, runner.dtype), rows=M * H)
+    kv = runner.linear(la["ukv"], ckv, M, slot=1)
+    timed("key / value layout", [lambda: runner.latent_kv(la, kv, k, v, entry(latent[0]), B, T)], M * H * (m.dim + m.vdim + dk + m.vdim) * 2)
+    timed("latent attention", [lambda: runner.plain_attention(m, q, k, v, dk, m.vdim, st.starts, col, B, T, T, H, y, m.vdim)],
+          M * H * (2 * dk + 2 * m.vdim) * 2, 2.0 * B * H * pairs * (dk + m.vdim))
+  else:
+    fk, fv = la["absorb_k"], la["absorb_v"]
+    un, q, lat = runner._buf("q_un", H * fk.Kp, rows=M), runner._buf("q", H * row, rows=M), runner._buf("latent_out", H * fv.Kp, rows=M)
+    timed("query rotation", [lambda: runner.latent_q(la, qs, col, st.starts, B, T, un, fk.Kp, fk.Kp, q, fk.N, row, row - fk.N)], M * H * dk * 4)
+    timed("absorb k", [(lambda f=model.layers[i]["absorb_k"]: runner.bank(f, un, H * fk.Kp, fk.Kp, q, H * row, row, M)) for i in latent],
+          fk.nbytes() + M * H * (fk.K + fk.N) * 2, 2.0 * M * H * fk.K * fk.N)
+    timed("latent attention", [(lambda i=i: runner.latent_attend(model.layers[i], q, lat, fv.Kp, *at(i))) for i in latent],
+          B * ctx * (m.kv_rank + m.rot_dim) * 2 + M * H * (2 * m.kv_rank + m.rot_dim) * 2, 2.0 * B * H * pairs * (2 * m.kv_rank + m.rot_dim))
+    y, y_head = runner._buf("heads", H * fv.N, rows=M), fv.N
+    timed("absorb v", [(lambda f=model.layers[i]["absorb_v"]: runner.bank(f, lat, H * fv.Kp, fv.Kp, y, H * fv.N, fv.N, M)) for i in latent],
+          fv.nbytes() + M * H * (fv.K + fv.N) * 2, 2.0 * M * H * fv.K * fv.N)
+  timed("output gate", [lambda: runner.gate_mul(la, y, m.vdim, y_head, src, M)], M * H * m.vdim * 6)
+  lin("linear latent out", latent, "out", runner.gate_mul(la, y, m.vdim, y_head, src, M))
+  osrc = runner.linear(la["out"], runner._buf("gated", la["out"].Kp), M)
+  timed("post-norm + residual", [lambda: runner.residual_norm(("add", osrc, la["post1"]), None, h, M, runner.frag)], M * D * (2 + 8 + 2))
+  # experts
+  h.normal_()
+  e = la["spec"].mlp
+  both = range(len(model.layers))
+  lin("linear router", both, "router", h, fp32_out=True)
+  z = runner.linear(la["router"], h, M, fp32_out=True)
+  if z.split_k <= 1:
+    z.y = z.ws
+  ids = runner.topk_id[:M * e.top].view(M, e.top)
+  timed("choice of experts", [lambda: ops.route_softmax(z, M, e.experts, e.top, runner.topk_w, ids)], M * (e.experts + 2 * e.top) * 4)
+  timed("route sort", [lambda: ops.moe_sort_routes(ids, e.experts, runner.counts, runner.offsets, runner.sorted_route)], M * e.top * 8)
+  live = int((runner.counts[:e.experts] > 0).sum())
+  act = runner.experts_gate_up(la, h, M)
+  timed("experts gate_up", [(lambda ly=model.layers[i]: runner.experts_gate_up(ly, h, M)) for i in both],
+        la["gu"].nbytes() * live / e.experts + M * (D + e.top * e.ff) * 2, 4.0 * M * e.top * D * e.ff)
+  timed("experts down", [(lambda ly=model.layers[i]: runner.experts_down(ly, act, M)) for i in both],
+        la["down"].nbytes() * live / e.experts + M * e.top * (D + e.ff) * 2, 2.0 * M * e.top * D * e.ff)
+  routes = runner.experts_down(la, act, M)
+  shift = (ls["shift"], st.cache.entries[ssd[0]]["shift"].r, col, st.starts, B, T)
+  timed("routes + norm + residual + shift",
+        [lambda: runner.residual_norm(("routes", routes, la["post2"], runner.topk_w, e.top), None, h, M, runner.frag, shift)],
+        M * D * (2 * e.top + 8 + 2) + (0 if prompt else B * D * 8))
+  return out
+
+
+def expert_family_kernels(cfg, M, iters, dev):
+  """Router, choice, sort and grouped products of a qwen3-family model with int4 experts."""
+  import torch
+
+  from tunix_amd import _lib as L
+  from tunix_amd import dummy_model, ops
+  from tunix_amd.model import QLoRAModel
+  model = QLoRAModel(cfg, dummy_model.create_dummy_weights(cfg, 1, dev), dev)
+  k, E, D, F = cfg.num_experts_per_tok, cfg.num_experts, cfg.embed_dim, cfg.hidden_dim
+  bf, i32 = dict(dtype=torch.bfloat16, device=dev), dict(dtype=torch.int32, device=dev)
+  x, scores = torch.randn(M, D, **bf), torch.empty(M, E, **bf)
+  tw, ids = torch.empty(M, k, **bf), torch.empty(M, k, **i32)
+  counts, offsets, order = torch.empty(E, **i32), torch.empty(E + 1, **i32), torch.empty(M * k, **i32)
+  act, y = torch.zeros(M * k, F, **bf), torch.empty(M * k, D, **bf)
+  banks = [ly["experts"] for ly in model.layers]
+  out = {}
+
+  def timed(name, fns, nbytes, flops=0.0):
+    out[name] = roof_row(in_turn(fns, iters), nbytes, flops)
+
+  def gmm(ex, up):
+    d = L.MoeGmmDesc()
+    d.n_routes, d.E, d.k, d.group, d.qtype = M * k, E, k, cfg.group, cfg.qtype
+    d.offsets, d.sorted_route = offsets.data_ptr(), order.data_ptr()
+    if up:
+      d.K, d.N, d.x, d.x_div, d.codes, d.scales = D, 2 * F, x.data_ptr(), k, ex.gu_codes.data_ptr(), ex.gu_scales.data_ptr()
+      d.epilogue, d.y = L.TNX_EPI_SILU_MUL, act.data_ptr()
+    else:
+      d.K, d.N, d.x, d.x_div, d.codes, d.scales = F, D, act.data_ptr(), 1, ex.dn_codes.data_ptr(), ex.dn_scales.data_ptr()
+      d.epilogue, d.y = L.TNX_EPI_STORE, y.data_ptr()
+    ops.moe_gmm(d)
+
+  timed("router", [(lambda ex=ex: ops.lora_down(x, ex.router_t, scores, M=M)) for ex in banks], E * D * 2 + M * (D + E) * 2, 2.0 * M * D * E)
+  timed("choice of experts", [lambda: ops.moe_route_topk(scores, k, tw, ids)], M * (E * 2 + k * 6))
+  timed("route sort", [lambda: ops.moe_sort_routes(ids, E, counts, offsets, order)], M * k * 8)
+  share = int((counts > 0).sum()) / E
+  ex = banks[0]
+  nb = lambda c, s: (c.numel() * c.element_size() + s.numel() * s.element_size()) * share
+  timed("experts gate_up", [(lambda ex=ex: gmm(ex, True)) for ex in banks], nb(ex.gu_codes, ex.gu_scales) + M * (D + k * F) * 2, 4.0 * M * k * D * F)
+  timed("experts down", [(lambda ex=ex: gmm(ex, False)) for ex in banks], nb(ex.dn_codes, ex.dn_scales) + M * k * (D + F) * 2, 2.0 * M * k * D * F)
+  return out
+
+
+def lapevik_workload(size, iters, steps, kernels=True):
+  """Prefill and decode of a Lapevik decoder with layers of a real model's size (random weights), beside a Nunezen
+  decoder of the same width and a qwen3-family model with the same experts (int4), and the time of every kernel
+  against its roof and against the like kernel's."""
+  import numpy as np
+  import torch
+
+  from tunix_amd import config, dummy_model
+  from tunix_amd.generate import CacheConfig, Sampler
+  from tunix_amd.generate.sampler import _SamplingState
+  from tunix_amd.generate.utils import IdTokenizer
+  from tunix_amd.model import QLoRAModel
+  from tunix_amd.stack_model import StackModel
+  dev = torch.device("cuda:0")
+  width, nH, nG, nff, B = STACK_SIZES[size]
+  H, E, top, ff = LAPEVIK_SIZES[size]
+  new_cfg = config.lapevik_shape(width, H, E, top, ff)
+  near_cfg = config.nunezen_shape(width, nH, nG, nff)
+  moe_cfg = config.qwen3_30b_a3b(num_layers=len(new_cfg.layers), vocab_size=new_cfg.vocab_size, embed_dim=width, hidden_dim=ff, num_heads=nH,
+                                 num_kv_heads=nG, num_experts=E, num_experts_per_tok=top, lora_rank=0, lora_alpha=0.0)
+  P, T = 1024, 256
+  S = P + T
+  ids = np.random.Generator(np.random.PCG64(5)).integers(1, new_cfg.vocab_size, size=(B, P)).astype(np.int32)
+  result = {"size": {"width": width, "ssd_heads": new_cfg.layers[0].mixer.heads, "latent_heads": H, "experts": E, "top": top,
+                     "expert_width": ff, "batch": B, "prompt": P, "layers": len(new_cfg.layers)}}
+  models = (("lapevik", lambda: StackModel(new_cfg, dummy_model.create_stack_weights(new_cfg, 1, dev), dev), lapevik_kernels),
+            ("nunezen", lambda: StackModel(near_cfg, dummy_model.create_stack_weights(near_cfg, 1, dev), dev), stack_kernels),
+            ("qwen3-family", lambda: QLoRAModel(moe_cfg, dummy_model.create_dummy_weights(moe_cfg, 1, dev), dev), None))
+  pb = 8      # rows of a prefill group: 8 x 1024 tokens
+  for name, build, measure in models:
+    model = build()
+    sampler = Sampler(model, IdTokenizer(new_cfg.vocab_size, pad_id=0, eos_id=1), CacheConfig(S))
+    prompts, ms, pre = [r for r in ids], [], []
+    for n in (4, 4, 4 + steps):
+      sampler(prompts, n, max_prompt_length=P, eos_tokens=[-1])
+      ms.append(sampler.last_stats["decode_ms"])
+      pre.append(sampler.last_stats["prefill_ms"])
+    d_ms = (ms[2] - ms[1]) / steps
+    r = {"prefill_tokens_per_s": round(B * P / (min(pre[1:]) * 1e-3)), "prefill_ms": round(min(pre[1:]), 2),
+         "decode_tokens_per_s": round(B / (d_ms * 1e-3)), "decode_ms_per_step": round(d_ms, 4)}
+    log(size, name, r)
+    if kernels and measure is not None:
+      st = _SamplingState(model, ids, S, S, 0, False, False)
+      st.starts.zero_()
+      r["decode_kernels"] = measure(model, model.new_runner(B, 1, S, 0), st, P + T // 2, iters)
+      del st
+      torch.cuda.empty_cache()
+      stp = _SamplingState(model, ids[:pb], S, S, 0, False, False)
+      stp.starts.zero_()
+      r["prefill_kernels"] = measure(model, model.new_runner(pb, P, S, 0, kv_chunk=0), stp, P, max(2, iters // 4))
+      del stp
+    result[name] = r
+    del model, sampler
+    torch.cuda.empty_cache()
+    if kernels and measure is None:
+      r["decode_kernels"] = expert_family_kernels(moe_cfg, B, iters, dev)
+      r["prefill_kernels"] = expert_family_kernels(moe_cfg, pb * P, max(2, iters // 4), dev)
+      torch.cuda.empty_cache()
+  if kernels:
+    for phase in ("decode_kernels", "prefill_kernels"):
+      like = {**result["nunezen"][phase], **result["qwen3-family"][phase]}
+      for k, v in result["lapevik"][phase].items():
+        b = like[LAPEVIK_LIKE[k]]
+        v["vs_like"] = round(v["times_roof"] / b["times_roof"], 2)
+        log(f"  {size} {phase:16s} {k:34s} {v['us']:9.1f} us  {v['times_roof']:6.2f} x roof ({v['bound']})   {LAPEVIK_LIKE[k]}: "
+            f"{b['us']:9.1f} us  {b['times_roof']:6.2f} x ({b['bound']})   ratio {v['vs_like']}")
+  return result
+
+
 def main():
   ap = argparse.ArgumentParser()
   ap.add_argument("--gpus", type=int, default=1)
@@ -820,6 +1049,7 @@ def main():
                   help="instead of the decode benchmark: a Nunezen decoder with layers of a real model's size (model "
                        "width 2048 or 4096), prefill, decode and every kernel against its roof, beside a gemma3-family "
                        "model of the same size; its own JSON line")
+  ap.add_argument("--stack-design", choices=["nunezen", "lapevik"], default="nunezen", help="with --stack: the layer-list design to measure")
   ap.add_argument("--stack-no-kernels", action="store_true", help="with --stack: throughput only")
   ap.add_argument("--config", choices=["c1", "c2", "c3", "c4"], default="c3",
                   help="c3 (default): the headline workload; c1 / c2 / c4: the other rollout workloads through "
@@ -866,7 +1096,7 @@ def main():
     sizes = sorted(STACK_SIZES) if args.stack == "all" else [args.stack]
     print(json.dumps({"metric": "Nunezen prefill and decode tokens/sec @1 MI355X", "unit": "tokens/s", "n_gpus": 1,
                       "dtype": "bf16", "data": "synthetic",
-                      "sizes": {z: stack_workload(z, args.kernel_iters, 64, not args.stack_no_kernels) for z in sizes}}),
+                      "sizes": {z: (lapevik_workload if args.stack_design == "lapevik" else stack_workload)(z, args.kernel_iters, 64, not args.stack_no_kernels) for z in sizes}}),
           flush=True)
     return
 

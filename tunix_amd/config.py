@@ -421,3 +421,13 @@ def nunezen_shape(width: int, heads: int, kv_heads: int, ff: int, vocab: int = 3
   return StackConfig(family="nunezen", vocab_size=vocab, embed_dim=width, norm_eps=1e-6,
                      layers=tuple(attn if i % 2 == 0 else light for i in range(layers)),
                      loop=LayerLoop(1, layers - 1, 2) if layers > 2 else None)
+
+
+def lapevik_shape(width: int, heads: int, experts: int, top: int, ff: int, vocab: int = 32768, layers: int = 4) -> StackConfig:
+  """A Lapevik decoder with layers of a real model's size: state-space and latent-attention layers in turn, each
+  with routed experts."""
+  moe = ExpertsMlp(ff, experts, top)
+  ssd = LayerSpec(SsdMixer(heads=width // 32, vdim=64, state=128, groups=8, conv=4, norm_groups=8), moe)
+  attn = LayerSpec(LatentMixer(heads, 128, 64, 128, q_rank=3 * width // 8, kv_rank=512, rot_base=500_000.0, scale=192 ** -0.5), moe)
+  return StackConfig(family="lapevik", vocab_size=vocab, embed_dim=width, norm_eps=1e-5, norm_offset=0.0, norm_groups=8, pre_norm=False,
+                     embed_norm=True, token_shift=True, layers=tuple(ssd if i % 2 == 0 else attn for i in range(layers)))

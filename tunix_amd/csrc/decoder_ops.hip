@@ -656,8 +656,11 @@ int launch_act_mul(hipStream_t st, int dtype, const void* y, int64_t ld, int64_t
 // ---- choice of experts: the k largest logits (first among equals), softmax over them ---------------
 // One wave per token.  NaN logits rank below every number, so that k distinct experts are found whatever
 // the logits hold; they leave as NaN weights.
+// Up to 256 experts: every expert counts the ones ahead of it, which is its place among the chosen; more: one
+// pass over the logits per choice.
+constexpr int kRankExperts = 256;
 __global__ __launch_bounds__(64) void route_softmax_kernel(const RowSrc<float> src, int E, int k, float* topk_w, int32_t* topk_id) {
-  extern __shared__ float z[];   // logits [E], chosen logits [k]
+  extern __shared__ __align__(16) float z[];   // logits [E], chosen logits [k]
   float* sel = z + E;
   const int64_t m = blockIdx.x;
   const int lane = threadIdx.x;
@@ -670,7 +673,25 @@ __global__ __launch_bounds__(64) void route_softmax_kernel(const RowSrc<float> s
   }
   bad = __any(bad);
   __syncthreads();
-  for (int j = 0; j < k; ++j) {
+  if (E <= kRankExperts) {   // (uniform)
+    for (int e = lane; e < E; e += 64) {
+      const float v = z[e];
+      int ahead = 0;
+      int o = 0;
+      for (; o + 4 <= E; o += 4) {
+        const f32x4 w = *reinterpret_cast<const f32x4*>(z + o);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) ahead += w[i] > v || (w[i] == v && o + i < e);
+      }
+      for (; o < E; ++o) ahead += z[o] > v || (z[o] == v && o < e);
+      if (ahead < k) {
+        sel[ahead] = v;
+        topk_id[m * k + ahead] = e;
+      }
+    }
+    __syncthreads();
+  }
+  for (int j = 0; j < k && E > kRankExperts; ++j) {
     float best = ninf;
     int bi = 0x7fffffff;
     for (int e = lane; e < E; e += 64)

@@ -349,12 +349,14 @@ extern "C" int tnx_dense_linear(void* stream, const tnx_dense_desc* d) {
     TNX_CHECK_LAUNCH("dense_rows");
     return TNX_OK;
   }
-  // many rows: the 128 x 256 kernel (row-major operands, 32-bit offsets)
-  if (!batch && !d->x_frag && !d->y_frag && split == 1 && d->M > 64 && d->ldx == d->K && d->N % 16 == 0 &&
+  // many rows: the 128 x 256 kernel (row-major operands, 32-bit offsets); a few columns would leave its tiles
+  // and the device mostly empty: 32 rows per work-group then
+  const bool narrow = d->N <= 64 && !mul && d->M > 64 && d->M <= 32 * 65535;
+  if (!batch && !narrow && !d->x_frag && !d->y_frag && split == 1 && d->M > 64 && d->ldx == d->K && d->N % 16 == 0 &&
       offsets32)
     return tnx_internal_wide_dense(st, d->M, d->K, d->N, (const uint16_t*)d->x, (const uint16_t*)d->w, d->epilogue, d->y,
                                    d->ldy);
-  const int rt = d->M <= 32 ? 1 : d->M <= 64 ? 2 : 4;
+  const int rt = d->M <= 32 || narrow ? 1 : d->M <= 64 ? 2 : 4;
   TNX_REQUIRE(cdiv(d->M, 32 * rt) <= 65535 && split <= 65535, "dense_linear: too many rows or splits in one call");
   const dim3 grid((unsigned)cdiv(d->N, 64), (unsigned)cdiv(d->M, 32 * rt), batch ? (unsigned)d->batch : (unsigned)split);
   if (batch) launch_rows<kBatch>(st, a, rt, grid);

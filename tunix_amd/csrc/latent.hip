@@ -83,6 +83,76 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a
   }
 }
 
+// Latents, offsets and rows in whole runs of eight: a thread keeps its runs in registers.
+template <int MAXI, typename T>
+__global__ __launch_bounds__(256) void latent_prep_vec_kernel(const LatentPrepArgs a, const RowSrc<T> src, T* q_out, T* c_out, T* cache) {
+  __shared__ float red[2][4];
+  const int64_t row = blockIdx.x, b = row / a.T, t = row % a.T;
+  const int slot = *a.col_ptr + (int)t, tid = threadIdx.x;
+  if (slot >= a.S) return;                                    // (uniform)
+  const int nq = a.q_rank / 8, nkv = a.rank / 8, nr = a.rot / 8, n = nq + nkv + nr;
+  float f[MAXI][8], w[MAXI][8];
+  const RowSrc<float> wq{a.w_q, nullptr, 1, 0, 0}, wkv{a.w_kv, nullptr, 1, 0, 0};
+#pragma unroll
+  for (int c = 0; c < MAXI; ++c) {
+    const int i = min(c * 256 + tid, n - 1);
+    get8(src, row, i < nq ? a.q_off + i * 8 : a.kv_off + (i - nq) * 8, f[c]);
+    if (i < nq) get8(wq, 0, i * 8, w[c]);
+    else if (i < nq + nkv) get8(wkv, 0, (i - nq) * 8, w[c]);
+  }
+  const float pos = (float)max(slot - a.starts[b], 0);
+  float sq = 0.f, skv = 0.f;
+#pragma unroll
+  for (int c = 0; c < MAXI; ++c) {
+    const int i = c * 256 + tid;
+    float s = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) s += f[c][j] * f[c][j];
+    if (i < nq) sq += s;
+    else if (i < nq + nkv) skv += s;
+  }
+  sq = wave_sum(sq);
+  skv = wave_sum(skv);
+  if ((tid & 63) == 0) {
+    red[0][tid >> 6] = sq;
+    red[1][tid >> 6] = skv;
+  }
+  __syncthreads();
+  const float rq = 1.0f / sqrtf((red[0][0] + red[0][1] + red[0][2] + red[0][3]) / (float)a.q_rank + a.eps);
+  const float rkv = 1.0f / sqrtf((red[1][0] + red[1][1] + red[1][2] + red[1][3]) / (float)a.rank + a.eps);
+  T* dst = cache + (b * a.S + slot) * a.row;
+#pragma unroll
+  for (int c = 0; c < MAXI; ++c) {
+    const int i = c * 256 + tid;
+    if (i >= n) continue;
+    if (i < nq + nkv) {
+      const float r = i < nq ? rq : rkv;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) f[c][j] = f[c][j] * r * w[c][j];
+      if (i < nq) {
+        put8(q_out + (a.q_frag ? frag_index(row, i * 8, a.q_ld) : row * a.q_ld + i * 8), f[c]);
+      } else {
+        const int d = (i - nq) * 8;
+        put8(dst + d, f[c]);
+        if (c_out) put8(c_out + (a.c_frag ? frag_index(row, d, a.c_ld) : row * a.c_ld + d), f[c]);
+      }
+      continue;
+    }
+    const int j0 = (i - nq - nkv) * 8;
+    float o[8];
+#pragma unroll
+    for (int p = 0; p < 4; ++p) {
+      float sn, cs;
+      sincosf(pos * a.inv_freq[j0 / 2 + p], &sn, &cs);
+      o[2 * p] = f[c][2 * p] * cs - f[c][2 * p + 1] * sn;
+      o[2 * p + 1] = f[c][2 * p + 1] * cs + f[c][2 * p] * sn;
+    }
+    put8(dst + a.rank_pad + j0, o);
+  }
+  for (int i = a.rank + tid; i < a.row; i += 256)
+    if (i < a.rank_pad || i >= a.rank_pad + a.rot) st_elem(dst, i, 0.f);
+}
+
 // ---- queries: the unrotated part of every head to one place, the rotated part to another ----------
 struct LatentQArgs {
   int64_t T;
@@ -457,8 +527,15 @@ unsigned spread(int64_t rows, int64_t items) {
 template <typename T>
 int prep_launch(hipStream_t st, const tnx_latent_prep_desc* d, const LatentPrepArgs& a) {
   const size_t lds = (size_t)(d->q_rank + d->rank + d->rot) * 4;
-  hipLaunchKernelGGL(latent_prep_kernel<T>, dim3((unsigned)(d->B * d->T)), dim3(256), lds, st, a, row_src<T>(d->y), (T*)d->q_out, (T*)d->c_out,
-                     (T*)d->cache);
+  const int items = (d->q_rank + d->rank + d->rot) / 8;
+  const bool vec = (d->q_rank | d->rank | d->rot | d->row) % 8 == 0 && d->q_off % 8 == 0 && d->kv_off % 8 == 0 && d->y.ld % 8 == 0 &&
+                   d->y.plane % 8 == 0 && d->q_ld % 8 == 0 && d->c_ld % 8 == 0 && items <= 1024;
+  const dim3 grid((unsigned)(d->B * d->T));
+  T *q_out = (T*)d->q_out, *c_out = (T*)d->c_out, *cache = (T*)d->cache;
+  if (vec && items <= 256) hipLaunchKernelGGL((latent_prep_vec_kernel<1, T>), grid, dim3(256), 0, st, a, row_src<T>(d->y), q_out, c_out, cache);
+  else if (vec && items <= 512) hipLaunchKernelGGL((latent_prep_vec_kernel<2, T>), grid, dim3(256), 0, st, a, row_src<T>(d->y), q_out, c_out, cache);
+  else if (vec) hipLaunchKernelGGL((latent_prep_vec_kernel<4, T>), grid, dim3(256), 0, st, a, row_src<T>(d->y), q_out, c_out, cache);
+  else hipLaunchKernelGGL(latent_prep_kernel<T>, grid, dim3(256), lds, st, a, row_src<T>(d->y), q_out, c_out, cache);
   TNX_CHECK_LAUNCH("latent_prep");
   return TNX_OK;
 }

@@ -547,7 +547,7 @@ class StackRunner(HeadRunner):
     ops.gate_mul(d)
     return out
 
-  def _sink_free_attention(self, m, q, k, v, dk, dv, starts, col_ptr, B, T, S, G, out, out_head):
+  def plain_attention(self, m, q, k, v, dk, dv, starts, col_ptr, B, T, S, G, out, out_head):
     """softmax(scale q k) v over plain keys and values (one kv head per query head, or one for all)."""
     d = L.SinkAttnDesc()
     d.B, d.T, d.S, d.H, d.G = B, T, S, m.heads, G
@@ -556,21 +556,25 @@ class StackRunner(HeadRunner):
     d.ws, d.out, d.out_ld, d.out_head = self.attn_ws.data_ptr(), out.data_ptr(), m.heads * out_head, out_head
     ops.sink_attn(d)
 
+  def latent_kv(self, ly, src, k, v, entry, B, T):
+    """Lays the projected keys and values of a prompt out as plain attention reads them."""
+    m, c = ly["spec"].mixer, entry.c
+    d = L.LatentKvDesc()
+    d.B, d.T, d.S, d.H, d.n, d.r, d.vd = B, T, c.shape[1], m.heads, m.dim, m.rot_dim, m.vdim
+    d.dkp, d.dvp, d.rank_pad, d.row, d.dtype = k.shape[1], v.shape[1], _up(m.kv_rank, 16), c.shape[2], self.code
+    d.y, d.v_off, d.cache, d.k, d.v = src, ly["ukv"].offsets[1], c.data_ptr(), k.data_ptr(), v.data_ptr()
+    ops.latent_kv(d)
+
   def latent_prompt(self, ly, cq, ckv, entry, col_ptr, starts, B, T):
     """A prompt from its first column on: keys and values of all heads are formed for its tokens."""
-    m, M, c = ly["spec"].mixer, B * T, entry.c
+    m, M = ly["spec"].mixer, B * T
     dkp, dvp = ops.sink_attn_pad(m.dim + m.rot_dim, False, self.dtype), ops.sink_attn_pad(m.vdim, True, self.dtype)
     q = self._buf("q", m.heads * dkp, rows=self.M)
     self.latent_q(ly, self.linear(ly["uq"], cq, M, slot=1), col_ptr, starts, B, T, q, dkp, m.dim, q, m.dim, dkp, dkp - m.dim)
     k, v = self._buf("k_full", dkp, rows=self.M * m.heads), self._buf("v_full", dvp, rows=self.M * m.heads)
-    d = L.LatentKvDesc()
-    d.B, d.T, d.S, d.H, d.n, d.r, d.vd = B, T, c.shape[1], m.heads, m.dim, m.rot_dim, m.vdim
-    d.dkp, d.dvp, d.rank_pad, d.row, d.dtype = dkp, dvp, _up(m.kv_rank, 16), c.shape[2], self.code
-    d.y, d.v_off, d.cache = self.linear(ly["ukv"], ckv, M, slot=1), ly["ukv"].offsets[1], c.data_ptr()
-    d.k, d.v = k.data_ptr(), v.data_ptr()
-    ops.latent_kv(d)
+    self.latent_kv(ly, self.linear(ly["ukv"], ckv, M, slot=1), k, v, entry, B, T)
     out = self._buf("heads", m.heads * m.vdim, rows=self.M)
-    self._sink_free_attention(m, q, k, v, m.dim + m.rot_dim, m.vdim, starts, col_ptr, B, T, T, m.heads, out, m.vdim)
+    self.plain_attention(m, q, k, v, m.dim + m.rot_dim, m.vdim, starts, col_ptr, B, T, T, m.heads, out, m.vdim)
     return out, m.vdim
 
   def latent_rows(self, ly, cq, entry, col_ptr, starts, B, T):
@@ -590,7 +594,7 @@ class StackRunner(HeadRunner):
     m, c = ly["spec"].mixer, entry.c
     S, row = c.shape[1], c.shape[2]
     if self.dtype != torch.bfloat16 or not ops.latent_attn_ok(m.kv_rank, row, S):
-      self._sink_free_attention(m, q, c, c, _up(m.kv_rank, 16) + m.rot_dim, m.kv_rank, starts, col_ptr, B, T, S, 1, out, out_head)
+      self.plain_attention(m, q, c, c, _up(m.kv_rank, 16) + m.rot_dim, m.kv_rank, starts, col_ptr, B, T, S, 1, out, out_head)
       return
     d = L.LatentAttnDesc()
     d.B, d.T, d.S, d.H, d.rank, d.row, d.scale = B, T, S, m.heads, m.kv_rank, row, m.scale
