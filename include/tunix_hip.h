@@ -847,7 +847,7 @@ typedef struct {
 } tnx_latent_kv_desc;
 int tnx_latent_kv(void* stream, const tnx_latent_kv_desc* d);
 /* bf16: q [B * T, H, row] against the cache rows of columns starts[b] .. col + t, softmax(scale * q . row), out[row, head]
- * [out_head] = the weighted sum of the rows' first `rank` elements.  kv_chunk > 0 (a multiple of 128) splits the key
+ * [out_head] = the weighted sum of the rows' first `rank` elements.  kv_chunk > 0 (a multiple of 64) splits the key
  * range (workspace of tnx_latent_attn_ws_bytes).  Rows of other lengths, and fp32: tnx_sink_attn with one kv head whose
  * keys and values are the cache rows. */
 typedef struct {

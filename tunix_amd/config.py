@@ -330,7 +330,7 @@ def lapevik_from_dict(d: dict) -> StackConfig:
       mixer = SsdMixer(heads=int(m["heads"]), vdim=int(m["vdim"]), state=int(m["state"]), groups=int(m["groups"]),
                        conv=int(m["conv"]), norm_groups=int(m["norm_groups"]))
     elif ly["type"] == "latent_attention":
-      rot = m["rot"]
+      rot = m["rot"] if int(m["rot_dim"]) else {"dims": 0, "base": 1.0}
       if int(rot["dims"]) != int(m["rot_dim"]):
         raise ValueError(f"layer {i}: rotation over {rot['dims']} of {m['rot_dim']} dimensions")
       mixer = LatentMixer(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),

@@ -4,6 +4,8 @@
 // matrix operands leave in the model's dtype (bf16 or fp32).
 #include <string.h>
 
+#include <type_traits>
+
 #include "decoder.h"
 #include "rng.h"
 
@@ -202,9 +204,9 @@ __device__ __forceinline__ void part_scales(const float* part, float* gs, int gr
 // The general residual step: norms over equal parts of a row, weighted sums of routed rows, token shift.
 // A work-group walks `run` tokens of one sequence; with a shift it forms the token before its first one
 // as well (x and x_out are then different buffers, unless the call brings one token per sequence).
-template <int MAXC, typename T>
-__global__ __launch_bounds__(256) void resnorm_rows_kernel(const ResNormArgs a) {
-  __shared__ float red[4], part[MAXC * 256], gs[MAXC * 256];
+template <int NT, int MAXC, bool ROUTES, typename T>   // NT threads, MAXC runs of eight per thread
+__global__ __launch_bounds__(NT) void resnorm_rows_kernel(const ResNormArgs a) {
+  __shared__ float red[NT / 64], part[MAXC * NT], gs[MAXC * NT];
   const int64_t runs = (a.T + a.run - 1) / a.run, b = blockIdx.x / runs, t0 = blockIdx.x % runs * a.run;
   const int64_t t1 = min(a.T, t0 + a.run);
   const int nch = (int)(a.D / 8), per = nch / a.groups, tid = threadIdx.x;
@@ -220,7 +222,7 @@ __global__ __launch_bounds__(256) void resnorm_rows_kernel(const ResNormArgs a) 
     }
   };
   const float* wnext = a.shift ? a.shift : a.w_next;
-  auto column = [&](int c) { return (int64_t)min(c * 256 + tid, nch - 1) * 8; };
+  auto column = [&](int c) { return (int64_t)min(c * NT + tid, nch - 1) * 8; };
 #pragma unroll
   for (int c = 0; c < MAXC; ++c) {
     if (a.w_post) load8f(a.w_post + column(c), wp[c]);
@@ -234,12 +236,12 @@ __global__ __launch_bounds__(256) void resnorm_rows_kernel(const ResNormArgs a) 
     float ss = 0.f;
 #pragma unroll
     for (int c = 0; c < MAXC; ++c) {
-      if (c * 256 + tid >= nch) continue;
+      if (c * NT + tid >= nch) continue;
       float q = 0.f;
 #pragma unroll
       for (int j = 0; j < 8; ++j) q += v[c][j] * v[c][j];
       ss += q;
-      if (a.groups > 1) part[c * 256 + tid] = q;
+      if (a.groups > 1) part[c * NT + tid] = q;
     }
     if (a.groups == 1) {
       const float s = 1.0f / sqrtf(block_sum(ss, red) / (float)a.D + a.eps);
@@ -249,7 +251,7 @@ __global__ __launch_bounds__(256) void resnorm_rows_kernel(const ResNormArgs a) 
     }
     part_scales(part, gs, a.groups, per, (float)(per * 8), a.eps);
 #pragma unroll
-    for (int c = 0; c < MAXC; ++c) r[c] = gs[min(c * 256 + tid, nch - 1) / per];
+    for (int c = 0; c < MAXC; ++c) r[c] = gs[min(c * NT + tid, nch - 1) / per];
   };
   for (int64_t t = a.shift && t0 > 0 ? t0 - 1 : t0; t < t1; ++t) {
     const int64_t row = b * a.T + t;
@@ -259,13 +261,14 @@ __global__ __launch_bounds__(256) void resnorm_rows_kernel(const ResNormArgs a) 
       const int64_t col = column(c);
       if (a.mode != 2) load8f(a.x + row * a.D + col, xo[c]);
       if (a.mode == 1 || a.mode == 2) {
-        if (a.route_w) {
+        if constexpr (ROUTES) {
 #pragma unroll
           for (int j = 0; j < 8; ++j) h[c][j] = 0.f;
+#pragma unroll 4
           for (int k = 0; k < a.route_k; ++k) {
             const float w = a.route_w[row * a.route_k + k];
             float f[8];
-            get8(src, row * a.route_k + k, col, f);
+            get8(RowSrc<T>{src.y, nullptr, 1, 0, a.y_ld}, row * a.route_k + k, col, f);
 #pragma unroll
             for (int j = 0; j < 8; ++j) h[c][j] += w * f[j];
           }
@@ -294,7 +297,7 @@ __global__ __launch_bounds__(256) void resnorm_rows_kernel(const ResNormArgs a) 
       T* out = reinterpret_cast<T*>(a.out);
 #pragma unroll
       for (int c = 0; c < MAXC; ++c) {
-        if (c * 256 + tid >= nch) continue;
+        if (c * NT + tid >= nch) continue;
         const int64_t col = column(c);
         if (a.mode != 0 || a.x_out != a.x) put8(a.x_out + row * a.D + col, h[c]);
         float o[8];
@@ -315,7 +318,7 @@ __global__ __launch_bounds__(256) void resnorm_rows_kernel(const ResNormArgs a) 
   if (a.shift && a.T == 1)
 #pragma unroll
     for (int c = 0; c < MAXC; ++c)
-      if (c * 256 + tid < nch) put8(a.before + b * a.D + column(c), h[c]);
+      if (c * NT + tid < nch) put8(a.before + b * a.D + column(c), h[c]);
 }
 
 // the same for any D that fits LDS twice: h and the token before, a thread owning the columns tid + 256 i
@@ -386,10 +389,17 @@ int launch_resnorm_rows(hipStream_t st, ResNormArgs a) {
   if (!vec) {
     TNX_REQUIRE(a.D <= 7168 && a.groups <= 1024, "residual_norm: D=%lld in %d parts needs runs of eight", (long long)a.D, a.groups);
     hipLaunchKernelGGL((resnorm_rows_any_kernel<T>), grid, dim3(256), (size_t)a.D * 8, st, a);
-  } else if (a.D <= 2048) hipLaunchKernelGGL((resnorm_rows_kernel<1, T>), grid, dim3(256), 0, st, a);
-  else if (a.D <= 4096) hipLaunchKernelGGL((resnorm_rows_kernel<2, T>), grid, dim3(256), 0, st, a);
-  else if (a.D <= 8192) hipLaunchKernelGGL((resnorm_rows_kernel<4, T>), grid, dim3(256), 0, st, a);
-  else hipLaunchKernelGGL((resnorm_rows_kernel<8, T>), grid, dim3(256), 0, st, a);
+    return TNX_OK;
+  }
+  auto launch = [&](auto routes) {
+    constexpr bool R = decltype(routes)::value;
+    if (a.D <= 2048) hipLaunchKernelGGL((resnorm_rows_kernel<256, 1, R, T>), grid, dim3(256), 0, st, a);
+    else if (a.D <= 4096) hipLaunchKernelGGL((resnorm_rows_kernel<512, 1, R, T>), grid, dim3(512), 0, st, a);
+    else if (a.D <= 8192) hipLaunchKernelGGL((resnorm_rows_kernel<1024, 1, R, T>), grid, dim3(1024), 0, st, a);
+    else hipLaunchKernelGGL((resnorm_rows_kernel<1024, 2, R, T>), grid, dim3(1024), 0, st, a);
+  };
+  if (a.route_w) launch(std::true_type{});
+  else launch(std::false_type{});
   return TNX_OK;
 }
 
@@ -841,7 +851,7 @@ extern "C" int tnx_residual_norm(void* stream, const tnx_residual_norm_desc* d) 
   TNX_REQUIRE((d->mode != 1 && d->mode != 3) || d->w_post, "residual_norm: null post-norm weight");
   const int groups = d->groups < 1 ? 1 : d->groups;
   TNX_REQUIRE(d->D % groups == 0, "residual_norm: D=%lld does not divide into %d parts", (long long)d->D, groups);
-  TNX_REQUIRE(!d->route_w || (d->route_k > 0 && arrives), "residual_norm: routed rows need their number per row");
+  TNX_REQUIRE(!d->route_w || (d->route_k > 0 && arrives && d->y.y && d->y.split_k <= 1), "residual_norm: routed rows are finished, and need their number per row");
   TNX_REQUIRE(!d->shift || (!d->w_next && d->before && d->starts && d->col_ptr && d->B > 0 && d->T > 0 && d->B * d->T == d->M),
               "residual_norm: a shift needs the rows before, their columns and no next norm");
   TNX_REQUIRE(!d->shift || d->T == 1 || (d->x_out && d->x_out != d->x), "residual_norm: a shift over several tokens needs a second buffer");

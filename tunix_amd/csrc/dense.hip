@@ -356,7 +356,8 @@ extern "C" int tnx_dense_linear(void* stream, const tnx_dense_desc* d) {
       offsets32)
     return tnx_internal_wide_dense(st, d->M, d->K, d->N, (const uint16_t*)d->x, (const uint16_t*)d->w, d->epilogue, d->y,
                                    d->ldy);
-  const int rt = d->M <= 32 || narrow ? 1 : d->M <= 64 ? 2 : 4;
+  int rt = d->M <= 32 || narrow ? 1 : d->M <= 64 ? 2 : 4;
+  while (batch && rt > 1 && cdiv(d->N, 64) * cdiv(d->M, 32 * rt) * d->batch < 512) rt /= 2;
   TNX_REQUIRE(cdiv(d->M, 32 * rt) <= 65535 && split <= 65535, "dense_linear: too many rows or splits in one call");
   const dim3 grid((unsigned)cdiv(d->N, 64), (unsigned)cdiv(d->M, 32 * rt), batch ? (unsigned)d->batch : (unsigned)split);
   if (batch) launch_rows<kBatch>(st, a, rt, grid);

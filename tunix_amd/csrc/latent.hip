@@ -13,6 +13,7 @@
 #include <mutex>
 
 #include "decoder.h"
+#include "gemm_tile.h"
 
 namespace {
 
@@ -278,162 +279,194 @@ struct LatentAttnArgs {
   int64_t out_head;
 };
 
-constexpr int kKeys = 128;
-constexpr size_t latent_smem_bytes(int kd, int nv) {
-  const int lp = kd * 16, w = (lp > nv * 128 ? lp : nv * 128) + 8;
-  return (size_t)(kKeys * w + 32 * (kKeys + 8)) * 2 + 2 * 4 * 32 * 4;
+constexpr int kKeys = 64;
+constexpr size_t latent_smem_bytes(int ks) {
+  return (size_t)(2 * kKeys * ks * 32 + 32 * (kKeys + 8)) * 2 + 2 * 4 * 32 * 4;
 }
 
-// 32 query rows ((position, head) pairs, heads fastest) per work-group; 128 cache rows at a time in LDS, where
-// they serve the scores as keys and the output as values; the next 128 are on their way in registers.
-// Wave w forms the scores of keys 32 w .. + 31 and the output's columns 32 NV w .. + 32 NV - 1.  Both products are
-// transposed, so that a lane owns one query.
-template <int KD, int NV>   // 16-deep k-steps of a row; 32-column groups of the values per wave
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) void latent_attn_kernel(const LatentAttnArgs a) {
-  constexpr int LP = KD * 16, DV = NV * 128, LDW = (LP > DV ? LP : DV) + 8, PLD = kKeys + 8;
+// 32 query rows ((position, head) pairs, heads fastest) per work-group; 64 cache rows at a time in LDS, where
+// they serve the scores as keys and the output as values, while the next 64 are on their way into the other
+// buffer.  Wave w of eight forms the scores of keys 16 (w % 4) .. + 15 with one half of the queries and the output's
+// columns 16 NV w .. + 16 NV - 1 for all of them; both products are transposed, so that a lane owns one query.
+// The 16-byte chunks of a row are permuted within groups of eight (by the row's number), so that neither the 16
+// rows of a score fragment nor the columns of a value row meet in a bank.
+template <int KS, int NV>   // 32-deep k-steps of a row; 128-column groups of the values
+__global__ __launch_bounds__(512) __attribute__((amdgpu_waves_per_eu(2, 2))) void latent_attn_kernel(const LatentAttnArgs a) {
+  constexpr int LP = KS * 32, DV = NV * 128, PLD = kKeys + 8, CH = LP / 8, CW = NV / 2;   // CW: 32-column groups per wave
+  constexpr int PIECES = KS / 2;
+  constexpr uint32_t kBuf = kKeys * LP * 2;
+  constexpr bool kHalfStride = LP / 2 % 64 == 32;           // rows alternate between the halves of the banks
   extern __shared__ __align__(16) unsigned char smem[];
-  uint16_t* ks = reinterpret_cast<uint16_t*>(smem);
-  uint16_t* ps = ks + kKeys * LDW;
-  float* redm = reinterpret_cast<float*>(ps + 32 * PLD);   // [4][32]
+  uint16_t* ps = reinterpret_cast<uint16_t*>(smem + 2 * kBuf);
+  float* redm = reinterpret_cast<float*>(ps + 32 * PLD);    // [4][32]
   float* redl = redm + 128;
-  typedef uint32_t vfrag __attribute__((ext_vector_type(NV / 2)));
-  const int tid = threadIdx.x, lane = tid & 63, l32 = lane & 31, lh = lane >> 5;
-  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int tid = threadIdx.x, lane = tid & 63, l32 = lane & 31, lh = lane >> 5, lm = lane & 15, lq = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), kg = wave & 3, half = wave >> 2;
   const int chunk = blockIdx.x, tile = blockIdx.y;
   const int64_t b = blockIdx.z;
   const int col0 = *a.col_ptr, start = a.starts[b];
-  const unsigned rows = (unsigned)(a.T * a.H), qrow = (unsigned)tile * 32 + l32;
-  const bool qvalid = qrow < rows;
-  const unsigned qc = min(qrow, rows - 1);
-  const int tq = (int)(qc / a.H), head = (int)(qc % a.H);
-  const int64_t qv = (b * a.T + tq) * a.H + head;
+  const unsigned rows = (unsigned)(a.T * a.H);
   int k_lo = max(start, 0), k_hi = min(col0 + (int)(min((unsigned)tile * 32 + 31, rows - 1) / a.H), (int)a.S - 1);
   if (a.n_chunks > 1) {
     k_lo = max(k_lo, chunk * a.kv_chunk);
     k_hi = min(k_hi, chunk * a.kv_chunk + a.kv_chunk - 1);
   }
-  const int c_n = min(col0 + tq, k_hi);
-  u32x4 qf[KD];
+  auto swz = [](int row) { return kHalfStride ? (row >> 1) & 7 : row & 7; };
+  // cache rows -> LDS: piece c of this wave is one kilobyte
+  const u32x4 rk = raw_rsrc(a.cache + b * a.S * LP, (uint64_t)a.S * LP * 2);
+  const uint32_t lds0 = lds_addr(smem) + (uint32_t)wave * (PIECES * 1024u);
+  uint32_t off[PIECES];
 #pragma unroll
-  for (int j = 0; j < KD; ++j) qf[j] = *reinterpret_cast<const u32x4*>(a.q + qv * LP + j * 16 + lh * 8);
-  f32x16 O[NV];
+  for (int c = 0; c < PIECES; ++c) {
+    const int g = (wave * PIECES + c) * 64 + lane, row = g / CH, pc = g % CH;
+    off[c] = (uint32_t)(row * (LP * 2) + ((pc & ~7) | ((pc ^ swz(row)) & 7)) * 16);
+  }
+  auto fetch = [&](int kb, uint32_t buf) {
 #pragma unroll
-  for (int j = 0; j < NV; ++j)
-#pragma unroll
-    for (int i = 0; i < 16; ++i) O[j][i] = 0.f;
-  float m_run = kNegBig, l_run = 0.f;
-  const float sc2 = a.scale * kLog2e;
-  const rsrc_t rk = make_rsrc(a.cache + b * a.S * LP, (uint64_t)a.S * LP * 2);
-  u32x4 kr[KD];            // 128 rows x LP / 8 runs of eight / 256 threads
-  auto fetch = [&](int kb) {
-#pragma unroll
-    for (int c = 0; c < KD; ++c)
-      kr[c] = __builtin_amdgcn_raw_buffer_load_b128(rk, (uint32_t)(c * 256 + tid) * 16u + (uint32_t)kb * (LP * 2), 0, kStreamOnce);
+    for (int c = 0; c < PIECES; ++c) dma16(lds0 + buf + (uint32_t)c * 1024u, rk, off[c] + (uint32_t)kb * (LP * 2), 0);
   };
   const int kb0 = k_lo & ~(kKeys - 1);
-  if (kb0 <= k_hi) fetch(kb0);
-  for (int kb = kb0; kb <= k_hi; kb += kKeys) {
-    __syncthreads();
+  if (kb0 <= k_hi) fetch(kb0, 0);
+  const int hq = half * 16 + lm;                            // this lane's query in the scores
+  const unsigned sq = min((unsigned)tile * 32 + hq, rows - 1);
+  u32x4 qf[KS];
 #pragma unroll
-    for (int c = 0; c < KD; ++c) {
-      const int i = c * 256 + tid;
-      *reinterpret_cast<u32x4*>(&ks[(i / (LP / 8)) * LDW + (i % (LP / 8)) * 8]) = kr[c];
+  for (int j = 0; j < KS; ++j)
+    qf[j] = *reinterpret_cast<const u32x4*>(a.q + ((b * a.T + sq / a.H) * a.H + sq % a.H) * LP + lq * 8 + j * 32);
+  const int cn = min(col0 + (int)(sq / a.H), k_hi);
+  float m16 = kNegBig, l16 = 0.f, m32 = kNegBig;
+  f32x16 O[CW];
+#pragma unroll
+  for (int j = 0; j < CW; ++j)
+#pragma unroll
+    for (int i = 0; i < 16; ++i) O[j][i] = 0.f;
+  const float sc2 = a.scale * kLog2e;
+  // this lane's score fragment: row 16 kg + lm, chunk 4 j + lq; its value columns: CW from vcol on
+  const int krow = kg * 16 + lm, vcol = wave * (CW * 32) + l32 * CW, vch = vcol / 8;
+  const uint32_t kf0 = (uint32_t)(krow * (LP * 2) + ((lq ^ swz(krow)) & 7) * 16), kf1 = (uint32_t)(krow * (LP * 2) + (((4 + lq) ^ swz(krow)) & 7) * 16);
+  uint32_t buf = 0;
+  for (int kb = kb0; kb <= k_hi; kb += kKeys, buf ^= kBuf) {
+    tnx_wait_vm(0);
+    __syncthreads();            // these rows have landed; every wave is done with the other buffer
+    if (kb + kKeys <= k_hi) fetch(kb + kKeys, buf ^ kBuf);
+    const unsigned char* ks = smem + buf;
+    f32x4 st[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};   // even and odd k-steps
+    constexpr int PF = 4;
+    u32x4 kf[PF];
+    auto load_k = [&](int j) { kf[j % PF] = *reinterpret_cast<const u32x4*>(ks + ((j & 1) ? kf1 : kf0) + (j >> 1) * 128); };
+#pragma unroll
+    for (int j = 0; j < PF && j < KS; ++j) load_k(j);
+#pragma unroll
+    for (int j = 0; j < KS; ++j) {
+      st[j & 1] = mfma16(kf[j % PF], qf[j], st[j & 1]);
+      if (j + PF < KS) load_k(j + PF);
+      __builtin_amdgcn_sched_barrier(0);
     }
-    __syncthreads();
-    if (kb + kKeys <= k_hi) fetch(kb + kKeys);
-    f32x16 st;
+    // register i: key kb + 16 kg + 4 lq + i
+    float sc[4], mx = -__builtin_inff();
 #pragma unroll
-    for (int i = 0; i < 16; ++i) st[i] = 0.f;
-#pragma unroll
-    for (int j = 0; j < KD; ++j)
-      st = mfma32(*reinterpret_cast<const u32x4*>(&ks[(wave * 32 + l32) * LDW + j * 16 + lh * 8]), qf[j], st);
-    // register 4 b + e: key kb + 32 wave + 8 b + 4 lh + e
-    float mx = -__builtin_inff();
-#pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      const int key = kb + wave * 32 + 8 * (i >> 2) + 4 * lh + (i & 3);
-      st[i] = key >= k_lo && key <= c_n ? st[i] * sc2 : -__builtin_inff();
-      mx = fmaxf(mx, st[i]);
+    for (int i = 0; i < 4; ++i) {
+      const int key = kb + kg * 16 + 4 * lq + i;
+      sc[i] = key >= k_lo && key <= cn ? (st[0][i] + st[1][i]) * sc2 : -__builtin_inff();
+      mx = fmaxf(mx, sc[i]);
     }
+    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-    if (lh == 0) redm[wave * 32 + l32] = mx;
+    if (lq == 0) redm[kg * 32 + hq] = mx;
     __syncthreads();
-    mx = fmaxf(fmaxf(redm[l32], redm[32 + l32]), fmaxf(redm[64 + l32], redm[96 + l32]));
-    const float m_new = fmaxf(m_run, mx), alpha = exp2_hw(m_run - m_new);
-    m_run = m_new;
-    float psum = 0.f;
+    {
+      const float m_new = fmaxf(m16, fmaxf(fmaxf(redm[hq], redm[32 + hq]), fmaxf(redm[64 + hq], redm[96 + hq])));
+      float p[4], psum = 0.f;
 #pragma unroll
-    for (int bb = 0; bb < 4; ++bb) {
-      float p[4];
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        p[e] = exp2_hw(st[4 * bb + e] - m_new);   // (exp2(-inf) = 0: a masked key)
-        psum += p[e];
+      for (int i = 0; i < 4; ++i) {
+        p[i] = exp2_hw(sc[i] - m_new);   // (exp2(-inf) = 0: a masked key)
+        psum += p[i];
       }
-      *reinterpret_cast<u32x2*>(&ps[l32 * PLD + wave * 32 + 8 * bb + 4 * lh]) = u32x2{pack2bf(p[0], p[1]), pack2bf(p[2], p[3])};
+      *reinterpret_cast<u32x2*>(&ps[hq * PLD + kg * 16 + 4 * lq]) = u32x2{pack2bf(p[0], p[1]), pack2bf(p[2], p[3])};
+      l16 = l16 * exp2_hw(m16 - m_new) + psum;
+      m16 = m_new;
     }
-    l_run = l_run * alpha + psum;
+    const float m_new = fmaxf(m32, fmaxf(fmaxf(redm[l32], redm[32 + l32]), fmaxf(redm[64 + l32], redm[96 + l32])));
+    const float alpha = exp2_hw(m32 - m_new);
+    m32 = m_new;
     if (__builtin_amdgcn_ballot_w64(alpha != 1.0f) != 0) {
 #pragma unroll
-      for (int j = 0; j < NV; ++j)
+      for (int j = 0; j < CW; ++j)
 #pragma unroll
         for (int i = 0; i < 16; ++i) O[j][i] *= alpha;
     }
+    uint32_t v[2][8];
+    u32x4 pf[2];
+    auto load_v = [&](int s) {
+      // k index 8 lh + i of this step: key 16 s + 8 lh + i
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int row = 16 * s + 8 * lh + i;
+        const unsigned char* at = ks + row * (LP * 2) + ((vch & ~7) | ((vch ^ swz(row)) & 7)) * 16 + vcol % 8 * 2;
+        if constexpr (CW == 2) v[s & 1][i] = *reinterpret_cast<const uint32_t*>(at);
+        else v[s & 1][i] = *reinterpret_cast<const uint16_t*>(at);
+      }
+    };
+    load_v(0);
     __syncthreads();
+    auto load_p = [&](int s) { pf[s & 1] = *reinterpret_cast<const u32x4*>(&ps[l32 * PLD + 16 * s + 8 * lh]); };
+    load_p(0);
 #pragma unroll
     for (int s = 0; s < kKeys / 16; ++s) {
-      // k index 8 lh + i of this step: key 16 s + 8 lh + i; lane l32 holds columns NV l32 + j of the wave's
-      vfrag v[8];
+      if (s + 1 < kKeys / 16) {
+        load_v(s + 1);
+        load_p(s + 1);
+      }
+      __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-      for (int i = 0; i < 8; ++i)
-        v[i] = *reinterpret_cast<const vfrag*>(&ks[(16 * s + 8 * lh + i) * LDW + wave * (NV * 32) + NV * l32]);
-      const u32x4 pf = *reinterpret_cast<const u32x4*>(&ps[l32 * PLD + 16 * s + 8 * lh]);
-#pragma unroll
-      for (int j = 0; j < NV; ++j) {
-        const uint32_t sel = (j & 1) ? 0x07060302u : 0x05040100u;
+      for (int j = 0; j < CW; ++j) {
+        const uint32_t sel = j ? 0x07060302u : 0x05040100u;
         u32x4 af;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) af[r] = __builtin_amdgcn_perm(v[2 * r + 1][j >> 1], v[2 * r][j >> 1], sel);
-        O[j] = mfma32(af, pf, O[j]);
+        for (int r = 0; r < 4; ++r) af[r] = __builtin_amdgcn_perm(v[s & 1][2 * r + 1], v[s & 1][2 * r], sel);
+        O[j] = mfma32(af, pf[s & 1], O[j]);
       }
     }
   }
-  l_run += __shfl_xor(l_run, 32, 64);
-  if (lh == 0) redl[wave * 32 + l32] = l_run;
+  l16 += __shfl_xor(l16, 16, 64);
+  l16 += __shfl_xor(l16, 32, 64);
+  if (lq == 0) redl[kg * 32 + hq] = l16;
   __syncthreads();
   const float l = redl[l32] + redl[32 + l32] + redl[64 + l32] + redl[96 + l32];
-  if (!qvalid) return;
-  // register 4 b + e of O[j]: column 32 NV wave + NV (8 b + 4 lh + e) + j: runs of 4 NV columns
+  const unsigned qrow = (unsigned)tile * 32 + l32;
+  if (qrow >= rows) return;
+  const int64_t qv = (b * a.T + qrow / a.H) * a.H + qrow % a.H;
+  // register 4 b + e of O[j]: column 32 CW wave + CW (8 b + 4 lh + e) + j: runs of 4 CW columns
   const float w = a.n_chunks > 1 ? 1.0f : l > 0.f ? 1.0f / l : 0.f;
 #pragma unroll
   for (int bb = 0; bb < 4; ++bb) {
-    const int d0 = wave * (NV * 32) + NV * (8 * bb + 4 * lh);
-    float x[4 * NV];
+    const int d0 = wave * (CW * 32) + CW * (8 * bb + 4 * lh);
+    float x[4 * CW];
 #pragma unroll
     for (int e = 0; e < 4; ++e)
 #pragma unroll
-      for (int j = 0; j < NV; ++j) x[e * NV + j] = O[j][4 * bb + e] * w;
+      for (int j = 0; j < CW; ++j) x[e * CW + j] = O[j][4 * bb + e] * w;
     if (a.n_chunks > 1) {
       float* po = a.ws + (qv * a.n_chunks + chunk) * DV + d0;
 #pragma unroll
-      for (int c = 0; c < 4 * NV; c += 4) *reinterpret_cast<f32x4*>(po + c) = f32x4{x[c], x[c + 1], x[c + 2], x[c + 3]};
+      for (int c = 0; c < 4 * CW; c += 4) *reinterpret_cast<f32x4*>(po + c) = f32x4{x[c], x[c + 1], x[c + 2], x[c + 3]};
       continue;
     }
     uint16_t* out = a.out + qv * a.out_head + d0;
 #pragma unroll
-    for (int c = 0; c < 4 * NV; c += 8) {
-      if (d0 + c + 8 <= a.rank) {
-        *reinterpret_cast<u32x4*>(out + c) = u32x4{pack2bf(x[c], x[c + 1]), pack2bf(x[c + 2], x[c + 3]), pack2bf(x[c + 4], x[c + 5]), pack2bf(x[c + 6], x[c + 7])};
+    for (int c = 0; c < 4 * CW; c += 4) {
+      if (d0 + c + 4 <= a.rank) {
+        *reinterpret_cast<u32x2*>(out + c) = u32x2{pack2bf(x[c], x[c + 1]), pack2bf(x[c + 2], x[c + 3])};
       } else {
 #pragma unroll
-        for (int e = 0; e < 8; ++e)
+        for (int e = 0; e < 4; ++e)
           if (d0 + c + e < a.rank) out[c + e] = f2bf(x[c + e]);
       }
     }
   }
   if (a.n_chunks > 1 && wave == 0 && lh == 0) {
     float* ml = a.ws + a.B * a.T * a.H * a.n_chunks * DV + (qv * a.n_chunks + chunk) * 2;
-    ml[0] = m_run;
+    ml[0] = m32;
     ml[1] = l;
   }
 }
@@ -470,20 +503,20 @@ __global__ __launch_bounds__(128) void latent_merge_kernel(const LatentAttnArgs 
   }
 }
 
-template <int KD, int NV>
+template <int KS, int NV>
 int launch_latent(hipStream_t st, const LatentAttnArgs& a) {
   static std::once_flag once;
   static hipError_t e = hipSuccess;
-  constexpr size_t kSmem = latent_smem_bytes(KD, NV);
+  constexpr size_t kSmem = latent_smem_bytes(KS);
   static_assert(kSmem <= 160 * 1024, "the tile fits LDS");
   std::call_once(once, [] {
-    e = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_attn_kernel<KD, NV>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)kSmem);
+    e = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_attn_kernel<KS, NV>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)kSmem);
   });
   if (e != hipSuccess) {
     tnx_set_error("latent_attn: cannot raise the dynamic LDS limit: %s", hipGetErrorString(e));
     return TNX_ELAUNCH;
   }
-  hipLaunchKernelGGL((latent_attn_kernel<KD, NV>), dim3((unsigned)a.n_chunks, (unsigned)cdiv(a.T * a.H, 32), (unsigned)a.B), dim3(256), kSmem, st, a);
+  hipLaunchKernelGGL((latent_attn_kernel<KS, NV>), dim3((unsigned)a.n_chunks, (unsigned)cdiv(a.T * a.H, 32), (unsigned)a.B), dim3(512), kSmem, st, a);
   if (a.n_chunks > 1)
     hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)(a.B * a.T * a.H)), dim3(128), (size_t)a.n_chunks * 4, st, a, NV * 128);
   TNX_CHECK_LAUNCH("latent_attn");
@@ -650,13 +683,13 @@ extern "C" int tnx_latent_attn(void* stream, const tnx_latent_attn_desc* d) {
   a.B = d->B; a.T = d->T; a.S = d->S; a.H = d->H; a.rank = d->rank; a.scale = d->scale; a.q = (const uint16_t*)d->q; a.cache = (const uint16_t*)d->cache;
   a.starts = d->starts; a.col_ptr = d->col_ptr; a.kv_chunk = d->kv_chunk; a.ws = d->ws; a.out = (uint16_t*)d->out; a.out_head = d->out_head;
   a.n_chunks = d->kv_chunk > 0 && d->kv_chunk < d->S ? (int)cdiv(d->S, d->kv_chunk) : 1;
-  TNX_REQUIRE(a.n_chunks == 1 || (d->ws && d->kv_chunk % kKeys == 0), "latent_attn: a split key range needs a workspace and chunks of whole 128 keys");
+  TNX_REQUIRE(a.n_chunks == 1 || (d->ws && d->kv_chunk % kKeys == 0), "latent_attn: a split key range needs a workspace and chunks of whole 64 keys");
   hipStream_t st = as_stream(stream);
   switch (d->row) {
-    case 128: return launch_latent<8, 2>(st, a);
-    case 256: return launch_latent<16, 2>(st, a);
-    case 320: return launch_latent<20, 2>(st, a);
-    default: return launch_latent<36, 4>(st, a);
+    case 128: return launch_latent<4, 2>(st, a);
+    case 256: return launch_latent<8, 2>(st, a);
+    case 320: return launch_latent<10, 2>(st, a);
+    default: return launch_latent<18, 4>(st, a);
   }
 }
 

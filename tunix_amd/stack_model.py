@@ -350,9 +350,9 @@ class StackRunner(HeadRunner):
   def _latent_chunk(self, m: LatentMixer) -> int:
     """The same for latent attention, whose work-groups have a compute unit to themselves."""
     groups = self.B * math.ceil(self.T * m.heads / 32)
-    if self.T != 1 or groups >= 256 or self.S <= 128:
+    if self.T != 1 or groups >= 256 or self.S <= 256:
       return 0
-    chunk = _up(math.ceil(self.S / math.ceil(256 / groups)), 128)
+    chunk = max(256, _up(math.ceil(self.S / math.ceil(256 / groups)), 64))
     return 0 if chunk >= self.S else chunk
 
   def _split(self, f: DenseLinear) -> int:
