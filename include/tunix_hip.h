@@ -448,7 +448,7 @@ int tnx_sample_commit(void* stream, const int32_t* ids, const float* logp, int64
 int tnx_moe_route_topk(void* stream, const uint16_t* scores, int64_t M, int E, int k,
                        uint16_t* topk_w, int32_t* topk_id);
 /* Builds the expert-sorted route list: counts[E], offsets[E+1], sorted_route[M*k] (route =
- * m*k + j).  Single work-group; M*k <= 1<<20. */
+ * m*k + j), stable in route order.  M*k <= 1<<20. */
 int tnx_moe_sort_routes(void* stream, const int32_t* topk_id, int64_t M, int k, int E,
                         int32_t* counts, int32_t* offsets, int32_t* sorted_route);
 typedef struct tnx_moe_gmm_desc {

@@ -162,6 +162,20 @@ def test_choice_of_experts(gpu):
   assert torch.isnan(w[0]).all() and torch.isfinite(w[1]).all()
 
 
+@pytest.mark.parametrize("M,k,E", [(1, 1, 1), (1, 3, 9), (32, 8, 64), (37, 5, 130), (128, 8, 512), (700, 6, 7), (4099, 8, 64), (20000, 4, 100), (50, 2, 600)])
+def test_routes_sorted_by_expert(gpu, M, k, E):
+  """Stable: an expert's routes in increasing order; experts without a route, and one with most of them."""
+  g = torch.Generator().manual_seed(M)
+  ids = torch.randint(0, E, (M, k), generator=g)
+  ids[torch.rand(M, k, generator=g) < 0.4] = E // 2
+  counts, offsets, order = (torch.full((n,), -7, dtype=torch.int32, device=gpu) for n in (E, E + 1, M * k))
+  ops.moe_sort_routes(ids.int().to(gpu), E, counts, offsets, order)
+  flat = ids.reshape(-1)
+  want = torch.bincount(flat, minlength=E)
+  assert torch.equal(counts.cpu().long(), want) and torch.equal(order.cpu().long(), torch.sort(flat, stable=True).indices)
+  assert offsets[0] == 0 and torch.equal(offsets[1:].cpu().long(), torch.cumsum(want, 0))
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("M,K,F,E,k", [(1, 64, 40, 3, 2), (5, 100, 33, 6, 6), (70, 128, 256, 8, 3), (300, 256, 96, 5, 2), (700, 128, 272, 3, 1)])
 def test_experts(gpu, dtype, M, K, F, E, k):
