@@ -9,6 +9,7 @@
 #include <string.h>
 
 #include <mutex>
+#include <type_traits>
 
 #include "decoder.h"
 
@@ -76,9 +77,9 @@ constexpr int kDenseKT = 128;   // k-tile of the fragment layout: eight 16-deep 
 // consecutive columns of one row.
 // MODE kBatch: blockIdx.z is the weight; kExperts: blockIdx.y is a block of 32 RT routes of one expert.
 template <int RT, int MODE>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(RT == 1 ? 4 : 1, RT == 4 ? 1 : RT == 2 ? 2 : 4)))
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(RT == 1 ? 3 : 1, RT == 4 ? 1 : RT == 2 ? 2 : 4)))
 void dense_rows_kernel(const DenseArgs a) {
-  constexpr int CG = 2, XD = 4;   // column groups; slabs of activations in flight
+  constexpr int CG = 2, XD = RT == 1 ? 8 : 4;   // column groups; slabs of activations in flight
   __shared__ __align__(16) float red[4][CG * 16 * 64];
   const int tid = threadIdx.x, lane = tid & 63, l32 = lane & 31, lh = lane >> 5;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -113,22 +114,24 @@ void dense_rows_kernel(const DenseArgs a) {
   const u32x4* wb = reinterpret_cast<const u32x4*>(a.w + w_at) + ((int64_t)(c64 >> 2) * ktiles * 8 + (c64 & 3) * 2) * 512 + lane;
   // lane: row l32 of every 32, eight k from 8 lh on; rows past the end repeat the last one
   const int64_t kslabs = a.K / 16;
-  const uint16_t* xp[RT];
-  int64_t orow[RT];                       // the row this lane stores, -1: none
+  const unsigned char* xb = reinterpret_cast<const unsigned char*>(a.x + x_at);
+  uint32_t xo[RT];                        // byte offsets (the host checks that they fit)
+  int orow[RT];                       // the row this lane stores, -1: none
 #pragma unroll
   for (int rt = 0; rt < RT; ++rt) {
-    const int64_t r = m0 + rt * 32 + l32, rc = min(r, m_end - 1);
-    int64_t row = rc;
+    const int r = (int)m0 + rt * 32 + l32, rc = min(r, (int)m_end - 1);
+    int row = rc;
     orow[rt] = r < m_end ? r : -1;
     if constexpr (MODE == kExperts) {
       const int route = a.sorted_route[rc];
       row = route / a.x_div;
       if (orow[rt] >= 0) orow[rt] = route;
     }
-    xp[rt] = a.x + x_at + (a.x_frag ? ((row >> 5) * kslabs << 9) + (lh << 8) + ((row & 31) << 3) : row * a.ldx + lh * 8);
+    xo[rt] = a.x_frag ? ((uint32_t)(row >> 5) * (uint32_t)kslabs << 10) + (lh << 9) + ((row & 31) << 4)
+                      : ((uint32_t)row * (uint32_t)a.ldx + lh * 8) * 2;
   }
-  const int xstep = a.x_frag ? 512 : 16;
-  auto load_x = [&](int slab, int rt) -> u32x4 { return *reinterpret_cast<const u32x4*>(xp[rt] + (int64_t)slab * xstep); };
+  const int xstep = a.x_frag ? 1024 : 32;
+  auto load_x = [&](int slab, int rt) -> u32x4 { return *reinterpret_cast<const u32x4*>(xb + slab * xstep + xo[rt]); };
   u32x4 wr[8][CG];
   auto load_w = [&](int kt, int u) {
 #pragma unroll
@@ -136,29 +139,34 @@ void dense_rows_kernel(const DenseArgs a) {
   };
   int kt = kt0 + wave;
   if (kt < kt1) {
-#pragma unroll
-    for (int u = 0; u < 8; ++u) load_w(kt, u);
     u32x4 xr[XD][RT];
+    // in the loop's order, so that its counted waits are the same on the way in
 #pragma unroll
-    for (int u = 0; u < XD - 1; ++u)
+    for (int u = 0; u < 8; ++u) {
+      if (u + XD - 1 >= 8)
 #pragma unroll
-      for (int rt = 0; rt < RT; ++rt) xr[u][rt] = load_x(kt * 8 + u, rt);
-    __builtin_amdgcn_sched_barrier(0);
-    for (; kt < kt1; kt += 4) {
-      const int ktn = min(kt + 4, kt1 - 1);   // (past the end: a valid tile, loaded and not used)
+        for (int rt = 0; rt < RT; ++rt) xr[(u + XD - 1) % XD][rt] = load_x(kt * 8 + u + XD - 9, rt);
+      load_w(kt, u);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    // a tile's products; `more`: the wave has another tile, whose operands are requested meanwhile
+    auto tile = [&](auto more) {
 #pragma unroll
       for (int u = 0; u < 8; ++u) {
-        const int n = u + XD - 1, nslab = n < 8 ? kt * 8 + n : ktn * 8 + n - 8;
+        const int n = u + XD - 1;
+        if (n < 8 || more)
 #pragma unroll
-        for (int rt = 0; rt < RT; ++rt) xr[n % XD][rt] = load_x(nslab, rt);
+          for (int rt = 0; rt < RT; ++rt) xr[n % XD][rt] = load_x(n < 8 ? kt * 8 + n : kt * 8 + 24 + n, rt);
 #pragma unroll
         for (int cg = 0; cg < CG; ++cg)
 #pragma unroll
           for (int rt = 0; rt < RT; ++rt) acc[rt][cg] = mfma32(wr[u][cg], xr[u % XD][rt], acc[rt][cg]);
-        load_w(ktn, u);
+        if (more) load_w(kt + 4, u);
         __builtin_amdgcn_sched_barrier(0);   // (a load sunk to its use would leave nothing in flight)
       }
-    }
+    };
+    for (; kt + 4 < kt1; kt += 4) tile(std::true_type{});
+    tile(std::false_type{});
   }
 
   // the four waves' parts meet, one row tile at a time; wave w then owns one quarter of the tile
@@ -332,6 +340,8 @@ extern "C" int tnx_dense_linear(void* stream, const tnx_dense_desc* d) {
   TNX_REQUIRE(split == 1 || d->ws, "dense_linear: split_k > 1 needs a workspace");
   TNX_REQUIRE(((uintptr_t)d->x & 15) == 0 && ((uintptr_t)d->w & 15) == 0, "dense_linear: x and w must be 16-byte aligned");
   TNX_REQUIRE(!batch || (d->x_stride % 8 == 0 && d->w_stride % 8 == 0 && d->y_stride % 4 == 0), "dense_linear: operands of a batch must stay aligned");
+  const int64_t x_rows = experts ? cdiv(d->M, (int64_t)d->x_div) : cdiv(d->M, 128) * 128;
+  const bool x32 = x_rows * (d->x_frag ? d->K : d->ldx) < (int64_t)1 << 31;
   const bool offsets32 = cdiv(d->N, 256) * (d->K / kDenseKT) * 65536 < (int64_t)1 << 31;
   if (experts) {
     // rows per block: as many as an expert gets on average, and the 128 x 256 kernel from about 24 on (a
@@ -342,6 +352,7 @@ extern "C" int tnx_dense_linear(void* stream, const tnx_dense_desc* d) {
         (uint64_t)(d->M / d->x_div) * (uint64_t)d->K * 2 < 0xfffff000ull && ((uintptr_t)d->y & 15) == 0 && d->epilogue != TNX_EPI_F32)
       return tnx_internal_wide_dense_grouped(st, d->M, d->K, d->N, a.x, a.w, d->epilogue, d->y, d->ldy, d->n_experts, d->offsets,
                                              d->sorted_route, d->x_div);
+    TNX_REQUIRE(x32, "dense_linear: x must stay below 4 GiB");
     const int rt = avg <= 32 ? 1 : avg <= 64 ? 2 : 4;
     const int64_t blocks = d->M / (32 * rt) + (d->n_experts < d->M ? d->n_experts : d->M);
     TNX_REQUIRE(blocks <= 65535, "dense_linear: too many routes in one call");
@@ -356,6 +367,7 @@ extern "C" int tnx_dense_linear(void* stream, const tnx_dense_desc* d) {
       offsets32)
     return tnx_internal_wide_dense(st, d->M, d->K, d->N, (const uint16_t*)d->x, (const uint16_t*)d->w, d->epilogue, d->y,
                                    d->ldy);
+  TNX_REQUIRE(x32, "dense_linear: x must stay below 4 GiB");
   int rt = d->M <= 32 || narrow ? 1 : d->M <= 64 ? 2 : 4;
   while (batch && rt > 1 && cdiv(d->N, 64) * cdiv(d->M, 32 * rt) * d->batch < 512) rt /= 2;
   TNX_REQUIRE(cdiv(d->M, 32 * rt) <= 65535 && split <= 65535, "dense_linear: too many rows or splits in one call");
