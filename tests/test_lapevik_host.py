@@ -26,7 +26,7 @@ def test_config_reader_names_every_tensor(name):
       assert all(getattr(ly.mixer, k) == m[k] for k in ("heads", "vdim", "state", "groups", "conv", "norm_groups"))
     else:
       assert all(getattr(ly.mixer, k) == m[k] for k in ("heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank", "scale"))
-      assert ly.mixer.rot_base == m["rot"]["base"]
+      assert not m["rot_dim"] or ly.mixer.rot_base == m["rot"]["base"]
     e = src["mlp"]
     assert (ly.mlp is None) == (e is None)
     if e is not None:
