@@ -73,8 +73,10 @@ const char* tnx_last_error(void);
  * points of decoders with dense weights (tnx_dense_linear to tnx_logits_stats); 4.0 adds batches and experts
  * to tnx_dense_desc, parts, routed rows and the token shift to tnx_residual_norm_desc, the gate in front
  * to tnx_gated_norm_desc, out_head to tnx_sink_attn_desc, and tnx_silu_mul, tnx_route_softmax,
- * tnx_short_conv, tnx_ring_write, tnx_ssd, tnx_latent_* and tnx_gate_mul. */
-#define TNX_ABI_VERSION_MAJOR 4
+ * tnx_short_conv, tnx_ring_write, tnx_ssd, tnx_latent_* and tnx_gate_mul; 5.0 adds softcap to tnx_lmhead_desc,
+ * a scale to tnx_embed_rows, a first column to tnx_ring_write, parts behind the norm of tnx_gated_norm, and
+ * tnx_parallel_step, tnx_conv_kvwrite, tnx_mixed_attn, tnx_memory and tnx_soft_cap. */
+#define TNX_ABI_VERSION_MAJOR 5
 #define TNX_ABI_VERSION_MINOR 0
 #define TNX_ABI_VERSION ((TNX_ABI_VERSION_MAJOR << 16) | TNX_ABI_VERSION_MINOR)
 int tnx_version(void);
@@ -387,6 +389,8 @@ typedef struct tnx_lmhead_desc {
   int logits_fp32;
   const uint16_t* w_expanded; /* optional: tnx_qw_expand of (codes, scales), or
                                  tnx_dense_expand of w_bf16                                   */
+  /* > 0: a logit is softcap * tanh(w . x / softcap), formed in fp32 before it is rounded */
+  float softcap;
 } tnx_lmhead_desc;
 int64_t tnx_lmhead_nblocks(int64_t V);
 int tnx_lmhead_logp(void* stream, const tnx_lmhead_desc* h_desc);
@@ -597,10 +601,10 @@ typedef struct {
 } tnx_dense_desc;
 int tnx_dense_linear(void* stream, const tnx_dense_desc* d);
 
-/* x[row] (fp32) = table[ids[b, col + t]]; optionally also cat[row, cat_off ..] = the same row in the
+/* x[row] (fp32) = scale * table[ids[b, col + t]]; optionally also cat[row, cat_off ..] = the table's row in the
  * model's dtype.  Ids outside [0, V) read row 0. */
 int tnx_embed_rows(void* stream, int dtype, const void* table, int64_t V, int64_t D, const int32_t* ids,
-                   int64_t ids_ld, const int32_t* col_ptr, int64_t B, int64_t T, float* x, void* cat,
+                   int64_t ids_ld, const int32_t* col_ptr, int64_t B, int64_t T, float scale, float* x, void* cat,
                    int64_t cat_ld, int64_t cat_off, int cat_frag);
 
 /* The residual step between two sublayers, in fp32:
@@ -703,8 +707,8 @@ typedef struct {
 size_t tnx_lightning_ws_bytes(int64_t B, int64_t T, int H, int dk, int dv);
 int tnx_lightning(void* stream, const tnx_lightning_desc* d);
 
-/* out = norm(o) * (w_offset + w) * sigmoid(g[:, g_off ..]) over whole rows of W values; gate_first: out =
- * norm(o * silu(g[:, g_off ..])) * (w_offset + w) over each of `groups` equal parts of a row (0: one). */
+/* out = norm(o) * (w_offset + w) * sigmoid(g[:, g_off ..]), gate_first: out = norm(o * silu(g[:, g_off ..])) *
+ * (w_offset + w), the norms over each of `groups` equal parts of a row of W values (0: one). */
 typedef struct {
   int64_t M, W;
   int dtype;
@@ -750,9 +754,9 @@ typedef struct {
   int64_t out_ld;
 } tnx_short_conv_desc;
 int tnx_short_conv(void* stream, const tnx_short_conv_desc* d);
-/* ring[b, (col + t) % slots, :] = y[b * T + t, off .. off + C) for the last min(T, slots) tokens. */
+/* ring[b, (col + t0 + t) % slots, :] = y[b * T + t, off .. off + C) for the last min(T, slots) tokens. */
 int tnx_ring_write(void* stream, int dtype, const tnx_rows_src* y, int64_t off, int64_t B, int64_t T, int64_t C, int slots,
-                   const int32_t* col_ptr, void* ring);
+                   const int32_t* col_ptr, int64_t t0, void* ring);
 
 /* State-space duality: per head h (group h / (H / G)), dt = softplus(y[:, dt_off + h] + dt_bias[h]),
  *   S <- exp(-exp(A_log[h]) dt) S + dt B x^T,  o[row, h * P ..] = S^T C + D[h] x.
@@ -881,6 +885,127 @@ typedef struct {
   int out_frag;
 } tnx_gate_mul_desc;
 int tnx_gate_mul(void* stream, const tnx_gate_mul_desc* d);
+
+/* The step between layers whose sublayers read one norm, in fp32:
+ *   x += mult * sum_p y_scale[p] * (w_post[p] ? norm(y[p]) * w_post[p] : y[p]),   then x += add[:] (null: nothing);
+ *   h = norm(x) * w_next,   out1 = h + conv1(h),  out2 = h + conv2(h)   (model dtype)
+ * over n_in (0 .. 3) incoming rows, norm(v) = v / sqrt(mean(v^2) + eps), conv(h)_t = sum_j w[taps - 1 - j, :] h_(t - j) with
+ * zeros before starts[b] (w [taps, D]; conv1 null: out1 = h, taps is then not read; out2 null: not written).  The rows
+ * are T tokens for each of B sequences; h of the columns before the call is read from the ring fp32 [B, slots, D]
+ * (slot = column % slots, slots >= taps - 1).  x_out takes the new x; null: x stays as it is (n_in == 0, add null).
+ * T == 1: the ring takes h, x_out may be x.  T > 1 and taps > 1: x_out is another buffer than x, and `tail` fp32
+ * [B, min(T, taps - 1), D] takes h of the last tokens, which the caller moves to the ring (tnx_ring_write). */
+typedef struct {
+  int64_t M, D;
+  int dtype;
+  float eps, mult;
+  int n_in;
+  tnx_rows_src y[3];
+  const float* w_post[3];
+  float y_scale[3];
+  float* x;
+  float* x_out;
+  const float* add;
+  const float* w_next;
+  int taps, slots;
+  const float* conv1;
+  const float* conv2;
+  void* out1;
+  void* out2;
+  int64_t out_ld;
+  int out_frag;
+  float* ring;
+  float* tail;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  int64_t B, T;
+} tnx_parallel_step_desc;
+int tnx_parallel_step(void* stream, const tnx_parallel_step_desc* d);
+
+/* Causal convolution per channel of projected q, k and v, then: q times 1 + temp_coef * ln(floor((p + 1) /
+ * temp_every) + 1) at position p (temp_coef 0: nothing); each value head divided by sqrt(mean(v^2) + eps) with
+ * value_norm; cache write at slot col + t.  y's channels off .. off + C - 1 hold q heads from q_off, k from k_off, v
+ * from v_off (offsets from `off`); w [taps, C] fp32, the last row for the current token; ring (model dtype) [B, slots, C],
+ * zeros before starts[b].  T == 1: slots >= taps, the ring takes the current channels; T > 1: it is only read.
+ * q_out [B*T, H, dkp], kcache [B, G, S, dkp], vcache [B, G, S, dvp]; dimensions past dk / dv are written as zeros. */
+typedef struct {
+  int64_t B, T, S;
+  int H, G, dk, dv, dkp, dvp;
+  int taps, slots, dtype;
+  float temp_coef, temp_every, eps;
+  int value_norm;
+  tnx_rows_src y;
+  int64_t off, C, q_off, k_off, v_off;
+  const float* w;
+  void* ring;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  void* q_out;
+  void* kcache;
+  void* vcache;
+} tnx_conv_kvwrite_desc;
+int tnx_conv_kvwrite(void* stream, const tnx_conv_kvwrite_desc* d);
+
+/* Causal attention whose softmax weights are mixed between the heads: with p_g the softmax of head g over keys
+ * starts[b] .. col + t, out[row, h] = (sum_g talk[h, g] p_g) V_h * sigmoid(gate[row, g_off + h * dv ..]) (gate.ld 0: no gate),
+ * V_h the values of head h's own kv head h / (H / G); caches as tnx_sink_attn's.  talk fp32 [H, H].  kv_chunk (64, 128 or
+ * 256): keys of a work-group where T == 1.  ws: tnx_mixed_attn_ws_bytes.  tnx_mixed_attn_ok: whether a bf16 shape runs
+ * on MFMA kernels; others, and fp32, run a plain kernel. */
+typedef struct {
+  int64_t B, T, S;
+  int H, G, dk, dv, dkp, dvp;
+  float scale;
+  int dtype;
+  const void* q;
+  const void* kcache;
+  const void* vcache;
+  const float* talk;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  int kv_chunk;
+  float* ws;
+  tnx_rows_src gate;
+  int64_t g_off;
+  void* out;
+  int64_t out_ld;
+  int out_frag;
+} tnx_mixed_attn_desc;
+int tnx_mixed_attn_ok(int64_t T, int64_t S, int H, int G, int dkp, int dvp);
+size_t tnx_mixed_attn_ws_bytes(int64_t B, int64_t T, int64_t S, int H, int dvp, int kv_chunk);
+int tnx_mixed_attn(void* stream, const tnx_mixed_attn_desc* d);
+
+/* Matrix memory with exponential gates.  Per head, with i = cap tanh((gates[row, i_off + h] + bias_i[h]) / cap), f =
+ * log sigmoid(cap tanh((gates[row, f_off + h] + bias_f[h]) / cap)) and the running maximum m (0 at a sequence's start):
+ *   m' = max(f + m, i),  S' = e^(f + m - m') S + e^(i - m') k v^T,  n' the same with k alone,
+ *   o[row, h * dv ..] = q_scale S'^T q / (max(|q_scale n'.q|, e^(-m')) + 1e-6).
+ * y: q from q_off, k from k_off, v from v_off, head by head; gates: fp32 rows or planes.  state fp32 [B, H, dk, dv], sum
+ * [B, H, dk] and top [B, H] are read unless col <= starts[b] and written back; o fp32 [B*T, o_ld].  ws:
+ * tnx_memory_ws_bytes. */
+typedef struct {
+  int64_t B, T;
+  int H, dk, dv;
+  int dtype;
+  float q_scale, cap;
+  tnx_rows_src y;
+  int64_t q_off, k_off, v_off;
+  tnx_rows_src gates;
+  int64_t i_off, f_off;
+  const float* bias_i;
+  const float* bias_f;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  float* state;
+  float* sum;
+  float* top;
+  float* o;
+  int64_t o_ld;
+  float* ws;
+} tnx_memory_desc;
+size_t tnx_memory_ws_bytes(int64_t B, int64_t T, int H, int dk, int dv);
+int tnx_memory(void* stream, const tnx_memory_desc* d);
+
+/* z <- cap * tanh(z / cap), n fp32 values in place. */
+int tnx_soft_cap(void* stream, float* z, int64_t n, float cap);
 
 /* Statistics and the whole-vocabulary draw of tnx_lmhead_logp over finished fp32 logits [M, V]
  * (any V); the fields mean what they mean there. */

@@ -89,7 +89,9 @@ def test_struct_layouts_match_the_header(tmp_path):
            "tnx_part_rope_desc": L.PartRopeDesc, "tnx_sink_attn_desc": L.SinkAttnDesc, "tnx_lightning_desc": L.LightningDesc,
            "tnx_gated_norm_desc": L.GatedNormDesc, "tnx_logits_desc": L.LogitsDesc, "tnx_short_conv_desc": L.ShortConvDesc,
            "tnx_ssd_desc": L.SsdDesc, "tnx_latent_prep_desc": L.LatentPrepDesc, "tnx_latent_q_desc": L.LatentQDesc,
-           "tnx_latent_kv_desc": L.LatentKvDesc, "tnx_latent_attn_desc": L.LatentAttnDesc, "tnx_gate_mul_desc": L.GateMulDesc}
+           "tnx_latent_kv_desc": L.LatentKvDesc, "tnx_latent_attn_desc": L.LatentAttnDesc, "tnx_gate_mul_desc": L.GateMulDesc,
+           "tnx_parallel_step_desc": L.ParallelStepDesc, "tnx_conv_kvwrite_desc": L.ConvKvDesc, "tnx_mixed_attn_desc": L.MixedAttnDesc,
+           "tnx_memory_desc": L.MemoryDesc}
   lines = ['#include <stdio.h>', '#include <stddef.h>', '#include "tunix_hip.h"', 'int main(void) {']
   for cname, cls in pairs.items():
     lines.append(f'  printf("{cname} %zu\\n", sizeof({cname}));')

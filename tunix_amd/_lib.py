@@ -12,7 +12,7 @@ _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libtunix_hip.so")
 
 # the ABI this binding was written against (TNX_ABI_VERSION_MAJOR / _MINOR of include/tunix_hip.h)
-ABI_VERSION = (4, 0)
+ABI_VERSION = (5, 0)
 
 TNX_Q_INT4, TNX_Q_NF4 = 0, 1
 TNX_NORM_LLAMA, TNX_NORM_QWEN3, TNX_NORM_GEMMA3 = 0, 1, 2
@@ -80,7 +80,7 @@ class LmHeadDesc(C.Structure):
       ("part_entropy", _p), ("entropy", _p),
       ("part_draw", _p), ("draw_key0", C.c_uint32), ("draw_key1", C.c_uint32), ("draw_rng_variant", _i32),
       ("draw_step_ptr", _p), ("draw_id", _p), ("draw_logp", _p), ("logits_fp32", _i32),
-      ("w_expanded", _p),
+      ("w_expanded", _p), ("softcap", _f32),
   ]
 
 
@@ -209,6 +209,43 @@ class GateMulDesc(C.Structure):
   ]
 
 
+class ParallelStepDesc(C.Structure):
+  _fields_ = [
+      ("M", _i64), ("D", _i64), ("dtype", _i32), ("eps", _f32), ("mult", _f32), ("n_in", _i32),
+      ("y", RowsSrc * 3), ("w_post", _p * 3), ("y_scale", _f32 * 3), ("x", _p), ("x_out", _p), ("add", _p), ("w_next", _p),
+      ("taps", _i32), ("slots", _i32), ("conv1", _p), ("conv2", _p), ("out1", _p), ("out2", _p), ("out_ld", _i64), ("out_frag", _i32),
+      ("ring", _p), ("tail", _p), ("starts", _p), ("col_ptr", _p), ("B", _i64), ("T", _i64),
+  ]
+
+
+class ConvKvDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("S", _i64),
+      ("H", _i32), ("G", _i32), ("dk", _i32), ("dv", _i32), ("dkp", _i32), ("dvp", _i32),
+      ("taps", _i32), ("slots", _i32), ("dtype", _i32), ("temp_coef", _f32), ("temp_every", _f32), ("eps", _f32), ("value_norm", _i32),
+      ("y", RowsSrc), ("off", _i64), ("C", _i64), ("q_off", _i64), ("k_off", _i64), ("v_off", _i64), ("w", _p), ("ring", _p),
+      ("starts", _p), ("col_ptr", _p), ("q_out", _p), ("kcache", _p), ("vcache", _p),
+  ]
+
+
+class MixedAttnDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("S", _i64),
+      ("H", _i32), ("G", _i32), ("dk", _i32), ("dv", _i32), ("dkp", _i32), ("dvp", _i32), ("scale", _f32), ("dtype", _i32),
+      ("q", _p), ("kcache", _p), ("vcache", _p), ("talk", _p), ("starts", _p), ("col_ptr", _p), ("kv_chunk", _i32), ("ws", _p),
+      ("gate", RowsSrc), ("g_off", _i64), ("out", _p), ("out_ld", _i64), ("out_frag", _i32),
+  ]
+
+
+class MemoryDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("H", _i32), ("dk", _i32), ("dv", _i32), ("dtype", _i32), ("q_scale", _f32), ("cap", _f32),
+      ("y", RowsSrc), ("q_off", _i64), ("k_off", _i64), ("v_off", _i64), ("gates", RowsSrc), ("i_off", _i64), ("f_off", _i64),
+      ("bias_i", _p), ("bias_f", _p), ("starts", _p), ("col_ptr", _p), ("state", _p), ("sum", _p), ("top", _p),
+      ("o", _p), ("o_ld", _i64), ("ws", _p),
+  ]
+
+
 class LogitsDesc(C.Structure):
   _fields_ = [
       ("M", _i64), ("V", _i64), ("logits", _p), ("temperature", _f32), ("forbidden", _p), ("n_forbidden", _i32),
@@ -265,7 +302,7 @@ SIGNATURES = {
     "tnx_logp_drift_static_max_rows": (_i64, []),
     "tnx_logp_drift_static": (_i32, [_p, _p, _p, _p, _i64, _i64, _p]),
     "tnx_dense_linear": (_i32, [_p, C.POINTER(DenseDesc)]),
-    "tnx_embed_rows": (_i32, [_p, _i32, _p, _i64, _i64, _p, _i64, _p, _i64, _i64, _p, _p, _i64, _i64, _i32]),
+    "tnx_embed_rows": (_i32, [_p, _i32, _p, _i64, _i64, _p, _i64, _p, _i64, _i64, _f32, _p, _p, _i64, _i64, _i32]),
     "tnx_residual_norm": (_i32, [_p, C.POINTER(ResidualNormDesc)]),
     "tnx_part_rope_kvwrite": (_i32, [_p, C.POINTER(PartRopeDesc)]),
     "tnx_sink_attn_pad": (_i32, [_i32, _i32]),
@@ -278,7 +315,7 @@ SIGNATURES = {
     "tnx_silu_mul": (_i32, [_p, _i32, _p, _i64, _i64, _i64, _i64, _p, _i64]),
     "tnx_route_softmax": (_i32, [_p, C.POINTER(RowsSrc), _i64, _i32, _i32, _p, _p]),
     "tnx_short_conv": (_i32, [_p, C.POINTER(ShortConvDesc)]),
-    "tnx_ring_write": (_i32, [_p, _i32, C.POINTER(RowsSrc), _i64, _i64, _i64, _i64, _i32, _p, _p]),
+    "tnx_ring_write": (_i32, [_p, _i32, C.POINTER(RowsSrc), _i64, _i64, _i64, _i64, _i32, _p, _i64, _p]),
     "tnx_ssd_step_ok": (_i32, [_i32, _i32]),
     "tnx_ssd_ws_bytes": (C.c_size_t, [_i64, _i64, _i32, _i32, _i32, _i32]),
     "tnx_ssd": (_i32, [_p, C.POINTER(SsdDesc)]),
@@ -290,6 +327,14 @@ SIGNATURES = {
     "tnx_latent_attn_ws_bytes": (C.c_size_t, [_i64, _i64, _i64, _i32, _i32, _i32]),
     "tnx_latent_attn": (_i32, [_p, C.POINTER(LatentAttnDesc)]),
     "tnx_gate_mul": (_i32, [_p, C.POINTER(GateMulDesc)]),
+    "tnx_parallel_step": (_i32, [_p, C.POINTER(ParallelStepDesc)]),
+    "tnx_conv_kvwrite": (_i32, [_p, C.POINTER(ConvKvDesc)]),
+    "tnx_mixed_attn_ok": (_i32, [_i64, _i64, _i32, _i32, _i32, _i32]),
+    "tnx_mixed_attn_ws_bytes": (C.c_size_t, [_i64, _i64, _i64, _i32, _i32, _i32]),
+    "tnx_mixed_attn": (_i32, [_p, C.POINTER(MixedAttnDesc)]),
+    "tnx_memory_ws_bytes": (C.c_size_t, [_i64, _i64, _i32, _i32, _i32]),
+    "tnx_memory": (_i32, [_p, C.POINTER(MemoryDesc)]),
+    "tnx_soft_cap": (_i32, [_p, _p, _i64, _f32]),
     "tnx_logits_stats": (_i32, [_p, C.POINTER(LogitsDesc)]),
     "tnx_fill_u32": (_i32, [_p, _p, _i64, C.c_uint32]),
 }

@@ -136,6 +136,73 @@ class AttentionMixer:
 
 
 @dataclasses.dataclass(frozen=True)
+class MixedAttentionMixer:
+  """Causal grouped-query attention without rotation: q, k and v behind a short causal convolution of `conv`
+  taps, queries scaled by 1 + temp_coef ln(floor((p + 1) / temp_every) + 1) at position p, value heads divided
+  by their root mean square (value_norm), softmax weights mixed between the heads, output gate."""
+  heads: int
+  kv_heads: int
+  dim: int
+  vdim: int
+  conv: int
+  scale: float
+  temp_coef: float = 0.0
+  temp_every: float = 1.0
+  value_norm: bool = True
+
+  def __post_init__(self):
+    if self.heads % self.kv_heads:
+      raise ValueError("heads must be a multiple of kv_heads")
+    if self.conv < 1:
+      raise ValueError("the convolution needs a tap")
+    if not self.temp_every > 0:
+      raise ValueError(f"temp_every={self.temp_every} must be positive")
+
+  def weight_shapes(self, D: int) -> dict[str, tuple]:
+    H, rows = self.heads, {"q": self.heads * self.dim, "k": self.kv_heads * self.dim, "v": self.kv_heads * self.vdim}
+    out = {n: (r, D) for n, r in rows.items()}
+    out.update({n + ".conv": (r, self.conv) for n, r in rows.items()})
+    out.update({"talk": (H, H), "g": (H * self.vdim, D), "o": (D, H * self.vdim)})
+    return out
+
+
+@dataclasses.dataclass(frozen=True)
+class MemoryMixer:
+  """Matrix memory with exponential gates (mLSTM): per head a matrix state [dim, vdim], a sum of keys and a
+  running maximum; gates capped at gate_cap; heads normed on their own, gated and projected."""
+  heads: int
+  dim: int
+  vdim: int
+  gate_cap: float
+
+  def __post_init__(self):
+    if not self.gate_cap > 0:
+      raise ValueError(f"gate_cap={self.gate_cap} must be positive")
+
+  def weight_shapes(self, D: int) -> dict[str, tuple]:
+    H, qk, v = self.heads, self.heads * self.dim, self.heads * self.vdim
+    return {"q": (qk, D), "k": (qk, D), "v": (v, D), "g": (v, D), "i": (H, D), "i.b": (H,), "f": (H, D), "f.b": (H,), "norm": (v,), "o": (D, v)}
+
+
+@dataclasses.dataclass(frozen=True)
+class ParallelMixer:
+  """Two mixers side by side that read one input; half the sum of their outputs, each normed over the width."""
+  left: MixedAttentionMixer
+  right: MemoryMixer
+
+  @property
+  def sides(self) -> tuple:
+    return (("left", self.left), ("right", self.right))
+
+  def weight_shapes(self, D: int) -> dict[str, tuple]:
+    out = {}
+    for side, m in self.sides:
+      out.update({f"{side}.{k}": s for k, s in m.weight_shapes(D).items()})
+      out[side + ".out"] = (D,)
+    return out
+
+
+@dataclasses.dataclass(frozen=True)
 class LightningMixer:
   """Linear attention with one constant decay per head and a matrix state per head; the heads'
   outputs are normed together, gated and projected."""
@@ -244,24 +311,28 @@ class ExpertsMlp:
 
 @dataclasses.dataclass(frozen=True)
 class LayerSpec:
-  mixer: AttentionMixer | LightningMixer | SsdMixer | LatentMixer
+  mixer: AttentionMixer | LightningMixer | SsdMixer | LatentMixer | ParallelMixer
   mlp: GatedMlp | ExpertsMlp | None
 
 
 @dataclasses.dataclass(frozen=True)
 class LayerLoop:
-  """Layers start .. stop - 1 run `times` times; before each pass x <- W [x; embedding output]."""
+  """Layers start .. stop - 1 run `times` times; before each pass x <- W [x; embedding output], or with `step` x <- x + the
+  pass's own vector."""
   start: int
   stop: int
   times: int
+  step: bool = False
 
 
 @dataclasses.dataclass(frozen=True)
 class StackConfig:
   """A decoder given layer by layer.  Every sublayer is x += norm(f(norm(x))), or x += norm(f(x)) without
   pre_norm, with norm weights stored as an offset from `norm_offset` and norms taken over norm_groups equal
-  parts of the row; the head is the embedding table.  embed_norm: the embedding is normed.  token_shift:
-  what a mixer reads is first moved towards the same of the token before, per element."""
+  parts of the row.  embed_norm: the embedding is normed.  token_shift:
+  what a mixer reads is first moved towards the same of the token before, per element.
+  parallel: x += residual_mult (mixer(h1) + mlp(h2)) with h = norm(x) and h1, h2 = h + a causal convolution of input_conv
+  taps of h, per sublayer.  tied_head: the head is the embedding table.  logit_softcap > 0: logits <- cap tanh(logits / cap)."""
   family: str
   vocab_size: int
   embed_dim: int
@@ -273,9 +344,21 @@ class StackConfig:
   pre_norm: bool = True
   embed_norm: bool = False
   token_shift: bool = False
+  parallel: bool = False
+  residual_mult: float = 1.0
+  input_conv: int = 0
+  embed_scale: float = 1.0
+  tied_head: bool = True
+  logit_softcap: float = 0.0
 
   def __post_init__(self):
     n, lp = len(self.layers), self.loop
+    if any(isinstance(ly.mixer, ParallelMixer) != self.parallel for ly in self.layers):
+      raise ValueError("parallel layers are made of parallel mixers, and no others are")
+    if self.parallel and (self.input_conv < 1 or self.norm_groups != 1 or self.norm_offset != 0.0 or not self.pre_norm or self.embed_norm or self.token_shift):
+      raise ValueError("parallel layers have one plain norm in front and input convolutions")
+    if lp is not None and lp.step != self.parallel:
+      raise ValueError("a loop over parallel layers adds its pass's vector, no other does")
     if lp is not None and not (0 <= lp.start < lp.stop <= n and lp.times >= 1):
       raise ValueError(f"the loop {lp} does not fit {n} layers")
     if self.embed_dim % self.norm_groups:
@@ -306,17 +389,22 @@ class StackConfig:
     out = {"embed": (self.vocab_size, D), "final.norm": (D,)}
     if self.embed_norm:
       out["embed.norm"] = (D,)
+    if not self.tied_head:
+      out["head"] = (self.vocab_size, D)
     if self.loop is not None:
-      out["loop.in"] = (D, 2 * D)
+      out.update({"loop.step": (self.loop.times, D)} if self.loop.step else {"loop.in": (D, 2 * D)})
     for i, ly in enumerate(self.layers):
       p = f"l{i}."
       parts = [(1, "mix.", ly.mixer)] + ([(2, "mlp.", ly.mlp)] if ly.mlp is not None else [])
       if self.token_shift:
         out[p + "shift"] = (D,)
       for n, at, part in parts:
-        if self.pre_norm:
+        if self.pre_norm and not (self.parallel and n == 2):
           out[p + f"norm{n}"] = (D,)
-        out[p + self.post_norm(n)] = (D,)
+        if self.parallel:
+          out[p + f"canon{n}"] = (D, self.input_conv)
+        else:
+          out[p + self.post_norm(n)] = (D,)
         out.update({p + at + k: s for k, s in part.weight_shapes(D).items()})
     return out
 
@@ -370,6 +458,27 @@ def nunezen_from_dict(d: dict) -> StackConfig:
   return StackConfig(family="nunezen", vocab_size=int(d["vocab"]), embed_dim=int(d["width"]), layers=tuple(layers),
                      norm_eps=float(d["norm"]["eps"]),
                      loop=None if lp is None else LayerLoop(int(lp["start"]), int(lp["stop"]), int(lp["times"])))
+
+
+def kuzezen_from_dict(d: dict) -> StackConfig:
+  """Reads a Kuzezen config.json."""
+  layers = []
+  for i, ly in enumerate(d["layers"]):
+    if ly["type"] != "parallel":
+      raise ValueError(f"layer {i}: unknown mixer type {ly['type']!r}")
+    a, b = ly["mixer"]["left"], ly["mixer"]["right"]
+    left = MixedAttentionMixer(heads=int(a["heads"]), kv_heads=int(a["kv_heads"]), dim=int(a["dim"]), vdim=int(a["vdim"]), conv=int(a["conv"]),
+                               scale=float(a["scale"]), temp_coef=float(a["q_temp"]["coef"]), temp_every=float(a["q_temp"]["every"]))
+    right = MemoryMixer(heads=int(b["heads"]), dim=int(b["dim"]), vdim=int(b["vdim"]), gate_cap=float(b["gate_cap"]))
+    mlp = ly.get("mlp")
+    if mlp is not None and mlp["kind"] != "dense":
+      raise ValueError(f"layer {i}: unknown feed-forward kind {mlp['kind']!r}")
+    layers.append(LayerSpec(ParallelMixer(left, right), None if mlp is None else GatedMlp(int(mlp["ff"]))))
+  lp = d.get("loop")
+  return StackConfig(family="kuzezen", vocab_size=int(d["vocab"]), embed_dim=int(d["width"]), layers=tuple(layers), norm_eps=float(d["norm"]["eps"]),
+                     loop=None if lp is None else LayerLoop(int(lp["start"]), int(lp["stop"]), int(lp["times"]), step=True), norm_offset=0.0,
+                     parallel=True, residual_mult=float(d["residual_mult"]), input_conv=int(d["canon"]["taps"]),
+                     embed_scale=float(d["embedding"]["scale"]), tied_head=False, logit_softcap=float(d["logit_softcap"]))
 
 
 # ---- the shapes the headline metric and the parity cases are quoted on ------------------------
@@ -431,3 +540,12 @@ def lapevik_shape(width: int, heads: int, experts: int, top: int, ff: int, vocab
   attn = LayerSpec(LatentMixer(heads, 128, 64, 128, q_rank=3 * width // 8, kv_rank=512, rot_base=500_000.0, scale=192 ** -0.5), moe)
   return StackConfig(family="lapevik", vocab_size=vocab, embed_dim=width, norm_eps=1e-5, norm_offset=0.0, norm_groups=8, pre_norm=False,
                      embed_norm=True, token_shift=True, layers=tuple(ssd if i % 2 == 0 else attn for i in range(layers)))
+
+
+def kuzezen_shape(width: int, heads: int, kv_heads: int, ff: int, vocab: int = 32768, dim: int = 128, layers: int = 4) -> StackConfig:
+  """A Kuzezen decoder with layers of a real model's size: mixed attention and matrix memory side by side, each with as many
+  heads, the middle layers run twice."""
+  mixer = ParallelMixer(MixedAttentionMixer(heads, kv_heads, dim, dim, 4, dim ** -0.5, 0.1, 8192.0), MemoryMixer(heads, dim, dim, 15.0))
+  return StackConfig(family="kuzezen", vocab_size=vocab, embed_dim=width, norm_eps=1e-6, layers=(LayerSpec(mixer, GatedMlp(ff)),) * layers,
+                     loop=LayerLoop(1, layers - 1, 2, step=True) if layers > 2 else None, norm_offset=0.0, parallel=True, residual_mult=0.5,
+                     input_conv=4, embed_scale=width ** 0.5, tied_head=False, logit_softcap=30.0)

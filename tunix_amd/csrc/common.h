@@ -175,6 +175,11 @@ __device__ __forceinline__ float wave_max(float v) {
   return v;
 }
 
+// cap * tanh(z / cap) with an absolute error of a few ulp of cap
+__device__ __forceinline__ float soft_cap_fast(float z, float cap) {
+  return cap * (1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(2.8853900817779268f * z / cap)));
+}
+
 static inline hipStream_t as_stream(void* s) { return (hipStream_t)s; }
 static inline int64_t cdiv(int64_t a, int64_t b) { return (a + b - 1) / b; }
 

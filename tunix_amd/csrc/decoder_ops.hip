@@ -1,9 +1,10 @@
 // The small operations of decoders with dense weights and an fp32 residual stream: embedding,
-// post-norm + residual + next pre-norm or token shift, partial rotation + cache write, gated norms,
-// gated unit, the choice of experts, and the statistics / sampling of finished logits.  Norms, angles and the residual are 32-bit;
+// post-norm + residual + next pre-norm or token shift, parallel sublayers' residual + norm + input convolutions,
+// partial rotation + cache write, convolution + cache write, gated norms, gated unit, the choice of experts, and the statistics / sampling of finished logits.  Norms, angles and the residual are 32-bit;
 // matrix operands leave in the model's dtype (bf16 or fp32).
 #include <string.h>
 
+#include <mutex>
 #include <type_traits>
 
 #include "decoder.h"
@@ -25,7 +26,7 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 // ---- embedding ---------------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void embed_rows_kernel(const T* table, int64_t V, int64_t D, const int32_t* ids,
-                                                         int64_t ids_ld, const int32_t* col_ptr, int64_t Tn, float* x,
+                                                         int64_t ids_ld, const int32_t* col_ptr, int64_t Tn, float scale, float* x,
                                                          T* cat, int64_t cat_ld, int64_t cat_off, int cat_frag) {
   const int64_t row = blockIdx.x, b = row / Tn, t = row % Tn;
   const int col = col_ptr ? *col_ptr : 0;
@@ -36,14 +37,16 @@ __global__ __launch_bounds__(256) void embed_rows_kernel(const T* table, int64_t
     for (int64_t i = (int64_t)threadIdx.x * 8; i < D; i += 2048) {
       float f[8];
       get8(src, id, i, f);
-      put8(x + row * D + i, f);
       if (cat) put8(cat + (cat_frag ? frag_index(row, cat_off + i, cat_ld) : row * cat_ld + cat_off + i), f);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) f[j] *= scale;
+      put8(x + row * D + i, f);
     }
     return;
   }
   for (int64_t i = threadIdx.x; i < D; i += 256) {
     const T v = table[id * D + i];
-    x[row * D + i] = ld_elem(&v, 0);
+    x[row * D + i] = scale * ld_elem(&v, 0);
     if (cat) cat[cat_frag ? frag_index(row, cat_off + i, cat_ld) : row * cat_ld + cat_off + i] = v;
   }
 }
@@ -414,6 +417,459 @@ void launch_resnorm(hipStream_t st, const ResNormArgs& a) {
   else hipLaunchKernelGGL((resnorm_vec_kernel<8, T>), grid, dim3(256), 0, st, a);
 }
 
+// ---- layers whose sublayers read one norm: residual + norm + input convolutions --------------------
+struct ParallelArgs {
+  int64_t D, B, T;
+  float eps, mult;
+  int n_in;
+  const void* y[3];
+  const float* ws[3];
+  int split[3];
+  int64_t plane[3], y_ld[3];
+  const float* w_post[3];
+  float y_scale[3];
+  const float* x;
+  float* x_out;
+  const float* add;
+  const float* w_next;
+  int taps, slots;
+  const float* conv1;
+  const float* conv2;
+  void* out1;
+  void* out2;
+  int64_t out_ld;
+  int out_frag;
+  float* ring;
+  float* tail;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  int run;                // tokens of a work-group
+};
+__device__ __forceinline__ void block_sum2(float& a, float& b, float (*red)[2]) {
+  a = wave_sum(a);
+  b = wave_sum(b);
+  const int wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
+  __syncthreads();
+  if ((threadIdx.x & 63) == 0) {
+    red[wave][0] = a;
+    red[wave][1] = b;
+  }
+  __syncthreads();
+  a = b = 0.f;
+  for (int w = 0; w < nw; ++w) {
+    a += red[w][0];
+    b += red[w][1];
+  }
+}
+
+// A work-group walks `run` tokens of one sequence; it forms h of the taps - 1 tokens in front of them as well, or
+// takes it from the ring where they belong to an earlier call.  A thread owns runs of eight columns.
+template <int NT, int MAXC, int TAPS, typename T>
+__global__ __launch_bounds__(NT) void parallel_step_kernel(const ParallelArgs a) {
+  __shared__ float red[NT / 64][2];
+  const int64_t runs = (a.T + a.run - 1) / a.run, b = blockIdx.x / runs, t0 = blockIdx.x % runs * a.run;
+  const int64_t t1 = min(a.T, t0 + a.run);
+  const int nch = (int)(a.D / 8), tid = threadIdx.x;
+  const bool conv = a.conv1 != nullptr;
+  const int col0 = conv ? *a.col_ptr : 0, start = conv ? a.starts[b] : 0;
+  auto column = [&](int c) { return (int64_t)min(c * NT + tid, nch - 1) * 8; };
+  auto load8f = [](const float* p, float (&f)[8]) {
+    const f32x4 u = *reinterpret_cast<const f32x4*>(p), v = *reinterpret_cast<const f32x4*>(p + 4);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      f[j] = u[j];
+      f[4 + j] = v[j];
+    }
+  };
+  float wn[MAXC][8], c1[TAPS][MAXC][8], c2[TAPS][MAXC][8], prev[TAPS][MAXC][8];   // prev[j]: h of j + 1 tokens before
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    load8f(a.w_next + column(c), wn[c]);
+#pragma unroll
+    for (int k = 0; k < TAPS; ++k) {
+      if (conv) load8f(a.conv1 + k * a.D + column(c), c1[k][c]);
+      if (a.conv2) load8f(a.conv2 + k * a.D + column(c), c2[k][c]);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) prev[k][c][j] = 0.f;
+    }
+  }
+  const int64_t first = conv ? t0 - (TAPS - 1) : t0;
+  for (int64_t t = first; t < t1; ++t) {
+    const bool live = col0 + t >= start;   // (uniform) otherwise h counts as zero for the tokens behind
+    float h[MAXC][8];
+    if (t < 0) {
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) {
+        if (live) load8f(a.ring + (b * a.slots + (col0 + t) % a.slots) * a.D + column(c), h[c]);
+        else
+#pragma unroll
+          for (int j = 0; j < 8; ++j) h[c][j] = 0.f;
+      }
+    } else {
+      const int64_t row = b * a.T + t;
+      float in[3][MAXC][8], s0 = 0.f, s1 = 0.f, s2 = 0.f;
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) {
+        load8f(a.x + row * a.D + column(c), h[c]);
+#pragma unroll
+        for (int p = 0; p < 3; ++p)
+          if (p < a.n_in) get8(RowSrc<T>{reinterpret_cast<const T*>(a.y[p]), a.ws[p], a.split[p], a.plane[p], a.y_ld[p]}, row, column(c), in[p][c]);
+      }
+      if (a.n_in > 0) {
+        // (uniform) the norms of the incoming rows; the third one's sum shares the second reduction
+#pragma unroll
+        for (int c = 0; c < MAXC; ++c)
+          if (c * NT + tid < nch)
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+              if (a.w_post[0]) s0 += in[0][c][j] * in[0][c][j];
+              if (a.w_post[1]) s1 += in[1][c][j] * in[1][c][j];
+              if (a.w_post[2]) s2 += in[2][c][j] * in[2][c][j];
+            }
+        if (a.w_post[0] || a.w_post[1]) block_sum2(s0, s1, red);
+        if (a.w_post[2]) {
+          float z = 0.f;
+          block_sum2(s2, z, red);
+        }
+        const float sums[3] = {s0, s1, s2};
+#pragma unroll
+        for (int p = 0; p < 3; ++p) {
+          if (p >= a.n_in) continue;
+          const float f = a.mult * a.y_scale[p], r = a.w_post[p] ? 1.0f / sqrtf(sums[p] / (float)a.D + a.eps) : 1.f;
+#pragma unroll
+          for (int c = 0; c < MAXC; ++c) {
+            float w[8];
+            if (a.w_post[p]) load8f(a.w_post[p] + column(c), w);
+#pragma unroll
+            for (int j = 0; j < 8; ++j) h[c][j] += f * (a.w_post[p] ? in[p][c][j] * r * w[j] : in[p][c][j]);
+          }
+        }
+      }
+      float ss = 0.f, zero = 0.f;
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) {
+        if (a.add) {
+          float v[8];
+          load8f(a.add + column(c), v);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) h[c][j] += v[j];
+        }
+        if (c * NT + tid < nch) {
+          if (a.x_out && t >= t0) put8(a.x_out + row * a.D + column(c), h[c]);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) ss += h[c][j] * h[c][j];
+        }
+      }
+      block_sum2(ss, zero, red);
+      const float rn = 1.0f / sqrtf(ss / (float)a.D + a.eps);
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) h[c][j] *= rn * wn[c][j];
+      if (t >= t0) {
+#pragma unroll
+        for (int c = 0; c < MAXC; ++c) {
+          if (c * NT + tid >= nch) continue;
+          const int64_t col = column(c), at = a.out_frag ? frag_index(row, col, a.out_ld) : row * a.out_ld + col;
+          float o[8];
+#pragma unroll
+          for (int j = 0; j < 8; ++j) o[j] = h[c][j];
+          if (conv) {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+              o[j] += c1[TAPS - 1][c][j] * h[c][j];
+#pragma unroll
+              for (int k = 0; k + 1 < TAPS; ++k) o[j] += c1[TAPS - 2 - k][c][j] * prev[k][c][j];
+            }
+          }
+          put8(reinterpret_cast<T*>(a.out1) + at, o);
+          if (a.out2) {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+              o[j] = h[c][j] + c2[TAPS - 1][c][j] * h[c][j];
+#pragma unroll
+              for (int k = 0; k + 1 < TAPS; ++k) o[j] += c2[TAPS - 2 - k][c][j] * prev[k][c][j];
+            }
+            put8(reinterpret_cast<T*>(a.out2) + at, o);
+          }
+          if (TAPS > 1 && conv) {
+            const int64_t keep = min(a.T, (int64_t)TAPS - 1);
+            if (a.T == 1) put8(a.ring + (b * a.slots + col0 % a.slots) * a.D + col, h[c]);
+            else if (t >= a.T - keep) put8(a.tail + (b * keep + t - (a.T - keep)) * a.D + col, h[c]);
+          }
+        }
+      }
+    }
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+#pragma unroll
+        for (int k = TAPS - 1; k > 0; --k) prev[k][c][j] = prev[k - 1][c][j];
+        prev[0][c][j] = live ? h[c][j] : 0.f;
+      }
+  }
+}
+
+// the same for any width and number of taps that fit LDS: a ring of `taps` rows of h, a thread owning the columns
+// tid + 256 i
+template <typename T>
+__global__ __launch_bounds__(256) void parallel_step_any_kernel(const ParallelArgs a) {
+  extern __shared__ __align__(16) float hbuf[];
+  __shared__ float red[4][2];
+  const int64_t runs = (a.T + a.run - 1) / a.run, b = blockIdx.x / runs, t0 = blockIdx.x % runs * a.run;
+  const int64_t t1 = min(a.T, t0 + a.run);
+  const int tid = threadIdx.x, taps = a.conv1 ? a.taps : 1;
+  const int col0 = a.conv1 ? *a.col_ptr : 0, start = a.conv1 ? a.starts[b] : 0;
+  const int64_t first = t0 - (taps - 1);
+  for (int64_t t = first; t < t1; ++t) {
+    const bool live = col0 + t >= start;
+    float* hr = hbuf + (t - first) % taps * a.D;
+    if (t < 0) {
+      for (int64_t i = tid; i < a.D; i += 256) hr[i] = live ? a.ring[(b * a.slots + (col0 + t) % a.slots) * a.D + i] : 0.f;
+      continue;
+    }
+    const int64_t row = b * a.T + t;
+    auto incoming = [&](int p, int64_t i) {
+      return RowSrc<T>{reinterpret_cast<const T*>(a.y[p]), a.ws[p], a.split[p], a.plane[p], a.y_ld[p]}.get(row, i);
+    };
+    float r[3] = {1.f, 1.f, 1.f};
+    for (int p = 0; p < a.n_in; ++p) {
+      if (!a.w_post[p]) continue;
+      float s = 0.f, z = 0.f;
+      for (int64_t i = tid; i < a.D; i += 256) {
+        const float v = incoming(p, i);
+        s += v * v;
+      }
+      block_sum2(s, z, red);
+      r[p] = 1.0f / sqrtf(s / (float)a.D + a.eps);
+    }
+    float ss = 0.f, z = 0.f;
+    for (int64_t i = tid; i < a.D; i += 256) {
+      float v = a.x[row * a.D + i];
+      for (int p = 0; p < a.n_in; ++p) v += a.mult * a.y_scale[p] * (incoming(p, i) * (a.w_post[p] ? r[p] * a.w_post[p][i] : 1.f));
+      if (a.add) v += a.add[i];
+      if (a.x_out && t >= t0) a.x_out[row * a.D + i] = v;
+      hr[i] = v;
+      ss += v * v;
+    }
+    block_sum2(ss, z, red);
+    const float rn = 1.0f / sqrtf(ss / (float)a.D + a.eps);
+    for (int64_t i = tid; i < a.D; i += 256) {
+      const float h = hr[i] * (rn * a.w_next[i]);
+      hr[i] = live ? h : 0.f;
+      if (t < t0) continue;
+      const int64_t at = a.out_frag ? frag_index(row, i, a.out_ld) : row * a.out_ld + i;
+      float o1 = h, o2 = h;
+      if (a.conv1)
+        for (int k = 0; k < taps; ++k) {
+          const float u = k == 0 ? h : hbuf[(t - k - first) % taps * a.D + i];
+          o1 += a.conv1[(int64_t)(taps - 1 - k) * a.D + i] * u;
+          if (a.conv2) o2 += a.conv2[(int64_t)(taps - 1 - k) * a.D + i] * u;
+        }
+      st_elem(reinterpret_cast<T*>(a.out1), at, o1);
+      if (a.out2) st_elem(reinterpret_cast<T*>(a.out2), at, o2);
+      if (taps > 1) {
+        const int64_t keep = min(a.T, (int64_t)taps - 1);
+        if (a.T == 1) a.ring[(b * a.slots + col0 % a.slots) * a.D + i] = h;
+        else if (t >= a.T - keep) a.tail[(b * keep + t - (a.T - keep)) * a.D + i] = h;
+      }
+    }
+  }
+}
+
+template <int NT, int MAXC, typename T>
+void launch_parallel_taps(hipStream_t st, const ParallelArgs& a, const dim3& grid) {
+  const int taps = a.conv1 ? a.taps : 1;
+  if (taps == 1) hipLaunchKernelGGL((parallel_step_kernel<NT, MAXC, 1, T>), grid, dim3(NT), 0, st, a);
+  else if (taps == 2) hipLaunchKernelGGL((parallel_step_kernel<NT, MAXC, 2, T>), grid, dim3(NT), 0, st, a);
+  else if (taps == 3) hipLaunchKernelGGL((parallel_step_kernel<NT, MAXC, 3, T>), grid, dim3(NT), 0, st, a);
+  else hipLaunchKernelGGL((parallel_step_kernel<NT, MAXC, 4, T>), grid, dim3(NT), 0, st, a);
+}
+constexpr size_t kParallelLds = 144 * 1024;
+template <typename T>
+int launch_parallel(hipStream_t st, ParallelArgs a) {
+  a.run = 16;
+  while (a.run > 1 && a.B * cdiv(a.T, a.run) < 1024) a.run /= 2;
+  const dim3 grid((unsigned)(a.B * cdiv(a.T, a.run)));
+  bool vec = a.D % 8 == 0 && a.D <= 8192 && a.out_ld % 8 == 0 && (!a.conv1 || a.taps <= 4);
+  for (int p = 0; p < a.n_in; ++p) vec = vec && a.y_ld[p] % 8 == 0 && a.plane[p] % 8 == 0;
+  if (!vec) {
+    const size_t lds = (size_t)a.D * (a.conv1 ? a.taps : 1) * 4;
+    TNX_REQUIRE(lds <= kParallelLds, "parallel_step: D=%lld with %d taps does not fit LDS", (long long)a.D, a.taps);
+    static std::once_flag once;
+    static hipError_t e = hipSuccess;
+    std::call_once(once, [] {
+      e = hipFuncSetAttribute(reinterpret_cast<const void*>(&parallel_step_any_kernel<T>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)kParallelLds);
+    });
+    if (e != hipSuccess) {
+      tnx_set_error("parallel_step: cannot raise the dynamic LDS limit: %s", hipGetErrorString(e));
+      return TNX_ELAUNCH;
+    }
+    hipLaunchKernelGGL((parallel_step_any_kernel<T>), grid, dim3(256), lds, st, a);
+  } else if (a.D <= 2048) launch_parallel_taps<256, 1, T>(st, a, grid);
+  else if (a.D <= 4096) launch_parallel_taps<512, 1, T>(st, a, grid);
+  else launch_parallel_taps<512, 2, T>(st, a, grid);
+  TNX_CHECK_LAUNCH("parallel_step");
+  return TNX_OK;
+}
+
+// ---- short convolution of q, k and v, query temperature, value norm, cache write ----------------------
+struct ConvKvArgs {
+  int64_t B, T, S;
+  int H, G, dk, dv, dkp, dvp, taps, slots;
+  float coef, every, eps;
+  int value_norm;
+  int64_t off, C, q_off, k_off, v_off;
+  const float* w;          // [taps, C]
+  void* ring;              // [B, slots, C]
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  int run, lanes;          // vec: tokens of a lane group, lanes of a head
+};
+__device__ __forceinline__ float query_temperature(int pos, float coef, float every) {
+  return 1.0f + coef * logf(floorf((float)(pos + 1) / every) + 1.0f);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void conv_kvwrite_kernel(const ConvKvArgs a, const RowSrc<T> src, T* q_out, T* kc, T* vc) {
+  extern __shared__ __align__(16) float vals[];   // v [G, dv], then its heads' scales [G]
+  float* vs = vals + a.G * a.dv;
+  const int64_t row = blockIdx.x, b = row / a.T, t = row % a.T;
+  const int tid = threadIdx.x, col0 = *a.col_ptr, start = a.starts[b], slot = col0 + (int)t;
+  if (slot >= a.S) return;                                    // (uniform; the host sizes the cache)
+  T* ring = reinterpret_cast<T*>(a.ring) + b * a.slots * a.C;
+  auto convolved = [&](int64_t c) {
+    float v = 0.f;
+    for (int j = a.taps - 1; j >= 0; --j) {
+      const int64_t col = (int64_t)slot - j;
+      if (col < start) continue;
+      const float u = t >= j ? src.get(row - j, a.off + c) : ld_elem(ring, (col % a.slots) * a.C + c);
+      v += a.w[(int64_t)(a.taps - 1 - j) * a.C + c] * u;
+    }
+    if (a.T == 1) st_elem(ring, (int64_t)(slot % a.slots) * a.C + c, src.get(row, a.off + c));
+    return v;
+  };
+  const float temp = query_temperature(max(slot - start, 0), a.coef, a.every);
+  for (int it = tid; it < a.H * a.dkp; it += 256) {
+    const int h = it / a.dkp, i = it % a.dkp;
+    st_elem(q_out, (row * a.H + h) * a.dkp + i, i < a.dk ? convolved(a.q_off + (int64_t)h * a.dk + i) * temp : 0.f);
+  }
+  for (int it = tid; it < a.G * a.dkp; it += 256) {
+    const int g = it / a.dkp, i = it % a.dkp;
+    st_elem(kc, ((b * a.G + g) * a.S + slot) * a.dkp + i, i < a.dk ? convolved(a.k_off + (int64_t)g * a.dk + i) : 0.f);
+  }
+  for (int it = tid; it < a.G * a.dv; it += 256) vals[it] = convolved(a.v_off + it);
+  __syncthreads();
+  for (int g = tid >> 6; g < a.G; g += 4) {
+    float s = 0.f;
+    for (int i = tid & 63; i < a.dv; i += 64) s += vals[g * a.dv + i] * vals[g * a.dv + i];
+    s = wave_sum(s);
+    if ((tid & 63) == 0) vs[g] = a.value_norm ? 1.0f / sqrtf(s / (float)a.dv + a.eps) : 1.f;
+  }
+  __syncthreads();
+  for (int it = tid; it < a.G * a.dvp; it += 256) {
+    const int g = it / a.dvp, i = it % a.dvp;
+    st_elem(vc, ((b * a.G + g) * a.S + slot) * a.dvp + i, i < a.dv ? vals[g * a.dv + i] * vs[g] : 0.f);
+  }
+}
+
+// A group of `lanes` lanes (a power of two) owns one head over `run` tokens, a lane eight of its dimensions; the
+// inputs of the tokens before stay in registers.
+template <int TAPS, typename T>
+__global__ __launch_bounds__(256) void conv_kvwrite_vec_kernel(const ConvKvArgs a, const RowSrc<T> src, T* q_out, T* kc, T* vc) {
+  const int heads = a.H + 2 * a.G, runs = (int)((a.T + a.run - 1) / a.run), gl = threadIdx.x % a.lanes;
+  const int64_t item = (int64_t)blockIdx.x * (256 / a.lanes) + threadIdx.x / a.lanes;
+  if (item >= a.B * runs * heads) return;
+  const int hd = (int)(item % heads), d0 = gl * 8;
+  const int64_t b = item / heads / runs, t0 = item / heads % runs * a.run;
+  const int kind = hd < a.H ? 0 : hd < a.H + a.G ? 1 : 2, g = kind == 0 ? hd : kind == 1 ? hd - a.H : hd - a.H - a.G;
+  const int dim = kind == 2 ? a.dv : a.dk, pad = kind == 2 ? a.dvp : a.dkp;
+  const bool real = d0 < dim;
+  const int64_t c = (kind == 0 ? a.q_off : kind == 1 ? a.k_off : a.v_off) + (int64_t)g * dim + (real ? d0 : 0);
+  const int col0 = *a.col_ptr, start = a.starts[b];
+  T* ring = reinterpret_cast<T*>(a.ring) + b * a.slots * a.C;
+  const RowSrc<T> rsrc{ring, nullptr, 1, 0, a.C};
+  const RowSrc<float> wsrc{a.w, nullptr, 1, 0, a.C};
+  float w[TAPS][8], u[TAPS][8];
+#pragma unroll
+  for (int k = 0; k < TAPS; ++k) get8(wsrc, k, c, w[k]);
+  auto input = [&](int64_t t, float (&f)[8]) {
+    const int64_t col = col0 + t;
+    if (col < start) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) f[i] = 0.f;
+    } else if (t >= 0) {
+      get8(src, b * a.T + t, a.off + c, f);
+    } else {
+      get8(rsrc, col % a.slots, c, f);
+    }
+  };
+#pragma unroll
+  for (int k = 0; k + 1 < TAPS; ++k) input(t0 - (TAPS - 1) + k, u[k]);
+  const int64_t t1 = min(a.T, t0 + a.run);
+  for (int64_t t = t0; t < t1; ++t) {
+    const int64_t row = b * a.T + t, slot = col0 + t;
+    if (slot >= a.S) break;
+    input(t, u[TAPS - 1]);
+    float v[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      v[i] = 0.f;
+#pragma unroll
+      for (int k = 0; k < TAPS; ++k) v[i] += w[k][i] * u[k][i];
+    }
+    float f = 1.f;
+    if (kind == 0) f = query_temperature(max((int)slot - start, 0), a.coef, a.every);
+    if (kind == 2 && a.value_norm) {
+      float s = 0.f;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) s += v[i] * v[i];
+      if (!real) s = 0.f;
+      for (int o = a.lanes / 2; o > 0; o >>= 1) s += __shfl_xor(s, o, 64);
+      f = 1.0f / sqrtf(s / (float)dim + a.eps);
+    }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = real ? v[i] * f : 0.f;
+    if (d0 < pad) {
+      T* dst = kind == 0 ? q_out + (row * a.H + g) * a.dkp : kind == 1 ? kc + ((b * a.G + g) * a.S + slot) * a.dkp : vc + ((b * a.G + g) * a.S + slot) * a.dvp;
+      put8(dst + d0, v);
+    }
+    if (a.T == 1 && real) put8(ring + (slot % a.slots) * a.C + c, u[TAPS - 1]);
+#pragma unroll
+    for (int k = 0; k + 1 < TAPS; ++k)
+#pragma unroll
+      for (int i = 0; i < 8; ++i) u[k][i] = u[k + 1][i];
+  }
+}
+template <typename T>
+int launch_conv_kv(hipStream_t st, ConvKvArgs a, const RowSrc<T>& src, T* q_out, T* kc, T* vc) {
+  const bool vec = a.taps <= 4 && (a.dk | a.dv | a.dkp | a.dvp) % 8 == 0 && a.dkp <= 512 && a.dvp <= 512 && (a.off | a.C | a.q_off | a.k_off | a.v_off) % 8 == 0 &&
+                   src.ld % 8 == 0 && src.plane % 8 == 0;
+  if (!vec) {
+    TNX_REQUIRE((int64_t)a.G * (a.dv + 1) <= 16000, "conv_kvwrite: values of one row above 16000");
+    hipLaunchKernelGGL((conv_kvwrite_kernel<T>), dim3((unsigned)(a.B * a.T)), dim3(256), (size_t)a.G * (a.dv + 1) * 4, st, a, src, q_out, kc, vc);
+    TNX_CHECK_LAUNCH("conv_kvwrite");
+    return TNX_OK;
+  }
+  a.lanes = 1;
+  while (a.lanes * 8 < (a.dkp > a.dvp ? a.dkp : a.dvp)) a.lanes *= 2;
+  const int heads = a.H + 2 * a.G;
+  a.run = 16;
+  while (a.run > 1 && a.B * cdiv(a.T, a.run) * heads * a.lanes < 262144) a.run /= 2;
+  const dim3 grid((unsigned)cdiv(a.B * cdiv(a.T, a.run) * heads, 256 / a.lanes));
+  if (a.taps == 1) hipLaunchKernelGGL((conv_kvwrite_vec_kernel<1, T>), grid, dim3(256), 0, st, a, src, q_out, kc, vc);
+  else if (a.taps == 2) hipLaunchKernelGGL((conv_kvwrite_vec_kernel<2, T>), grid, dim3(256), 0, st, a, src, q_out, kc, vc);
+  else if (a.taps == 3) hipLaunchKernelGGL((conv_kvwrite_vec_kernel<3, T>), grid, dim3(256), 0, st, a, src, q_out, kc, vc);
+  else hipLaunchKernelGGL((conv_kvwrite_vec_kernel<4, T>), grid, dim3(256), 0, st, a, src, q_out, kc, vc);
+  TNX_CHECK_LAUNCH("conv_kvwrite");
+  return TNX_OK;
+}
+
+__global__ __launch_bounds__(256) void soft_cap_kernel(float* z, int64_t n, float cap) {
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) z[i] = cap * tanhf(z[i] / cap);
+}
+
 // ---- rotation of the first rot_dims dimensions of q and k, cache write --------------------------
 struct PartRopeArgs {
   int64_t T, S;
@@ -506,7 +962,7 @@ __global__ __launch_bounds__(256) void part_rope_vec_kernel(const PartRopeArgs a
   }
 }
 
-// ---- RMS norm and a gate: norm(o) . w . sigmoid(g) over the whole row, or norm(o . silu(g)) . w in parts --
+// ---- RMS norm and a gate, in parts of a row: norm(o) . w . sigmoid(g), or norm(o . silu(g)) . w --------------
 struct GatedNormArgs {
   int64_t W, o_ld, out_ld, g_off;
   float eps, w_offset;
@@ -585,22 +1041,34 @@ int launch_gate_first(hipStream_t st, int64_t M, const GatedNormArgs& a, const R
 }
 template <typename T>
 __global__ __launch_bounds__(256) void gated_norm_kernel(const GatedNormArgs a, const RowSrc<T> g, T* out) {
-  __shared__ float red[4];
+  __shared__ float gs[1024];
   const int64_t row = blockIdx.x;
   const float* o = a.o + row * a.o_ld;
-  float ss = 0.f;
-  for (int64_t i = threadIdx.x; i < a.W; i += 256) ss += o[i] * o[i];
-  const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)a.W + a.eps);
+  const int per = (int)(a.W / a.groups), lane = threadIdx.x & 63;
+  if (a.groups == 1) {
+    float ss = 0.f;
+    for (int64_t i = threadIdx.x; i < a.W; i += 256) ss += o[i] * o[i];
+    ss = block_sum(ss, gs + 4);
+    if (threadIdx.x == 0) gs[0] = 1.0f / sqrtf(ss / (float)a.W + a.eps);
+  } else {
+    for (int p = threadIdx.x >> 6; p < a.groups; p += 4) {
+      float s = 0.f;
+      for (int i = lane; i < per; i += 64) s += o[p * per + i] * o[p * per + i];
+      s = wave_sum(s);
+      if (lane == 0) gs[p] = 1.0f / sqrtf(s / (float)per + a.eps);
+    }
+  }
+  __syncthreads();
   for (int64_t i = threadIdx.x; i < a.W; i += 256)
     st_elem(out, a.out_frag ? frag_index(row, i, a.out_ld) : row * a.out_ld + i,
-            o[i] * r * (a.w_offset + a.w[i]) * sigmoid_f32(g.get(row, a.g_off + i)));
+            o[i] * gs[i / per] * (a.w_offset + a.w[i]) * sigmoid_f32(g.get(row, a.g_off + i)));
 }
 // eight elements per thread and turn, everything requested ahead of the sum
-template <int MAXC, typename T>
+template <int MAXC, bool PARTS, typename T>
 __global__ __launch_bounds__(256) void gated_norm_vec_kernel(const GatedNormArgs a, const RowSrc<T> g, T* out) {
-  __shared__ float red[4];
+  __shared__ float red[4], part[PARTS ? MAXC * 256 : 1], gs[PARTS ? MAXC * 256 : 1];
   const int64_t row = blockIdx.x;
-  const int nch = (int)(a.W / 8);
+  const int nch = (int)(a.W / 8), per = nch / a.groups;
   float o[MAXC][8], w[MAXC][8], gv[MAXC][8];
   const RowSrc<float> os{a.o, nullptr, 1, 0, a.o_ld}, wsrc{a.w, nullptr, 1, 0, 0};
 #pragma unroll
@@ -612,29 +1080,41 @@ __global__ __launch_bounds__(256) void gated_norm_vec_kernel(const GatedNormArgs
   }
   float ss = 0.f;
 #pragma unroll
-  for (int c = 0; c < MAXC; ++c)
-    if (c * 256 + (int)threadIdx.x < nch)
+  for (int c = 0; c < MAXC; ++c) {
+    float q = 0.f;
 #pragma unroll
-      for (int j = 0; j < 8; ++j) ss += o[c][j] * o[c][j];
-  const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)a.W + a.eps);
+    for (int j = 0; j < 8; ++j) q += o[c][j] * o[c][j];
+    if constexpr (PARTS) part[c * 256 + threadIdx.x] = q;
+    else if (c * 256 + (int)threadIdx.x < nch) ss += q;
+  }
+  float r = 1.f;
+  if constexpr (PARTS) part_scales(part, gs, a.groups, per, (float)(per * 8), a.eps);
+  else r = 1.0f / sqrtf(block_sum(ss, red) / (float)a.W + a.eps);
 #pragma unroll
   for (int c = 0; c < MAXC; ++c) {
     const int ch = c * 256 + threadIdx.x;
     if (ch >= nch) continue;
+    if constexpr (PARTS) r = gs[ch / per];
 #pragma unroll
     for (int j = 0; j < 8; ++j) o[c][j] = o[c][j] * r * (a.w_offset + w[c][j]) * sigmoid_f32(gv[c][j]);
     put8(out + (a.out_frag ? frag_index(row, (int64_t)ch * 8, a.out_ld) : row * a.out_ld + (int64_t)ch * 8), o[c]);
   }
 }
+template <bool PARTS, typename T>
+void launch_gated_norm_vec(hipStream_t st, int64_t M, const GatedNormArgs& a, const RowSrc<T>& g, T* out) {
+  const dim3 grid((unsigned)M);
+  if (a.W <= 2048) hipLaunchKernelGGL((gated_norm_vec_kernel<1, PARTS, T>), grid, dim3(256), 0, st, a, g, out);
+  else if (a.W <= 4096) hipLaunchKernelGGL((gated_norm_vec_kernel<2, PARTS, T>), grid, dim3(256), 0, st, a, g, out);
+  else if (a.W <= 8192) hipLaunchKernelGGL((gated_norm_vec_kernel<4, PARTS, T>), grid, dim3(256), 0, st, a, g, out);
+  else hipLaunchKernelGGL((gated_norm_vec_kernel<8, PARTS, T>), grid, dim3(256), 0, st, a, g, out);
+}
 template <typename T>
 void launch_gated_norm(hipStream_t st, int64_t M, const GatedNormArgs& a, const RowSrc<T>& g, T* out) {
-  const dim3 grid((unsigned)M);
-  const bool vec = a.W % 8 == 0 && a.W <= 16384 && a.o_ld % 8 == 0 && g.ld % 8 == 0 && g.plane % 8 == 0 && a.g_off % 8 == 0 && a.out_ld % 8 == 0;
-  if (!vec) hipLaunchKernelGGL((gated_norm_kernel<T>), grid, dim3(256), 0, st, a, g, out);
-  else if (a.W <= 2048) hipLaunchKernelGGL((gated_norm_vec_kernel<1, T>), grid, dim3(256), 0, st, a, g, out);
-  else if (a.W <= 4096) hipLaunchKernelGGL((gated_norm_vec_kernel<2, T>), grid, dim3(256), 0, st, a, g, out);
-  else if (a.W <= 8192) hipLaunchKernelGGL((gated_norm_vec_kernel<4, T>), grid, dim3(256), 0, st, a, g, out);
-  else hipLaunchKernelGGL((gated_norm_vec_kernel<8, T>), grid, dim3(256), 0, st, a, g, out);
+  const bool vec = a.W % 8 == 0 && a.W / a.groups % 8 == 0 && a.W <= 16384 && a.o_ld % 8 == 0 && g.ld % 8 == 0 && g.plane % 8 == 0 && a.g_off % 8 == 0 &&
+                   a.out_ld % 8 == 0;
+  if (!vec) hipLaunchKernelGGL((gated_norm_kernel<T>), dim3((unsigned)M), dim3(256), 0, st, a, g, out);
+  else if (a.groups > 1) launch_gated_norm_vec<true>(st, M, a, g, out);
+  else launch_gated_norm_vec<false>(st, M, a, g, out);
 }
 
 // ---- gated unit on finished projections: out = act(y[:, :F]) * y[:, u_off : u_off + F] -----------
@@ -825,7 +1305,7 @@ RowSrc<T> row_src(const tnx_rows_src& s) {
 }  // namespace
 
 extern "C" int tnx_embed_rows(void* stream, int dtype, const void* table, int64_t V, int64_t D, const int32_t* ids,
-                              int64_t ids_ld, const int32_t* col_ptr, int64_t B, int64_t T, float* x, void* cat,
+                              int64_t ids_ld, const int32_t* col_ptr, int64_t B, int64_t T, float scale, float* x, void* cat,
                               int64_t cat_ld, int64_t cat_off, int cat_frag) {
   TNX_REQUIRE(table && ids && x, "embed_rows: null pointer");
   TNX_REQUIRE(V > 0 && D > 0 && B > 0 && T > 0, "embed_rows: bad shape");
@@ -833,10 +1313,10 @@ extern "C" int tnx_embed_rows(void* stream, int dtype, const void* table, int64_
   TNX_REQUIRE(dtype == TNX_BF16 || dtype == TNX_F32, "embed_rows: bad dtype %d", dtype);
   if (dtype == TNX_BF16)
     hipLaunchKernelGGL(embed_rows_kernel<uint16_t>, dim3((unsigned)(B * T)), dim3(256), 0, as_stream(stream), (const uint16_t*)table,
-                       V, D, ids, ids_ld, col_ptr, T, x, (uint16_t*)cat, cat_ld, cat_off, cat_frag);
+                       V, D, ids, ids_ld, col_ptr, T, scale, x, (uint16_t*)cat, cat_ld, cat_off, cat_frag);
   else
     hipLaunchKernelGGL(embed_rows_kernel<float>, dim3((unsigned)(B * T)), dim3(256), 0, as_stream(stream), (const float*)table, V, D,
-                       ids, ids_ld, col_ptr, T, x, (float*)cat, cat_ld, cat_off, cat_frag);
+                       ids, ids_ld, col_ptr, T, scale, x, (float*)cat, cat_ld, cat_off, cat_frag);
   TNX_CHECK_LAUNCH("embed_rows");
   return TNX_OK;
 }
@@ -872,6 +1352,62 @@ extern "C" int tnx_residual_norm(void* stream, const tnx_residual_norm_desc* d) 
   if (d->dtype == TNX_BF16) launch_resnorm<uint16_t>(as_stream(stream), a);
   else launch_resnorm<float>(as_stream(stream), a);
   TNX_CHECK_LAUNCH("residual_norm");
+  return TNX_OK;
+}
+
+extern "C" int tnx_parallel_step(void* stream, const tnx_parallel_step_desc* d) {
+  TNX_REQUIRE(d, "parallel_step: null descriptor");
+  TNX_REQUIRE(d->M > 0 && d->D > 0 && d->B > 0 && d->T > 0 && d->B * d->T == d->M && d->M < (int64_t)1 << 31, "parallel_step: bad shape");
+  TNX_REQUIRE(d->dtype == TNX_BF16 || d->dtype == TNX_F32, "parallel_step: bad dtype %d", d->dtype);
+  TNX_REQUIRE(d->n_in >= 0 && d->n_in <= 3, "parallel_step: %d incoming rows, at most three", d->n_in);
+  TNX_REQUIRE(d->x && d->w_next && d->out1 && d->out_ld >= d->D, "parallel_step: null pointer or short output rows");
+  TNX_REQUIRE(d->x_out || (d->n_in == 0 && !d->add), "parallel_step: the new residual needs a buffer");
+  TNX_REQUIRE(!d->out2 || (d->conv1 && d->conv2), "parallel_step: a second output needs both convolutions");
+  const int taps = d->conv1 ? d->taps : 1;
+  if (d->conv1) {
+    TNX_REQUIRE(taps >= 1 && taps <= 4096 && d->starts && d->col_ptr, "parallel_step: the convolutions need taps and columns");
+    TNX_REQUIRE(taps == 1 || (d->ring && d->slots >= taps - 1 && (d->T == 1 || (d->tail && (!d->x_out || d->x_out != d->x)))),
+                "parallel_step: the convolutions need a ring and, over several tokens, a tail and a second residual buffer");
+  }
+  ParallelArgs a;
+  memset(&a, 0, sizeof(a));
+  a.D = d->D; a.B = d->B; a.T = d->T; a.eps = d->eps; a.mult = d->mult; a.n_in = d->n_in;
+  for (int p = 0; p < d->n_in; ++p) {
+    TNX_REQUIRE(src_given(d->y[p]) && d->y[p].ld >= d->D, "parallel_step: incoming rows %d are missing", p);
+    a.y[p] = d->y[p].y; a.ws[p] = d->y[p].ws; a.split[p] = d->y[p].split_k < 1 ? 1 : d->y[p].split_k; a.plane[p] = a.split[p] > 1 ? d->y[p].plane : 0;
+    a.y_ld[p] = d->y[p].ld; a.w_post[p] = d->w_post[p]; a.y_scale[p] = d->y_scale[p];
+  }
+  a.x = d->x; a.x_out = d->x_out; a.add = d->add; a.w_next = d->w_next; a.taps = taps; a.slots = d->slots; a.conv1 = d->conv1;
+  a.conv2 = d->out2 ? d->conv2 : nullptr; a.out1 = d->out1; a.out2 = d->out2; a.out_ld = d->out_ld; a.out_frag = d->out_frag;
+  a.ring = d->ring; a.tail = d->tail; a.starts = d->starts; a.col_ptr = d->col_ptr;
+  return d->dtype == TNX_BF16 ? launch_parallel<uint16_t>(as_stream(stream), a) : launch_parallel<float>(as_stream(stream), a);
+}
+
+extern "C" int tnx_conv_kvwrite(void* stream, const tnx_conv_kvwrite_desc* d) {
+  TNX_REQUIRE(d, "conv_kvwrite: null descriptor");
+  TNX_REQUIRE(d->B > 0 && d->T > 0 && d->S > 0 && d->H > 0 && d->G > 0 && d->H % d->G == 0 && d->B * d->T < (int64_t)1 << 31, "conv_kvwrite: bad shape");
+  TNX_REQUIRE(d->dk > 0 && d->dv > 0 && d->dkp >= d->dk && d->dvp >= d->dv, "conv_kvwrite: bad head sizes");
+  TNX_REQUIRE(d->taps >= 1 && d->taps <= 4096 && d->slots >= 1 && d->slots >= (d->T == 1 ? d->taps : d->taps - 1), "conv_kvwrite: the ring is shorter than the taps");
+  TNX_REQUIRE(d->off >= 0 && d->q_off >= 0 && d->k_off >= 0 && d->v_off >= 0 && d->q_off + (int64_t)d->H * d->dk <= d->C && d->k_off + (int64_t)d->G * d->dk <= d->C &&
+                  d->v_off + (int64_t)d->G * d->dv <= d->C,
+              "conv_kvwrite: heads outside the channels");
+  TNX_REQUIRE(src_given(d->y) && d->w && d->ring && d->starts && d->col_ptr && d->q_out && d->kcache && d->vcache && d->temp_every > 0.f, "conv_kvwrite: null pointer");
+  TNX_REQUIRE(d->dtype == TNX_BF16 || d->dtype == TNX_F32, "conv_kvwrite: bad dtype %d", d->dtype);
+  ConvKvArgs a;
+  memset(&a, 0, sizeof(a));
+  a.B = d->B; a.T = d->T; a.S = d->S; a.H = d->H; a.G = d->G; a.dk = d->dk; a.dv = d->dv; a.dkp = d->dkp; a.dvp = d->dvp; a.taps = d->taps; a.slots = d->slots;
+  a.coef = d->temp_coef; a.every = d->temp_every; a.eps = d->eps; a.value_norm = d->value_norm; a.off = d->off; a.C = d->C; a.q_off = d->q_off;
+  a.k_off = d->k_off; a.v_off = d->v_off; a.w = d->w; a.ring = d->ring; a.starts = d->starts; a.col_ptr = d->col_ptr;
+  if (d->dtype == TNX_BF16)
+    return launch_conv_kv(as_stream(stream), a, row_src<uint16_t>(d->y), (uint16_t*)d->q_out, (uint16_t*)d->kcache, (uint16_t*)d->vcache);
+  return launch_conv_kv(as_stream(stream), a, row_src<float>(d->y), (float*)d->q_out, (float*)d->kcache, (float*)d->vcache);
+}
+
+extern "C" int tnx_soft_cap(void* stream, float* z, int64_t n, float cap) {
+  TNX_REQUIRE(z && n > 0 && cap > 0.f, "soft_cap: null pointer or bad shape");
+  const int64_t blocks = cdiv(n, 1024);
+  hipLaunchKernelGGL(soft_cap_kernel, dim3((unsigned)(blocks < 65535 ? blocks : 65535)), dim3(256), 0, as_stream(stream), z, n, cap);
+  TNX_CHECK_LAUNCH("soft_cap");
   return TNX_OK;
 }
 
@@ -919,7 +1455,7 @@ extern "C" int tnx_gated_norm(void* stream, const tnx_gated_norm_desc* d) {
   GatedNormArgs a;
   a.W = d->W; a.o_ld = d->o_ld; a.out_ld = d->out_ld; a.g_off = d->g_off; a.eps = d->eps; a.w_offset = d->w_offset;
   a.w = d->w; a.o = d->o; a.out_frag = d->out_frag; a.groups = d->groups < 1 ? 1 : d->groups;
-  TNX_REQUIRE(d->W % a.groups == 0 && (d->gate_first || a.groups == 1), "gated_norm: the row does not divide into %d parts", a.groups);
+  TNX_REQUIRE(d->W % a.groups == 0 && a.groups <= 1024, "gated_norm: the row does not divide into %d parts, or into more than 1024", a.groups);
   if (d->gate_first)
     return d->dtype == TNX_BF16 ? launch_gate_first(as_stream(stream), d->M, a, row_src<uint16_t>(d->g), (uint16_t*)d->out)
                                 : launch_gate_first(as_stream(stream), d->M, a, row_src<float>(d->g), (float*)d->out);

@@ -42,6 +42,7 @@ struct LHArgs {
   int variant;
   const int32_t* step_ptr;
   int logits_fp32;   // keep the fp32 accumulator as the logit (reference mode)
+  float softcap;     // > 0: softcap * tanh(acc / softcap), before any rounding
 };
 
 constexpr float kNegInf = -__builtin_inff();
@@ -151,7 +152,8 @@ __global__ __launch_bounds__(DENSE && NT == 2 ? 512 : 256) void lmhead_kernel(co
       float raw[NT], l[NT];
 #pragma unroll
       for (int nt = 0; nt < NT; ++nt) {
-        raw[nt] = a.logits_fp32 ? acc[mt][nt][i] : rbf(acc[mt][nt][i]);
+        const float z = a.softcap > 0.f ? soft_cap_fast(acc[mt][nt][i], a.softcap) : acc[mt][nt][i];
+        raw[nt] = a.logits_fp32 ? z : rbf(z);
         l[nt] = ok[nt] ? __fdiv_rn(raw[nt], a.temperature) : kNegInf;
       }
       if (a.logits_out && rok) {  // raw model logits: no temperature, no forbidden mask
@@ -373,6 +375,7 @@ extern "C" int tnx_lmhead_logp(void* stream, const tnx_lmhead_desc* d) {
   a.part_ent = d->entropy ? d->part_entropy : nullptr;
   a.part_draw = nullptr; a.key0 = a.key1 = 0; a.variant = 0; a.step_ptr = nullptr;
   a.logits_fp32 = d->logits_fp32 != 0;
+  a.softcap = d->softcap;
   if (d->draw_id) {
     TNX_REQUIRE(d->part_draw && d->draw_step_ptr, "lmhead: the draw needs the part_draw workspace [M, n_vblocks, 3] and a step pointer");
     TNX_REQUIRE(d->draw_rng_variant == 0 || d->draw_rng_variant == 1, "lmhead: rng_variant must be 0 or 1");

@@ -566,6 +566,16 @@ void qgemm_wide_kernel(const QLArgs a, const WideHead h) {
       return;
     }
   }
+  if constexpr (PRE) {
+    if (h.part != nullptr && h.softcap > 0.f) {
+#pragma unroll
+      for (int rt = 0; rt < RT; ++rt)
+#pragma unroll
+        for (int cg = 0; cg < CG; ++cg)
+#pragma unroll
+          for (int i = 0; i < 16; ++i) acc[rt][cg][i] = soft_cap_fast(acc[rt][cg][i], h.softcap);
+    }
+  }
   const int cols = mul ? kWideCols / 2 : kWideCols;      // output columns of the work-group
   const int sld = cols + 8;
   const uint32_t stage = 0;   // 128 rows x (256 + 8) columns: over both tiles and into the table, all dead now

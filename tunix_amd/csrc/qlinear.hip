@@ -63,6 +63,7 @@ struct WideHead {
   int variant;
   const int32_t* step_ptr;
   int64_t rows_total;        // M of the whole call: the noise of element (row, v) is number row * V + v of M * V
+  float softcap;             // > 0: logits are softcap * tanh(acc / softcap) before they are rounded (dense heads)
 };
 
 __device__ __forceinline__ float silu_bf16(float g) {
@@ -975,6 +976,7 @@ int tnx_internal_wide_head(hipStream_t st, const tnx_lmhead_desc* d, float tempe
   if (dense) {
     if (!pre_ok || d->V % 16 != 0 || d->lora_rank > 0) return 1;
   } else {
+    if (d->softcap > 0.f) return 1;
     if (d->group < 32 || d->group % 32 != 0 || (d->group <= KTILE ? KTILE % d->group != 0 : d->group % KTILE != 0) ||
         d->D % d->group != 0)
       return 1;
@@ -994,7 +996,7 @@ int tnx_internal_wide_head(hipStream_t st, const tnx_lmhead_desc* d, float tempe
   // 128 x 128 head kernel re-reads them once per 128, as many bytes again as the weights.
   if (!wide_shape(a, dense ? 1 : 512)) return 1;
   a.y = nullptr;
-  WideHead h{d->part, part_ent, d->targets, nvb, temperature, d->logits_out, nullptr, 0u, 0u, 0, nullptr, d->M};
+  WideHead h{d->part, part_ent, d->targets, nvb, temperature, d->logits_out, nullptr, 0u, 0u, 0, nullptr, d->M, d->softcap};
   if (d->draw_id) {
     h.part_draw = d->part_draw; h.key0 = d->draw_key0; h.key1 = d->draw_key1; h.variant = d->draw_rng_variant;
     h.step_ptr = d->draw_step_ptr;

@@ -101,10 +101,10 @@ __global__ __launch_bounds__(256) void short_conv_vec_kernel(const ConvArgs a, c
 // ring[b, (col + t) % slots, :] = rows of the last min(T, slots) tokens
 template <typename T>
 __global__ __launch_bounds__(256) void ring_write_kernel(int64_t Tn, int64_t C, int64_t off, int slots, const int32_t* col_ptr,
-                                                         const RowSrc<T> src, T* ring) {
+                                                         int64_t t0, const RowSrc<T> src, T* ring) {
   const int64_t c = (int64_t)blockIdx.x * 256 + threadIdx.x, b = blockIdx.z, t = Tn - 1 - blockIdx.y;
   if (c >= C) return;
-  st_elem(ring, (b * slots + (*col_ptr + t) % slots) * C + c, src.get(b * Tn + t, off + c));
+  st_elem(ring, (b * slots + (*col_ptr + t0 + t) % slots) * C + c, src.get(b * Tn + t, off + c));
 }
 
 // ---- the recurrence -----------------------------------------------------------------------------
@@ -624,17 +624,17 @@ extern "C" int tnx_short_conv(void* stream, const tnx_short_conv_desc* d) {
 }
 
 extern "C" int tnx_ring_write(void* stream, int dtype, const tnx_rows_src* y, int64_t off, int64_t B, int64_t T, int64_t C, int slots,
-                              const int32_t* col_ptr, void* ring) {
+                              const int32_t* col_ptr, int64_t t0, void* ring) {
   TNX_REQUIRE(y && src_given(*y) && col_ptr && ring, "ring_write: null pointer");
-  TNX_REQUIRE(B > 0 && B <= 65535 && T > 0 && C > 0 && slots > 0 && slots <= 65535 && off >= 0, "ring_write: bad shape");
+  TNX_REQUIRE(B > 0 && B <= 65535 && T > 0 && C > 0 && slots > 0 && slots <= 65535 && off >= 0 && t0 >= 0, "ring_write: bad shape");
   TNX_REQUIRE(dtype == TNX_BF16 || dtype == TNX_F32, "ring_write: bad dtype %d", dtype);
   const dim3 grid((unsigned)cdiv(C, 256), (unsigned)(T < slots ? T : slots), (unsigned)B);
   if (dtype == TNX_BF16) {
     const RowSrc<uint16_t> s{(const uint16_t*)y->y, y->ws, y->split_k, y->plane, y->ld};
-    hipLaunchKernelGGL(ring_write_kernel<uint16_t>, grid, dim3(256), 0, as_stream(stream), T, C, off, slots, col_ptr, s, (uint16_t*)ring);
+    hipLaunchKernelGGL(ring_write_kernel<uint16_t>, grid, dim3(256), 0, as_stream(stream), T, C, off, slots, col_ptr, t0, s, (uint16_t*)ring);
   } else {
     const RowSrc<float> s{(const float*)y->y, y->ws, y->split_k, y->plane, y->ld};
-    hipLaunchKernelGGL(ring_write_kernel<float>, grid, dim3(256), 0, as_stream(stream), T, C, off, slots, col_ptr, s, (float*)ring);
+    hipLaunchKernelGGL(ring_write_kernel<float>, grid, dim3(256), 0, as_stream(stream), T, C, off, slots, col_ptr, t0, s, (float*)ring);
   }
   TNX_CHECK_LAUNCH("ring_write");
   return TNX_OK;

@@ -67,7 +67,8 @@ def create_dummy_weights(cfg: ModelConfig, seed: int = 0, device="cpu", scale: f
 
 def create_stack_weights(cfg: StackConfig, seed: int = 0, device="cpu", scale: float | None = None) -> dict:
   """Random weights of a layer-list decoder, by file name: linears ~ N(0, 1) / sqrt(inputs) (or
-  `scale`), norm weights near zero, or around one where they are not stored around zero, sinks ~ N(0, 1)."""
+  `scale`), norm weights near zero, or around one where they are not stored around zero, sinks ~ N(0, 1), head mixtures
+  around the identity."""
   dev = torch.device(device)
   gen = torch.Generator(device=dev)
   gen.manual_seed(seed)
@@ -76,9 +77,11 @@ def create_stack_weights(cfg: StackConfig, seed: int = 0, device="cpu", scale: f
     t = torch.randn(*shape, generator=gen, device=dev, dtype=torch.float32)
     if name.endswith(("mix.sink", "mix.dt_bias")):
       pass
+    elif name.endswith(".talk"):
+      t = torch.eye(shape[0], device=dev) + t * (0.3 * shape[0] ** -0.5)
     elif name.endswith("mix.A_log"):
       t = 0.5 * t + 0.5
-    elif name.endswith(("mix.norm", "mix.D", "dq.norm", "dkv.norm")) or (not cfg.pre_norm and "norm" in name):
+    elif name.endswith(("mix.norm", "mix.D", "dq.norm", "dkv.norm")) or (cfg.norm_offset == 0.0 and ("norm" in name or name.endswith(".out"))):
       t = 1.0 + 0.1 * t
     elif name.endswith(".shift"):
       t = 0.5 + 0.2 * t

@@ -311,10 +311,10 @@ def dense_linear(desc: L.DenseDesc):
   L.check(L.lib().tnx_dense_linear(_stream(), C.byref(desc)), "tnx_dense_linear")
 
 
-def embed_rows(table, ids, col_ptr, B, T, V, D, x, cat=None, cat_off=0, cat_frag=False):
-  """x fp32 [B*T, D] = rows of `table` [V, D]; cat: a second copy in the table's dtype."""
+def embed_rows(table, ids, col_ptr, B, T, V, D, x, cat=None, cat_off=0, cat_frag=False, scale=1.0):
+  """x fp32 [B*T, D] = scaled rows of `table` [V, D]; cat: a second, unscaled copy in the table's dtype."""
   L.check(L.lib().tnx_embed_rows(_stream(), DTYPES[table.dtype], _ptr(table), V, D, _ptr(ids), ids.shape[1],
-                                 _ptr(col_ptr), B, T, _ptr(x), _ptr(cat), 0 if cat is None else cat.shape[1], cat_off,
+                                 _ptr(col_ptr), B, T, float(scale), _ptr(x), _ptr(cat), 0 if cat is None else cat.shape[1], cat_off,
                                  1 if cat_frag else 0), "tnx_embed_rows")
 
 
@@ -376,10 +376,10 @@ def short_conv(desc: L.ShortConvDesc):
   L.check(L.lib().tnx_short_conv(_stream(), C.byref(desc)), "tnx_short_conv")
 
 
-def ring_write(src: L.RowsSrc, off, B, T, col_ptr, ring):
-  """The last min(T, slots) rows of every sequence into ring [B, slots, width]."""
+def ring_write(src: L.RowsSrc, off, B, T, col_ptr, ring, t0=0):
+  """The last min(T, slots) rows of every sequence into ring [B, slots, width]; the first row belongs to column col + t0."""
   L.check(L.lib().tnx_ring_write(_stream(), DTYPES[ring.dtype], C.byref(src), off, B, T, ring.shape[2], ring.shape[1],
-                                 _ptr(col_ptr), _ptr(ring)), "tnx_ring_write")
+                                 _ptr(col_ptr), t0, _ptr(ring)), "tnx_ring_write")
 
 
 def ssd_step_ok(N, P) -> bool:
@@ -424,6 +424,40 @@ def latent_attn(desc: L.LatentAttnDesc):
 
 def gate_mul(desc: L.GateMulDesc):
   L.check(L.lib().tnx_gate_mul(_stream(), C.byref(desc)), "tnx_gate_mul")
+
+
+def parallel_step(desc: L.ParallelStepDesc):
+  L.check(L.lib().tnx_parallel_step(_stream(), C.byref(desc)), "tnx_parallel_step")
+
+
+def conv_kvwrite(desc: L.ConvKvDesc):
+  L.check(L.lib().tnx_conv_kvwrite(_stream(), C.byref(desc)), "tnx_conv_kvwrite")
+
+
+def mixed_attn_ok(T, S, H, G, dkp, dvp) -> bool:
+  return bool(L.lib().tnx_mixed_attn_ok(T, S, H, G, dkp, dvp))
+
+
+def mixed_attn_ws_bytes(B, T, S, H, dvp, kv_chunk) -> int:
+  return int(L.lib().tnx_mixed_attn_ws_bytes(B, T, S, H, dvp, kv_chunk))
+
+
+def mixed_attn(desc: L.MixedAttnDesc):
+  L.check(L.lib().tnx_mixed_attn(_stream(), C.byref(desc)), "tnx_mixed_attn")
+
+
+def memory_ws_bytes(B, T, H, dk, dv) -> int:
+  return int(L.lib().tnx_memory_ws_bytes(B, T, H, dk, dv))
+
+
+def memory(desc: L.MemoryDesc):
+  L.check(L.lib().tnx_memory(_stream(), C.byref(desc)), "tnx_memory")
+
+
+def soft_cap(z: torch.Tensor, cap: float):
+  """z <- cap tanh(z / cap), in place."""
+  _expect(z, torch.float32, "soft_cap")
+  L.check(L.lib().tnx_soft_cap(_stream(), _ptr(z), z.numel(), float(cap)), "tnx_soft_cap")
 
 
 def logits_stats(desc: L.LogitsDesc):

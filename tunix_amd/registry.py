@@ -42,6 +42,7 @@ ARCHITECTURES: dict[str, Architecture] = {
     "gemma3": _QLORA,
     "Nunezen": _stack(config.nunezen_from_dict),
     "Lapevik": _stack(config.lapevik_from_dict),
+    "Kuzezen": _stack(config.kuzezen_from_dict),
 }
 
 

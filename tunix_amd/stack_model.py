@@ -16,7 +16,7 @@ import torch
 from . import _lib as L
 from . import ops
 from .cache import KVSpec, LatentSpec, PartsSpec, RingSpec, SequenceCache, StateSpec
-from .config import AttentionMixer, ExpertsMlp, LatentMixer, LightningMixer, SsdMixer, StackConfig
+from .config import AttentionMixer, ExpertsMlp, LatentMixer, LightningMixer, MemoryMixer, MixedAttentionMixer, ParallelMixer, SsdMixer, StackConfig
 from .model import HeadRunner
 
 
@@ -95,6 +95,13 @@ class LinearBank:
     return sum(f.nbytes() for f in self.linears)
 
 
+class LinearPart:
+  """Some members of a projection, where a layer reads only them."""
+
+  def __init__(self, linear: DenseLinear, first: int, count: int):
+    self.linear, self.offsets = linear, linear.offsets[first:first + count]
+
+
 class StackModel:
   """Weights of one layer-list decoder on one GPU."""
 
@@ -111,6 +118,7 @@ class StackModel:
     self.embed = torch.zeros(V, D, dtype=dtype, device=dev)
     self.final_norm = vec("final.norm")
     self.linears: dict[str, list[DenseLinear]] = {}    # the projections a weight takes part in
+    self.transposed: set[str] = set()                  # vectors kept as [taps, channels]
     self.vectors: dict[str, torch.Tensor] = {"final.norm": self.final_norm}
 
     def linear(members, paired=False, transpose=False):
@@ -123,19 +131,31 @@ class StackModel:
       self.vectors[name] = vec(name)
       return self.vectors[name]
 
+    def taps(name, buf=None):
+      """A convolution's weights [channels, taps] as [taps, channels], of their own or in given columns."""
+      t = vec(name).T
+      if buf is None:
+        buf = torch.empty(t.shape, dtype=torch.float32, device=dev)
+      buf.copy_(t)
+      self.vectors[name] = buf
+      self.transposed.add(name)
+      return buf
+
     self.embed_norm = vector("embed.norm") if cfg.embed_norm else None
-    self.loop_in = linear(["loop.in"]) if cfg.loop is not None else None
+    looped = cfg.loop is not None
+    self.loop_in = linear(["loop.in"]) if looped and not cfg.loop.step else None
+    self.loop_step = vector("loop.step") if looped and cfg.loop.step else None
     self.layers = []
     for i, spec in enumerate(cfg.layers):
       p, m = f"l{i}.", spec.mixer
-      ly = {"spec": spec, "norm1": vector(p + "norm1") if cfg.pre_norm else None, "post1": vector(p + cfg.post_norm(1))}
+      ly = {"spec": spec, "norm1": vector(p + "norm1") if cfg.pre_norm else None, "post1": None if cfg.parallel else vector(p + cfg.post_norm(1))}
       if cfg.token_shift:
         ly["shift"] = vector(p + "shift")
       if isinstance(m, SsdMixer):
         x = p + "mix."
         ly["in"] = linear([(x + "in", 0, m.inner), (x + "in", m.inner, m.inner + m.channels),
                            (x + "in", m.inner + m.channels, m.inner + m.channels + m.heads)])
-        self.vectors[x + "conv"] = ly["conv"] = vec(x + "conv").T.contiguous()      # [taps, channels]
+        ly["conv"] = taps(x + "conv")
         for key, name in (("conv_b", "conv.b"), ("dt_bias", "dt_bias"), ("A_log", "A_log"), ("D", "D"), ("norm", "norm")):
           ly[key] = vector(x + name)
       elif isinstance(m, LatentMixer):
@@ -148,6 +168,21 @@ class StackModel:
         ly["q_norm"], ly["kv_norm"] = vector(x + "dq.norm"), vector(x + "dkv.norm")
         freq = np.float64(m.rot_base) ** (-2.0 * np.arange(m.rot_dim // 2) / max(m.rot_dim, 1))
         ly["inv_freq"] = torch.from_numpy(freq.astype(np.float32)).to(dev)
+      elif isinstance(m, ParallelMixer):
+        # everything that reads the input is one projection, but the memory's gates: they stay fp32
+        a, b = p + "mix.left.", p + "mix.right."
+        f = ly["in"] = linear([x + n for x in (a, b) for n in "qkvg"])
+        left = {"spec": type(spec)(m.left, None), "in": LinearPart(f, 0, 4), "out": linear([a + "o"]), "post": vector(a + "out"), "talk": vector(a + "talk")}
+        n_conv = f.offsets[3] - f.offsets[0]
+        left["conv"] = torch.zeros(m.left.conv, n_conv, dtype=torch.float32, device=dev)
+        for n, off, size in zip("qkv", f.offsets, f.shapes):
+          taps(a + n + ".conv", left["conv"][:, off:off + size[0]])
+        right = {"spec": type(spec)(m.right, None), "in": LinearPart(f, 4, 4), "out": linear([b + "o"]), "post": vector(b + "out"), "gates": linear([b + "i", b + "f"]),
+                 "bias_i": vector(b + "i.b"), "bias_f": vector(b + "f.b"), "norm": vector(b + "norm")}
+        ly["left"], ly["right"] = left, right
+        ly["canon1"] = taps(p + "canon1")
+        if spec.mlp is not None:
+          ly["canon2"] = taps(p + "canon2")
       elif isinstance(m, AttentionMixer):
         ly["in"] = linear([p + "mix.q", p + "mix.k", p + "mix.v"])
         ly["sink"] = vector(p + "mix.sink") if m.sink else None
@@ -157,8 +192,9 @@ class StackModel:
         ly["in"] = linear([p + "mix.q", p + "mix.k", p + "mix.v", p + "mix.g"])
         ly["norm"] = vector(p + "mix.norm")
         ly["decay"] = torch.tensor(m.decay, dtype=torch.float32, device=dev)
-      ly["out"] = linear([p + "mix.o"])
-      if spec.mlp is not None:
+      if not isinstance(m, ParallelMixer):
+        ly["out"] = linear([p + "mix.o"])
+      if spec.mlp is not None and not cfg.parallel:
         ly["norm2"], ly["post2"] = vector(p + "norm2") if cfg.pre_norm else None, vector(p + cfg.post_norm(2))
       if isinstance(spec.mlp, ExpertsMlp):
         e = [p + f"mlp.e{j}." for j in range(spec.mlp.experts)]
@@ -169,25 +205,31 @@ class StackModel:
         ly["gu"] = linear([p + "mlp.gate", p + "mlp.up"], paired=True)
         ly["down"] = linear([p + "mlp.down"])
       self.layers.append(ly)
-    # the head is the embedding table: through the statistics head when its shape is one that
-    # kernel takes, else as a plain linear into fp32 logits
-    self.head = self.head_w = self.head_expanded = None
+    # the head (the embedding table, or a weight of its own) runs through the statistics head when its shape is
+    # one that kernel takes, else as a plain linear into fp32 logits
+    self.head = self.head_expanded = self.head_linear = None
+    self.head_w = self.embed if cfg.tied_head else torch.zeros_like(self.embed)
     self.block_head = dtype == torch.bfloat16 and D % 128 == 0 and V % 16 == 0
-    self.head_linear = None
-    self._load_embed(weights["embed"])
+    self._load_tables(weights)
     torch.cuda.synchronize(dev)
 
-  def _load_embed(self, table):
-    self.embed.copy_(table.to(self.device, self.dtype))
+  def _load_tables(self, weights: dict):
+    """The embedding table and the head, as far as `weights` has them."""
+    head = "embed" if self.cfg.tied_head else "head"
+    for name, table in (("embed", self.embed), (head, self.head_w)):
+      if name in weights:
+        table.copy_(weights[name].to(self.device, self.dtype))
+    if head not in weights:
+      return
     if self.block_head:
       if self.head_expanded is None:
-        self.head_expanded = ops.dense_expand(self.embed)
+        self.head_expanded = ops.dense_expand(self.head_w)
       else:
-        self.head_expanded.copy_(ops.dense_expand(self.embed))
+        self.head_expanded.copy_(ops.dense_expand(self.head_w))
     elif self.head_linear is None:
-      self.head_linear = DenseLinear(["embed"], {"embed": self.embed}, self.dtype, self.device)
+      self.head_linear = DenseLinear([head], {head: self.head_w}, self.dtype, self.device)
     else:
-      self.head_linear.load({"embed": self.embed})
+      self.head_linear.load({head: self.head_w})
 
   def _check_names(self, weights: dict, complete: bool):
     extra = sorted(set(weights) - set(self.shapes))
@@ -210,6 +252,13 @@ class StackModel:
         spec = PartsSpec((("state", StateSpec(m.heads, m.state, m.vdim)), ("conv", RingSpec(m.conv, m.channels, self.dtype))))
       elif isinstance(m, LatentMixer):
         spec = LatentSpec(ops.latent_row(m.kv_rank, m.rot_dim, self.dtype), self.dtype)
+      elif isinstance(m, ParallelMixer):
+        a, b = m.left, m.right
+        ring = self.layers[i]["left"]["conv"]
+        left = PartsSpec((("kv", KVSpec(a.kv_heads, ops.sink_attn_pad(a.dim, True, self.dtype), ops.sink_attn_pad(a.vdim, True, self.dtype), self.dtype)),
+                          ("conv", RingSpec(a.conv, ring.shape[1], self.dtype))))
+        right = PartsSpec((("state", StateSpec(b.heads, b.dim, b.vdim)), ("sum", StateSpec(b.heads, b.dim, 1)), ("top", StateSpec(b.heads, 1, 1))))
+        spec = PartsSpec((("left", left), ("right", right), ("input", RingSpec(max(self.cfg.input_conv - 1, 1), self.cfg.embed_dim, torch.float32))))
       else:
         spec = StateSpec(m.heads, m.dim, m.vdim)
       if self.cfg.token_shift:
@@ -239,9 +288,8 @@ class StackModel:
     for n, t in new_state.items():
       if n in self.vectors:
         t = t.to(self.device, torch.float32)
-        self.vectors[n].copy_(t.T if t.dim() == 2 else t)
-    if "embed" in new_state:
-      self._load_embed(new_state["embed"])
+        self.vectors[n].copy_(t.T if n in self.transposed else t)
+    self._load_tables(new_state)
     torch.cuda.synchronize(self.device)
 
   def weight_bytes(self) -> dict:
@@ -249,9 +297,10 @@ class StackModel:
     n = 0
     for i, begins in self.cfg.layer_runs:
       ly = self.layers[i]
-      n += sum(ly[k].nbytes() for k in ("in", "uq", "absorb_k", "absorb_v", "out", "router", "gu", "down") if k in ly)
-      n += self.loop_in.nbytes() if begins else 0
-    return {"dense": n, "head": self.embed.numel() * self.embed.element_size()}
+      n += sum(part[k].nbytes() for part in (ly, ly.get("left", {}), ly.get("right", {}))
+               for k in ("in", "uq", "absorb_k", "absorb_v", "out", "router", "gates", "gu", "down") if hasattr(part.get(k), "nbytes"))
+      n += self.loop_in.nbytes() if begins and self.loop_in is not None else 0
+    return {"dense": n, "head": self.head_w.numel() * self.head_w.element_size()}
 
 
 class StackRunner(HeadRunner):
@@ -273,23 +322,29 @@ class StackRunner(HeadRunner):
     self._bufs: dict = {}
     D = cfg.embed_dim
     self.x = torch.empty(M, D, dtype=torch.float32, device=dev)
-    # a token shift reads the row in front of a row: over several tokens the new rows go to a second buffer
-    self.x_next = torch.empty_like(self.x) if cfg.token_shift and T > 1 else None
+    # a token shift or an input convolution reads the rows in front of a row: over several tokens the new rows go to a
+    # second buffer
+    self.x_next = torch.empty_like(self.x) if (cfg.token_shift or cfg.input_conv > 1) and T > 1 else None
+    self.tail = torch.empty(B * min(T, max(cfg.input_conv - 1, 1)), D, dtype=torch.float32, device=dev) if cfg.input_conv > 1 and T > 1 else None
     # the final-normed rows (row-major, zero columns behind the model width)
     width = D if model.block_head else model.Dp
     self.xn = torch.zeros(M, width, dtype=self.dtype, device=dev)
     self.split_k_override = dict(split_k_override or {})
     n_light = n_attn = n_routes = n_experts = 1
-    n_y, n_ws = [1, 1], [1, 1]     # a projection's output, and that of one which runs while the first is still read
+    n_y, n_ws = [1, 1, 1], [1, 1, 1]     # a projection's output, and those of some which run while the first is still read
     for i, begins in cfg.layer_runs:
       ly = model.layers[i]
       m = ly["spec"].mixer
-      for key, slot in (("in", 0), ("out", 0), ("router", 0), ("gu", 0), ("down", 0), ("uq", 1), ("ukv", 1)):
-        f = ly.get(key)
+      mlp_slot = 2 if cfg.parallel else 0
+      uses = [(ly, k, s) for k, s in (("in", 0), ("out", 0), ("router", 0), ("gu", mlp_slot), ("down", mlp_slot), ("uq", 1), ("ukv", 1))]
+      if cfg.parallel:
+        uses += [(ly["right"], "gates", 1), (ly["left"], "out", 0), (ly["right"], "out", 1)]
+      for part, key, slot in uses:
+        f = part.get(key)
         if isinstance(f, DenseLinear):
           n_y[slot] = max(n_y[slot], M * f.N)
-          n_ws[slot] = max(n_ws[slot], self._split(f) * M * f.N if self._split(f) > 1 or key == "router" else 1)
-      if begins:
+          n_ws[slot] = max(n_ws[slot], self._split(f) * M * f.N if self._split(f) > 1 or key in ("router", "gates") else 1)
+      if begins and model.loop_in is not None:
         n_ws[0] = max(n_ws[0], self._split(model.loop_in) * M * model.loop_in.N)
       if isinstance(ly["spec"].mlp, ExpertsMlp):
         e = ly["spec"].mlp
@@ -303,6 +358,10 @@ class StackRunner(HeadRunner):
       elif isinstance(m, LatentMixer):
         if self.dtype == torch.bfloat16:
           n_attn = max(n_attn, ops.latent_attn_ws_bytes(B, T, S, m.heads, m.kv_rank, self._latent_chunk(m)) // 4)
+      elif isinstance(m, ParallelMixer):
+        a, r = m.left, m.right
+        n_light = max([n_light] + [ops.memory_ws_bytes(b, T, r.heads, r.dim, r.vdim) // 4 for b in range(1, B + 1)])
+        n_attn = max(n_attn, ops.mixed_attn_ws_bytes(B, T, S, a.heads, ops.sink_attn_pad(a.vdim, True, self.dtype), self._mixed_chunk(kv_chunk)) // 4)
       else:
         n_attn = max(n_attn, ops.sink_attn_ws_bytes(B, T, S, m.heads, ops.sink_attn_pad(m.vdim, True, self.dtype),
                                                     self._kv_chunk(m, kv_chunk)) // 4)
@@ -354,6 +413,15 @@ class StackRunner(HeadRunner):
       return 0
     chunk = max(256, _up(math.ceil(self.S / math.ceil(256 / groups)), 64))
     return 0 if chunk >= self.S else chunk
+
+  def _mixed_chunk(self, given) -> int:
+    """Keys of a work-group in a decode step of mixed attention: as many as leave about two work-groups per compute unit."""
+    if given:
+      return given
+    for chunk in (256, 128):
+      if self.B * math.ceil(self.S / chunk) >= 512:
+        return chunk
+    return 64
 
   def _split(self, f: DenseLinear) -> int:
     """k split of a few-row linear whose reader sums fp32 planes."""
@@ -463,14 +531,114 @@ class StackRunner(HeadRunner):
     return o
 
   def gate(self, ly, o, src, M: int) -> torch.Tensor:
-    """norm(o) . weight * sigmoid(gate columns of the projection)."""
-    out = self._buf("gated", ly["out"].Kp)
+    """norm(o) . weight * sigmoid(gate columns of the projection); a memory's heads are normed on their own."""
+    m, out = ly["spec"].mixer, self._buf("gated", ly["out"].Kp)
     d = L.GatedNormDesc()
-    d.M, d.W, d.dtype, d.eps, d.w_offset = M, o.shape[1], self.code, self.cfg.norm_eps, 0.0
+    d.M, d.W, d.dtype, d.eps, d.w_offset, d.groups = M, o.shape[1], self.code, self.cfg.norm_eps, 0.0, m.heads if isinstance(m, MemoryMixer) else 1
     d.o, d.o_ld, d.g, d.g_off, d.w = o.data_ptr(), o.shape[1], src, ly["in"].offsets[3], ly["norm"].data_ptr()
     d.out, d.out_ld, d.out_frag = out.data_ptr(), out.shape[1], 1 if self.frag else 0
     ops.gated_norm(d)
     return out
+
+  # parallel layers
+  def parallel_step(self, pending, ly, out, out2, at, entry, add=None):
+    """x takes the pending sublayers (rows of the left and right mixer and of the feed-forward with their layer, or None)
+    and the vector `add`; out, out2 = norm(x) behind the layer's input convolutions.  ly None: out = the final norm of x."""
+    cfg, (col_ptr, starts, B, T) = self.cfg, at
+    d = L.ParallelStepDesc()
+    d.M, d.D, d.dtype, d.eps, d.mult, d.B, d.T = B * T, cfg.embed_dim, self.code, cfg.norm_eps, cfg.residual_mult, B, T
+    if pending is not None:
+      sides, mlp, before = pending
+      for i, (side, rows) in enumerate(zip(("left", "right"), sides)):
+        d.y[i], d.w_post[i], d.y_scale[i] = rows, before[side]["post"].data_ptr(), 0.5
+      d.n_in = 2
+      if mlp is not None:
+        d.y[2], d.y_scale[2], d.n_in = mlp, 1.0, 3
+    moved = ly is not None and cfg.input_conv > 1 and T > 1
+    d.x, d.add = self.x.data_ptr(), None if add is None else add.data_ptr()
+    if d.n_in or add is not None:
+      d.x_out = (self.x_next if moved else self.x).data_ptr()
+    d.out1, d.out_ld, d.out_frag = out.data_ptr(), out.shape[1], 1 if self.frag and ly is not None else 0
+    if ly is None:
+      d.w_next = self.model.final_norm.data_ptr()
+    else:
+      ring = entry["input"].r
+      d.w_next, d.conv1, d.taps, d.slots, d.ring = ly["norm1"].data_ptr(), ly["canon1"].data_ptr(), cfg.input_conv, ring.shape[1], ring.data_ptr()
+      if "canon2" in ly:
+        d.conv2, d.out2 = ly["canon2"].data_ptr(), out2.data_ptr()
+      d.starts, d.col_ptr = starts.data_ptr(), col_ptr.data_ptr()
+      if moved:
+        d.tail = self.tail.data_ptr()
+    ops.parallel_step(d)
+    if moved:
+      if d.x_out:
+        self.x, self.x_next = self.x_next, self.x
+      keep = min(T, cfg.input_conv - 1)
+      ops.ring_write(ops.rows_src(y=self.tail, ld=cfg.embed_dim), 0, B, keep, col_ptr, ring, t0=T - keep)
+
+  def conv_kv(self, ly, src, entry, col_ptr, starts, B, T) -> torch.Tensor:
+    """Convolution of q, k and v, query temperature, value norm, cache write; returns q."""
+    m, f, kv, ring = ly["spec"].mixer, ly["in"], entry["kv"], entry["conv"].r
+    dkp, dvp = kv.k.shape[3], kv.v.shape[3]
+    q = self._buf("q", m.heads * dkp)
+    d = L.ConvKvDesc()
+    d.B, d.T, d.S, d.H, d.G = B, T, kv.k.shape[2], m.heads, m.kv_heads
+    d.dk, d.dv, d.dkp, d.dvp, d.taps, d.slots, d.dtype = m.dim, m.vdim, dkp, dvp, m.conv, ring.shape[1], self.code
+    d.temp_coef, d.temp_every, d.eps, d.value_norm = m.temp_coef, m.temp_every, self.cfg.norm_eps, 1 if m.value_norm else 0
+    d.y, d.off, d.C = src, f.offsets[0], ring.shape[2]
+    d.q_off, d.k_off, d.v_off = (o - f.offsets[0] for o in f.offsets[:3])
+    d.w, d.ring, d.starts, d.col_ptr = ly["conv"].data_ptr(), ring.data_ptr(), starts.data_ptr(), col_ptr.data_ptr()
+    d.q_out, d.kcache, d.vcache = q.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr()
+    ops.conv_kvwrite(d)
+    if T > 1:
+      ops.ring_write(src, f.offsets[0], B, T, col_ptr, ring)
+    return q
+
+  def mixed_attend(self, ly, q, src, entry, col_ptr, starts, B, T) -> torch.Tensor:
+    """Attention with mixed heads and the output gate (the projection's fourth part)."""
+    m, kv = ly["spec"].mixer, entry["kv"]
+    out = self._buf("mixed", ly["out"].Kp)
+    d = L.MixedAttnDesc()
+    d.B, d.T, d.S, d.H, d.G = B, T, kv.k.shape[2], m.heads, m.kv_heads
+    d.dk, d.dv, d.dkp, d.dvp, d.scale, d.dtype = m.dim, m.vdim, kv.k.shape[3], kv.v.shape[3], m.scale, self.code
+    d.q, d.kcache, d.vcache, d.talk = q.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr(), ly["talk"].data_ptr()
+    d.starts, d.col_ptr, d.kv_chunk, d.ws = starts.data_ptr(), col_ptr.data_ptr(), self._mixed_chunk(self.kv_chunk_arg), self.attn_ws.data_ptr()
+    d.gate, d.g_off = src, ly["in"].offsets[3]
+    d.out, d.out_ld, d.out_frag = out.data_ptr(), out.shape[1], 1 if self.frag else 0
+    ops.mixed_attn(d)
+    return out
+
+  def remember(self, ly, src, gates, entry, col_ptr, starts, B, T) -> torch.Tensor:
+    """The matrix memory of a projection's rows: fp32 [rows, heads * vdim]."""
+    m, f = ly["spec"].mixer, ly["in"]
+    o = self._buf("state_out", m.heads * m.vdim, torch.float32)
+    d = L.MemoryDesc()
+    d.B, d.T, d.H, d.dk, d.dv, d.dtype, d.q_scale, d.cap = B, T, m.heads, m.dim, m.vdim, self.code, m.dim ** -0.5, m.gate_cap
+    d.y, d.q_off, d.k_off, d.v_off = src, *f.offsets[:3]
+    d.gates, d.i_off, d.f_off = gates, *ly["gates"].offsets
+    d.bias_i, d.bias_f, d.starts, d.col_ptr = ly["bias_i"].data_ptr(), ly["bias_f"].data_ptr(), starts.data_ptr(), col_ptr.data_ptr()
+    d.state, d.sum, d.top = (entry[n].s.data_ptr() for n in ("state", "sum", "top"))
+    d.o, d.o_ld, d.ws = o.data_ptr(), o.shape[1], self.light_ws.data_ptr()
+    ops.memory(d)
+    return o
+
+  def fp32_rows(self, f: DenseLinear, x, M: int, slot: int) -> L.RowsSrc:
+    """A projection whose rows stay fp32 (finished, or planes)."""
+    src = self.linear(f, x, M, fp32_out=True, slot=slot)
+    if src.split_k <= 1 and src.ws:
+      src.y = src.ws
+    return src
+
+  def parallel_sublayers(self, ly, h, h2, entry, col_ptr, starts, B, T):
+    """Both mixers of h and the feed-forward of h2, as `parallel_step` takes them."""
+    M, at, left, right = B * T, (col_ptr, starts, B, T), ly["left"], ly["right"]
+    src = self.linear(ly["in"], h, M)
+    gates = self.fp32_rows(right["gates"], h, M, slot=1)
+    a = self.mixed_attend(left, self.conv_kv(left, src, entry["left"], *at), src, entry["left"], *at)
+    b = self.gate(right, self.remember(right, src, gates, entry["right"], *at), src, M)
+    sides = self.linear(left["out"], a, M), self.linear(right["out"], b, M, slot=1)
+    mlp = self.linear(ly["down"], self.gate_up(ly, h2, M, slot=2), M, slot=2) if "gu" in ly else None
+    return sides, mlp, ly
 
   # state-space duality
   def convolve(self, ly, src, entry, col_ptr, starts, B, T) -> torch.Tensor:
@@ -624,9 +792,7 @@ class StackRunner(HeadRunner):
   def route(self, ly, h, M: int):
     """Chooses every row's experts and sorts the routes by expert."""
     e = ly["spec"].mlp
-    src = self.linear(ly["router"], h, M, fp32_out=True)
-    if src.split_k <= 1 and src.ws:
-      src.y = src.ws
+    src = self.fp32_rows(ly["router"], h, M, slot=0)
     ids = self.topk_id[:M * e.top].view(M, e.top)
     ops.route_softmax(src, M, e.experts, e.top, self.topk_w, ids)
     ops.moe_sort_routes(ids, e.experts, self.counts, self.offsets, self.sorted_route)
@@ -665,12 +831,12 @@ class StackRunner(HeadRunner):
       return ("routes", self.experts_down(ly, self.experts_gate_up(ly, h, M), M), ly["post2"], self.topk_w, e.top)
     return ("add", self.linear(ly["down"], self.gate_up(ly, h, M), M), ly["post2"])
 
-  def gate_up(self, ly, h, M: int) -> torch.Tensor:
+  def gate_up(self, ly, h, M: int, slot: int = 0) -> torch.Tensor:
     f = ly["gu"]
     act = self._buf("act", ly["down"].Kp)
     if self.dtype == torch.float32:
-      self.linear(f, h, M)
-      ops.gelu_mul(self.y[0][:M * f.N].view(M, f.N), f.offsets[1], M, ly["spec"].mlp.ff, act)
+      self.linear(f, h, M, slot=slot)
+      ops.gelu_mul(self.y[slot][:M * f.N].view(M, f.N), f.offsets[1], M, ly["spec"].mlp.ff, act)
     else:
       d = L.DenseDesc()
       d.M, d.K, d.N, d.dtype = M, f.Kp, f.N, self.code
@@ -692,8 +858,10 @@ class StackRunner(HeadRunner):
     starts = self.no_starts if starts is None else starts
     D = cfg.embed_dim
     cat = None if m.loop_in is None else self._buf("cat", m.loop_in.Kp)
-    ops.embed_rows(m.embed, tokens, col_ptr, B, T, cfg.vocab_size, D, self.x, cat=cat, cat_off=D, cat_frag=self.frag)
+    ops.embed_rows(m.embed, tokens, col_ptr, B, T, cfg.vocab_size, D, self.x, cat=cat, cat_off=D, cat_frag=self.frag, scale=cfg.embed_scale)
     h = self._buf("h", m.Dp)
+    if cfg.parallel:
+      return self._forward_parallel(h, col_ptr, cache, B, T, starts)
     pending, behind_layer = None if m.embed_norm is None else ("norm", None, m.embed_norm), False
 
     def norm(w_next, out, frag, shift=None):
@@ -721,7 +889,30 @@ class StackRunner(HeadRunner):
     norm(m.final_norm, self.xn, False)
     return self.xn
 
+  def _forward_parallel(self, h, col_ptr, cache, B, T, starts):
+    m, cfg, at = self.model, self.cfg, (col_ptr, starts, B, T)
+    h2, pending, passes = self._buf("h2", m.Dp), None, 0
+    for (i, begins), entry in zip(cfg.layer_runs, cache.entries):
+      add = None
+      if begins:   # a pass of the loop: x <- x + the pass's vector
+        add, passes = m.loop_step[passes], passes + 1
+      if self.residual_sink is not None and pending is not None:   # (the layer's own result is asked for, without what comes ahead of the next)
+        self.parallel_step(pending, None, self.xn, None, at, None)
+        self.residual_sink(self.x[:B * T])
+        pending = None
+      self.parallel_step(pending, m.layers[i], h, h2, at, entry, add)
+      pending = self.parallel_sublayers(m.layers[i], h, h2, entry, *at)
+    self.parallel_step(pending, None, self.xn, None, at, None)
+    if self.residual_sink is not None:
+      self.residual_sink(self.x[:B * T])
+    return self.xn
+
   # ---- head ----------------------------------------------------------------------------------
+  def head_desc(self, *args, **kw) -> L.LmHeadDesc:
+    d = super().head_desc(*args, **kw)
+    d.softcap = self.cfg.logit_softcap
+    return d
+
   def run_head(self, x, rows, temperature=1.0, targets=None, best_id=None, best_logp=None, target_logp=None, lse=None,
                logits_out=None, forbidden=None, entropy=None, part_entropy=None, draw=None, logits_fp32=False):
     m = self.model
@@ -738,6 +929,8 @@ class StackRunner(HeadRunner):
     d.x, d.ldx, d.w, d.epilogue = x.data_ptr(), x.shape[1], f.w.data_ptr(), L.TNX_EPI_F32
     d.y, d.ldy, d.split_k = logits_out.data_ptr(), V, 1
     ops.dense_linear(d)
+    if self.cfg.logit_softcap > 0.0:
+      ops.soft_cap(logits_out[:rows], self.cfg.logit_softcap)
     s = L.LogitsDesc()
     s.M, s.V, s.logits, s.temperature = rows, V, logits_out.data_ptr(), float(temperature)
     if forbidden is not None:
