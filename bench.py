@@ -951,6 +951,43 @@ def expert_family_kernels(cfg, M, iters, dev):
   return out
 
 
+PREFILL_ROWS = 8      # sequences of the prefill group whose kernels are timed
+
+
+def measure_model(name, build, measure, size, ids, P, T, steps, iters):
+  """Prefill and decode throughput of a model over the prompts `ids` [B, P], and with `measure` the time of every kernel."""
+  import torch
+
+  from tunix_amd.generate import CacheConfig, Sampler
+  from tunix_amd.generate.sampler import _SamplingState
+  from tunix_amd.generate.utils import IdTokenizer
+  B, S = len(ids), P + T
+  model = build()
+  sampler = Sampler(model, IdTokenizer(model.cfg.vocab_size, pad_id=0, eos_id=1), CacheConfig(S))
+  prompts, ms, pre = [r for r in ids], [], []
+  for n in (4, 4, 4 + steps):
+    sampler(prompts, n, max_prompt_length=P, eos_tokens=[-1])
+    ms.append(sampler.last_stats["decode_ms"])
+    pre.append(sampler.last_stats["prefill_ms"])
+  d_ms = (ms[2] - ms[1]) / steps
+  r = {"prefill_tokens_per_s": round(B * P / (min(pre[1:]) * 1e-3)), "prefill_ms": round(min(pre[1:]), 2),
+       "decode_tokens_per_s": round(B / (d_ms * 1e-3)), "decode_ms_per_step": round(d_ms, 4)}
+  log(size, name, r)
+  if measure is not None:
+    st = _SamplingState(model, ids, S, S, 0, False, False)
+    st.starts.zero_()
+    r["decode_kernels"] = measure(model, model.new_runner(B, 1, S, 0), st, P + T // 2, iters)
+    del st
+    torch.cuda.empty_cache()
+    st = _SamplingState(model, ids[:PREFILL_ROWS], S, S, 0, False, False)
+    st.starts.zero_()
+    r["prefill_kernels"] = measure(model, model.new_runner(PREFILL_ROWS, P, S, 0, kv_chunk=0), st, P, max(2, iters // 4))
+    del st
+  del model, sampler
+  torch.cuda.empty_cache()
+  return r
+
+
 def lapevik_workload(size, iters, steps, kernels=True):
   """Prefill and decode of a Lapevik decoder with layers of a real model's size (random weights), beside a Nunezen
   decoder of the same width and a qwen3-family model with the same experts (int4), and the time of every kernel
@@ -959,9 +996,6 @@ def lapevik_workload(size, iters, steps, kernels=True):
   import torch
 
   from tunix_amd import config, dummy_model
-  from tunix_amd.generate import CacheConfig, Sampler
-  from tunix_amd.generate.sampler import _SamplingState
-  from tunix_amd.generate.utils import IdTokenizer
   from tunix_amd.model import QLoRAModel
   from tunix_amd.stack_model import StackModel
   dev = torch.device("cuda:0")
@@ -972,42 +1006,18 @@ def lapevik_workload(size, iters, steps, kernels=True):
   moe_cfg = config.qwen3_30b_a3b(num_layers=len(new_cfg.layers), vocab_size=new_cfg.vocab_size, embed_dim=width, hidden_dim=ff, num_heads=nH,
                                  num_kv_heads=nG, num_experts=E, num_experts_per_tok=top, lora_rank=0, lora_alpha=0.0)
   P, T = 1024, 256
-  S = P + T
   ids = np.random.Generator(np.random.PCG64(5)).integers(1, new_cfg.vocab_size, size=(B, P)).astype(np.int32)
   result = {"size": {"width": width, "ssd_heads": new_cfg.layers[0].mixer.heads, "latent_heads": H, "experts": E, "top": top,
                      "expert_width": ff, "batch": B, "prompt": P, "layers": len(new_cfg.layers)}}
   models = (("lapevik", lambda: StackModel(new_cfg, dummy_model.create_stack_weights(new_cfg, 1, dev), dev), lapevik_kernels),
             ("nunezen", lambda: StackModel(near_cfg, dummy_model.create_stack_weights(near_cfg, 1, dev), dev), stack_kernels),
             ("qwen3-family", lambda: QLoRAModel(moe_cfg, dummy_model.create_dummy_weights(moe_cfg, 1, dev), dev), None))
-  pb = 8      # rows of a prefill group: 8 x 1024 tokens
   for name, build, measure in models:
-    model = build()
-    sampler = Sampler(model, IdTokenizer(new_cfg.vocab_size, pad_id=0, eos_id=1), CacheConfig(S))
-    prompts, ms, pre = [r for r in ids], [], []
-    for n in (4, 4, 4 + steps):
-      sampler(prompts, n, max_prompt_length=P, eos_tokens=[-1])
-      ms.append(sampler.last_stats["decode_ms"])
-      pre.append(sampler.last_stats["prefill_ms"])
-    d_ms = (ms[2] - ms[1]) / steps
-    r = {"prefill_tokens_per_s": round(B * P / (min(pre[1:]) * 1e-3)), "prefill_ms": round(min(pre[1:]), 2),
-         "decode_tokens_per_s": round(B / (d_ms * 1e-3)), "decode_ms_per_step": round(d_ms, 4)}
-    log(size, name, r)
-    if kernels and measure is not None:
-      st = _SamplingState(model, ids, S, S, 0, False, False)
-      st.starts.zero_()
-      r["decode_kernels"] = measure(model, model.new_runner(B, 1, S, 0), st, P + T // 2, iters)
-      del st
-      torch.cuda.empty_cache()
-      stp = _SamplingState(model, ids[:pb], S, S, 0, False, False)
-      stp.starts.zero_()
-      r["prefill_kernels"] = measure(model, model.new_runner(pb, P, S, 0, kv_chunk=0), stp, P, max(2, iters // 4))
-      del stp
+    r = measure_model(name, build, measure if kernels else None, size, ids, P, T, steps, iters)
     result[name] = r
-    del model, sampler
-    torch.cuda.empty_cache()
     if kernels and measure is None:
       r["decode_kernels"] = expert_family_kernels(moe_cfg, B, iters, dev)
-      r["prefill_kernels"] = expert_family_kernels(moe_cfg, pb * P, max(2, iters // 4), dev)
+      r["prefill_kernels"] = expert_family_kernels(moe_cfg, PREFILL_ROWS * P, max(2, iters // 4), dev)
       torch.cuda.empty_cache()
   if kernels:
     for phase in ("decode_kernels", "prefill_kernels"):
@@ -1016,6 +1026,97 @@ def lapevik_workload(size, iters, steps, kernels=True):
         b = like[LAPEVIK_LIKE[k]]
         v["vs_like"] = round(v["times_roof"] / b["times_roof"], 2)
         log(f"  {size} {phase:16s} {k:34s} {v['us']:9.1f} us  {v['times_roof']:6.2f} x roof ({v['bound']})   {LAPEVIK_LIKE[k]}: "
+            f"{b['us']:9.1f} us  {b['times_roof']:6.2f} x ({b['bound']})   ratio {v['vs_like']}")
+  return result
+
+
+# the like kernel of each, of a Nunezen decoder
+KUZEZEN_LIKE = {
+    "linear in": "linear lightning in", "linear gates": "linear o", "linear attention out": "linear o", "linear memory out": "linear o",
+    "linear gate_up": "linear gate_up", "linear down": "linear down", "convolution + cache write": "rotation + cache write",
+    "mixed attention": "attention", "matrix memory": "lightning", "head norms + gate": "gated norm",
+    "norms + residual + norm + convolutions": "post-norm + residual + norm",
+}
+
+
+def kuzezen_kernels(model, runner, st, ctx, iters):
+  """Per-kernel times of a Kuzezen model's pass: T = runner.T tokens per row, the last of them at context `ctx`."""
+  import torch
+  B, T, M, D = runner.B, runner.T, runner.M, model.cfg.embed_dim
+  prompt = T > 1
+  col = torch.tensor([ctx - T], dtype=torch.int32, device=model.device)
+  at = (col, st.starts, B, T)
+  layers, first = range(len(model.layers)), {}
+  for (i, _), e in zip(model.cfg.layer_runs, st.cache.entries):
+    first.setdefault(i, e)
+  for e in first.values():
+    e["left"]["kv"].k.normal_()
+    e["left"]["kv"].v.normal_()
+  out = {}
+
+  def timed(name, fn, nbytes, flops=0.0):
+    out[name] = roof_row(in_turn([(lambda i=i: fn(model.layers[i], first[i])) for i in layers], iters), nbytes, flops)
+
+  def lin(name, pick, x, slot, n_out=None, fp32=False):
+    f = pick(model.layers[0])
+    timed(name, lambda ly, e: runner.linear(pick(ly), x, M, fp32_out=fp32, slot=slot), f.nbytes() + M * (f.K * 2 + f.N * (4 if fp32 else 2)), 2.0 * M * f.K * f.N)
+
+  h, h2 = runner._buf("h", model.Dp), runner._buf("h2", model.Dp)
+  h.normal_()
+  h2.normal_()
+  ly = model.layers[0]
+  a, m = ly["spec"].mixer.left, ly["spec"].mixer.right
+  lin("linear in", lambda ly: ly["in"], h, 0)
+  src = runner.linear(ly["in"], h, M)
+  lin("linear gates", lambda ly: ly["right"]["gates"], h, 1, fp32=True)
+  gates = runner.fp32_rows(ly["right"]["gates"], h, M, slot=1)
+  rows = (a.heads * a.dim + a.kv_heads * (a.dim + a.vdim)) * 2
+  timed("convolution + cache write", lambda ly, e: runner.conv_kv(ly["left"], src, e["left"], *at), 2 * M * rows + (0 if prompt else B * rows * a.conv))
+  q = runner.conv_kv(ly["left"], src, first[0]["left"], *at)
+  pairs = T * ctx - T * (T - 1) / 2
+  timed("mixed attention", lambda ly, e: runner.mixed_attend(ly["left"], q, src, e["left"], *at),
+        B * a.kv_heads * ctx * (a.dim + a.vdim) * 2 + M * a.heads * (a.dim + 2 * a.vdim) * 2,
+        2.0 * B * a.heads * pairs * (a.dim + a.vdim + a.heads))
+  timed("matrix memory", lambda ly, e: runner.remember(ly["right"], src, gates, e["right"], *at),
+        M * m.heads * ((2 * m.dim + m.vdim) * 2 + m.vdim * 4 + 8) + B * m.heads * m.dim * m.vdim * 8,
+        2.0 * M * m.heads * (2 * m.dim * m.vdim + (32 * (m.dim + m.vdim) if prompt else 0)))
+  o = runner.remember(ly["right"], src, gates, first[0]["right"], *at)
+  timed("head norms + gate", lambda ly, e: runner.gate(ly["right"], o, src, M), M * o.shape[1] * 8)
+  lin("linear attention out", lambda ly: ly["left"]["out"], runner._buf("mixed", ly["left"]["out"].Kp), 0)
+  lin("linear memory out", lambda ly: ly["right"]["out"], runner._buf("gated", ly["right"]["out"].Kp), 1)
+  f = ly["gu"]
+  timed("linear gate_up", lambda ly, e: runner.gate_up(ly, h2, M, slot=2), f.nbytes() + M * (f.K + f.N // 2) * 2, 2.0 * M * f.K * f.N)
+  lin("linear down", lambda ly: ly["down"], runner._buf("act", ly["down"].Kp), 2)
+  sides = runner.linear(ly["left"]["out"], runner._buf("mixed", ly["left"]["out"].Kp), M), runner.linear(ly["right"]["out"], runner._buf("gated", ly["right"]["out"].Kp), M, slot=1)
+  pending = sides, runner.linear(ly["down"], runner._buf("act", ly["down"].Kp), M, slot=2), ly
+  timed("norms + residual + norm + convolutions", lambda ly, e: runner.parallel_step(pending, ly, h, h2, at, e), M * D * (6 + 8 + 4) + (0 if prompt else B * D * 16))
+  return out
+
+
+def kuzezen_workload(size, iters, steps, kernels=True):
+  """Prefill and decode of a Kuzezen decoder with layers of a real model's size (random weights) beside a Nunezen decoder
+  of the same width, heads, feed-forward and number of layers, and every kernel against its roof and the like one's."""
+  import numpy as np
+  import torch
+
+  from tunix_amd import config, dummy_model
+  from tunix_amd.stack_model import StackModel
+  dev = torch.device("cuda:0")
+  width, H, G, ff, B = STACK_SIZES[size]
+  new_cfg, near_cfg = config.kuzezen_shape(width, H, G, ff), config.nunezen_shape(width, H, G, ff)
+  P, T = 1024, 256
+  ids = np.random.Generator(np.random.PCG64(5)).integers(1, new_cfg.vocab_size, size=(B, P)).astype(np.int32)
+  result = {"size": {"width": width, "heads": H, "kv_heads": G, "memory_heads": H, "head_dim": 128, "feed_forward": ff, "batch": B, "prompt": P,
+                     "layer_runs": len(new_cfg.layer_runs)}}
+  for name, cfg, measure in (("kuzezen", new_cfg, kuzezen_kernels), ("nunezen", near_cfg, stack_kernels)):
+    result[name] = measure_model(name, lambda: StackModel(cfg, dummy_model.create_stack_weights(cfg, 1, dev), dev), measure if kernels else None, size, ids, P, T,
+                                 steps, iters)
+  if kernels:
+    for phase in ("decode_kernels", "prefill_kernels"):
+      for k, v in result["kuzezen"][phase].items():
+        b = result["nunezen"][phase][KUZEZEN_LIKE[k]]
+        v["vs_like"] = round(v["times_roof"] / b["times_roof"], 2)
+        log(f"  {size} {phase:16s} {k:40s} {v['us']:9.1f} us  {v['times_roof']:6.2f} x roof ({v['bound']})   {KUZEZEN_LIKE[k]}: "
             f"{b['us']:9.1f} us  {b['times_roof']:6.2f} x ({b['bound']})   ratio {v['vs_like']}")
   return result
 
@@ -1049,7 +1150,7 @@ def main():
                   help="instead of the decode benchmark: a Nunezen decoder with layers of a real model's size (model "
                        "width 2048 or 4096), prefill, decode and every kernel against its roof, beside a gemma3-family "
                        "model of the same size; its own JSON line")
-  ap.add_argument("--stack-design", choices=["nunezen", "lapevik"], default="nunezen", help="with --stack: the layer-list design to measure")
+  ap.add_argument("--stack-design", choices=["nunezen", "lapevik", "kuzezen"], default="nunezen", help="with --stack: the layer-list design to measure")
   ap.add_argument("--stack-no-kernels", action="store_true", help="with --stack: throughput only")
   ap.add_argument("--config", choices=["c1", "c2", "c3", "c4"], default="c3",
                   help="c3 (default): the headline workload; c1 / c2 / c4: the other rollout workloads through "
@@ -1094,9 +1195,10 @@ def main():
 
   if args.stack:
     sizes = sorted(STACK_SIZES) if args.stack == "all" else [args.stack]
-    print(json.dumps({"metric": "Nunezen prefill and decode tokens/sec @1 MI355X", "unit": "tokens/s", "n_gpus": 1,
+    measure = {"nunezen": stack_workload, "lapevik": lapevik_workload, "kuzezen": kuzezen_workload}[args.stack_design]
+    print(json.dumps({"metric": f"{args.stack_design.capitalize()} prefill and decode tokens/sec @1 MI355X", "unit": "tokens/s", "n_gpus": 1,
                       "dtype": "bf16", "data": "synthetic",
-                      "sizes": {z: (lapevik_workload if args.stack_design == "lapevik" else stack_workload)(z, args.kernel_iters, 64, not args.stack_no_kernels) for z in sizes}}),
+                      "sizes": {z: measure(z, args.kernel_iters, 64, not args.stack_no_kernels) for z in sizes}}),
           flush=True)
     return
 
