@@ -948,8 +948,8 @@ int tnx_conv_kvwrite(void* stream, const tnx_conv_kvwrite_desc* d);
 
 /* Causal attention whose softmax weights are mixed between the heads: with p_g the softmax of head g over keys
  * starts[b] .. col + t, out[row, h] = (sum_g talk[h, g] p_g) V_h * sigmoid(gate[row, g_off + h * dv ..]) (gate.ld 0: no gate),
- * V_h the values of head h's own kv head h / (H / G); caches as tnx_sink_attn's.  talk fp32 [H, H].  kv_chunk (64, 128 or
- * 256): keys of a work-group where T == 1.  ws: tnx_mixed_attn_ws_bytes.  tnx_mixed_attn_ok: whether a bf16 shape runs
+ * V_h the values of head h's own kv head h / (H / G); caches as tnx_sink_attn's.  talk fp32 [H, H].  kv_chunk (a
+ * multiple of 64 up to 320): keys of a work-group where T == 1.  ws: tnx_mixed_attn_ws_bytes.  tnx_mixed_attn_ok: whether a bf16 shape runs
  * on MFMA kernels; others, and fp32, run a plain kernel. */
 typedef struct {
   int64_t B, T, S;

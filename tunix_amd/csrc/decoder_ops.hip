@@ -445,6 +445,211 @@ struct ParallelArgs {
   const int32_t* col_ptr;
   int run;                // tokens of a work-group
 };
+// eight values of a row as they lie in memory
+template <typename T>
+struct Raw8;
+template <>
+struct Raw8<uint16_t> {
+  u32x4 v;
+  __device__ __forceinline__ void load(const uint16_t* p) { v = *reinterpret_cast<const u32x4*>(p); }
+  __device__ __forceinline__ void get(float (&f)[8]) const {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      f[2 * j] = bflo(v[j]);
+      f[2 * j + 1] = bfhi(v[j]);
+    }
+  }
+};
+template <>
+struct Raw8<float> {
+  f32x4 v[2];
+  __device__ __forceinline__ void load(const float* p) {
+    v[0] = *reinterpret_cast<const f32x4*>(p);
+    v[1] = *reinterpret_cast<const f32x4*>(p + 4);
+  }
+  __device__ __forceinline__ void get(float (&f)[8]) const {
+#pragma unroll
+    for (int j = 0; j < 8; ++j) f[j] = v[j >> 2][j & 3];
+  }
+};
+
+// A work-group walks `run` tokens of one sequence; it forms h of the taps - 1 tokens in front of them as well, or
+// takes it from the ring where they belong to an earlier call.  A thread owns runs of eight columns.  The next
+// token's rows are requested before this one's sums (PLANES: incoming rows in partial planes, one token at a time).
+template <int NT, int MAXC, int TAPS, bool PLANES, typename T>
+__global__ __launch_bounds__(NT) void parallel_step_kernel(const ParallelArgs a) {
+  constexpr int NW = NT / 64;
+  __shared__ float red[2][NW][3];   // (two reductions a token take turns: one barrier each)
+  const int64_t runs = (a.T + a.run - 1) / a.run, b = blockIdx.x / runs, t0 = blockIdx.x % runs * a.run;
+  const int64_t t1 = min(a.T, t0 + a.run);
+  const int nch = (int)(a.D / 8), tid = threadIdx.x, wave = tid >> 6;
+  const bool conv = a.conv1 != nullptr;
+  const int col0 = conv ? *a.col_ptr : 0, start = conv ? a.starts[b] : 0;
+  auto column = [&](int c) { return (int64_t)min(c * NT + tid, nch - 1) * 8; };
+  auto load8f = [](const float* p, float (&f)[8]) {
+    Raw8<float> r;
+    r.load(p);
+    r.get(f);
+  };
+  struct Rows {
+    Raw8<float> x[MAXC];
+    Raw8<T> y[3][MAXC];
+  };
+  auto request = [&](int64_t row, Rows& r) {
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      r.x[c].load(a.x + row * a.D + column(c));
+      if constexpr (!PLANES)
+#pragma unroll
+        for (int p = 0; p < 3; ++p)
+          if (p < a.n_in) r.y[p][c].load(reinterpret_cast<const T*>(a.y[p]) + row * a.y_ld[p] + column(c));
+    }
+  };
+  const int64_t first = conv ? t0 - (TAPS - 1) : t0, tb = max(first, (int64_t)0);
+  Rows cur, nxt;
+  request(b * a.T + tb, cur);
+  float wn[MAXC][8], wp[2][MAXC][8], c1[TAPS][MAXC][8], c2[TAPS][MAXC][8], prev[TAPS][MAXC][8];   // prev[j]: h of j + 1 tokens before
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    load8f(a.w_next + column(c), wn[c]);
+#pragma unroll
+    for (int p = 0; p < 2; ++p)
+      if (a.w_post[p]) load8f(a.w_post[p] + column(c), wp[p][c]);
+#pragma unroll
+    for (int k = 0; k < TAPS; ++k) {
+      if (conv) load8f(a.conv1 + k * a.D + column(c), c1[k][c]);
+      if (a.conv2) load8f(a.conv2 + k * a.D + column(c), c2[k][c]);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) prev[k][c][j] = 0.f;
+    }
+  }
+#pragma unroll
+  for (int k = 0; k + 1 < TAPS; ++k) {   // tokens of an earlier call
+    const int64_t t = tb - 1 - k;
+    if (conv && t < 0 && col0 + t >= start)
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) load8f(a.ring + (b * a.slots + (col0 + t) % a.slots) * a.D + column(c), prev[k][c]);
+  }
+  for (int64_t t = tb; t < t1; ++t) {
+    const int64_t row = b * a.T + t;
+    const bool live = col0 + t >= start;   // (uniform) otherwise h counts as zero for the tokens behind
+    float h[MAXC][8], in[3][MAXC][8], s[3] = {0.f, 0.f, 0.f};
+    if constexpr (!PLANES) request(b * a.T + min(t + 1, t1 - 1), nxt);
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      cur.x[c].get(h[c]);
+#pragma unroll
+      for (int p = 0; p < 3; ++p) {
+        if (p >= a.n_in) continue;
+        if constexpr (PLANES) get8(RowSrc<T>{reinterpret_cast<const T*>(a.y[p]), a.ws[p], a.split[p], a.plane[p], a.y_ld[p]}, row, column(c), in[p][c]);
+        else cur.y[p][c].get(in[p][c]);
+        if (a.w_post[p] && c * NT + tid < nch)
+#pragma unroll
+          for (int j = 0; j < 8; ++j) s[p] += in[p][c][j] * in[p][c][j];
+      }
+    }
+    if (a.n_in > 0) {   // (uniform)
+#pragma unroll
+      for (int p = 0; p < 3; ++p)
+        if (p < a.n_in && a.w_post[p]) {
+          s[p] = wave_sum(s[p]);
+          if ((tid & 63) == 0) red[0][wave][p] = s[p];
+        }
+      __syncthreads();
+#pragma unroll
+      for (int p = 0; p < 3; ++p) {
+        if (p >= a.n_in) continue;
+        float f = a.mult * a.y_scale[p];
+        if (a.w_post[p]) {
+          float sum = 0.f;
+#pragma unroll
+          for (int w = 0; w < NW; ++w) sum += red[0][w][p];
+          f *= 1.0f / sqrtf(sum / (float)a.D + a.eps);
+        }
+#pragma unroll
+        for (int c = 0; c < MAXC; ++c) {
+          float w2[8];
+          if (p == 2 && a.w_post[2]) load8f(a.w_post[2] + column(c), w2);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) h[c][j] += f * in[p][c][j] * (a.w_post[p] ? (p == 2 ? w2[j] : wp[p & 1][c][j]) : 1.f);
+        }
+      }
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      if (a.add) {
+        float v[8];
+        load8f(a.add + column(c), v);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) h[c][j] += v[j];
+      }
+      if (c * NT + tid < nch) {
+        if (a.x_out && t >= t0) put8(a.x_out + row * a.D + column(c), h[c]);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) ss += h[c][j] * h[c][j];
+      }
+    }
+    ss = wave_sum(ss);
+    if ((tid & 63) == 0) red[1][wave][0] = ss;
+    __syncthreads();
+    ss = 0.f;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) ss += red[1][w][0];
+    const float rn = 1.0f / sqrtf(ss / (float)a.D + a.eps);
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) h[c][j] *= rn * wn[c][j];
+    if (t >= t0) {
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) {
+        if (c * NT + tid >= nch) continue;
+        const int64_t col = column(c), at = a.out_frag ? frag_index(row, col, a.out_ld) : row * a.out_ld + col;
+        float o[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) o[j] = h[c][j];
+        if (conv) {
+#pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            o[j] += c1[TAPS - 1][c][j] * h[c][j];
+#pragma unroll
+            for (int k = 0; k + 1 < TAPS; ++k) o[j] += c1[TAPS - 2 - k][c][j] * prev[k][c][j];
+          }
+        }
+        put8(reinterpret_cast<T*>(a.out1) + at, o);
+        if (a.out2) {
+#pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            o[j] = h[c][j] + c2[TAPS - 1][c][j] * h[c][j];
+#pragma unroll
+            for (int k = 0; k + 1 < TAPS; ++k) o[j] += c2[TAPS - 2 - k][c][j] * prev[k][c][j];
+          }
+          put8(reinterpret_cast<T*>(a.out2) + at, o);
+        }
+        if (TAPS > 1 && conv) {
+          const int64_t keep = min(a.T, (int64_t)TAPS - 1);
+          if (a.T == 1) put8(a.ring + (b * a.slots + col0 % a.slots) * a.D + col, h[c]);
+          else if (t >= a.T - keep) put8(a.tail + (b * keep + t - (a.T - keep)) * a.D + col, h[c]);
+        }
+      }
+    }
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+#pragma unroll
+        for (int k = TAPS - 1; k > 0; --k) prev[k][c][j] = prev[k - 1][c][j];
+        prev[0][c][j] = live ? h[c][j] : 0.f;
+      }
+    if constexpr (PLANES) {
+      if (t + 1 < t1) request(b * a.T + t + 1, cur);
+    } else {
+      cur = nxt;
+    }
+  }
+}
+
 __device__ __forceinline__ void block_sum2(float& a, float& b, float (*red)[2]) {
   a = wave_sum(a);
   b = wave_sum(b);
@@ -459,155 +664,6 @@ __device__ __forceinline__ void block_sum2(float& a, float& b, float (*red)[2]) 
   for (int w = 0; w < nw; ++w) {
     a += red[w][0];
     b += red[w][1];
-  }
-}
-
-// A work-group walks `run` tokens of one sequence; it forms h of the taps - 1 tokens in front of them as well, or
-// takes it from the ring where they belong to an earlier call.  A thread owns runs of eight columns.
-template <int NT, int MAXC, int TAPS, typename T>
-__global__ __launch_bounds__(NT) void parallel_step_kernel(const ParallelArgs a) {
-  __shared__ float red[NT / 64][2];
-  const int64_t runs = (a.T + a.run - 1) / a.run, b = blockIdx.x / runs, t0 = blockIdx.x % runs * a.run;
-  const int64_t t1 = min(a.T, t0 + a.run);
-  const int nch = (int)(a.D / 8), tid = threadIdx.x;
-  const bool conv = a.conv1 != nullptr;
-  const int col0 = conv ? *a.col_ptr : 0, start = conv ? a.starts[b] : 0;
-  auto column = [&](int c) { return (int64_t)min(c * NT + tid, nch - 1) * 8; };
-  auto load8f = [](const float* p, float (&f)[8]) {
-    const f32x4 u = *reinterpret_cast<const f32x4*>(p), v = *reinterpret_cast<const f32x4*>(p + 4);
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      f[j] = u[j];
-      f[4 + j] = v[j];
-    }
-  };
-  float wn[MAXC][8], c1[TAPS][MAXC][8], c2[TAPS][MAXC][8], prev[TAPS][MAXC][8];   // prev[j]: h of j + 1 tokens before
-#pragma unroll
-  for (int c = 0; c < MAXC; ++c) {
-    load8f(a.w_next + column(c), wn[c]);
-#pragma unroll
-    for (int k = 0; k < TAPS; ++k) {
-      if (conv) load8f(a.conv1 + k * a.D + column(c), c1[k][c]);
-      if (a.conv2) load8f(a.conv2 + k * a.D + column(c), c2[k][c]);
-#pragma unroll
-      for (int j = 0; j < 8; ++j) prev[k][c][j] = 0.f;
-    }
-  }
-  const int64_t first = conv ? t0 - (TAPS - 1) : t0;
-  for (int64_t t = first; t < t1; ++t) {
-    const bool live = col0 + t >= start;   // (uniform) otherwise h counts as zero for the tokens behind
-    float h[MAXC][8];
-    if (t < 0) {
-#pragma unroll
-      for (int c = 0; c < MAXC; ++c) {
-        if (live) load8f(a.ring + (b * a.slots + (col0 + t) % a.slots) * a.D + column(c), h[c]);
-        else
-#pragma unroll
-          for (int j = 0; j < 8; ++j) h[c][j] = 0.f;
-      }
-    } else {
-      const int64_t row = b * a.T + t;
-      float in[3][MAXC][8], s0 = 0.f, s1 = 0.f, s2 = 0.f;
-#pragma unroll
-      for (int c = 0; c < MAXC; ++c) {
-        load8f(a.x + row * a.D + column(c), h[c]);
-#pragma unroll
-        for (int p = 0; p < 3; ++p)
-          if (p < a.n_in) get8(RowSrc<T>{reinterpret_cast<const T*>(a.y[p]), a.ws[p], a.split[p], a.plane[p], a.y_ld[p]}, row, column(c), in[p][c]);
-      }
-      if (a.n_in > 0) {
-        // (uniform) the norms of the incoming rows; the third one's sum shares the second reduction
-#pragma unroll
-        for (int c = 0; c < MAXC; ++c)
-          if (c * NT + tid < nch)
-#pragma unroll
-            for (int j = 0; j < 8; ++j) {
-              if (a.w_post[0]) s0 += in[0][c][j] * in[0][c][j];
-              if (a.w_post[1]) s1 += in[1][c][j] * in[1][c][j];
-              if (a.w_post[2]) s2 += in[2][c][j] * in[2][c][j];
-            }
-        if (a.w_post[0] || a.w_post[1]) block_sum2(s0, s1, red);
-        if (a.w_post[2]) {
-          float z = 0.f;
-          block_sum2(s2, z, red);
-        }
-        const float sums[3] = {s0, s1, s2};
-#pragma unroll
-        for (int p = 0; p < 3; ++p) {
-          if (p >= a.n_in) continue;
-          const float f = a.mult * a.y_scale[p], r = a.w_post[p] ? 1.0f / sqrtf(sums[p] / (float)a.D + a.eps) : 1.f;
-#pragma unroll
-          for (int c = 0; c < MAXC; ++c) {
-            float w[8];
-            if (a.w_post[p]) load8f(a.w_post[p] + column(c), w);
-#pragma unroll
-            for (int j = 0; j < 8; ++j) h[c][j] += f * (a.w_post[p] ? in[p][c][j] * r * w[j] : in[p][c][j]);
-          }
-        }
-      }
-      float ss = 0.f, zero = 0.f;
-#pragma unroll
-      for (int c = 0; c < MAXC; ++c) {
-        if (a.add) {
-          float v[8];
-          load8f(a.add + column(c), v);
-#pragma unroll
-          for (int j = 0; j < 8; ++j) h[c][j] += v[j];
-        }
-        if (c * NT + tid < nch) {
-          if (a.x_out && t >= t0) put8(a.x_out + row * a.D + column(c), h[c]);
-#pragma unroll
-          for (int j = 0; j < 8; ++j) ss += h[c][j] * h[c][j];
-        }
-      }
-      block_sum2(ss, zero, red);
-      const float rn = 1.0f / sqrtf(ss / (float)a.D + a.eps);
-#pragma unroll
-      for (int c = 0; c < MAXC; ++c)
-#pragma unroll
-        for (int j = 0; j < 8; ++j) h[c][j] *= rn * wn[c][j];
-      if (t >= t0) {
-#pragma unroll
-        for (int c = 0; c < MAXC; ++c) {
-          if (c * NT + tid >= nch) continue;
-          const int64_t col = column(c), at = a.out_frag ? frag_index(row, col, a.out_ld) : row * a.out_ld + col;
-          float o[8];
-#pragma unroll
-          for (int j = 0; j < 8; ++j) o[j] = h[c][j];
-          if (conv) {
-#pragma unroll
-            for (int j = 0; j < 8; ++j) {
-              o[j] += c1[TAPS - 1][c][j] * h[c][j];
-#pragma unroll
-              for (int k = 0; k + 1 < TAPS; ++k) o[j] += c1[TAPS - 2 - k][c][j] * prev[k][c][j];
-            }
-          }
-          put8(reinterpret_cast<T*>(a.out1) + at, o);
-          if (a.out2) {
-#pragma unroll
-            for (int j = 0; j < 8; ++j) {
-              o[j] = h[c][j] + c2[TAPS - 1][c][j] * h[c][j];
-#pragma unroll
-              for (int k = 0; k + 1 < TAPS; ++k) o[j] += c2[TAPS - 2 - k][c][j] * prev[k][c][j];
-            }
-            put8(reinterpret_cast<T*>(a.out2) + at, o);
-          }
-          if (TAPS > 1 && conv) {
-            const int64_t keep = min(a.T, (int64_t)TAPS - 1);
-            if (a.T == 1) put8(a.ring + (b * a.slots + col0 % a.slots) * a.D + col, h[c]);
-            else if (t >= a.T - keep) put8(a.tail + (b * keep + t - (a.T - keep)) * a.D + col, h[c]);
-          }
-        }
-      }
-    }
-#pragma unroll
-    for (int c = 0; c < MAXC; ++c)
-#pragma unroll
-      for (int j = 0; j < 8; ++j) {
-#pragma unroll
-        for (int k = TAPS - 1; k > 0; --k) prev[k][c][j] = prev[k - 1][c][j];
-        prev[0][c][j] = live ? h[c][j] : 0.f;
-      }
   }
 }
 
@@ -678,13 +734,20 @@ __global__ __launch_bounds__(256) void parallel_step_any_kernel(const ParallelAr
   }
 }
 
-template <int NT, int MAXC, typename T>
+template <int NT, int MAXC, bool PLANES, typename T>
 void launch_parallel_taps(hipStream_t st, const ParallelArgs& a, const dim3& grid) {
   const int taps = a.conv1 ? a.taps : 1;
-  if (taps == 1) hipLaunchKernelGGL((parallel_step_kernel<NT, MAXC, 1, T>), grid, dim3(NT), 0, st, a);
-  else if (taps == 2) hipLaunchKernelGGL((parallel_step_kernel<NT, MAXC, 2, T>), grid, dim3(NT), 0, st, a);
-  else if (taps == 3) hipLaunchKernelGGL((parallel_step_kernel<NT, MAXC, 3, T>), grid, dim3(NT), 0, st, a);
-  else hipLaunchKernelGGL((parallel_step_kernel<NT, MAXC, 4, T>), grid, dim3(NT), 0, st, a);
+  if (taps == 1) hipLaunchKernelGGL((parallel_step_kernel<NT, MAXC, 1, PLANES, T>), grid, dim3(NT), 0, st, a);
+  else if (taps == 2) hipLaunchKernelGGL((parallel_step_kernel<NT, MAXC, 2, PLANES, T>), grid, dim3(NT), 0, st, a);
+  else if (taps == 3) hipLaunchKernelGGL((parallel_step_kernel<NT, MAXC, 3, PLANES, T>), grid, dim3(NT), 0, st, a);
+  else hipLaunchKernelGGL((parallel_step_kernel<NT, MAXC, 4, PLANES, T>), grid, dim3(NT), 0, st, a);
+}
+template <int NT, int MAXC, typename T>
+void launch_parallel_planes(hipStream_t st, const ParallelArgs& a, const dim3& grid) {
+  bool planes = false;
+  for (int p = 0; p < a.n_in; ++p) planes = planes || a.split[p] > 1;
+  if (planes) launch_parallel_taps<NT, MAXC, true, T>(st, a, grid);
+  else launch_parallel_taps<NT, MAXC, false, T>(st, a, grid);
 }
 constexpr size_t kParallelLds = 144 * 1024;
 template <typename T>
@@ -707,9 +770,9 @@ int launch_parallel(hipStream_t st, ParallelArgs a) {
       return TNX_ELAUNCH;
     }
     hipLaunchKernelGGL((parallel_step_any_kernel<T>), grid, dim3(256), lds, st, a);
-  } else if (a.D <= 2048) launch_parallel_taps<256, 1, T>(st, a, grid);
-  else if (a.D <= 4096) launch_parallel_taps<512, 1, T>(st, a, grid);
-  else launch_parallel_taps<512, 2, T>(st, a, grid);
+  } else if (a.D <= 2048) launch_parallel_planes<256, 1, T>(st, a, grid);
+  else if (a.D <= 4096) launch_parallel_planes<512, 1, T>(st, a, grid);
+  else launch_parallel_planes<512, 2, T>(st, a, grid);
   TNX_CHECK_LAUNCH("parallel_step");
   return TNX_OK;
 }

@@ -30,10 +30,11 @@ struct MixedArgs {
   const float* talk;       // [H, H]
   const int32_t* starts;   // [B]
   const int32_t* col_ptr;
-  int kv_chunk, n_chunks;
+  int kv_chunk, n_chunks;  // one position: keys of a work-group of mixed_value_kernel
+  int s_chunk, s_chunks;   // the same of mixed_score_kernel
   float* lse;              // many positions: [B * T, H], log2 of the denominators
   float* scores;           // one position: [B, H, Sp], log2 units
-  float* ml;               // [B, H, n_chunks, 2]: maximum and sum of a chunk
+  float* ml;               // [B, H, s_chunks, 2]: maximum and sum of a chunk
   float* part;             // [B, n_chunks, H, dvp]
   int64_t Sp;
   int gated;
@@ -233,7 +234,8 @@ __device__ __forceinline__ void store_head(const MixedArgs& a, const RowSrc<uint
 //      [head][position][key];
 //   3. O = W . V of its heads; value rows as in mixed_value_kernel.
 // Two barriers a turn: the weights of a turn are read before its second one, the mixed weights before the next turn's first.
-template <int KS, int NH, int NJ, int HW, int NW>   // 32-deep k-steps; halves and value columns per lane and half; heads of a wave
+// ONE: the heads of a wave share their kv head, so that its keys and values are requested a phase ahead.
+template <int KS, int NH, int NJ, int HW, int NW, bool ONE>   // 32-deep k-steps; halves and value columns per lane and half; heads of a wave
 __global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(1, 2))) void mixed_tile_kernel(const MixedArgs a, const RowSrc<uint16_t> gate) {
   constexpr int DK = KS * 32, DV = NH * NJ * 16, HS = NW * HW;
   constexpr int HT = (HS + 15) / 16, GP = HT * 16;                 // 16-row tiles of heads; head slots
@@ -245,8 +247,9 @@ __global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(1, 2)))
   uint16_t* ws = pl + 32 * KSTR;             // [GP][16][WLD]
   const int tid = threadIdx.x, lane = tid & 63, lm = lane & 15, lq = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int tile = (int)gridDim.x - 1 - (int)blockIdx.x;           // the longest key ranges first
-  const int64_t b = blockIdx.y;
+  // sequences fastest: with a multiple of eight of them, the work-groups of one share an XCD and its keys stay in that L2
+  const int tile = (int)gridDim.y - 1 - (int)blockIdx.y;           // the longest key ranges first
+  const int64_t b = blockIdx.x;
   const int col0 = *a.col_ptr, start = a.starts[b];
   const int tp = tile * 16 + lm, tq = min(tp, (int)a.T - 1);       // this lane's position as a column
   const int c_n = col0 + tq, w_lo = col0 + tile * 16, t_hi = min(col0 + min(tile * 16 + 15, (int)a.T - 1), (int)a.S - 1);
@@ -319,9 +322,11 @@ __global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(1, 2)))
           for (int i = 0; i < 8; ++i) p[hh][i] = 0.f;
           continue;
         }
-        if (g / a.R != c) {
-          c = g / a.R;
-          load_k(c, kb);
+        if constexpr (!ONE) {
+          if (g / a.R != c) {
+            c = g / a.R;
+            load_k(c, kb);
+          }
         }
 #pragma unroll
         for (int s = 0; s < 2; ++s) {
@@ -388,15 +393,17 @@ __global__ __launch_bounds__(64 * NW) __attribute__((amdgpu_waves_per_eu(1, 2)))
     }
     __syncthreads();
     if (!busy) continue;
-    if (kb + 32 <= t_hi) load_k(c_first, kb + 32);
+    load_k(c_first, min(kb + 32, t_hi & ~31));
     int c = c_first;
 #pragma unroll
     for (int hh = 0; hh < HW; ++hh) {
       const int g = wave * HW + hh;
       if (g >= a.H) continue;
-      if (g / a.R != c) {
-        c = g / a.R;
-        load_v(c, kb);
+      if constexpr (!ONE) {
+        if (g / a.R != c) {
+          c = g / a.R;
+          load_v(c, kb);
+        }
       }
       const u32x4 wf = *reinterpret_cast<const u32x4*>(ws + (g * 16 + lm) * WLD + lq * 8);
 #pragma unroll
@@ -443,7 +450,7 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, KS > 4 ? 
   const int chunk = blockIdx.x, qts = (a.R + 15) / 16, g = blockIdx.y / qts, r = blockIdx.y % qts * 16 + lm;
   const int64_t b = blockIdx.z;
   const int start = a.starts[b], last = min(*a.col_ptr, (int)a.S - 1);
-  const int k_lo = max(start, chunk * a.kv_chunk), k_hi = min(last, chunk * a.kv_chunk + a.kv_chunk - 1);
+  const int k_lo = max(start, chunk * a.s_chunk), k_hi = min(last, chunk * a.s_chunk + a.s_chunk - 1);
   if (k_lo > k_hi) return;                                          // (its statistics are never read)
   const bool valid = r < a.R;
   const int head = g * a.R + min(r, a.R - 1);
@@ -492,12 +499,21 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, KS > 4 ? 
   };
   Stage sg[2];
   const int kb0 = k_lo & ~63, kb_last = k_hi & ~63;
+  // (no load behind the last keys, and none under a condition inside the loop: its waits count exactly)
   load(kb0, sg[0]);
-  for (int kb = kb0; kb <= kb_last; kb += 128) {
-    load(min(kb + 64, kb_last), sg[1]);
+  int kb = kb0;
+  for (; kb + 128 <= kb_last; kb += 128) {
+    load(kb + 64, sg[1]);
     compute(kb, sg[0]);
-    load(min(kb + 128, kb_last), sg[0]);
-    if (kb + 64 <= kb_last) compute(kb + 64, sg[1]);
+    load(kb + 128, sg[0]);
+    compute(kb + 64, sg[1]);
+  }
+  if (kb + 64 <= kb_last) {
+    load(kb + 64, sg[1]);
+    compute(kb, sg[0]);
+    compute(kb + 64, sg[1]);
+  } else {
+    compute(kb, sg[0]);
   }
   // a head's four lanes
 #pragma unroll
@@ -507,7 +523,7 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, KS > 4 ? 
     m = mn;
   }
   if (valid && lq == 0) {
-    float* s = a.ml + ((b * a.H + head) * a.n_chunks + chunk) * 2;
+    float* s = a.ml + ((b * a.H + head) * a.s_chunks + chunk) * 2;
     s[0] = m;
     s[1] = l;
   }
@@ -532,12 +548,30 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
   const int start = a.starts[b], last = min(*a.col_ptr, (int)a.S - 1), base = chunk * KC;
   const int k_lo = max(start, base), k_hi = min(last, base + KC - 1);
   if (k_lo > k_hi) return;                                          // (its part is never read)
+  // the first values are on their way while the weights are formed
+  struct Stage {
+    vfrag vf[NH][8];
+  };
+  const rsrc_t rv = make_rsrc(reinterpret_cast<const uint16_t*>(a.v) + b * a.G * a.S * DV, (uint64_t)a.G * a.S * DV * 2);
+  auto load = [&](int c, int kb, Stage& s) {
+#pragma unroll
+    for (int k = 0; k < 8; ++k)
+#pragma unroll
+      for (int h = 0; h < NH; ++h) {
+        const uint32_t o = (uint32_t)((c * (int)a.S + kb + 8 * lq + k) * DV + h * 16 * NJ + NJ * lm) * 2u;
+        if constexpr (NJ == 8) s.vf[h][k] = __builtin_amdgcn_raw_buffer_load_b128(rv, o, 0, kStreamOnce);
+        else s.vf[h][k] = __builtin_amdgcn_raw_buffer_load_b64(rv, o, 0, kStreamOnce);
+      }
+  };
+  Stage sg[2];
+  const int qts = (a.R + 15) / 16, kb0 = k_lo & ~31, kb_last = k_hi & ~31;
+  if (wave < a.G * qts) load(wave / qts, kb0, sg[0]);
   {
     const int h = tid >> 2;
     float m = kNegBig, l = 0.f;
     if (h < a.H)
-      for (int c = start / KC + (tid & 3); c <= last / KC; c += 4) {
-        const float* s = a.ml + ((b * a.H + h) * a.n_chunks + c) * 2;
+      for (int c = start / a.s_chunk + (tid & 3); c <= last / a.s_chunk; c += 4) {
+        const float* s = a.ml + ((b * a.H + h) * a.s_chunks + c) * 2;
         const float mn = fmaxf(m, s[0]);
         l = l * exp2_hw(m - mn) + s[1] * exp2_hw(s[0] - mn);
         m = mn;
@@ -551,8 +585,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
     if ((tid & 3) == 0) lse[h] = h < a.H ? m + __log2f(l) : -kNegBig;
   }
   __syncthreads();
-  for (int it = tid; it < GP * (KC / 4); it += 256) {
-    const int h = it / (KC / 4), k0 = it % (KC / 4) * 4;
+  for (int it = tid; it < GP * (KC / 4); it += 256) {   // (heads fastest: they lie side by side in LDS)
+    const int h = it % GP, k0 = it / GP * 4;
     f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
     if (h < a.H && base + k0 < a.Sp) s = *reinterpret_cast<const f32x4*>(a.scores + (b * a.H + h) * a.Sp + base + k0);
     const float e = lse[h];
@@ -595,29 +629,15 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
     }
   }
   __syncthreads();
-  const int qts = (a.R + 15) / 16;
   for (int it = wave; it < a.G * qts; it += 4) {
     const int c = it / qts, r0 = it % qts * 16, head = c * a.R + min(r0 + lm, a.R - 1);
-    const rsrc_t rv = make_rsrc(reinterpret_cast<const uint16_t*>(a.v) + (b * a.G + c) * a.S * DV, (uint64_t)a.S * DV * 2);
-    struct Stage {
-      vfrag vf[NH][8];
-    };
-    auto load = [&](int kb, Stage& sg) {
-#pragma unroll
-      for (int s = 0; s < 8; ++s)
-#pragma unroll
-        for (int h = 0; h < NH; ++h) {
-          const uint32_t o = (uint32_t)((kb + 8 * lq + s) * DV + h * 16 * NJ + NJ * lm) * 2u;
-          if constexpr (NJ == 8) sg.vf[h][s] = __builtin_amdgcn_raw_buffer_load_b128(rv, o, 0, kStreamOnce);
-          else sg.vf[h][s] = __builtin_amdgcn_raw_buffer_load_b64(rv, o, 0, kStreamOnce);
-        }
-    };
+    if (it != wave) load(c, kb0, sg[0]);
     f32x4 O[NH][NJ];
 #pragma unroll
     for (int h = 0; h < NH; ++h)
 #pragma unroll
       for (int j = 0; j < NJ; ++j) O[h][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-    auto compute = [&](int kb, const Stage& sg) {
+    auto compute = [&](int kb, const Stage& s) {
       const u32x4 wf = *reinterpret_cast<const u32x4*>(ws + head * wld + kb - base + lq * 8);
 #pragma unroll
       for (int h = 0; h < NH; ++h)
@@ -626,18 +646,23 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
           const uint32_t sel = (j & 1) ? 0x07060302u : 0x05040100u;
           u32x4 bf;
 #pragma unroll
-          for (int r = 0; r < 4; ++r) bf[r] = __builtin_amdgcn_perm(sg.vf[h][2 * r + 1][j >> 1], sg.vf[h][2 * r][j >> 1], sel);
+          for (int r = 0; r < 4; ++r) bf[r] = __builtin_amdgcn_perm(s.vf[h][2 * r + 1][j >> 1], s.vf[h][2 * r][j >> 1], sel);
           O[h][j] = mfma16(wf, bf, O[h][j]);
         }
     };
-    Stage sg[2];
-    const int kb0 = k_lo & ~31, kb_last = k_hi & ~31;
-    load(kb0, sg[0]);
-    for (int kb = kb0; kb <= kb_last; kb += 64) {
-      load(min(kb + 32, kb_last), sg[1]);
+    int kb = kb0;
+    for (; kb + 64 <= kb_last; kb += 64) {
+      load(c, kb + 32, sg[1]);
       compute(kb, sg[0]);
-      load(min(kb + 64, kb_last), sg[0]);
-      if (kb + 32 <= kb_last) compute(kb + 32, sg[1]);
+      load(c, kb + 64, sg[0]);
+      compute(kb + 32, sg[1]);
+    }
+    if (kb + 32 <= kb_last) {
+      load(c, kb + 32, sg[1]);
+      compute(kb, sg[0]);
+      compute(kb + 32, sg[1]);
+    } else {
+      compute(kb, sg[0]);
     }
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -668,6 +693,7 @@ __global__ __launch_bounds__(256) void mixed_join_kernel(const MixedArgs a, cons
   }
 }
 
+constexpr int kMaxChunk = 320;
 // ---- launches ---------------------------------------------------------------------------------------------
 template <class K>
 int raise_lds(K kern, size_t bytes) {
@@ -677,19 +703,26 @@ int raise_lds(K kern, size_t bytes) {
   return TNX_ELAUNCH;
 }
 
-template <int KS, int NH, int NJ, int HW, int NW>
-int launch_tile(hipStream_t st, const MixedArgs& a, const RowSrc<uint16_t>& gate) {
+template <int KS, int NH, int NJ, int HW, int NW, bool ONE>
+int launch_tile_as(hipStream_t st, const MixedArgs& a, const RowSrc<uint16_t>& gate) {
   constexpr int GP = (NW * HW + 15) / 16 * 16;
   constexpr size_t kLoop = (size_t)(2 * 32 * (16 * (GP + 8) + 8) + GP * 16 * 40) * 2, kOut = (size_t)NW * 16 * NH * NJ * 16 * 4;
   constexpr size_t kLds = kLoop > kOut ? kLoop : kOut;
   static std::once_flag once;
   static int rc = TNX_OK;
-  std::call_once(once, [] { rc = raise_lds(&mixed_tile_kernel<KS, NH, NJ, HW, NW>, kLds); });
+  std::call_once(once, [] { rc = raise_lds(&mixed_tile_kernel<KS, NH, NJ, HW, NW, ONE>, kLds); });
   if (rc) return rc;
   hipLaunchKernelGGL((mixed_stats_kernel<2 * KS>), dim3((unsigned)cdiv(a.T * a.R, 128), (unsigned)a.G, (unsigned)a.B), dim3(256), 0, st, a);
-  hipLaunchKernelGGL((mixed_tile_kernel<KS, NH, NJ, HW, NW>), dim3((unsigned)cdiv(a.T, 16), (unsigned)a.B), dim3(64 * NW), kLds, st, a, gate);
+  hipLaunchKernelGGL((mixed_tile_kernel<KS, NH, NJ, HW, NW, ONE>), dim3((unsigned)a.B, (unsigned)cdiv(a.T, 16)), dim3(64 * NW), kLds, st, a, gate);
   TNX_CHECK_LAUNCH("mixed_tile");
   return TNX_OK;
+}
+template <int KS, int NH, int NJ, int HW, int NW>
+int launch_tile(hipStream_t st, const MixedArgs& a, const RowSrc<uint16_t>& gate) {
+  if constexpr (HW > 1) {
+    if (a.R % HW != 0) return launch_tile_as<KS, NH, NJ, HW, NW, false>(st, a, gate);
+  }
+  return launch_tile_as<KS, NH, NJ, HW, NW, true>(st, a, gate);
 }
 template <int KS, int NH, int NJ>
 int launch_tile_heads(hipStream_t st, const MixedArgs& a, const RowSrc<uint16_t>& gate) {
@@ -714,7 +747,7 @@ int launch_value(hipStream_t st, const MixedArgs& a) {
   const size_t lds = (size_t)(2 * a.kv_chunk * (GP + 8) + GP * (a.kv_chunk + 8)) * 2;
   static std::once_flag once;
   static int rc = TNX_OK;
-  std::call_once(once, [] { rc = raise_lds(&mixed_value_kernel<NH, NJ, HT>, (size_t)(2 * 256 * (GP + 8) + GP * 264) * 2); });
+  std::call_once(once, [] { rc = raise_lds(&mixed_value_kernel<NH, NJ, HT>, (size_t)(2 * kMaxChunk * (GP + 8) + GP * (kMaxChunk + 8)) * 2); });
   if (rc) return rc;
   hipLaunchKernelGGL((mixed_value_kernel<NH, NJ, HT>), dim3((unsigned)a.n_chunks, (unsigned)a.B), dim3(256), lds, st, a);
   TNX_CHECK_LAUNCH("mixed_value");
@@ -756,7 +789,7 @@ extern "C" size_t tnx_mixed_attn_ws_bytes(int64_t B, int64_t T, int64_t S, int H
   if (B <= 0 || T <= 0 || S <= 0 || H <= 0) return 0;
   if (T > 1) return (size_t)(B * T) * (size_t)H * 4;
   if (kv_chunk <= 0) return 0;
-  return (size_t)(B * H) * ((size_t)score_row(S) + (size_t)cdiv(S, kv_chunk) * (size_t)(2 + dvp)) * 4;
+  return (size_t)(B * H) * ((size_t)score_row(S) + (size_t)cdiv(S, 64) * 2 + (size_t)cdiv(S, kv_chunk) * (size_t)dvp) * 4;
 }
 
 extern "C" int tnx_mixed_attn(void* stream, const tnx_mixed_attn_desc* d) {
@@ -779,7 +812,7 @@ extern "C" int tnx_mixed_attn(void* stream, const tnx_mixed_attn_desc* d) {
   if (!tnx_mixed_attn_ok(d->T, d->S, d->H, d->G, d->dkp, d->dvp)) return launch_any<uint16_t>(st, a, g16);
   TNX_REQUIRE(d->ws, "mixed_attn: needs the workspace of tnx_mixed_attn_ws_bytes");
   if (d->T > 1) {
-    TNX_REQUIRE(d->G <= 65535, "mixed_attn: too many kv heads");
+    TNX_REQUIRE(d->G <= 65535 && cdiv(d->T, 16) <= 65535, "mixed_attn: too many kv heads or positions");
     a.lse = d->ws;
     switch (d->dkp) {
       case 64: return launch_tile_v<2>(st, a, g16);
@@ -787,14 +820,18 @@ extern "C" int tnx_mixed_attn(void* stream, const tnx_mixed_attn_desc* d) {
       default: return launch_tile_v<8>(st, a, g16);
     }
   }
-  TNX_REQUIRE(d->kv_chunk == 64 || d->kv_chunk == 128 || d->kv_chunk == 256, "mixed_attn: kv_chunk must be 64, 128 or 256");
+  TNX_REQUIRE(d->kv_chunk > 0 && d->kv_chunk % 64 == 0 && d->kv_chunk <= kMaxChunk, "mixed_attn: kv_chunk must be a multiple of 64 up to %d", kMaxChunk);
   a.kv_chunk = d->kv_chunk;
   a.n_chunks = (int)cdiv(d->S, d->kv_chunk);
   a.Sp = score_row(d->S);
+  // a wave of the score kernel takes as many keys as leave one or two waves per SIMD
+  const int64_t streams = d->B * d->G * cdiv(a.R, 16), most = cdiv(d->S, 64), want = cdiv(1536, streams);
+  a.s_chunk = (int)(cdiv(most, want < most ? want : most) * 64);
+  a.s_chunks = (int)cdiv(d->S, a.s_chunk);
   a.scores = d->ws;
   a.ml = a.scores + d->B * d->H * a.Sp;
-  a.part = a.ml + d->B * d->H * (int64_t)a.n_chunks * 2;
-  const dim3 sg((unsigned)a.n_chunks, (unsigned)(d->G * cdiv(a.R, 16)), (unsigned)d->B);
+  a.part = a.ml + d->B * d->H * most * 2;
+  const dim3 sg((unsigned)a.s_chunks, (unsigned)(d->G * cdiv(a.R, 16)), (unsigned)d->B);
   TNX_REQUIRE(sg.y <= 65535, "mixed_attn: too many heads");
   switch (d->dkp) {
     case 64: hipLaunchKernelGGL(mixed_score_kernel<2>, sg, dim3(64), 0, st, a); break;

@@ -418,7 +418,7 @@ class StackRunner(HeadRunner):
     """Keys of a work-group in a decode step of mixed attention: as many as leave about two work-groups per compute unit."""
     if given:
       return given
-    for chunk in (256, 128):
+    for chunk in (320, 256, 192, 128):
       if self.B * math.ceil(self.S / chunk) >= 512:
         return chunk
     return 64
