@@ -1057,7 +1057,7 @@ def kuzezen_kernels(model, runner, st, ctx, iters):
   def timed(name, fn, nbytes, flops=0.0):
     out[name] = roof_row(in_turn([(lambda i=i: fn(model.layers[i], first[i])) for i in layers], iters), nbytes, flops)
 
-  def lin(name, pick, x, slot, n_out=None, fp32=False):
+  def lin(name, pick, x, slot, fp32=False):
     f = pick(model.layers[0])
     timed(name, lambda ly, e: runner.linear(pick(ly), x, M, fp32_out=fp32, slot=slot), f.nbytes() + M * (f.K * 2 + f.N * (4 if fp32 else 2)), 2.0 * M * f.K * f.N)
 
