@@ -54,6 +54,7 @@ extern "C" {
 #define TNX_EPI_SILU_MUL 2  /* y = bf16(bf16(silu(bf16 g)) * bf16 u) (llama3/model.py:493)    */
 #define TNX_EPI_GELU_MUL 3  /* y = bf16(bf16(gelu_tanh(bf16 g)) * bf16 u) (gemma3/model.py:785-797) */
 #define TNX_EPI_F32 4       /* y(fp32) = acc, no rounding                                   */
+#define TNX_EPI_RELU2 5     /* y = max(acc, 0)^2 (tnx_dense_linear alone)                   */
 
 const char* tnx_last_error(void);
 /* Library / ABI version: (major << 16) | minor, the value tnx_version() returns.
@@ -75,8 +76,11 @@ const char* tnx_last_error(void);
  * to tnx_gated_norm_desc, out_head to tnx_sink_attn_desc, and tnx_silu_mul, tnx_route_softmax,
  * tnx_short_conv, tnx_ring_write, tnx_ssd, tnx_latent_* and tnx_gate_mul; 5.0 adds softcap to tnx_lmhead_desc,
  * a scale to tnx_embed_rows, a first column to tnx_ring_write, parts behind the norm of tnx_gated_norm, and
- * tnx_parallel_step, tnx_conv_kvwrite, tnx_mixed_attn, tnx_memory and tnx_soft_cap. */
-#define TNX_ABI_VERSION_MAJOR 5
+ * tnx_parallel_step, tnx_conv_kvwrite, tnx_mixed_attn, tnx_memory and tnx_soft_cap; 6.0 adds learned positions to
+ * tnx_embed_rows, centred norms, a factor, an extra row and the depth average to tnx_residual_norm_desc, slopes and
+ * chunks to tnx_sink_attn_desc, an ungated form and shared weights to tnx_gated_norm_desc, TNX_EPI_RELU2, and
+ * tnx_rownorm_kvwrite, tnx_gated_state, tnx_poly_norm and tnx_route_scores. */
+#define TNX_ABI_VERSION_MAJOR 6
 #define TNX_ABI_VERSION_MINOR 0
 #define TNX_ABI_VERSION ((TNX_ABI_VERSION_MAJOR << 16) | TNX_ABI_VERSION_MINOR)
 int tnx_version(void);
@@ -573,7 +577,7 @@ typedef struct {
 
 /* y[M, N] = x[M, K] . w^T.  bf16: w is the fragment-order copy of tnx_dense_expand, K % 128 == 0
  * (zero-padded), N % 16 == 0 for bf16 outputs.  fp32: w row-major [N, K], K % 16 == 0.
- * epilogue: TNX_EPI_STORE (model dtype), TNX_EPI_F32, or (bf16) TNX_EPI_GELU_MUL / TNX_EPI_SILU_MUL: w's
+ * epilogue: TNX_EPI_STORE or TNX_EPI_RELU2 (model dtype; the square of the positive part, formed in fp32), TNX_EPI_F32, or (bf16) TNX_EPI_GELU_MUL / TNX_EPI_SILU_MUL: w's
  * rows come in alternating blocks of 16 gate and 16 up rows and y[M, N/2] = act(gate) * up with act =
  * gelu_tanh / silu, formed in fp32 and rounded once.  split_k > 1 (bf16, few rows): fp32 planes to ws
  * [split_k][M][ldy] instead.
@@ -602,10 +606,11 @@ typedef struct {
 int tnx_dense_linear(void* stream, const tnx_dense_desc* d);
 
 /* x[row] (fp32) = scale * table[ids[b, col + t]]; optionally also cat[row, cat_off ..] = the table's row in the
- * model's dtype.  Ids outside [0, V) read row 0. */
+ * model's dtype.  Ids outside [0, V) read row 0.  pos (null: none; [n_pos, D] in the table's dtype): pos[p] is added,
+ * unscaled, p = the token's position col + t - starts[b], held inside the table (the caller bounds sequences). */
 int tnx_embed_rows(void* stream, int dtype, const void* table, int64_t V, int64_t D, const int32_t* ids,
                    int64_t ids_ld, const int32_t* col_ptr, int64_t B, int64_t T, float scale, float* x, void* cat,
-                   int64_t cat_ld, int64_t cat_off, int cat_frag);
+                   int64_t cat_ld, int64_t cat_off, int cat_frag, const void* pos, int64_t n_pos, const int32_t* starts);
 
 /* The residual step between two sublayers, in fp32:
  *   mode 1: x += norm(y) * (w_offset + w_post);  mode 2: x = y;  mode 3: x = norm(x) * (w_offset + w_post);
@@ -617,7 +622,12 @@ int tnx_embed_rows(void* stream, int dtype, const void* table, int64_t V, int64_
  * shift (null: none; instead of w_next): out = x + (x' - x) * shift with x' the x of the token before: the row in
  * front of it, or `before` [B, D] for the first token of a call (zeros for the first token of a sequence).  The
  * rows are T tokens for each of B sequences.  T == 1: `before` takes the new x; T > 1: x_out is another
- * buffer than x, and the caller keeps the last rows (tnx_ring_write). */
+ * buffer than x, and the caller keeps the last rows (tnx_ring_write).
+ * center: norms are layer norms, (v - mean) / sqrt(mean((v - mean)^2) + eps).  mult (0: 1): mode 1 adds mult * norm(y).
+ * extra (extra.ld 0: none): rows that join y before its norm, times extra_w[row] (null: 1).
+ * hist (null: none): the results of earlier layers, X_j at hist + j * hist_plane, j < hist_n.  The new x is X_n
+ * (n = hist_n): it is stored there when hist_store is set, and x becomes sum_{j <= n} hist_w[j] X_j.  These four go with
+ * modes 0 and 1, one part and no shift. */
 typedef struct {
   int64_t M, D;
   int dtype;
@@ -639,6 +649,14 @@ typedef struct {
   const int32_t* starts;
   const int32_t* col_ptr;
   int64_t B, T;
+  int center;
+  float mult;
+  tnx_rows_src extra;
+  const float* extra_w;
+  float* hist;
+  int64_t hist_plane;
+  int hist_n, hist_store;
+  const float* hist_w;   /* [hist_n + 1] */
 } tnx_residual_norm_desc;
 int tnx_residual_norm(void* stream, const tnx_residual_norm_desc* d);
 
@@ -661,9 +679,30 @@ typedef struct {
 } tnx_part_rope_desc;
 int tnx_part_rope_kvwrite(void* stream, const tnx_part_rope_desc* d);
 
+/* Query and key norms over a whole projection and the cache write: q and k are divided by the root mean square of all
+ * their heads together (eps inside the root) times w_q [H * dk] and w_k [G * dk]; the rest as tnx_part_rope_kvwrite.
+ * kcache null: q alone (keys and values are another layer's). */
+typedef struct {
+  int64_t B, T, S;
+  int H, G, dk, dv, dkp, dvp;
+  int dtype;
+  float eps;
+  const float* w_q;
+  const float* w_k;
+  tnx_rows_src y;
+  int64_t k_off, v_off;
+  const int32_t* col_ptr;
+  void* q_out;
+  void* kcache;
+  void* vcache;
+} tnx_rownorm_kvwrite_desc;
+int tnx_rownorm_kvwrite(void* stream, const tnx_rownorm_kvwrite_desc* d);
+
 /* Causal attention over keys starts[b] .. col + t with softmax(scale * q.k) whose denominator also
  * holds exp(sinks[head]) (sinks null: none).  out[row, head * out_head ..] (out_head 0: dv).  kv_chunk > 0 splits the key range (few
- * query rows, workspace of tnx_sink_attn_ws_bytes).  tnx_sink_attn_pad: the padded head size the
+ * query rows, workspace of tnx_sink_attn_ws_bytes).  slopes (null: none; [H]): slopes[head] times the distance of the
+ * two positions is taken off a score.  chunk > 0: a position sees the keys of its own chunk alone, chunks of that many
+ * positions counted from starts[b].  tnx_sink_attn_pad: the padded head size the
  * MFMA kernels take (other sizes, and fp32, run a plain kernel). */
 typedef struct {
   int64_t B, T, S;
@@ -682,6 +721,8 @@ typedef struct {
   int64_t out_ld;
   int out_frag;
   int64_t out_head;
+  const float* slopes;
+  int chunk;
 } tnx_sink_attn_desc;
 int tnx_sink_attn_pad(int dim, int is_value);
 size_t tnx_sink_attn_ws_bytes(int64_t B, int64_t T, int64_t S, int H, int dvp, int kv_chunk);
@@ -707,8 +748,42 @@ typedef struct {
 size_t tnx_lightning_ws_bytes(int64_t B, int64_t T, int H, int dk, int dv);
 int tnx_lightning(void* stream, const tnx_lightning_desc* d);
 
+/* Linear attention with a forget gate per channel, whose complement writes (HGRN2): per head
+ *   f = lower + (1 - lower) sigmoid(z + bias),  S <- diag(f) S + (1 - f) v^T,  o = S^T silu(q)
+ * with q and v columns of y (from q_off and v_off, head by head) and z of the fp32 rows f (from f_off); bias and lower
+ * [H * dk].  y_f32: y's finished rows are fp32, whatever dtype says (planes always are).  state fp32 [B, H, dk, dv] is read
+ * unless col <= starts[b] and written back; o fp32 [B*T, o_ld].
+ * norm_w (null: none; [dv], T == 1 and tnx_gated_state_step_ok): heads are divided by their root mean square, times norm_w,
+ * and leave in out (model dtype) instead. */
+typedef struct {
+  int64_t B, T;
+  int H, dk, dv;
+  int dtype, y_f32;
+  tnx_rows_src y;
+  int64_t q_off, v_off;
+  tnx_rows_src f;
+  int64_t f_off;
+  const float* bias;
+  const float* lower;
+  const int32_t* starts;
+  const int32_t* col_ptr;
+  float* state;
+  float* o;
+  int64_t o_ld;
+  float* ws;
+  const float* norm_w;
+  float eps;
+  void* out;
+  int64_t out_ld;
+  int out_frag;
+} tnx_gated_state_desc;
+int tnx_gated_state_step_ok(int dk, int dv);
+size_t tnx_gated_state_ws_bytes(int64_t B, int64_t T, int H, int dk, int dv);
+int tnx_gated_state(void* stream, const tnx_gated_state_desc* d);
+
 /* out = norm(o) * (w_offset + w) * sigmoid(g[:, g_off ..]), gate_first: out = norm(o * silu(g[:, g_off ..])) *
- * (w_offset + w), the norms over each of `groups` equal parts of a row of W values (0: one). */
+ * (w_offset + w), the norms over each of `groups` equal parts of a row of W values (0: one).  g.ld 0: no gate.
+ * shared_w: w holds one part's weights, for every part. */
 typedef struct {
   int64_t M, W;
   int dtype;
@@ -722,6 +797,7 @@ typedef struct {
   int64_t out_ld;
   int out_frag;
   int gate_first, groups;
+  int shared_w;
 } tnx_gated_norm_desc;
 int tnx_gated_norm(void* stream, const tnx_gated_norm_desc* d);
 
@@ -735,6 +811,16 @@ int tnx_silu_mul(void* stream, int dtype, const void* y, int64_t ld, int64_t up_
 /* Choice of experts from fp32 logits z [M, E] (z.y fp32, or planes): topk_id int32 [M, k], the k largest logits in
  * descending order (lower id first among equals); topk_w fp32 [M, k], the softmax over these k alone. */
 int tnx_route_softmax(void* stream, const tnx_rows_src* z, int64_t M, int E, int k, float* topk_w, int32_t* topk_id);
+/* The same with scores s = softmax over all E logits: the k experts with the largest s + correction (correction [E], null:
+ * none) are chosen; topk_w = s / (sum of the chosen s + 1e-20) * scale.  gate_w (null: none) fp32 [M] = sigmoid of z's column
+ * gate_off. */
+int tnx_route_scores(void* stream, const tnx_rows_src* z, int64_t M, int E, int k, const float* correction, float scale, int64_t gate_off,
+                     float* topk_w, int32_t* topk_id, float* gate_w);
+
+/* out[M, F] = a norm(y) + b norm(y^2) + c norm(y^3) + e with norm(v) = v / sqrt(mean(v^2) + eps) over the F values of a row,
+ * powers element by element; coef [4] = a, b, c, e. */
+int tnx_poly_norm(void* stream, int dtype, const tnx_rows_src* y, int64_t M, int64_t F, const float* coef, float eps, void* out,
+                  int64_t out_ld, int out_frag);
 
 /* Causal convolution per channel and silu: out[row, c] = silu(bias[c] + sum_j w[taps - 1 - j, c] u(t - j, c)) for
  * the channels off .. off + C - 1 of y.  Tokens before the call's first one come from the ring [B, slots, C] (model

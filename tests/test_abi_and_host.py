@@ -91,7 +91,7 @@ def test_struct_layouts_match_the_header(tmp_path):
            "tnx_ssd_desc": L.SsdDesc, "tnx_latent_prep_desc": L.LatentPrepDesc, "tnx_latent_q_desc": L.LatentQDesc,
            "tnx_latent_kv_desc": L.LatentKvDesc, "tnx_latent_attn_desc": L.LatentAttnDesc, "tnx_gate_mul_desc": L.GateMulDesc,
            "tnx_parallel_step_desc": L.ParallelStepDesc, "tnx_conv_kvwrite_desc": L.ConvKvDesc, "tnx_mixed_attn_desc": L.MixedAttnDesc,
-           "tnx_memory_desc": L.MemoryDesc}
+           "tnx_memory_desc": L.MemoryDesc, "tnx_rownorm_kvwrite_desc": L.RowNormKvDesc, "tnx_gated_state_desc": L.GatedStateDesc}
   lines = ['#include <stdio.h>', '#include <stddef.h>', '#include "tunix_hip.h"', 'int main(void) {']
   for cname, cls in pairs.items():
     lines.append(f'  printf("{cname} %zu\\n", sizeof({cname}));')

@@ -12,12 +12,12 @@ _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libtunix_hip.so")
 
 # the ABI this binding was written against (TNX_ABI_VERSION_MAJOR / _MINOR of include/tunix_hip.h)
-ABI_VERSION = (5, 0)
+ABI_VERSION = (6, 0)
 
 TNX_Q_INT4, TNX_Q_NF4 = 0, 1
 TNX_NORM_LLAMA, TNX_NORM_QWEN3, TNX_NORM_GEMMA3 = 0, 1, 2
 TNX_ROPE_LLAMA, TNX_ROPE_QWEN3, TNX_ROPE_GEMMA3 = 0, 1, 2
-TNX_EPI_STORE, TNX_EPI_RESIDUAL, TNX_EPI_SILU_MUL, TNX_EPI_GELU_MUL, TNX_EPI_F32 = 0, 1, 2, 3, 4
+TNX_EPI_STORE, TNX_EPI_RESIDUAL, TNX_EPI_SILU_MUL, TNX_EPI_GELU_MUL, TNX_EPI_F32, TNX_EPI_RELU2 = 0, 1, 2, 3, 4, 5
 
 TNX_BF16, TNX_F32 = 0, 1
 
@@ -113,6 +113,8 @@ class ResidualNormDesc(C.Structure):
       ("y", RowsSrc), ("w_post", _p), ("x", _p), ("w_next", _p), ("out", _p), ("out_ld", _i64), ("out_frag", _i32),
       ("groups", _i32), ("x_out", _p), ("route_w", _p), ("route_k", _i32), ("shift", _p), ("before", _p),
       ("starts", _p), ("col_ptr", _p), ("B", _i64), ("T", _i64),
+      ("center", _i32), ("mult", _f32), ("extra", RowsSrc), ("extra_w", _p),
+      ("hist", _p), ("hist_plane", _i64), ("hist_n", _i32), ("hist_store", _i32), ("hist_w", _p),
   ]
 
 
@@ -125,13 +127,22 @@ class PartRopeDesc(C.Structure):
   ]
 
 
+class RowNormKvDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("S", _i64),
+      ("H", _i32), ("G", _i32), ("dk", _i32), ("dv", _i32), ("dkp", _i32), ("dvp", _i32), ("dtype", _i32), ("eps", _f32),
+      ("w_q", _p), ("w_k", _p), ("y", RowsSrc), ("k_off", _i64), ("v_off", _i64),
+      ("col_ptr", _p), ("q_out", _p), ("kcache", _p), ("vcache", _p),
+  ]
+
+
 class SinkAttnDesc(C.Structure):
   _fields_ = [
       ("B", _i64), ("T", _i64), ("S", _i64),
       ("H", _i32), ("G", _i32), ("dk", _i32), ("dv", _i32), ("dkp", _i32), ("dvp", _i32),
       ("scale", _f32), ("dtype", _i32), ("q", _p), ("kcache", _p), ("vcache", _p), ("sinks", _p),
       ("starts", _p), ("col_ptr", _p), ("kv_chunk", _i32), ("ws", _p), ("out", _p), ("out_ld", _i64), ("out_frag", _i32),
-      ("out_head", _i64),
+      ("out_head", _i64), ("slopes", _p), ("chunk", _i32),
   ]
 
 
@@ -147,7 +158,16 @@ class GatedNormDesc(C.Structure):
   _fields_ = [
       ("M", _i64), ("W", _i64), ("dtype", _i32), ("eps", _f32), ("w_offset", _f32),
       ("o", _p), ("o_ld", _i64), ("g", RowsSrc), ("g_off", _i64), ("w", _p),
-      ("out", _p), ("out_ld", _i64), ("out_frag", _i32), ("gate_first", _i32), ("groups", _i32),
+      ("out", _p), ("out_ld", _i64), ("out_frag", _i32), ("gate_first", _i32), ("groups", _i32), ("shared_w", _i32),
+  ]
+
+
+class GatedStateDesc(C.Structure):
+  _fields_ = [
+      ("B", _i64), ("T", _i64), ("H", _i32), ("dk", _i32), ("dv", _i32), ("dtype", _i32), ("y_f32", _i32),
+      ("y", RowsSrc), ("q_off", _i64), ("v_off", _i64), ("f", RowsSrc), ("f_off", _i64), ("bias", _p), ("lower", _p),
+      ("starts", _p), ("col_ptr", _p), ("state", _p), ("o", _p), ("o_ld", _i64), ("ws", _p),
+      ("norm_w", _p), ("eps", _f32), ("out", _p), ("out_ld", _i64), ("out_frag", _i32),
   ]
 
 
@@ -302,18 +322,24 @@ SIGNATURES = {
     "tnx_logp_drift_static_max_rows": (_i64, []),
     "tnx_logp_drift_static": (_i32, [_p, _p, _p, _p, _i64, _i64, _p]),
     "tnx_dense_linear": (_i32, [_p, C.POINTER(DenseDesc)]),
-    "tnx_embed_rows": (_i32, [_p, _i32, _p, _i64, _i64, _p, _i64, _p, _i64, _i64, _f32, _p, _p, _i64, _i64, _i32]),
+    "tnx_embed_rows": (_i32, [_p, _i32, _p, _i64, _i64, _p, _i64, _p, _i64, _i64, _f32, _p, _p, _i64, _i64, _i32, _p, _i64, _p]),
     "tnx_residual_norm": (_i32, [_p, C.POINTER(ResidualNormDesc)]),
     "tnx_part_rope_kvwrite": (_i32, [_p, C.POINTER(PartRopeDesc)]),
+    "tnx_rownorm_kvwrite": (_i32, [_p, C.POINTER(RowNormKvDesc)]),
     "tnx_sink_attn_pad": (_i32, [_i32, _i32]),
     "tnx_sink_attn_ws_bytes": (C.c_size_t, [_i64, _i64, _i64, _i32, _i32, _i32]),
     "tnx_sink_attn": (_i32, [_p, C.POINTER(SinkAttnDesc)]),
     "tnx_lightning_ws_bytes": (C.c_size_t, [_i64, _i64, _i32, _i32, _i32]),
     "tnx_lightning": (_i32, [_p, C.POINTER(LightningDesc)]),
+    "tnx_gated_state_step_ok": (_i32, [_i32, _i32]),
+    "tnx_gated_state_ws_bytes": (C.c_size_t, [_i64, _i64, _i32, _i32, _i32]),
+    "tnx_gated_state": (_i32, [_p, C.POINTER(GatedStateDesc)]),
     "tnx_gated_norm": (_i32, [_p, C.POINTER(GatedNormDesc)]),
     "tnx_gelu_mul": (_i32, [_p, _i32, _p, _i64, _i64, _i64, _i64, _p, _i64]),
     "tnx_silu_mul": (_i32, [_p, _i32, _p, _i64, _i64, _i64, _i64, _p, _i64]),
     "tnx_route_softmax": (_i32, [_p, C.POINTER(RowsSrc), _i64, _i32, _i32, _p, _p]),
+    "tnx_route_scores": (_i32, [_p, C.POINTER(RowsSrc), _i64, _i32, _i32, _p, _f32, _i64, _p, _p, _p]),
+    "tnx_poly_norm": (_i32, [_p, _i32, C.POINTER(RowsSrc), _i64, _i64, _p, _f32, _p, _i64, _i32]),
     "tnx_short_conv": (_i32, [_p, C.POINTER(ShortConvDesc)]),
     "tnx_ring_write": (_i32, [_p, _i32, C.POINTER(RowsSrc), _i64, _i64, _i64, _i64, _i32, _p, _i64, _p]),
     "tnx_ssd_step_ok": (_i32, [_i32, _i32]),

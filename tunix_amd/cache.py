@@ -1,6 +1,7 @@
 """What a batch of sequences carries from one forward pass to the next: one entry per layer run,
 a key / value slab (attention), a slab of latents, a recurrent state, a ring of the last columns' rows,
-or several of these.  A layer that runs several times has one entry per run.
+or several of these.  A layer that runs several times has one entry per run; one that reads another layer's keys
+and values has that layer's entry.
 
 Slabs are [B, heads, S, size] or [B, S, size] in the model's dtype, states [B, heads, dim, vdim] in fp32,
 rings [B, slots, width] with slot = column % slots.  Rows of
@@ -68,6 +69,12 @@ class PartsSpec:
 
   def allocate(self, B: int, S: int, device) -> "PartsEntry":
     return PartsEntry({name: spec.allocate(B, S, device) for name, spec in self.parts})
+
+
+@dataclasses.dataclass(frozen=True)
+class BorrowedSpec:
+  """Nothing of its own: the entry of an earlier layer run."""
+  run: int
 
 
 @dataclasses.dataclass
@@ -138,18 +145,23 @@ class PartsEntry:
 
 class SequenceCache:
   """The entries of one batch.  shared=True: layer runs with equal specs use one buffer (a scratch
-  cache for passes that never come back to it)."""
+  cache for passes that never come back to it), but those whose entry a later run reads."""
 
   def __init__(self, specs: list, B: int, S: int, device, shared: bool = False):
     self.B, self.S = B, S
     made: dict = {}
     self.entries = []
-    for spec in specs:
-      if shared and spec in made:
+    lent = {spec.run for spec in specs if isinstance(spec, BorrowedSpec)}
+    for i, spec in enumerate(specs):
+      if isinstance(spec, BorrowedSpec):
+        self.entries.append(self.entries[spec.run])
+        continue
+      if shared and spec in made and i not in lent:
         self.entries.append(made[spec])
         continue
       entry = spec.allocate(B, S, device)
-      made[spec] = entry
+      if i not in lent:
+        made[spec] = entry
       self.entries.append(entry)
 
   @property
@@ -170,6 +182,6 @@ class SequenceCache:
   def grow(self, S: int):
     """More columns, the ones in use kept."""
     if S > self.S:
-      for e in self.entries:
+      for e in {id(e): e for e in self.entries}.values():
         e.grow(S)
       self.S = S

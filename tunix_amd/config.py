@@ -111,7 +111,10 @@ class ModelConfig:
 @dataclasses.dataclass(frozen=True)
 class AttentionMixer:
   """Causal grouped-query attention: separate key and value head sizes, rotation of the first
-  rot_dims dimensions of q and k, any score scale, optionally a learned sink per query head."""
+  rot_dims dimensions of q and k, any score scale, optionally a learned sink per query head.
+  row_norm: q and k are normed, each over all its heads together (then nothing rotates).  slopes: what a head takes off a
+  score per position of distance (empty: nothing).  chunk > 0: a position sees its own chunk of that many positions only.
+  kv_from: the layer whose keys and values (its cache entry) this one reads instead of its own."""
   heads: int
   kv_heads: int
   dim: int
@@ -120,19 +123,38 @@ class AttentionMixer:
   rot_base: float
   scale: float
   sink: bool = True
+  row_norm: bool = False
+  slopes: tuple = ()
+  chunk: int = 0
+  kv_from: int | None = None
 
   def __post_init__(self):
     if self.heads % self.kv_heads:
       raise ValueError("heads must be a multiple of kv_heads")
     if self.rot_dims % 2 or not 0 <= self.rot_dims <= self.dim:
       raise ValueError(f"rot_dims={self.rot_dims} must be even and at most the head size {self.dim}")
+    if self.slopes and len(self.slopes) != self.heads:
+      raise ValueError(f"{len(self.slopes)} slopes for {self.heads} heads")
+    if self.chunk < 0:
+      raise ValueError(f"chunk={self.chunk} must not be negative")
+    if self.row_norm and self.rot_dims or self.kv_from is not None and not self.row_norm:
+      raise ValueError("normed projections do not rotate, and only they may borrow keys and values")
 
   def weight_shapes(self, D: int) -> dict[str, tuple]:
-    out = {"q": (self.heads * self.dim, D), "k": (self.kv_heads * self.dim, D), "v": (self.kv_heads * self.vdim, D),
-           "o": (D, self.heads * self.vdim)}
+    rows = {"q": self.heads * self.dim, "k": self.kv_heads * self.dim, "v": self.kv_heads * self.vdim}
+    own = ("q",) if self.kv_from is not None else ("q", "k", "v")
+    out = {n: (rows[n], D) for n in own}
+    out["o"] = (D, self.heads * self.vdim)
+    if self.row_norm:
+      out.update({n + ".norm": (rows[n],) for n in own if n != "v"})
     if self.sink:
       out["sink"] = (self.heads,)
     return out
+
+
+def distance_slopes(heads: int) -> tuple:
+  """2^(-8 (h + 1) / heads) for head h."""
+  return tuple(2.0 ** (-8.0 * (h + 1) / heads) for h in range(heads))
 
 
 @dataclasses.dataclass(frozen=True)
@@ -221,6 +243,19 @@ class LightningMixer:
 
 
 @dataclasses.dataclass(frozen=True)
+class GatedStateMixer:
+  """Linear attention with a forget gate per head and channel, bounded below, whose complement writes (HGRN2): a matrix state
+  [dim, vdim] per head; heads normed on their own with shared weights, then projected."""
+  heads: int
+  dim: int
+  vdim: int
+
+  def weight_shapes(self, D: int) -> dict[str, tuple]:
+    qk, v = self.heads * self.dim, self.heads * self.vdim
+    return {"q": (qk, D), "f": (qk, D), "f.b": (qk,), "lower": (qk,), "v": (v, D), "norm": (self.vdim,), "o": (D, v)}
+
+
+@dataclasses.dataclass(frozen=True)
 class SsdMixer:
   """State-space duality: per head a matrix state [state, vdim] whose decay depends on the token; inputs
   behind a short causal convolution, B and C shared by the heads of a group; the heads' outputs gated,
@@ -290,29 +325,51 @@ class GatedMlp:
 
 
 @dataclasses.dataclass(frozen=True)
+class PolyNormMlp:
+  """down(a norm(z) + b norm(z^2) + c norm(z^3) + e) with z = up h, norms over the row and four learned numbers."""
+  ff: int
+
+  def weight_shapes(self, D: int) -> dict[str, tuple]:
+    return {"up": (self.ff, D), "down": (D, self.ff), "act": (4,)}
+
+
+@dataclasses.dataclass(frozen=True)
 class ExpertsMlp:
-  """The weighted sum of down(silu(gate h) * (up h)) of the `top` experts with the largest router logits;
-  weights: softmax over the chosen logits."""
+  """The weighted sum of the `top` chosen experts: down(silu(gate h) * (up h)), or down(max(up h, 0)^2) when not gated.
+  Chosen are the largest router logits, weights the softmax over them; corrected: chosen are the largest of softmax over all
+  logits + a correction per expert, weights the chosen scores over their sum, times scale.  shared_ff > 0: one more expert of
+  that size for every token, times a sigmoid of its own (not gated and corrected experts only)."""
   ff: int
   experts: int
   top: int
+  gated: bool = True
+  corrected: bool = False
+  scale: float = 1.0
+  shared_ff: int = 0
 
   def __post_init__(self):
     if not 1 <= self.top <= self.experts:
       raise ValueError(f"{self.top} of {self.experts} experts")
+    if self.shared_ff and (self.gated or not self.corrected) or not self.corrected and self.scale != 1.0:
+      raise ValueError("a shared expert and a scale go with corrected scores")
 
   def weight_shapes(self, D: int) -> dict[str, tuple]:
     out = {"router": (self.experts, D)}
-    for e in range(self.experts):
-      out[f"e{e}.gate"] = out[f"e{e}.up"] = (self.ff, D)
-      out[f"e{e}.down"] = (D, self.ff)
+    if self.corrected:
+      out["correction"] = (self.experts,)
+    sizes = [(f"e{e}", self.ff) for e in range(self.experts)] + ([("shared", self.shared_ff)] if self.shared_ff else [])
+    for name, ff in sizes:
+      out.update({f"{name}.{n}": (ff, D) for n in (("gate", "up") if self.gated else ("up",))})
+      out[name + ".down"] = (D, ff)
+    if self.shared_ff:
+      out["shared.sg"] = (1, D)
     return out
 
 
 @dataclasses.dataclass(frozen=True)
 class LayerSpec:
-  mixer: AttentionMixer | LightningMixer | SsdMixer | LatentMixer | ParallelMixer
-  mlp: GatedMlp | ExpertsMlp | None
+  mixer: AttentionMixer | LightningMixer | SsdMixer | LatentMixer | ParallelMixer | GatedStateMixer
+  mlp: GatedMlp | PolyNormMlp | ExpertsMlp | None
 
 
 @dataclasses.dataclass(frozen=True)
@@ -327,12 +384,14 @@ class LayerLoop:
 
 @dataclasses.dataclass(frozen=True)
 class StackConfig:
-  """A decoder given layer by layer.  Every sublayer is x += norm(f(norm(x))), or x += norm(f(x)) without
+  """A decoder given layer by layer.  Every sublayer is x += residual_mult norm(f(norm(x))), or x += norm(f(x)) without
   pre_norm, with norm weights stored as an offset from `norm_offset` and norms taken over norm_groups equal
   parts of the row.  embed_norm: the embedding is normed.  token_shift:
   what a mixer reads is first moved towards the same of the token before, per element.
   parallel: x += residual_mult (mixer(h1) + mlp(h2)) with h = norm(x) and h1, h2 = h + a causal convolution of input_conv
-  taps of h, per sublayer.  tied_head: the head is the embedding table.  logit_softcap > 0: logits <- cap tanh(logits / cap)."""
+  taps of h, per sublayer.  center_norm: norms are layer norms.  max_positions > 0: a learned vector per position is added to the
+  embedding, and a sequence has at most so many positions.  depth_average: behind layer i, x <- sum over j <= i + 1 of
+  l<i>.dwa[j] X_j with X_0 the embedding output and X_(j+1) layer j's result.  tied_head: the head is the embedding table.  logit_softcap > 0: logits <- cap tanh(logits / cap)."""
   family: str
   vocab_size: int
   embed_dim: int
@@ -350,6 +409,9 @@ class StackConfig:
   embed_scale: float = 1.0
   tied_head: bool = True
   logit_softcap: float = 0.0
+  center_norm: bool = False
+  max_positions: int = 0
+  depth_average: bool = False
 
   def __post_init__(self):
     n, lp = len(self.layers), self.loop
@@ -365,6 +427,18 @@ class StackConfig:
       raise ValueError(f"width {self.embed_dim} does not divide into {self.norm_groups} norm groups")
     if self.token_shift and self.pre_norm:
       raise ValueError("a token shift goes with norms behind the sublayers only")
+    if self.center_norm or self.depth_average or (self.residual_mult != 1.0 and not self.parallel):
+      if self.parallel or self.token_shift or self.norm_groups != 1 or not self.pre_norm or self.embed_norm or lp is not None:
+        raise ValueError("layer norms, a residual factor and the depth average go with plain pre-normed layers that run once")
+    for i, ly in enumerate(self.layers):
+      j = getattr(ly.mixer, "kv_from", None)
+      if j is None:
+        continue
+      src = self.layers[j].mixer if 0 <= j < i else None
+      if lp is not None or not isinstance(src, AttentionMixer) or src.kv_from is not None:
+        raise ValueError(f"layer {i} reads the keys of layer {j}, which is no earlier attention layer with keys of its own")
+      if any(getattr(src, n) != getattr(ly.mixer, n) for n in ("heads", "kv_heads", "dim", "vdim")):
+        raise ValueError(f"layer {i} reads the keys of layer {j}, whose heads differ")
 
   def post_norm(self, n: int) -> str:
     """Name of the norm behind a layer's mixer (n = 1) or feed-forward (2)."""
@@ -391,6 +465,8 @@ class StackConfig:
       out["embed.norm"] = (D,)
     if not self.tied_head:
       out["head"] = (self.vocab_size, D)
+    if self.max_positions:
+      out["pos"] = (self.max_positions, D)
     if self.loop is not None:
       out.update({"loop.step": (self.loop.times, D)} if self.loop.step else {"loop.in": (D, 2 * D)})
     for i, ly in enumerate(self.layers):
@@ -398,6 +474,8 @@ class StackConfig:
       parts = [(1, "mix.", ly.mixer)] + ([(2, "mlp.", ly.mlp)] if ly.mlp is not None else [])
       if self.token_shift:
         out[p + "shift"] = (D,)
+      if self.depth_average:
+        out[p + "dwa"] = (i + 2,)
       for n, at, part in parts:
         if self.pre_norm and not (self.parallel and n == 2):
           out[p + f"norm{n}"] = (D,)
@@ -481,6 +559,38 @@ def kuzezen_from_dict(d: dict) -> StackConfig:
                      embed_scale=float(d["embedding"]["scale"]), tied_head=False, logit_softcap=float(d["logit_softcap"]))
 
 
+def kezolix_from_dict(d: dict) -> StackConfig:
+  """Reads a Kezolix config.json."""
+  layers = []
+  for i, ly in enumerate(d["layers"]):
+    m = ly["mixer"]
+    if ly["type"] == "attention":
+      heads, mask, kv_from = int(m["heads"]), m.get("mask"), m.get("kv_from")
+      if mask is not None and int(mask["size"]) < 1:
+        raise ValueError(f"layer {i}: a chunk of {mask['size']} positions")
+      mixer = AttentionMixer(heads=heads, kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]), rot_dims=0, rot_base=1.0,
+                             scale=float(m["scale"]), sink=False, row_norm=True, slopes=distance_slopes(heads),
+                             chunk=0 if mask is None else int(mask["size"]), kv_from=None if kv_from is None else int(kv_from))
+    elif ly["type"] == "hgrn2":
+      mixer = GatedStateMixer(heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]))
+    else:
+      raise ValueError(f"layer {i}: unknown mixer type {ly['type']!r}")
+    mlp = ly.get("mlp")
+    if mlp is not None:
+      if mlp["kind"] == "dense":
+        mlp = PolyNormMlp(int(mlp["ff"]))
+      elif mlp["kind"] == "moe":
+        r, shared = mlp["router"], mlp.get("shared")
+        mlp = ExpertsMlp(ff=int(mlp["expert"]["ff"]), experts=int(r["experts"]), top=int(r["top"]), gated=False, corrected=True,
+                         scale=float(r["scale"]), shared_ff=0 if shared is None else int(shared["ff"]))
+      else:
+        raise ValueError(f"layer {i}: unknown feed-forward kind {mlp['kind']!r}")
+    layers.append(LayerSpec(mixer, mlp))
+  return StackConfig(family="kezolix", vocab_size=int(d["vocab"]), embed_dim=int(d["width"]), layers=tuple(layers), norm_eps=float(d["norm"]["eps"]),
+                     norm_offset=0.0, residual_mult=float(d["residual_mult"]), tied_head=False, center_norm=True,
+                     max_positions=int(d["max_positions"]), depth_average=True)
+
+
 # ---- the shapes the headline metric and the parity cases are quoted on ------------------------
 def tiny_qwen3(**kw) -> ModelConfig:
   """2-layer Qwen3-style decoder: D512, 8q/2kv, dh64, MLP 1536, V32000, int4 g64, LoRA r8."""
@@ -549,3 +659,18 @@ def kuzezen_shape(width: int, heads: int, kv_heads: int, ff: int, vocab: int = 3
   return StackConfig(family="kuzezen", vocab_size=vocab, embed_dim=width, norm_eps=1e-6, layers=(LayerSpec(mixer, GatedMlp(ff)),) * layers,
                      loop=LayerLoop(1, layers - 1, 2, step=True) if layers > 2 else None, norm_offset=0.0, parallel=True, residual_mult=0.5,
                      input_conv=4, embed_scale=width ** 0.5, tied_head=False, logit_softcap=30.0)
+
+
+def kezolix_shape(width: int, heads: int, kv_heads: int, ff: int, experts: int, top: int, expert_ff: int, vocab: int = 32768, dim: int = 128,
+                  chunk: int = 2048, layers: int = 4, positions: int = 8192) -> StackConfig:
+  """A Kezolix decoder with layers of a real model's size: recurrent and attention layers in turn, the first with a dense
+  feed-forward, the others with routed and shared experts; the last attention layer reads the keys of the first."""
+  moe = ExpertsMlp(expert_ff, experts, top, gated=False, corrected=True, scale=2.5, shared_ff=expert_ff)
+  attn = lambda kv_from: AttentionMixer(heads, kv_heads, dim, dim, 0, 1.0, dim ** -0.5, sink=False, row_norm=True, slopes=distance_slopes(heads),
+                                        chunk=chunk, kv_from=kv_from)
+  out = []
+  for i in range(layers):
+    mixer = GatedStateMixer(heads, dim, dim) if i % 2 == 0 else attn(1 if i > 1 and i >= layers - 2 else None)
+    out.append(LayerSpec(mixer, PolyNormMlp(ff) if i == 0 else moe))
+  return StackConfig(family="kezolix", vocab_size=vocab, embed_dim=width, norm_eps=1e-6, layers=tuple(out), norm_offset=0.0, residual_mult=0.5,
+                     tied_head=False, center_norm=True, max_positions=positions, depth_average=True)

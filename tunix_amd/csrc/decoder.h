@@ -1,5 +1,6 @@
 // Device helpers shared by the dense-weight decoder kernels (dense.hip, decoder_ops.hip,
-// sink_attention.hip, lightning.hip, ssd.hip, latent.hip, memory.hip, mixed_attention.hip): element access by dtype, activations,
+// sink_attention.hip, lightning.hip, ssd.hip, latent.hip, memory.hip, mixed_attention.hip, layer_ops.hip,
+// gated_state.hip): element access by dtype, activations,
 // fragment order, MFMA.
 #pragma once
 #include "common.h"

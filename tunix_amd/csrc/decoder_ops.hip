@@ -10,6 +10,8 @@
 #include "decoder.h"
 #include "rng.h"
 
+int tnx_internal_layer_step(hipStream_t st, const tnx_residual_norm_desc* d);
+
 namespace {
 
 __device__ __forceinline__ float block_sum(float v, float* red) {
@@ -27,9 +29,11 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 template <typename T>
 __global__ __launch_bounds__(256) void embed_rows_kernel(const T* table, int64_t V, int64_t D, const int32_t* ids,
                                                          int64_t ids_ld, const int32_t* col_ptr, int64_t Tn, float scale, float* x,
-                                                         T* cat, int64_t cat_ld, int64_t cat_off, int cat_frag) {
+                                                         T* cat, int64_t cat_ld, int64_t cat_off, int cat_frag, const T* pos,
+                                                         int64_t n_pos, const int32_t* starts) {
   const int64_t row = blockIdx.x, b = row / Tn, t = row % Tn;
   const int col = col_ptr ? *col_ptr : 0;
+  const int64_t p = pos ? min(max((int64_t)col + t - starts[b], (int64_t)0), n_pos - 1) : 0;
   int64_t id = ids[b * ids_ld + col + t];
   if (id < 0 || id >= V) id = 0;   // padding columns: never read by a later token
   if (D % 8 == 0 && cat_ld % 8 == 0) {   // (cat_off is then a multiple of eight, too, where cat is given)
@@ -40,13 +44,19 @@ __global__ __launch_bounds__(256) void embed_rows_kernel(const T* table, int64_t
       if (cat) put8(cat + (cat_frag ? frag_index(row, cat_off + i, cat_ld) : row * cat_ld + cat_off + i), f);
 #pragma unroll
       for (int j = 0; j < 8; ++j) f[j] *= scale;
+      if (pos) {
+        float g[8];
+        get8(RowSrc<T>{pos, nullptr, 1, 0, D}, p, i, g);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) f[j] += g[j];
+      }
       put8(x + row * D + i, f);
     }
     return;
   }
   for (int64_t i = threadIdx.x; i < D; i += 256) {
     const T v = table[id * D + i];
-    x[row * D + i] = scale * ld_elem(&v, 0);
+    x[row * D + i] = scale * ld_elem(&v, 0) + (pos ? ld_elem(pos, p * D + i) : 0.f);
     if (cat) cat[cat_frag ? frag_index(row, cat_off + i, cat_ld) : row * cat_ld + cat_off + i] = v;
   }
 }
@@ -1032,6 +1042,7 @@ struct GatedNormArgs {
   const float* w;
   const float* o;
   int out_frag, groups;
+  int64_t w_len;           // weights repeat after so many columns
 };
 // the gate first, then norms over equal parts: any width that fits LDS
 template <typename T>
@@ -1124,7 +1135,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(const GatedNormArgs a, 
   __syncthreads();
   for (int64_t i = threadIdx.x; i < a.W; i += 256)
     st_elem(out, a.out_frag ? frag_index(row, i, a.out_ld) : row * a.out_ld + i,
-            o[i] * gs[i / per] * (a.w_offset + a.w[i]) * sigmoid_f32(g.get(row, a.g_off + i)));
+            o[i] * gs[i / per] * (a.w_offset + a.w[i % a.w_len]) * (g.ld > 0 ? sigmoid_f32(g.get(row, a.g_off + i)) : 1.f));
 }
 // eight elements per thread and turn, everything requested ahead of the sum
 template <int MAXC, bool PARTS, typename T>
@@ -1138,8 +1149,8 @@ __global__ __launch_bounds__(256) void gated_norm_vec_kernel(const GatedNormArgs
   for (int c = 0; c < MAXC; ++c) {
     const int64_t col = (int64_t)min(c * 256 + (int)threadIdx.x, nch - 1) * 8;
     get8(os, row, col, o[c]);
-    get8(wsrc, 0, col, w[c]);
-    get8(g, row, a.g_off + col, gv[c]);
+    get8(wsrc, 0, PARTS ? col % a.w_len : col, w[c]);
+    if (g.ld > 0) get8(g, row, a.g_off + col, gv[c]);   // (uniform)
   }
   float ss = 0.f;
 #pragma unroll
@@ -1159,7 +1170,7 @@ __global__ __launch_bounds__(256) void gated_norm_vec_kernel(const GatedNormArgs
     if (ch >= nch) continue;
     if constexpr (PARTS) r = gs[ch / per];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) o[c][j] = o[c][j] * r * (a.w_offset + w[c][j]) * sigmoid_f32(gv[c][j]);
+    for (int j = 0; j < 8; ++j) o[c][j] = o[c][j] * r * (a.w_offset + w[c][j]) * (g.ld > 0 ? sigmoid_f32(gv[c][j]) : 1.f);
     put8(out + (a.out_frag ? frag_index(row, (int64_t)ch * 8, a.out_ld) : row * a.out_ld + (int64_t)ch * 8), o[c]);
   }
 }
@@ -1369,17 +1380,19 @@ RowSrc<T> row_src(const tnx_rows_src& s) {
 
 extern "C" int tnx_embed_rows(void* stream, int dtype, const void* table, int64_t V, int64_t D, const int32_t* ids,
                               int64_t ids_ld, const int32_t* col_ptr, int64_t B, int64_t T, float scale, float* x, void* cat,
-                              int64_t cat_ld, int64_t cat_off, int cat_frag) {
+                              int64_t cat_ld, int64_t cat_off, int cat_frag, const void* pos, int64_t n_pos,
+                              const int32_t* starts) {
   TNX_REQUIRE(table && ids && x, "embed_rows: null pointer");
   TNX_REQUIRE(V > 0 && D > 0 && B > 0 && T > 0, "embed_rows: bad shape");
   TNX_REQUIRE(!cat || (cat_ld >= cat_off + D && cat_off % D == 0), "embed_rows: the second copy does not fit its rows");
+  TNX_REQUIRE(!pos || (n_pos > 0 && starts), "embed_rows: learned positions need their number and the first columns");
   TNX_REQUIRE(dtype == TNX_BF16 || dtype == TNX_F32, "embed_rows: bad dtype %d", dtype);
   if (dtype == TNX_BF16)
     hipLaunchKernelGGL(embed_rows_kernel<uint16_t>, dim3((unsigned)(B * T)), dim3(256), 0, as_stream(stream), (const uint16_t*)table,
-                       V, D, ids, ids_ld, col_ptr, T, scale, x, (uint16_t*)cat, cat_ld, cat_off, cat_frag);
+                       V, D, ids, ids_ld, col_ptr, T, scale, x, (uint16_t*)cat, cat_ld, cat_off, cat_frag, (const uint16_t*)pos, n_pos, starts);
   else
     hipLaunchKernelGGL(embed_rows_kernel<float>, dim3((unsigned)(B * T)), dim3(256), 0, as_stream(stream), (const float*)table, V, D,
-                       ids, ids_ld, col_ptr, T, scale, x, (float*)cat, cat_ld, cat_off, cat_frag);
+                       ids, ids_ld, col_ptr, T, scale, x, (float*)cat, cat_ld, cat_off, cat_frag, (const float*)pos, n_pos, starts);
   TNX_CHECK_LAUNCH("embed_rows");
   return TNX_OK;
 }
@@ -1399,6 +1412,7 @@ extern "C" int tnx_residual_norm(void* stream, const tnx_residual_norm_desc* d) 
               "residual_norm: a shift needs the rows before, their columns and no next norm");
   TNX_REQUIRE(!d->shift || d->T == 1 || (d->x_out && d->x_out != d->x), "residual_norm: a shift over several tokens needs a second buffer");
   TNX_REQUIRE(d->dtype == TNX_BF16 || d->dtype == TNX_F32, "residual_norm: bad dtype %d", d->dtype);
+  if (d->center || (d->mult != 0.f && d->mult != 1.f) || d->extra.ld > 0 || d->hist) return tnx_internal_layer_step(as_stream(stream), d);
   ResNormArgs a;
   a.M = d->M; a.D = d->D; a.eps = d->eps; a.w_offset = d->w_offset; a.y = d->y.y; a.ws = d->y.ws;
   a.split = d->y.split_k < 1 ? 1 : d->y.split_k; a.plane = d->y.plane; a.y_ld = arrives ? d->y.ld : 8; a.mode = d->mode;
@@ -1512,12 +1526,14 @@ extern "C" int tnx_part_rope_kvwrite(void* stream, const tnx_part_rope_desc* d) 
 
 extern "C" int tnx_gated_norm(void* stream, const tnx_gated_norm_desc* d) {
   TNX_REQUIRE(d, "gated_norm: null descriptor");
-  TNX_REQUIRE(d->M > 0 && d->W > 0 && d->o && d->o_ld >= d->W && src_given(d->g) && d->w && d->out && d->out_ld >= d->W,
+  TNX_REQUIRE(d->M > 0 && d->W > 0 && d->o && d->o_ld >= d->W && (src_given(d->g) || (d->g.ld == 0 && !d->gate_first)) && d->w && d->out && d->out_ld >= d->W,
               "gated_norm: null pointer or bad shape");
   TNX_REQUIRE(d->dtype == TNX_BF16 || d->dtype == TNX_F32, "gated_norm: bad dtype %d", d->dtype);
   GatedNormArgs a;
   a.W = d->W; a.o_ld = d->o_ld; a.out_ld = d->out_ld; a.g_off = d->g_off; a.eps = d->eps; a.w_offset = d->w_offset;
   a.w = d->w; a.o = d->o; a.out_frag = d->out_frag; a.groups = d->groups < 1 ? 1 : d->groups;
+  a.w_len = d->shared_w ? d->W / a.groups : d->W;
+  TNX_REQUIRE(!d->shared_w || !d->gate_first, "gated_norm: shared weights go with the gate behind the norm");
   TNX_REQUIRE(d->W % a.groups == 0 && a.groups <= 1024, "gated_norm: the row does not divide into %d parts, or into more than 1024", a.groups);
   if (d->gate_first)
     return d->dtype == TNX_BF16 ? launch_gate_first(as_stream(stream), d->M, a, row_src<uint16_t>(d->g), (uint16_t*)d->out)

@@ -67,6 +67,12 @@ __device__ __forceinline__ bool find_block(const int32_t* offsets, int n_experts
   return true;
 }
 
+__device__ __forceinline__ f32x4 square_relu(f32x4 v) {
+#pragma unroll
+  for (int e = 0; e < 4; ++e) v[e] = fmaxf(v[e], 0.f) * fmaxf(v[e], 0.f);
+  return v;
+}
+
 constexpr int kDenseKT = 128;   // k-tile of the fragment layout: eight 16-deep slabs
 
 // A work-group of four waves owns 32 * RT rows x 64 columns (two 32-column groups); its waves take
@@ -219,8 +225,9 @@ void dense_rows_kernel(const DenseArgs a) {
         }
       } else if (col < a.N) {   // bf16: N is a multiple of 16
         uint16_t* y = reinterpret_cast<uint16_t*>(a.y) + y_at;
+        const f32x4 u = a.epilogue == TNX_EPI_RELU2 ? square_relu(v) : v;
         *reinterpret_cast<u32x2*>(y + (a.y_frag ? frag_index(row, col, a.ldy) : row * a.ldy + col)) =
-            u32x2{pack2bf(v[0], v[1]), pack2bf(v[2], v[3])};
+            u32x2{pack2bf(u[0], u[1]), pack2bf(u[2], u[3])};
       }
     }
   }
@@ -280,7 +287,7 @@ __global__ __launch_bounds__(256) void dense_f32_kernel(const DenseArgs a) {
     if constexpr (MODE == kExperts) row = a.sorted_route[row];
 #pragma unroll
     for (int j = 0; j < 4; ++j)
-      if (n0 + tx * 4 + j < N) y[row * ldy + n0 + tx * 4 + j] = acc[i][j];
+      if (n0 + tx * 4 + j < N) y[row * ldy + n0 + tx * 4 + j] = a.epilogue == TNX_EPI_RELU2 ? fmaxf(acc[i][j], 0.f) * fmaxf(acc[i][j], 0.f) : acc[i][j];
   }
 }
 
@@ -314,7 +321,7 @@ extern "C" int tnx_dense_linear(void* stream, const tnx_dense_desc* d) {
   if (d->dtype == TNX_F32) {
     TNX_REQUIRE(d->K % 16 == 0 && d->ldx % 4 == 0 && d->ldx >= d->K && d->ldy >= d->N,
                 "dense_linear: fp32 needs K %% 16 == 0 and row strides that hold the rows");
-    TNX_REQUIRE((d->epilogue == TNX_EPI_STORE || d->epilogue == TNX_EPI_F32) && d->split_k <= 1 && !d->x_frag && !d->y_frag,
+    TNX_REQUIRE((d->epilogue == TNX_EPI_STORE || d->epilogue == TNX_EPI_F32 || d->epilogue == TNX_EPI_RELU2) && d->split_k <= 1 && !d->x_frag && !d->y_frag,
                 "dense_linear: fp32 stores row-major results only");
     const int64_t blocks = experts ? d->M / 64 + (d->n_experts < d->M ? d->n_experts : d->M) : cdiv(d->M, 64);
     TNX_REQUIRE(blocks <= 65535, "dense_linear: too many rows in one call");
@@ -328,7 +335,8 @@ extern "C" int tnx_dense_linear(void* stream, const tnx_dense_desc* d) {
   }
   TNX_REQUIRE(d->K % kDenseKT == 0, "dense_linear: K=%lld must be a multiple of 128 (zero-pad)", (long long)d->K);
   const bool mul = d->epilogue == TNX_EPI_GELU_MUL || d->epilogue == TNX_EPI_SILU_MUL;
-  TNX_REQUIRE(d->epilogue == TNX_EPI_STORE || d->epilogue == TNX_EPI_F32 || mul, "dense_linear: bad epilogue %d", d->epilogue);
+  TNX_REQUIRE(d->epilogue == TNX_EPI_STORE || d->epilogue == TNX_EPI_F32 || d->epilogue == TNX_EPI_RELU2 || mul, "dense_linear: bad epilogue %d", d->epilogue);
+  TNX_REQUIRE(d->epilogue != TNX_EPI_RELU2 || d->split_k <= 1, "dense_linear: an activation needs whole sums: no k split");
   TNX_REQUIRE(d->epilogue == TNX_EPI_F32 || d->split_k > 1 || d->N % 16 == 0, "dense_linear: N=%lld must be a multiple of 16", (long long)d->N);
   if (mul) TNX_REQUIRE(d->N % 32 == 0 && d->split_k <= 1, "dense_linear: a gated unit needs N %% 32 == 0 and no k split");
   const int64_t ncols = mul ? d->N / 2 : d->N;

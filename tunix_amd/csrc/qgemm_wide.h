@@ -567,6 +567,14 @@ void qgemm_wide_kernel(const QLArgs a, const WideHead h) {
     }
   }
   if constexpr (PRE) {
+    if (a.epilogue == TNX_EPI_RELU2) {
+#pragma unroll
+      for (int rt = 0; rt < RT; ++rt)
+#pragma unroll
+        for (int cg = 0; cg < CG; ++cg)
+#pragma unroll
+          for (int i = 0; i < 16; ++i) acc[rt][cg][i] = fmaxf(acc[rt][cg][i], 0.f) * fmaxf(acc[rt][cg][i], 0.f);
+    }
     if (h.part != nullptr && h.softcap > 0.f) {
 #pragma unroll
       for (int rt = 0; rt < RT; ++rt)

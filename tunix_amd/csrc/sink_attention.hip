@@ -1,7 +1,8 @@
 // Causal grouped-query attention with a learned sink per head, separate key and value head sizes
 // and an arbitrary score scale, over caches K [B, G, S, dkp] and V [B, G, S, dvp] whose rows are
 // zero-padded.  Scores, softmax and its running sums are fp32.  A row's keys start at starts[b]
-// (left padding), whatever their token ids.
+// (left padding), whatever their token ids.  A head may take off its score a slope times the distance, and a position may
+// see its own chunk of positions only (BIAS).
 //
 //   sink_attn_tile_kernel   many query positions: 128 query rows per work-group, keys and values
 //                           staged through LDS, 32x32x16 MFMAs
@@ -30,7 +31,14 @@ struct SinkArgs {
   int64_t out_ld;
   int out_frag;
   int64_t out_head;        // distance of two heads in an output row
+  const float* slopes;     // [H] or null
+  int chunk;               // positions of a chunk, 0: no chunks
 };
+
+// the first column that the position in column `col` sees
+__device__ __forceinline__ int first_seen(int col, int start, int chunk) {
+  return chunk > 0 && col > start ? start + (col - start) / chunk * chunk : start;
+}
 
 constexpr float kNegBig = -1.0e30f;
 constexpr float kLog2e = 1.4426950408889634f;
@@ -50,7 +58,8 @@ __global__ __launch_bounds__(256) void sink_attn_any_kernel(const SinkArgs a) {
   __shared__ float p[256], red[4];
   const int h = blockIdx.x, g = h / a.R;
   const int64_t row = blockIdx.y, b = row / a.T, t = row % a.T;
-  const int tid = threadIdx.x, last = *a.col_ptr + (int)t, first = a.starts[b];
+  const int tid = threadIdx.x, last = *a.col_ptr + (int)t, first = first_seen(last, a.starts[b], a.chunk);
+  const float slope = a.slopes ? a.slopes[h] : 0.f;
   const T* q = reinterpret_cast<const T*>(a.q) + (row * a.H + h) * a.dkp;
   const T* k = reinterpret_cast<const T*>(a.k) + (b * a.G + g) * a.S * a.dkp;
   const T* v = reinterpret_cast<const T*>(a.v) + (b * a.G + g) * a.S * a.dvp;
@@ -64,7 +73,7 @@ __global__ __launch_bounds__(256) void sink_attn_any_kernel(const SinkArgs a) {
       if (tid < n) {
         float d = 0.f;
         for (int i = 0; i < a.dk; ++i) d += ld_elem(q, i) * ld_elem(k, (int64_t)key * a.dkp + i);
-        s = d * a.scale * kLog2e;
+        s = (d * a.scale - slope * (float)(last - key)) * kLog2e;
       }
       float mx = wave_max(s);
       __syncthreads();
@@ -111,7 +120,7 @@ __global__ __launch_bounds__(256) void sink_attn_any_kernel(const SinkArgs a) {
 // One wave per (16 query rows of a (row, kv head), key chunk).  S^T = K . q^T leaves every lane with
 // the scores of one query for eight keys: the A fragment of the P . V product.  Keys and values flow
 // through a ring of register stages; every load is unconditional so the waits count exactly.
-template <int KS, int NH, int NJ>   // 32-deep k-steps, halves of V, value columns per lane and half
+template <int KS, int NH, int NJ, bool BIAS>   // 32-deep k-steps, halves of V, value columns per lane and half
 __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 2))) void sink_attn_step_kernel(const SinkArgs a) {
   constexpr int DK = KS * 32, DV = NH * NJ * 16;
   constexpr int NS = KS * 8 + NH * 4 * NJ <= 64 ? 2 : 1;
@@ -127,10 +136,17 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 2))) void
   const int tq = qvalid ? (int)(qrow / a.R) : 0, rq = qvalid ? (int)(qrow % a.R) : 0;
   const int c_n = min(col0 + tq, (int)a.S - 1);
   const uint16_t* q = reinterpret_cast<const uint16_t*>(a.q) + ((b * a.T + tq) * a.H + g * a.R + rq) * DK;
-  int k_lo = start, k_hi = min(col0 + (int)a.T - 1, (int)a.S - 1);
+  int k_lo = start, k_hi = min(col0 + (int)a.T - 1, (int)a.S - 1), split0 = 0, seen = start;
+  float slope2 = 0.f;
+  if constexpr (BIAS) {
+    k_lo = first_seen(col0 + (int)(qt * 16u / a.R), start, a.chunk);   // (of the tile's first position; later ones see no earlier key)
+    seen = first_seen(c_n, start, a.chunk);
+    split0 = a.chunk > 0 ? first_seen(col0, start, a.chunk) & ~31 : 0;
+    if (a.slopes) slope2 = a.slopes[g * a.R + rq] * kLog2e;
+  }
   if (a.n_chunks > 1) {
-    k_lo = max(k_lo, chunk * a.kv_chunk);
-    k_hi = min(k_hi, chunk * a.kv_chunk + a.kv_chunk - 1);
+    k_lo = max(k_lo, split0 + chunk * a.kv_chunk);
+    k_hi = min(k_hi, split0 + chunk * a.kv_chunk + a.kv_chunk - 1);
   }
   u32x4 qf[KS];
 #pragma unroll
@@ -179,7 +195,9 @@ __global__ __launch_bounds__(64) __attribute__((amdgpu_waves_per_eu(1, 2))) void
     for (int s = 0; s < 8; ++s) {
       const int key = kb + (s < 4 ? 4 * lq + s : 16 + 4 * lq + (s - 4));
       ok[s] = qvalid && key >= k_lo && key <= min(k_hi, c_n);
+      if constexpr (BIAS) ok[s] = ok[s] && key >= seen;
       sv[s] = st[s >> 2][s & 3] * sc2;
+      if constexpr (BIAS) sv[s] = __builtin_fmaf(slope2, (float)(key - c_n), sv[s]);
       if (ok[s]) bmax = fmaxf(bmax, sv[s]);
     }
     bmax = fmaxf(bmax, __shfl_xor(bmax, 16, 64));
@@ -311,7 +329,7 @@ __global__ __launch_bounds__(128) void sink_attn_merge_kernel(const SinkArgs a) 
 // transposed, S^T = K . Q^T and O^T = V^T . P^T: a lane holds the scores, the probabilities (already
 // the B operand of the second product, in a permuted key order that the V fragments follow) and the
 // output of ONE query, so the softmax state is per lane.
-template <int KD, int NV>   // 16-deep k-steps of the head size; 32-column groups of the value size
+template <int KD, int NV, bool BIAS>   // 16-deep k-steps of the head size; 32-column groups of the value size
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(KD + NV > 11 ? 1 : 2, 2)))
 void sink_attn_tile_kernel(const SinkArgs a) {
   constexpr int DK = KD * 16, DV = NV * 32, KT = 64;
@@ -343,7 +361,11 @@ void sink_attn_tile_kernel(const SinkArgs a) {
 #pragma unroll
     for (int i = 0; i < 16; ++i) O[j][i] = 0.f;
   float m_run = kNegBig, l_run = 0.f;
-  const float sc2 = a.scale * kLog2e, factor = sc2 > 0.f ? sc2 : 1.0f;
+  const float sc2 = a.scale * kLog2e, factor = !BIAS && sc2 > 0.f ? sc2 : 1.0f;
+  // columns that this position, and the first and last one of the wave, see first
+  const int seen = BIAS ? first_seen(c_n, start, a.chunk) : start;
+  const int w_first = BIAS ? first_seen(w_lo, start, a.chunk) : start, w_last = BIAS ? first_seen(w_hi, start, a.chunk) : start;
+  const float slope2 = BIAS && a.slopes ? a.slopes[head] * kLog2e : 0.f;
   const rsrc_t rk = make_rsrc(reinterpret_cast<const uint16_t*>(a.k) + (b * a.G + g) * a.S * DK, (uint64_t)a.S * DK * 2);
   const rsrc_t rv = make_rsrc(reinterpret_cast<const uint16_t*>(a.v) + (b * a.G + g) * a.S * DV, (uint64_t)a.S * DV * 2);
   constexpr int KC = KT * DK / 8 / 256, VC = KT * DV / 8 / 256;   // 16-byte chunks per thread
@@ -360,7 +382,8 @@ void sink_attn_tile_kernel(const SinkArgs a) {
       vr[c] = __builtin_amdgcn_raw_buffer_load_b128(rv, (uint32_t)((kb + r) * DV + ch * 8) * 2u, 0, 0);
     }
   };
-  const int kb0 = max(start, 0) & ~(KT - 1);
+  int kb0 = max(start, 0) & ~(KT - 1);
+  if constexpr (BIAS) kb0 = first_seen(col0 + (int)(min((unsigned)tile * 128, rows - 1) / a.R), start, a.chunk) & ~(KT - 1);
   if (kb0 <= t_hi) fetch(kb0);
   for (int kb = kb0; kb <= t_hi; kb += KT) {
     __syncthreads();
@@ -376,7 +399,7 @@ void sink_attn_tile_kernel(const SinkArgs a) {
     }
     __syncthreads();
     if (kb + KT <= t_hi) fetch(kb + KT);
-    if (kb > w_hi) continue;                                   // (wave-uniform: nothing visible in this tile)
+    if (kb > w_hi || (BIAS && kb + KT - 1 < w_first)) continue;   // (wave-uniform: nothing visible in this tile)
     f32x16 st[2];
 #pragma unroll
     for (int hf = 0; hf < 2; ++hf) {
@@ -386,20 +409,26 @@ void sink_attn_tile_kernel(const SinkArgs a) {
       for (int j = 0; j < KD; ++j)
         st[hf] = mfma32(*reinterpret_cast<const u32x4*>(&ks[(hf * 32 + l32) * KLD + j * 16 + lh * 8]), qf[j], st[hf]);
     }
-    if (sc2 <= 0.f) {   // (uniform; the maximum below is taken over unscaled scores)
+    if constexpr (BIAS) {
+      const float far = slope2 * (float)(kb + 4 * lh - c_n);
+#pragma unroll
+      for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) st[hf][i] = __builtin_fmaf(st[hf][i], sc2, __builtin_fmaf(slope2, (float)(hf * 32 + 8 * (i >> 2) + (i & 3)), far));
+    } else if (sc2 <= 0.f) {   // (uniform; the maximum below is taken over unscaled scores)
 #pragma unroll
       for (int hf = 0; hf < 2; ++hf)
 #pragma unroll
         for (int i = 0; i < 16; ++i) st[hf][i] *= sc2;
     }
     // register 4 b + e of st[hf]: key kb + 32 hf + 8 b + 4 lh + e
-    if (!(kb >= start && kb + KT - 1 <= w_lo)) {
+    if (!(kb >= w_last && kb + KT - 1 <= w_lo)) {
 #pragma unroll
       for (int hf = 0; hf < 2; ++hf)
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
           const int key = kb + hf * 32 + 8 * (i >> 2) + 4 * lh + (i & 3);
-          if (key < start || key > c_n) st[hf][i] = -__builtin_inff();
+          if (key < seen || key > c_n) st[hf][i] = -__builtin_inff();
         }
     }
     float mx = st[0][0];
@@ -488,7 +517,9 @@ void sink_attn_tile_kernel(const SinkArgs a) {
 template <int KS, int NH, int NJ>
 void launch_step(hipStream_t st, const SinkArgs& a) {
   const unsigned qts = (unsigned)cdiv(a.T * a.R, 16);
-  hipLaunchKernelGGL((sink_attn_step_kernel<KS, NH, NJ>), dim3((unsigned)a.n_chunks, (unsigned)a.G * qts, (unsigned)a.B), dim3(64), 0, st, a);
+  const dim3 grid((unsigned)a.n_chunks, (unsigned)a.G * qts, (unsigned)a.B);
+  if (a.slopes || a.chunk > 0) hipLaunchKernelGGL((sink_attn_step_kernel<KS, NH, NJ, true>), grid, dim3(64), 0, st, a);
+  else hipLaunchKernelGGL((sink_attn_step_kernel<KS, NH, NJ, false>), grid, dim3(64), 0, st, a);
 }
 template <int KS>
 int launch_step_v(hipStream_t st, const SinkArgs& a) {
@@ -500,8 +531,9 @@ int launch_step_v(hipStream_t st, const SinkArgs& a) {
 }
 template <int KD, int NV>
 void launch_tile(hipStream_t st, const SinkArgs& a) {
-  hipLaunchKernelGGL((sink_attn_tile_kernel<KD, NV>), dim3((unsigned)cdiv(a.T * a.R, 128), (unsigned)a.G, (unsigned)a.B), dim3(256), 0,
-                     st, a);
+  const dim3 grid((unsigned)cdiv(a.T * a.R, 128), (unsigned)a.G, (unsigned)a.B);
+  if (a.slopes || a.chunk > 0) hipLaunchKernelGGL((sink_attn_tile_kernel<KD, NV, true>), grid, dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((sink_attn_tile_kernel<KD, NV, false>), grid, dim3(256), 0, st, a);
 }
 template <int KD>
 int launch_tile_v(hipStream_t st, const SinkArgs& a) {
@@ -542,7 +574,10 @@ extern "C" int tnx_sink_attn(void* stream, const tnx_sink_attn_desc* d) {
   a.dvp = d->dvp; a.scale = d->scale; a.q = d->q; a.k = d->kcache; a.v = d->vcache; a.sinks = d->sinks; a.starts = d->starts;
   a.col_ptr = d->col_ptr; a.ws = d->ws; a.out = d->out; a.out_ld = d->out_ld; a.out_frag = d->out_frag;
   a.out_head = d->out_head ? d->out_head : d->dv;
-  a.kv_chunk = d->kv_chunk; a.n_chunks = d->kv_chunk > 0 && d->kv_chunk < d->S ? (int)cdiv(d->S, d->kv_chunk) : 1;
+  a.slopes = d->slopes; a.chunk = d->chunk > 0 && d->chunk < d->S ? d->chunk : 0;
+  // one position sees at most its chunk; the splits begin at a block's edge in front of it
+  const int64_t span = a.chunk > 0 && d->T == 1 && a.chunk + 31 < d->S ? a.chunk + 31 : d->S;
+  a.kv_chunk = d->kv_chunk; a.n_chunks = d->kv_chunk > 0 && d->kv_chunk < span ? (int)cdiv(span, d->kv_chunk) : 1;
   hipStream_t st = as_stream(stream);
   const bool mfma = d->dtype == TNX_BF16 && mfma_sizes(d->dkp, d->dvp) && (uint64_t)d->S * (uint64_t)(d->dkp > d->dvp ? d->dkp : d->dvp) * 2 < (1ull << 31);
   if (!mfma) {

@@ -77,6 +77,13 @@ def create_stack_weights(cfg: StackConfig, seed: int = 0, device="cpu", scale: f
     t = torch.randn(*shape, generator=gen, device=dev, dtype=torch.float32)
     if name.endswith(("mix.sink", "mix.dt_bias")):
       pass
+    elif name.endswith("mix.lower"):
+      t = torch.sigmoid(t)
+    elif name.endswith(".dwa"):
+      t = 0.1 * t
+      t[-1] += 1.0
+    elif name.endswith(("mlp.act", "mlp.correction")):
+      t = 0.3 * t
     elif name.endswith(".talk"):
       t = torch.eye(shape[0], device=dev) + t * (0.3 * shape[0] ** -0.5)
     elif name.endswith("mix.A_log"):

@@ -23,6 +23,7 @@ class _Batch:
     self.rows = {r: i for i, r in enumerate(ids)}     # live request -> slot
     self.st = st
     self.column = st.num_input_tokens                 # column of the next token
+    self.first = st.starts.tolist()                   # column of each row's first token
     self.runner = None
 
 
@@ -59,6 +60,7 @@ class Replay:
   def _start(self, entries: list[dict]) -> list[np.ndarray]:
     lengths = [len(e["tokens"]) for e in entries]
     P = max(lengths)
+    utils.check_positions(self.model, P)
     ids = np.array([utils.pad_to_length(np.asarray(e["tokens"], dtype=np.int32), P, PAD_ID, left=True) for e in entries])
     S = utils.next_power_of_2(P + 64)
     st = _SamplingState(self.model, ids, S, S, PAD_ID, False, False, lengths=lengths)
@@ -81,6 +83,8 @@ class Replay:
       raise ValueError("the requests of a running batch go on together, one token each")
     st, model = batch.st, self.model
     B, S = st.token_buffer.shape
+    for e in entries:
+      utils.check_positions(model, batch.column + 1 - batch.first[batch.rows[e["id"]]])
     if batch.column >= S:
       S *= 2
       st.cache.grow(S)

@@ -251,6 +251,7 @@ class Sampler:
     max_tokens_length = max(len(x) for x in tokens)
     if max_prompt_length is None or max_prompt_length < max_tokens_length:
       max_prompt_length = utils.next_power_of_2(max_tokens_length)
+    utils.check_positions(model, max_tokens_length + max_generation_steps - 1)   # (the last token is not fed back)
     pad = self.tokenizer.pad_id()
     all_input_ids = np.array([
         utils.pad_to_length(x, target_length=max_prompt_length, pad_value=pad, left=True)

@@ -79,3 +79,10 @@ class IdTokenizer:
     while i + 1 < len(ids) and ids[i] == self._bos and ids[i + 1] == self._bos:
       i += 1
     return ids[i:]
+
+
+def check_positions(model, n: int):
+  """Whether a sequence of n tokens fits a model that learns a vector per position."""
+  most = getattr(model.cfg, "max_positions", 0)
+  if most and n > most:
+    raise ValueError(f"a sequence of {n} tokens, but the model has {most} positions")

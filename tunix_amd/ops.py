@@ -311,11 +311,12 @@ def dense_linear(desc: L.DenseDesc):
   L.check(L.lib().tnx_dense_linear(_stream(), C.byref(desc)), "tnx_dense_linear")
 
 
-def embed_rows(table, ids, col_ptr, B, T, V, D, x, cat=None, cat_off=0, cat_frag=False, scale=1.0):
-  """x fp32 [B*T, D] = scaled rows of `table` [V, D]; cat: a second, unscaled copy in the table's dtype."""
+def embed_rows(table, ids, col_ptr, B, T, V, D, x, cat=None, cat_off=0, cat_frag=False, scale=1.0, pos=None, starts=None):
+  """x fp32 [B*T, D] = scaled rows of `table` [V, D], plus the rows of `pos` at the tokens' positions; cat: a second, unscaled
+  copy in the table's dtype."""
   L.check(L.lib().tnx_embed_rows(_stream(), DTYPES[table.dtype], _ptr(table), V, D, _ptr(ids), ids.shape[1],
                                  _ptr(col_ptr), B, T, float(scale), _ptr(x), _ptr(cat), 0 if cat is None else cat.shape[1], cat_off,
-                                 1 if cat_frag else 0), "tnx_embed_rows")
+                                 1 if cat_frag else 0, _ptr(pos), 0 if pos is None else pos.shape[0], _ptr(starts)), "tnx_embed_rows")
 
 
 def rows_src(y=None, ws=None, split_k=1, plane=0, ld=0) -> L.RowsSrc:
@@ -331,6 +332,10 @@ def residual_norm(desc: L.ResidualNormDesc):
 
 def part_rope_kvwrite(desc: L.PartRopeDesc):
   L.check(L.lib().tnx_part_rope_kvwrite(_stream(), C.byref(desc)), "tnx_part_rope_kvwrite")
+
+
+def rownorm_kvwrite(desc: L.RowNormKvDesc):
+  L.check(L.lib().tnx_rownorm_kvwrite(_stream(), C.byref(desc)), "tnx_rownorm_kvwrite")
 
 
 def sink_attn_pad(dim: int, value: bool, dtype) -> int:
@@ -354,6 +359,18 @@ def lightning(desc: L.LightningDesc):
   L.check(L.lib().tnx_lightning(_stream(), C.byref(desc)), "tnx_lightning")
 
 
+def gated_state_step_ok(dk, dv) -> bool:
+  return bool(L.lib().tnx_gated_state_step_ok(dk, dv))
+
+
+def gated_state_ws_bytes(B, T, H, dk, dv) -> int:
+  return int(L.lib().tnx_gated_state_ws_bytes(B, T, H, dk, dv))
+
+
+def gated_state(desc: L.GatedStateDesc):
+  L.check(L.lib().tnx_gated_state(_stream(), C.byref(desc)), "tnx_gated_state")
+
+
 def gated_norm(desc: L.GatedNormDesc):
   L.check(L.lib().tnx_gated_norm(_stream(), C.byref(desc)), "tnx_gated_norm")
 
@@ -370,6 +387,16 @@ def silu_mul(y, up_off, M, F, out):
 
 def route_softmax(src: L.RowsSrc, M, E, k, topk_w, topk_id):
   L.check(L.lib().tnx_route_softmax(_stream(), C.byref(src), M, E, k, _ptr(topk_w), _ptr(topk_id)), "tnx_route_softmax")
+
+
+def route_scores(src: L.RowsSrc, M, E, k, correction, scale, topk_w, topk_id, gate_off=0, gate_w=None):
+  L.check(L.lib().tnx_route_scores(_stream(), C.byref(src), M, E, k, _ptr(correction), float(scale), gate_off, _ptr(topk_w), _ptr(topk_id),
+                                   _ptr(gate_w)), "tnx_route_scores")
+
+
+def poly_norm(src: L.RowsSrc, dtype, M, F, coef, eps, out, out_frag):
+  L.check(L.lib().tnx_poly_norm(_stream(), DTYPES[dtype], C.byref(src), M, F, _ptr(coef), float(eps), _ptr(out), out.shape[1],
+                                1 if out_frag else 0), "tnx_poly_norm")
 
 
 def short_conv(desc: L.ShortConvDesc):

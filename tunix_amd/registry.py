@@ -43,6 +43,7 @@ ARCHITECTURES: dict[str, Architecture] = {
     "Nunezen": _stack(config.nunezen_from_dict),
     "Lapevik": _stack(config.lapevik_from_dict),
     "Kuzezen": _stack(config.kuzezen_from_dict),
+    "Kezolix": _stack(config.kezolix_from_dict),
 }
 
 

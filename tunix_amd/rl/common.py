@@ -18,6 +18,7 @@ import numpy as np
 import torch
 
 from .. import ops
+from ..generate.utils import check_positions
 from ..model import QLoRAModel
 
 
@@ -106,6 +107,9 @@ def compute_per_token_logps(model: QLoRAModel, prompt_tokens, completion_tokens,
   cache = model.new_cache(rows_b, Ltot, shared=True)
   # column of each row's first token: behind the prompt's leading padding
   starts = torch.cumprod((ids == pad_id).to(torch.int32), dim=1).sum(dim=1).to(torch.int32)
+  if getattr(cfg, "max_positions", 0):   # (padding behind a completion has no position)
+    behind = torch.cumprod((ids.flip(1) == pad_id).to(torch.int32), dim=1).sum(dim=1)
+    check_positions(model, int((Ltot - behind - starts).max()))
   head_rows = rows_b * T if chunk_size <= 0 else rows_b * min(T, chunk_size)
   head_rows = min(head_rows, 8192)
   part = torch.empty(head_rows * runner.nvb * 4, dtype=torch.float32, device=dev)

@@ -15,8 +15,8 @@ import torch
 
 from . import _lib as L
 from . import ops
-from .cache import KVSpec, LatentSpec, PartsSpec, RingSpec, SequenceCache, StateSpec
-from .config import AttentionMixer, ExpertsMlp, LatentMixer, LightningMixer, MemoryMixer, MixedAttentionMixer, ParallelMixer, SsdMixer, StackConfig
+from .cache import BorrowedSpec, KVSpec, LatentSpec, PartsSpec, RingSpec, SequenceCache, StateSpec
+from .config import AttentionMixer, ExpertsMlp, GatedStateMixer, LatentMixer, LightningMixer, MemoryMixer, MixedAttentionMixer, ParallelMixer, PolyNormMlp, SsdMixer, StackConfig
 from .model import HeadRunner
 
 
@@ -30,12 +30,13 @@ FRAG_ROWS = 512
 
 class DenseLinear:
   """One dense projection, possibly several weights [N_i, K] that share an input.  A member is a name, or
-  (name, first row, end row) for some rows of a weight.  Every member starts at a multiple of 16 output
-  columns (`offsets`), K is zero-padded to a multiple of 128.
+  (name, first row, end row) for some rows of a weight.  Every member starts at a multiple of `align` (16) output
+  columns (`offsets`), K is zero-padded to a multiple of 128.  Runs of 256 columns lie behind each other in memory: at an
+  offset that is a multiple of 256 a call may begin or end.
   paired: two members of one shape whose rows alternate in blocks of 16 (gate | up), so that the
   kernel's epilogue finds both in one wave (bf16).  transpose: the members' transposes."""
 
-  def __init__(self, members: list, weights: dict, dtype, device, paired: bool = False, transpose: bool = False):
+  def __init__(self, members: list, weights: dict, dtype, device, paired: bool = False, transpose: bool = False, align: int = 16):
     self.members = [m if isinstance(m, tuple) else (m, 0, weights[m].shape[0]) for m in members]
     self.names, self.dtype, self.device, self.paired = [m[0] for m in self.members], dtype, device, paired
     self.transpose = transpose
@@ -43,7 +44,7 @@ class DenseLinear:
     self.shapes = [(r1 - r0, s[1])[::-1 if transpose else 1] for (_, r0, r1), s in zip(self.members, self.full_shapes)]
     self.K = self.shapes[0][1]
     self.Kp = _up(self.K, 128)
-    widths = [_up(s[0], 16) for s in self.shapes]
+    widths = [_up(s[0], align) for s in self.shapes]
     self.offsets = [sum(widths[:i]) for i in range(len(widths))]
     self.N = sum(widths)
     self.w = None
@@ -121,8 +122,8 @@ class StackModel:
     self.transposed: set[str] = set()                  # vectors kept as [taps, channels]
     self.vectors: dict[str, torch.Tensor] = {"final.norm": self.final_norm}
 
-    def linear(members, paired=False, transpose=False):
-      f = DenseLinear(members, weights, dtype, dev, paired, transpose)
+    def linear(members, paired=False, transpose=False, align=16):
+      f = DenseLinear(members, weights, dtype, dev, paired, transpose, align)
       for n in dict.fromkeys(f.names):
         self.linears.setdefault(n, []).append(f)
       return f
@@ -141,6 +142,7 @@ class StackModel:
       self.transposed.add(name)
       return buf
 
+    self.pos = torch.empty(cfg.max_positions, D, dtype=dtype, device=dev) if cfg.max_positions else None
     self.embed_norm = vector("embed.norm") if cfg.embed_norm else None
     looped = cfg.loop is not None
     self.loop_in = linear(["loop.in"]) if looped and not cfg.loop.step else None
@@ -151,6 +153,8 @@ class StackModel:
       ly = {"spec": spec, "norm1": vector(p + "norm1") if cfg.pre_norm else None, "post1": None if cfg.parallel else vector(p + cfg.post_norm(1))}
       if cfg.token_shift:
         ly["shift"] = vector(p + "shift")
+      if cfg.depth_average:
+        ly["dwa"] = vector(p + "dwa")
       if isinstance(m, SsdMixer):
         x = p + "mix."
         ly["in"] = linear([(x + "in", 0, m.inner), (x + "in", m.inner, m.inner + m.channels),
@@ -183,8 +187,15 @@ class StackModel:
         ly["canon1"] = taps(p + "canon1")
         if spec.mlp is not None:
           ly["canon2"] = taps(p + "canon2")
+      elif isinstance(m, GatedStateMixer):
+        # (the gates' columns begin at a run of 256, so that a prompt pass can keep them, and only them, in fp32)
+        ly["in"] = linear([p + "mix.q", p + "mix.v", p + "mix.f"], align=256)
+        ly["bias"], ly["lower"], ly["norm"] = vector(p + "mix.f.b"), vector(p + "mix.lower"), vector(p + "mix.norm")
       elif isinstance(m, AttentionMixer):
-        ly["in"] = linear([p + "mix.q", p + "mix.k", p + "mix.v"])
+        ly["in"] = linear([p + "mix.q"] if m.kv_from is not None else [p + "mix.q", p + "mix.k", p + "mix.v"])
+        if m.row_norm:
+          ly["q_norm"], ly["k_norm"] = vector(p + "mix.q.norm"), None if m.kv_from is not None else vector(p + "mix.k.norm")
+        ly["slopes"] = torch.tensor(m.slopes, dtype=torch.float32, device=dev) if m.slopes else None
         ly["sink"] = vector(p + "mix.sink") if m.sink else None
         freq = np.float64(m.rot_base) ** (-2.0 * np.arange(m.rot_dims // 2) / max(m.rot_dims, 1))
         ly["inv_freq"] = torch.from_numpy(freq.astype(np.float32)).to(dev)
@@ -198,9 +209,15 @@ class StackModel:
         ly["norm2"], ly["post2"] = vector(p + "norm2") if cfg.pre_norm else None, vector(p + cfg.post_norm(2))
       if isinstance(spec.mlp, ExpertsMlp):
         e = [p + f"mlp.e{j}." for j in range(spec.mlp.experts)]
-        ly["router"] = linear([p + "mlp.router"])
-        ly["gu"] = LinearBank([linear([n + "gate", n + "up"], paired=True) for n in e])
+        ly["router"] = linear([p + "mlp.router"] + ([p + "mlp.shared.sg"] if spec.mlp.shared_ff else []))
+        ly["gu"] = LinearBank([linear([n + "gate", n + "up"], paired=True) if spec.mlp.gated else linear([n + "up"]) for n in e])
         ly["down"] = LinearBank([linear([n + "down"]) for n in e])
+        if spec.mlp.corrected:
+          ly["correction"] = vector(p + "mlp.correction")
+        if spec.mlp.shared_ff:
+          ly["shared_up"], ly["shared_down"] = linear([p + "mlp.shared.up"]), linear([p + "mlp.shared.down"])
+      elif isinstance(spec.mlp, PolyNormMlp):
+        ly["gu"], ly["down"], ly["act"] = linear([p + "mlp.up"]), linear([p + "mlp.down"]), vector(p + "mlp.act")
       elif spec.mlp is not None:
         ly["gu"] = linear([p + "mlp.gate", p + "mlp.up"], paired=True)
         ly["down"] = linear([p + "mlp.down"])
@@ -216,8 +233,8 @@ class StackModel:
   def _load_tables(self, weights: dict):
     """The embedding table and the head, as far as `weights` has them."""
     head = "embed" if self.cfg.tied_head else "head"
-    for name, table in (("embed", self.embed), (head, self.head_w)):
-      if name in weights:
+    for name, table in (("embed", self.embed), ("pos", self.pos), (head, self.head_w)):
+      if table is not None and name in weights:
         table.copy_(weights[name].to(self.device, self.dtype))
     if head not in weights:
       return
@@ -245,7 +262,9 @@ class StackModel:
     specs = []
     for i, _ in self.cfg.layer_runs:
       m = self.cfg.layers[i].mixer
-      if isinstance(m, AttentionMixer):
+      if isinstance(m, AttentionMixer) and m.kv_from is not None:
+        spec = BorrowedSpec(m.kv_from)   # (layers with borrowed keys run once: a layer is its run)
+      elif isinstance(m, AttentionMixer):
         spec = KVSpec(m.kv_heads, ops.sink_attn_pad(m.dim, False, self.dtype),
                       ops.sink_attn_pad(m.vdim, True, self.dtype), self.dtype)
       elif isinstance(m, SsdMixer):
@@ -298,7 +317,7 @@ class StackModel:
     for i, begins in self.cfg.layer_runs:
       ly = self.layers[i]
       n += sum(part[k].nbytes() for part in (ly, ly.get("left", {}), ly.get("right", {}))
-               for k in ("in", "uq", "absorb_k", "absorb_v", "out", "router", "gates", "gu", "down") if hasattr(part.get(k), "nbytes"))
+               for k in ("in", "uq", "absorb_k", "absorb_v", "out", "router", "gates", "gu", "down", "shared_up", "shared_down") if hasattr(part.get(k), "nbytes"))
       n += self.loop_in.nbytes() if begins and self.loop_in is not None else 0
     return {"dense": n, "head": self.head_w.numel() * self.head_w.element_size()}
 
@@ -322,6 +341,9 @@ class StackRunner(HeadRunner):
     self._bufs: dict = {}
     D = cfg.embed_dim
     self.x = torch.empty(M, D, dtype=torch.float32, device=dev)
+    # the embedding output and every layer's result but the last one's, where they are averaged over depth
+    self.hist = torch.empty(cfg.num_layers, M, D, dtype=torch.float32, device=dev) if cfg.depth_average else None
+    self.first = None           # the embedding output, until a sublayer has been added
     # a token shift or an input convolution reads the rows in front of a row: over several tokens the new rows go to a
     # second buffer
     self.x_next = torch.empty_like(self.x) if (cfg.token_shift or cfg.input_conv > 1) and T > 1 else None
@@ -336,14 +358,15 @@ class StackRunner(HeadRunner):
       ly = model.layers[i]
       m = ly["spec"].mixer
       mlp_slot = 2 if cfg.parallel else 0
-      uses = [(ly, k, s) for k, s in (("in", 0), ("out", 0), ("router", 0), ("gu", mlp_slot), ("down", mlp_slot), ("uq", 1), ("ukv", 1))]
+      uses = [(ly, k, s) for k, s in (("in", 0), ("out", 0), ("router", 0), ("gu", mlp_slot), ("down", mlp_slot), ("uq", 1), ("ukv", 1), ("shared_down", 0))]
       if cfg.parallel:
         uses += [(ly["right"], "gates", 1), (ly["left"], "out", 0), (ly["right"], "out", 1)]
       for part, key, slot in uses:
         f = part.get(key)
         if isinstance(f, DenseLinear):
           n_y[slot] = max(n_y[slot], M * f.N)
-          n_ws[slot] = max(n_ws[slot], self._split(f) * M * f.N if self._split(f) > 1 or key in ("router", "gates") else 1)
+          n_ws[slot] = max(n_ws[slot], self._split(f) * M * f.N if self._split(f) > 1 or key in ("router", "gates") or
+                         key == "in" and isinstance(m, GatedStateMixer) else 1)
       if begins and model.loop_in is not None:
         n_ws[0] = max(n_ws[0], self._split(model.loop_in) * M * model.loop_in.N)
       if isinstance(ly["spec"].mlp, ExpertsMlp):
@@ -353,6 +376,8 @@ class StackRunner(HeadRunner):
           n_y[0] = max(n_y[0], M * e.top * ly["gu"].N)
       if isinstance(m, LightningMixer):   # (a call may bring fewer rows, and cut them into more spans)
         n_light = max([n_light] + [ops.lightning_ws_bytes(b, T, m.heads, m.dim, m.vdim) // 4 for b in range(1, B + 1)])
+      elif isinstance(m, GatedStateMixer):
+        n_light = max([n_light] + [ops.gated_state_ws_bytes(b, T, m.heads, m.dim, m.vdim) // 4 for b in range(1, B + 1)])
       elif isinstance(m, SsdMixer):
         n_light = max([n_light] + [ops.ssd_ws_bytes(b, T, m.heads, m.groups, m.state, m.vdim) // 4 for b in range(1, B + 1)])
       elif isinstance(m, LatentMixer):
@@ -368,10 +393,11 @@ class StackRunner(HeadRunner):
     self.kv_chunk_arg = kv_chunk
     self.y = [torch.empty(n, dtype=self.dtype, device=dev) for n in n_y]
     self.ws = [torch.empty(n, dtype=torch.float32, device=dev) for n in n_ws]
-    if n_routes > 1 or n_experts > 1:
+    if any(isinstance(ly.mlp, ExpertsMlp) for ly in cfg.layers):
       i32 = lambda n: torch.empty(n, dtype=torch.int32, device=dev)
       self.topk_id, self.counts, self.offsets, self.sorted_route = i32(n_routes), i32(n_experts), i32(n_experts + 1), i32(n_routes)
       self.topk_w = torch.empty(n_routes, dtype=torch.float32, device=dev)
+      self.gate_w = torch.empty(M, dtype=torch.float32, device=dev)
     self.light_ws = torch.empty(n_light, dtype=torch.float32, device=dev)
     self.attn_ws = torch.empty(n_attn, dtype=torch.float32, device=dev)
     self.zero = torch.zeros(1, dtype=torch.int32, device=dev)
@@ -400,11 +426,12 @@ class StackRunner(HeadRunner):
     if given is not None:
       return given
     waves = self.B * m.kv_heads * math.ceil(self.T * (m.heads // m.kv_heads) / 16)
-    if self.dtype != torch.bfloat16 or self.T != 1 or waves >= 1024 or self.S <= 64:
+    S = min(self.S, m.chunk + 31) if m.chunk else self.S      # (columns that one position may see, from a block's edge on)
+    if self.dtype != torch.bfloat16 or self.T != 1 or waves >= 1024 or S <= 64:
       return 0
-    n = min(math.ceil(1024 / waves), self.S // 32)
-    chunk = max(32, _up(math.ceil(self.S / n), 32))
-    return 0 if chunk >= self.S else chunk
+    n = min(math.ceil(1024 / waves), S // 32)
+    chunk = max(32, _up(math.ceil(S / n), 32))
+    return 0 if chunk >= S else chunk
 
   def _latent_chunk(self, m: LatentMixer) -> int:
     """The same for latent attention, whose work-groups have a compute unit to themselves."""
@@ -433,15 +460,17 @@ class StackRunner(HeadRunner):
     groups = math.ceil(f.N / 64) * math.ceil(self.M / 128)
     return int(max(1, min(8, (256 if self.M > 32 else 512) // groups, f.Kp // 512)))
 
-  def linear(self, f: DenseLinear, x, M: int, fp32_out: bool = False, slot: int = 0) -> L.RowsSrc:
-    """Runs one projection of x [M, f.Kp]; returns its output as the reading kernel wants it.  It holds until
-    the next projection of the same slot."""
+  def linear(self, f: DenseLinear, x, M: int, fp32_out: bool = False, slot: int = 0, cols: tuple | None = None) -> L.RowsSrc:
+    """Runs one projection of x [M, f.Kp], or its columns cols[0] .. cols[1] (runs of 256); returns its output as the reading
+    kernel wants it.  It holds until the next projection of the same slot."""
+    c0, c1 = cols or (0, f.N)
+    N = c1 - c0
     d = L.DenseDesc()
-    d.M, d.K, d.N, d.dtype = M, f.Kp, f.N, self.code
-    d.x, d.ldx, d.x_frag, d.w = x.data_ptr(), x.shape[1], 1 if self.frag else 0, f.w.data_ptr()
-    d.ldy, d.split_k = f.N, self._split(f)
+    d.M, d.K, d.N, d.dtype = M, f.Kp, N, self.code
+    d.x, d.ldx, d.x_frag, d.w = x.data_ptr(), x.shape[1], 1 if self.frag else 0, f.w.data_ptr() + c0 * f.Kp * f.w.element_size()
+    d.ldy, d.split_k = N, self._split(f)
     src = L.RowsSrc()
-    src.ld, src.plane, src.split_k = f.N, M * f.N, d.split_k
+    src.ld, src.plane, src.split_k = N, M * N, d.split_k
     if d.split_k > 1:
       d.epilogue, d.ws = L.TNX_EPI_F32, self.ws[slot].data_ptr()
       src.ws = d.ws
@@ -462,14 +491,16 @@ class StackRunner(HeadRunner):
     d.epilogue, d.y, d.ldy, d.y_stride, d.split_k, d.batch = L.TNX_EPI_STORE, y.data_ptr(), ldy, y_stride, 1, len(f)
     ops.dense_linear(d)
 
-  def residual_norm(self, pending, w_next, out, M: int, frag: bool, shift=None):
+  def residual_norm(self, pending, w_next, out, M: int, frag: bool, shift=None, behind=None):
     """x takes what is pending: None, ("add", rows, post-norm weight), ("set", rows, None), ("norm", None, weight) --
-    x itself normed -- or ("routes", rows, post-norm weight, route weights, routes per row);
+    x itself normed -- or ("routes", rows, post-norm weight, route weights, routes per row[, extra rows, their weights]);
     out = norm(x) . w_next, or x itself when w_next is None, or x moved towards the token before:
-    shift = (weight, ring of the rows before, col_ptr, starts, B, T)."""
+    shift = (weight, ring of the rows before, col_ptr, starts, B, T).
+    behind: the layer that ends with what is pending, when results are averaged over depth."""
     cfg = self.cfg
     d = L.ResidualNormDesc()
     d.M, d.D, d.dtype, d.eps, d.w_offset, d.groups = M, cfg.embed_dim, self.code, cfg.norm_eps, cfg.norm_offset, cfg.norm_groups
+    d.center, d.mult = 1 if cfg.center_norm else 0, cfg.residual_mult
     if pending is not None:
       kind, rows, w_post = pending[:3]
       d.mode = {"add": 1, "routes": 1, "set": 2, "norm": 3}[kind]
@@ -478,7 +509,16 @@ class StackRunner(HeadRunner):
       d.w_post = None if w_post is None else w_post.data_ptr()
       if kind == "routes":
         d.route_w, d.route_k = pending[3].data_ptr(), pending[4]
+        if len(pending) > 5:
+          d.extra, d.extra_w = pending[5], pending[6].data_ptr()
     d.x, d.w_next = self.x.data_ptr(), None if w_next is None else w_next.data_ptr()
+    if self.first is not None:
+      d.x = self.first.data_ptr()
+      if pending is not None:
+        d.x_out, self.first = self.x.data_ptr(), None
+    if behind is not None:
+      d.hist, d.hist_plane, d.hist_n, d.hist_w = self.hist.data_ptr(), self.M * cfg.embed_dim, behind + 1, self.model.layers[behind]["dwa"].data_ptr()
+      d.hist_store = 1 if behind + 1 < cfg.num_layers else 0
     d.out, d.out_ld, d.out_frag = out.data_ptr(), out.shape[1], 1 if frag else 0
     if shift is not None:
       w, ring, col_ptr, starts, B, T = shift
@@ -504,6 +544,21 @@ class StackRunner(HeadRunner):
     ops.part_rope_kvwrite(d)
     return q
 
+  def norm_kv(self, ly, src, entry, col_ptr, starts, B, T):
+    """Norms q and k over their projections and writes the cache (with borrowed keys: q alone); returns q."""
+    m, f = ly["spec"].mixer, ly["in"]
+    dkp, dvp = entry.k.shape[3], entry.v.shape[3]
+    q = self._buf("q", m.heads * dkp)
+    d = L.RowNormKvDesc()
+    d.B, d.T, d.S, d.H, d.G = B, T, entry.k.shape[2], m.heads, m.kv_heads
+    d.dk, d.dv, d.dkp, d.dvp, d.dtype, d.eps = m.dim, m.vdim, dkp, dvp, self.code, self.cfg.norm_eps
+    d.w_q, d.y, d.col_ptr, d.q_out = ly["q_norm"].data_ptr(), src, col_ptr.data_ptr(), q.data_ptr()
+    if m.kv_from is None:
+      d.w_k, d.k_off, d.v_off = ly["k_norm"].data_ptr(), f.offsets[1], f.offsets[2]
+      d.kcache, d.vcache = entry.k.data_ptr(), entry.v.data_ptr()
+    ops.rownorm_kvwrite(d)
+    return q
+
   def attend(self, ly, q, entry, col_ptr, starts, B, T) -> torch.Tensor:
     m = ly["spec"].mixer
     out = self._buf("attn", ly["out"].Kp)
@@ -512,6 +567,7 @@ class StackRunner(HeadRunner):
     d.dk, d.dv, d.dkp, d.dvp, d.scale, d.dtype = m.dim, m.vdim, entry.k.shape[3], entry.v.shape[3], m.scale, self.code
     d.q, d.kcache, d.vcache = q.data_ptr(), entry.k.data_ptr(), entry.v.data_ptr()
     d.sinks = None if ly["sink"] is None else ly["sink"].data_ptr()
+    d.slopes, d.chunk = None if ly["slopes"] is None else ly["slopes"].data_ptr(), m.chunk
     d.starts, d.col_ptr = starts.data_ptr(), col_ptr.data_ptr()
     d.kv_chunk = self._kv_chunk(m, self.kv_chunk_arg) if T == 1 else 0
     d.ws, d.out, d.out_ld, d.out_frag = self.attn_ws.data_ptr(), out.data_ptr(), out.shape[1], 1 if self.frag else 0
@@ -536,6 +592,43 @@ class StackRunner(HeadRunner):
     d = L.GatedNormDesc()
     d.M, d.W, d.dtype, d.eps, d.w_offset, d.groups = M, o.shape[1], self.code, self.cfg.norm_eps, 0.0, m.heads if isinstance(m, MemoryMixer) else 1
     d.o, d.o_ld, d.g, d.g_off, d.w = o.data_ptr(), o.shape[1], src, ly["in"].offsets[3], ly["norm"].data_ptr()
+    d.out, d.out_ld, d.out_frag = out.data_ptr(), out.shape[1], 1 if self.frag else 0
+    ops.gated_norm(d)
+    return out
+
+  # forget gates whose complement writes
+  def gated_in(self, f: DenseLinear, h, M: int):
+    """The projection of h as the recurrence reads it: (rows of q and v, whether they are fp32, rows of the gates -- fp32
+    always --, the gates' first column)."""
+    if self.dtype == torch.float32 or self.frag:
+      src = self.fp32_rows(f, h, M, slot=0)
+      return src, 1, src, f.offsets[2]
+    return self.linear(f, h, M, cols=(0, f.offsets[2])), 0, self.fp32_rows(f, h, M, slot=0, cols=(f.offsets[2], f.N)), 0
+
+  def gated_state(self, ly, rows, entry, col_ptr, starts, B, T) -> torch.Tensor:
+    """The recurrence and its heads' norms: what the output projection reads."""
+    m, f, M = ly["spec"].mixer, ly["in"], B * T
+    out = self._buf("gated", ly["out"].Kp)
+    d = L.GatedStateDesc()
+    d.B, d.T, d.H, d.dk, d.dv, d.dtype = B, T, m.heads, m.dim, m.vdim, self.code
+    d.y, d.y_f32, d.f, d.f_off = rows
+    d.q_off, d.v_off, d.bias, d.lower = f.offsets[0], f.offsets[1], ly["bias"].data_ptr(), ly["lower"].data_ptr()
+    d.starts, d.col_ptr, d.state, d.ws = starts.data_ptr(), col_ptr.data_ptr(), entry.s.data_ptr(), self.light_ws.data_ptr()
+    if T == 1 and ops.gated_state_step_ok(m.dim, m.vdim):
+      d.norm_w, d.eps, d.out, d.out_ld, d.out_frag = ly["norm"].data_ptr(), self.cfg.norm_eps, out.data_ptr(), out.shape[1], 1 if self.frag else 0
+      ops.gated_state(d)
+      return out
+    o = self._buf("state_out", m.heads * m.vdim, torch.float32)
+    d.o, d.o_ld = o.data_ptr(), o.shape[1]
+    ops.gated_state(d)
+    return self.head_norm(ly, o, M)
+
+  def head_norm(self, ly, o, M: int) -> torch.Tensor:
+    """Heads of o normed on their own, with shared weights."""
+    m, out = ly["spec"].mixer, self._buf("gated", ly["out"].Kp)
+    d = L.GatedNormDesc()
+    d.M, d.W, d.dtype, d.eps, d.groups, d.shared_w = M, o.shape[1], self.code, self.cfg.norm_eps, m.heads, 1
+    d.o, d.o_ld, d.w = o.data_ptr(), o.shape[1], ly["norm"].data_ptr()
     d.out, d.out_ld, d.out_frag = out.data_ptr(), out.shape[1], 1 if self.frag else 0
     ops.gated_norm(d)
     return out
@@ -622,9 +715,9 @@ class StackRunner(HeadRunner):
     ops.memory(d)
     return o
 
-  def fp32_rows(self, f: DenseLinear, x, M: int, slot: int) -> L.RowsSrc:
+  def fp32_rows(self, f: DenseLinear, x, M: int, slot: int, cols: tuple | None = None) -> L.RowsSrc:
     """A projection whose rows stay fp32 (finished, or planes)."""
-    src = self.linear(f, x, M, fp32_out=True, slot=slot)
+    src = self.linear(f, x, M, fp32_out=True, slot=slot, cols=cols)
     if src.split_k <= 1 and src.ws:
       src.y = src.ws
     return src
@@ -772,10 +865,12 @@ class StackRunner(HeadRunner):
 
   def _mixer(self, ly, h, entry, col_ptr, starts, B, T) -> L.RowsSrc:
     m, M = ly["spec"].mixer, B * T
-    src = self.linear(ly["in"], h, M)
     at = (entry, col_ptr, starts, B, T)
+    if isinstance(m, GatedStateMixer):
+      return self.linear(ly["out"], self.gated_state(ly, self.gated_in(ly["in"], h, M), *at), M)
+    src = self.linear(ly["in"], h, M)
     if isinstance(m, AttentionMixer):
-      out = self.attend(ly, self.rotate(ly, src, *at), *at)
+      out = self.attend(ly, self.norm_kv(ly, src, *at) if m.row_norm else self.rotate(ly, src, *at), *at)
     elif isinstance(m, SsdMixer):
       u = None if T == 1 and ops.ssd_step_ok(m.state, m.vdim) else self.convolve(ly, src, *at)
       out = self.ssd_gate(ly, self.ssd(ly, src, u, *at), src, M)
@@ -794,7 +889,12 @@ class StackRunner(HeadRunner):
     e = ly["spec"].mlp
     src = self.fp32_rows(ly["router"], h, M, slot=0)
     ids = self.topk_id[:M * e.top].view(M, e.top)
-    ops.route_softmax(src, M, e.experts, e.top, self.topk_w, ids)
+    if e.corrected:
+      shared = e.shared_ff > 0
+      ops.route_scores(src, M, e.experts, e.top, ly["correction"], e.scale, self.topk_w, ids, ly["router"].offsets[1] if shared else 0,
+                       self.gate_w if shared else None)
+    else:
+      ops.route_softmax(src, M, e.experts, e.top, self.topk_w, ids)
     ops.moe_sort_routes(ids, e.experts, self.counts, self.offsets, self.sorted_route)
 
   def experts_linear(self, f: LinearBank, x, x_frag: bool, x_div: int, routes: int, epilogue: int, y, ldy: int):
@@ -808,7 +908,9 @@ class StackRunner(HeadRunner):
   def experts_gate_up(self, ly, h, M: int) -> torch.Tensor:
     e, f = ly["spec"].mlp, ly["gu"]
     act = self._buf("act", ly["down"].Kp, rows=self.M * e.top)
-    if self.dtype == torch.float32:
+    if not e.gated:
+      self.experts_linear(f, h, self.frag, e.top, M * e.top, L.TNX_EPI_RELU2, act, act.shape[1])
+    elif self.dtype == torch.float32:
       y = self.y[0][:M * e.top * f.N].view(M * e.top, f.N)
       self.experts_linear(f, h, False, e.top, M * e.top, L.TNX_EPI_STORE, y, f.N)
       ops.silu_mul(y, f.offsets[1], M * e.top, e.ff, act)
@@ -828,8 +930,28 @@ class StackRunner(HeadRunner):
     e = ly["spec"].mlp
     if isinstance(e, ExpertsMlp):
       self.route(ly, h, M)
-      return ("routes", self.experts_down(ly, self.experts_gate_up(ly, h, M), M), ly["post2"], self.topk_w, e.top)
+      routes = ("routes", self.experts_down(ly, self.experts_gate_up(ly, h, M), M), ly["post2"], self.topk_w, e.top)
+      if e.shared_ff:
+        routes += (self.linear(ly["shared_down"], self.shared_up(ly, h, M), M), self.gate_w)
+      return routes
+    if isinstance(e, PolyNormMlp):
+      return ("add", self.linear(ly["down"], self.poly_up(ly, h, M), M), ly["post2"])
     return ("add", self.linear(ly["down"], self.gate_up(ly, h, M), M), ly["post2"])
+
+  def shared_up(self, ly, h, M: int) -> torch.Tensor:
+    """max(up h, 0)^2 of the expert that every token uses."""
+    f, act = ly["shared_up"], self._buf("shared", ly["shared_down"].Kp)
+    d = L.DenseDesc()
+    d.M, d.K, d.N, d.dtype = M, f.Kp, f.N, self.code
+    d.x, d.ldx, d.x_frag, d.w = h.data_ptr(), h.shape[1], 1 if self.frag else 0, f.w.data_ptr()
+    d.epilogue, d.y, d.ldy, d.y_frag, d.split_k = L.TNX_EPI_RELU2, act.data_ptr(), act.shape[1], 1 if self.frag else 0, 1
+    ops.dense_linear(d)
+    return act
+
+  def poly_up(self, ly, h, M: int) -> torch.Tensor:
+    act = self._buf("act", ly["down"].Kp)
+    ops.poly_norm(self.linear(ly["gu"], h, M), self.dtype, M, ly["spec"].mlp.ff, ly["act"], self.cfg.norm_eps, act, self.frag)
+    return act
 
   def gate_up(self, ly, h, M: int, slot: int = 0) -> torch.Tensor:
     f = ly["gu"]
@@ -858,15 +980,17 @@ class StackRunner(HeadRunner):
     starts = self.no_starts if starts is None else starts
     D = cfg.embed_dim
     cat = None if m.loop_in is None else self._buf("cat", m.loop_in.Kp)
-    ops.embed_rows(m.embed, tokens, col_ptr, B, T, cfg.vocab_size, D, self.x, cat=cat, cat_off=D, cat_frag=self.frag, scale=cfg.embed_scale)
+    self.first = self.hist[0] if cfg.depth_average else None
+    ops.embed_rows(m.embed, tokens, col_ptr, B, T, cfg.vocab_size, D, self.x if self.first is None else self.first, pos=m.pos, starts=starts, cat=cat, cat_off=D, cat_frag=self.frag, scale=cfg.embed_scale)
     h = self._buf("h", m.Dp)
     if cfg.parallel:
       return self._forward_parallel(h, col_ptr, cache, B, T, starts)
     pending, behind_layer = None if m.embed_norm is None else ("norm", None, m.embed_norm), False
+    ended = None                                     # the layer that what is pending completes
 
     def norm(w_next, out, frag, shift=None):
       nonlocal behind_layer
-      self.residual_norm(pending, w_next, out, M, frag, shift)
+      self.residual_norm(pending, w_next, out, M, frag, shift, behind=ended if behind_layer and cfg.depth_average else None)
       if behind_layer and self.residual_sink is not None:
         self.residual_sink(self.x[:M])
       behind_layer = False
@@ -885,7 +1009,7 @@ class StackRunner(HeadRunner):
       if "gu" in ly:
         norm(ly["norm2"], h, self.frag)
         pending = self._mlp(ly, h, M)
-      behind_layer = True
+      behind_layer, ended = True, i
     norm(m.final_norm, self.xn, False)
     return self.xn
 
