@@ -1121,6 +1121,130 @@ def kuzezen_workload(size, iters, steps, kernels=True):
   return result
 
 
+# the like kernel of each, of a Nunezen decoder or (experts) of a Lapevik one
+KEZOLIX_LIKE = {
+    "linear recurrent in": "linear lightning in", "linear recurrent out": "linear o", "linear qkv": "linear qkv", "linear q": "linear qkv", "linear attention out": "linear o",
+    "linear up": "linear gate_up", "linear down": "linear down",
+    "recurrence": "lightning", "head norms": "gated norm", "row norms + cache write": "rotation + cache write", "attention": "attention", "PolyNorm": "gated norm",
+    "linear router": "linear router", "choice of experts": "choice of experts", "route sort": "route sort", "experts up": "experts gate_up", "experts down": "experts down",
+    "norm + residual + norm": "post-norm + residual + norm", "routes + norm + residual + depth + norm": "routes + norm + residual + shift",
+}
+
+
+def kezolix_kernels(model, runner, st, ctx, iters):
+  """Per-kernel times of a Kezolix model's pass: T = runner.T tokens per row, the last of them at context `ctx`."""
+  import torch
+
+  from tunix_amd import ops
+  from tunix_amd.config import ExpertsMlp, GatedStateMixer
+  B, T, M, D = runner.B, runner.T, runner.M, model.cfg.embed_dim
+  prompt = T > 1
+  col = torch.tensor([ctx - T], dtype=torch.int32, device=model.device)
+  at = lambda i: (st.cache.entries[i], col, st.starts, B, T)
+  pick = lambda test: [i for i, ly in enumerate(model.layers) if test(ly["spec"])]
+  rec, moe = pick(lambda s: isinstance(s.mixer, GatedStateMixer)), pick(lambda s: isinstance(s.mlp, ExpertsMlp))
+  attn = [i for i in range(len(model.layers)) if i not in rec]
+  lent = [i for i in attn if model.layers[i]["spec"].mixer.kv_from is not None]
+  own, poly = [i for i in attn if i not in lent], [i for i in range(len(model.layers)) if i not in moe]
+  for i in own:
+    st.cache.entries[i].k.normal_()
+    st.cache.entries[i].v.normal_()
+  out = {}
+
+  def timed(name, idx, fn, nbytes, flops=0.0):
+    out[name] = roof_row(in_turn([(lambda i=i: fn(model.layers[i], i)) for i in idx], iters), nbytes, flops)
+
+  def lin(name, idx, key, x, fp32=False):
+    f = model.layers[idx[0]][key]
+    timed(name, idx, lambda ly, i: runner.linear(ly[key], x, M, fp32_out=fp32), f.nbytes() + M * (f.K * 2 + f.N * (4 if fp32 else 2)), 2.0 * M * f.K * f.N)
+
+  h = runner._buf("h", model.Dp)
+  h.normal_()
+  # recurrent layers
+  lr, m = model.layers[rec[0]], model.layers[rec[0]]["spec"].mixer
+  qk, v, f = m.heads * m.dim, m.heads * m.vdim, lr["in"]
+  timed("linear recurrent in", rec, lambda ly, i: runner.gated_in(ly["in"], h, M), f.nbytes() + M * (f.K * 2 + (qk + v) * 2 + qk * 4), 2.0 * M * f.K * f.N)
+  rows = runner.gated_in(f, h, M)
+  timed("recurrence", rec, lambda ly, i: runner.gated_state(ly, rows, *at(i)), M * (qk * 6 + v * (6 if prompt else 4)) + B * m.heads * m.dim * m.vdim * 8,
+        2.0 * M * m.heads * (2 * m.dim * m.vdim + (32 * (m.dim + m.vdim) if prompt else 0)))
+  o, normed = runner.gated_state(lr, rows, *at(rec[0]))
+  if not normed:
+    timed("head norms", rec[:1], lambda ly, i: runner.head_norm(ly, o, M), M * v * 6)
+    o = runner.head_norm(lr, o, M)
+  lin("linear recurrent out", rec, "out", o)
+  # attention layers
+  la, a = model.layers[own[0]], model.layers[own[0]]["spec"].mixer
+  lin("linear qkv", own, "in", h)
+  lin("linear q", lent, "in", h)
+  src = runner.linear(la["in"], h, M)
+  timed("row norms + cache write", own, lambda ly, i: runner.norm_kv(ly, src, *at(i)), 2 * M * (a.heads * a.dim + a.kv_heads * (a.dim + a.vdim)) * 2)
+  q = runner.norm_kv(la, src, *at(own[0]))
+  pairs = T * ctx - T * (T - 1) / 2
+  timed("attention", own, lambda ly, i: runner.attend(ly, q, *at(i)), B * a.kv_heads * ctx * (a.dim + a.vdim) * 2 + 2 * M * a.heads * a.dim * 2,
+        2.0 * B * a.heads * pairs * (a.dim + a.vdim))
+  lin("linear attention out", attn, "out", runner.attend(la, q, *at(own[0])))
+  # dense feed-forward
+  lp, ff = model.layers[poly[0]], model.layers[poly[0]]["spec"].mlp.ff
+  lin("linear up", poly, "gu", h)
+  y, act = runner.linear(lp["gu"], h, M), runner._buf("act", lp["down"].Kp)
+  timed("PolyNorm", poly, lambda ly, i: ops.poly_norm(y, runner.dtype, M, ff, ly["act"], model.cfg.norm_eps, act, runner.frag), M * ff * 4)
+  lin("linear down", poly, "down", act)
+  # experts
+  lm, e = model.layers[moe[0]], model.layers[moe[0]]["spec"].mlp
+  lin("linear router", moe, "router", h, fp32=True)
+  z = runner.fp32_rows(lm["router"], h, M, slot=0)
+  n, E = e.routes, len(lm["gu"])       # the shared expert among them
+  ids = runner.topk_id[:M * n].view(M, n)
+  timed("choice of experts", moe, lambda ly, i: ops.route_scores(z, M, e.experts, e.top, ly["correction"], e.scale, runner.topk_w, ids, ly["router"].offsets[1], ld=n),
+        M * (e.experts + 1 + 2 * n) * 4)
+  timed("route sort", moe[:1], lambda ly, i: ops.moe_sort_routes(ids, E, runner.counts, runner.offsets, runner.sorted_route), M * n * 8)
+  live = int((runner.counts[:E] > 0).sum())
+  xact = runner.experts_gate_up(lm, h, M)
+  timed("experts up", moe, lambda ly, i: runner.experts_gate_up(ly, h, M), lm["gu"].nbytes() * live / E + M * (D + n * e.ff) * 2, 2.0 * M * n * D * e.ff)
+  timed("experts down", moe, lambda ly, i: runner.experts_down(ly, xact, M), lm["down"].nbytes() * live / E + M * n * (D + e.ff) * 2, 2.0 * M * n * D * e.ff)
+  routes = ("routes", runner.experts_down(lm, xact, M), lm["post2"], runner.topk_w, n)
+  # the residual: between a layer's sublayers, and behind the layer with the most earlier results but the last
+  last = max(i for i in moe if i + 1 < len(model.layers))
+  runner.hist.normal_()
+  timed("routes + norm + residual + depth + norm", [last], lambda ly, i: runner.residual_norm(routes, ly["norm1"], h, M, runner.frag, behind=i),
+        M * D * (2 * n + 4 * (last + 1) + 4 + 8 + 2))
+  osrc = runner.linear(la["out"], runner._buf("attn", la["out"].Kp), M)
+  timed("norm + residual + norm", moe, lambda ly, i: runner.residual_norm(("add", osrc, ly["post1"]), ly["norm2"], h, M, runner.frag), M * D * (2 + 8 + 2))
+  return out
+
+
+def kezolix_workload(size, iters, steps, kernels=True):
+  """Prefill and decode of a Kezolix decoder with layers of a real model's size (random weights) beside a Nunezen decoder
+  of the same width, heads, feed-forward and number of layer runs and a Lapevik one with the same routed experts, and every
+  kernel against its roof and the like one's."""
+  import numpy as np
+  import torch
+
+  from tunix_amd import config, dummy_model
+  from tunix_amd.stack_model import StackModel
+  dev = torch.device("cuda:0")
+  width, H, G, ff, B = STACK_SIZES[size]
+  lH, E, top, eff = LAPEVIK_SIZES[size]
+  new_cfg = config.kezolix_shape(width, H, G, ff, E, top, eff)
+  P, T = 1024, 256
+  ids = np.random.Generator(np.random.PCG64(5)).integers(1, new_cfg.vocab_size, size=(B, P)).astype(np.int32)
+  result = {"size": {"width": width, "heads": H, "kv_heads": G, "head_dim": 128, "feed_forward": ff, "experts": E, "top": top, "expert_width": eff, "batch": B,
+                     "prompt": P, "chunk": new_cfg.layers[1].mixer.chunk, "layers": new_cfg.num_layers}}
+  for name, cfg, measure in (("kezolix", new_cfg, kezolix_kernels), ("nunezen", config.nunezen_shape(width, H, G, ff), stack_kernels),
+                             ("lapevik", config.lapevik_shape(width, lH, E, top, eff), lapevik_kernels)):
+    result[name] = measure_model(name, lambda: StackModel(cfg, dummy_model.create_stack_weights(cfg, 1, dev), dev), measure if kernels else None, size, ids, P, T,
+                                 steps, iters)
+  if kernels:
+    for phase in ("decode_kernels", "prefill_kernels"):
+      like = {**result["lapevik"][phase], **result["nunezen"][phase]}
+      for k, v in result["kezolix"][phase].items():
+        b = like[KEZOLIX_LIKE[k]]
+        v["vs_like"] = round(v["times_roof"] / b["times_roof"], 2)
+        log(f"  {size} {phase:16s} {k:40s} {v['us']:9.1f} us  {v['times_roof']:6.2f} x roof ({v['bound']})   {KEZOLIX_LIKE[k]}: "
+            f"{b['us']:9.1f} us  {b['times_roof']:6.2f} x ({b['bound']})   ratio {v['vs_like']}")
+  return result
+
+
 def main():
   ap = argparse.ArgumentParser()
   ap.add_argument("--gpus", type=int, default=1)
@@ -1150,7 +1274,7 @@ def main():
                   help="instead of the decode benchmark: a Nunezen decoder with layers of a real model's size (model "
                        "width 2048 or 4096), prefill, decode and every kernel against its roof, beside a gemma3-family "
                        "model of the same size; its own JSON line")
-  ap.add_argument("--stack-design", choices=["nunezen", "lapevik", "kuzezen"], default="nunezen", help="with --stack: the layer-list design to measure")
+  ap.add_argument("--stack-design", choices=["nunezen", "lapevik", "kuzezen", "kezolix"], default="nunezen", help="with --stack: the layer-list design to measure")
   ap.add_argument("--stack-no-kernels", action="store_true", help="with --stack: throughput only")
   ap.add_argument("--config", choices=["c1", "c2", "c3", "c4"], default="c3",
                   help="c3 (default): the headline workload; c1 / c2 / c4: the other rollout workloads through "
@@ -1195,7 +1319,7 @@ def main():
 
   if args.stack:
     sizes = sorted(STACK_SIZES) if args.stack == "all" else [args.stack]
-    measure = {"nunezen": stack_workload, "lapevik": lapevik_workload, "kuzezen": kuzezen_workload}[args.stack_design]
+    measure = {"nunezen": stack_workload, "lapevik": lapevik_workload, "kuzezen": kuzezen_workload, "kezolix": kezolix_workload}[args.stack_design]
     print(json.dumps({"metric": f"{args.stack_design.capitalize()} prefill and decode tokens/sec @1 MI355X", "unit": "tokens/s", "n_gpus": 1,
                       "dtype": "bf16", "data": "synthetic",
                       "sizes": {z: measure(z, args.kernel_iters, 64, not args.stack_no_kernels) for z in sizes}}),

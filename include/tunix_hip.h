@@ -813,9 +813,10 @@ int tnx_silu_mul(void* stream, int dtype, const void* y, int64_t ld, int64_t up_
 int tnx_route_softmax(void* stream, const tnx_rows_src* z, int64_t M, int E, int k, float* topk_w, int32_t* topk_id);
 /* The same with scores s = softmax over all E logits: the k experts with the largest s + correction (correction [E], null:
  * none) are chosen; topk_w = s / (sum of the chosen s + 1e-20) * scale.  gate_w (null: none) fp32 [M] = sigmoid of z's column
- * gate_off. */
+ * gate_off.  ld: entries of a row of topk_w and topk_id, k, or k + 1: then every row's last one is expert E with that sigmoid
+ * as its weight (an expert that all rows use). */
 int tnx_route_scores(void* stream, const tnx_rows_src* z, int64_t M, int E, int k, const float* correction, float scale, int64_t gate_off,
-                     float* topk_w, int32_t* topk_id, float* gate_w);
+                     int ld, float* topk_w, int32_t* topk_id, float* gate_w);
 
 /* out[M, F] = a norm(y) + b norm(y^2) + c norm(y^3) + e with norm(v) = v / sqrt(mean(v^2) + eps) over the F values of a row,
  * powers element by element; coef [4] = a, b, c, e. */

@@ -35,14 +35,14 @@ def config(vocab, width, layers, eps=1e-6, mult=0.7, positions=320):
 CONFIGS = {
     # every kind of layer and feed-forward, with and without one; keys borrowed twice, over a layer of the same sizes
     "mixed": config(320, 128, [state(3, 32, 48, dense(160)), attention(6, 2, 32, 48, 20, moe(48, 9, 3, 80, 1.7)), state(2, 64, 40),
-                               attention(6, 2, 32, 48, 33, None, 0.3), attention(6, 2, 32, 48, 50, moe(64, 4, 1, 24, 0.6), 0.25, kv_from=1),
+                               attention(6, 2, 32, 48, 33, None, 0.3), attention(6, 2, 32, 48, 50, moe(64, 4, 1, 64, 0.6), 0.25, kv_from=1),
                                attention(6, 2, 32, 48, 17, dense(96), kv_from=1)]),
     # every expert of every token: nothing hangs on a close call of a router
-    "all": config(320, 128, [attention(4, 1, 64, 24, 40, moe(48, 6, 6, 64, 2.5)), state(5, 16, 32, moe(80, 2, 2, 16)), attention(4, 1, 64, 24, 9, dense(200), kv_from=0),
+    "all": config(320, 128, [attention(4, 1, 64, 24, 40, moe(48, 6, 6, 64, 2.5)), state(5, 16, 32, moe(80, 2, 2, 80)), attention(4, 1, 64, 24, 9, dense(200), kv_from=0),
                              state(2, 128, 64, moe(32, 1, 1, 40, 0.4))], mult=0.5),
     # nothing a multiple of eight
     "odd": config(211, 100, [attention(3, 3, 21, 13, 7, moe(33, 5, 2, 21, 3.0)), state(3, 11, 9, dense(70)), attention(3, 3, 21, 13, 1000, kv_from=0, scale=0.31),
-                             state(1, 20, 30, moe(20, 6, 1, 50)), attention(10, 5, 12, 45, 1)], eps=1e-3, mult=1.0, positions=200),
+                             state(1, 20, 30, moe(20, 6, 1, 20)), attention(10, 5, 12, 45, 1)], eps=1e-3, mult=1.0, positions=200),
     # wide heads and many of them
     "wide": config(512, 192, [state(1, 200, 136, dense(256)), attention(16, 2, 136, 200, 64, moe(128, 3, 3, 128)), state(2, 256, 264),
                               attention(20, 5, 64, 96, 130, dense(64)), attention(16, 2, 136, 200, 45, kv_from=1), state(4, 96, 24)], eps=1e-4, mult=0.4, positions=400),

@@ -529,6 +529,10 @@ def test_choice_by_corrected_scores(gpu, E, k):
     ok = (ti.cpu() == ids).all(1)
     assert rel(tw.cpu()[ok], w[ok]) < 2e-6
     torch.testing.assert_close(gw.cpu(), torch.sigmoid(both[:, -1]), rtol=2e-6, atol=1e-7)
+    # beside an expert that every row uses: the same, one entry longer
+    tw2, ti2 = torch.empty(M, k + 1, device=gpu), torch.empty(M, k + 1, dtype=torch.int32, device=gpu)
+    ops.route_scores(src, M, E, k, cg, scale, tw2, ti2, up(E, 16), ld=k + 1)
+    assert torch.equal(ti2[:, :k], ti) and torch.equal(tw2[:, :k], tw) and bool((ti2[:, k] == E).all()) and torch.equal(tw2[:, k], gw)
   plain = torch.empty(M, k, device=gpu)
   ops.route_scores(src, M, E, k, None, 1.0, plain, ti)
   assert torch.equal(ti.cpu().long().sort(1).values[:1], R.route(z.double(), torch.zeros(E), k, 1.0)[0].sort(1).values[:1])
@@ -749,7 +753,7 @@ def test_rollout_log_probabilities_and_weight_updates(gpu):
   with pytest.raises(ValueError, match="same structure"):
     roll.update_params({"l0.mix.q": w2["l0.mix.q"]})                    # a member of a fused projection without the others
   assert np.array_equal(all_logits(model, [prompts[0]], 2)[0], before)
-  for part in ("head", "l0.mix.lower", "l2.dwa", "l4.mix.q.norm", "l4.mix.q", "l1.mlp.e3.up", "l1.mlp.shared.down", "l1.mlp.correction", "l0.mlp.act", "pos", "embed"):
+  for part in ("head", "l0.mix.lower", "l2.dwa", "l4.mix.q.norm", "l4.mix.q", "l1.mlp.e3.up", "l1.mlp.shared.down", "l4.mlp.shared.up", "l1.mlp.correction", "l0.mlp.act", "pos", "embed"):
     w[part] = w2[part]                                                    # alone, one after another
     roll.update_params({part: w2[part]})
     assert err(all_logits(model, [prompts[0]], 2)[0], R.forward(d, w, prompts[0]).numpy()) < TOL[F32], part

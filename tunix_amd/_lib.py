@@ -338,7 +338,7 @@ SIGNATURES = {
     "tnx_gelu_mul": (_i32, [_p, _i32, _p, _i64, _i64, _i64, _i64, _p, _i64]),
     "tnx_silu_mul": (_i32, [_p, _i32, _p, _i64, _i64, _i64, _i64, _p, _i64]),
     "tnx_route_softmax": (_i32, [_p, C.POINTER(RowsSrc), _i64, _i32, _i32, _p, _p]),
-    "tnx_route_scores": (_i32, [_p, C.POINTER(RowsSrc), _i64, _i32, _i32, _p, _f32, _i64, _p, _p, _p]),
+    "tnx_route_scores": (_i32, [_p, C.POINTER(RowsSrc), _i64, _i32, _i32, _p, _f32, _i64, _i32, _p, _p, _p]),
     "tnx_poly_norm": (_i32, [_p, _i32, C.POINTER(RowsSrc), _i64, _i64, _p, _f32, _p, _i64, _i32]),
     "tnx_short_conv": (_i32, [_p, C.POINTER(ShortConvDesc)]),
     "tnx_ring_write": (_i32, [_p, _i32, C.POINTER(RowsSrc), _i64, _i64, _i64, _i64, _i32, _p, _i64, _p]),

@@ -353,6 +353,16 @@ class ExpertsMlp:
     if self.shared_ff and (self.gated or not self.corrected) or not self.corrected and self.scale != 1.0:
       raise ValueError("a shared expert and a scale go with corrected scores")
 
+  @property
+  def shared_routed(self) -> bool:
+    """A shared expert of the others' size is one more expert, to which every token is routed."""
+    return self.shared_ff == self.ff
+
+  @property
+  def routes(self) -> int:
+    """Experts that a token is routed to."""
+    return self.top + (1 if self.shared_routed else 0)
+
   def weight_shapes(self, D: int) -> dict[str, tuple]:
     out = {"router": (self.experts, D)}
     if self.corrected:
@@ -662,7 +672,7 @@ def kuzezen_shape(width: int, heads: int, kv_heads: int, ff: int, vocab: int = 3
 
 
 def kezolix_shape(width: int, heads: int, kv_heads: int, ff: int, experts: int, top: int, expert_ff: int, vocab: int = 32768, dim: int = 128,
-                  chunk: int = 2048, layers: int = 4, positions: int = 8192) -> StackConfig:
+                  chunk: int = 2048, layers: int = 6, positions: int = 8192) -> StackConfig:
   """A Kezolix decoder with layers of a real model's size: recurrent and attention layers in turn, the first with a dense
   feed-forward, the others with routed and shared experts; the last attention layer reads the keys of the first."""
   moe = ExpertsMlp(expert_ff, experts, top, gated=False, corrected=True, scale=2.5, shared_ff=expert_ff)

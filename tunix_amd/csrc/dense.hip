@@ -370,7 +370,7 @@ extern "C" int tnx_dense_linear(void* stream, const tnx_dense_desc* d) {
   }
   // many rows: the 128 x 256 kernel (row-major operands, 32-bit offsets); a few columns would leave its tiles
   // and the device mostly empty: 32 rows per work-group then
-  const bool narrow = d->N <= 64 && !mul && d->M > 64 && d->M <= 32 * 65535;
+  const bool narrow = d->N <= 128 && !mul && d->M > 64 && d->M <= 32 * 65535;
   if (!batch && !narrow && !d->x_frag && !d->y_frag && split == 1 && d->M > 64 && d->ldx == d->K && d->N % 16 == 0 &&
       offsets32)
     return tnx_internal_wide_dense(st, d->M, d->K, d->N, (const uint16_t*)d->x, (const uint16_t*)d->w, d->epilogue, d->y,

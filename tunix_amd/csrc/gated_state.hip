@@ -187,6 +187,7 @@ struct GateLds {
   static constexpr int score = vt + 128 * kTokLd * 2;     // high and low [32][kTokLd]
   static constexpr int total = score + 2 * kTok * kTokLd * 2;   // fp32: per token group [512 / DK][DK], then of the chunk [DK]
   static constexpr int bytes = total + (512 + DK) * 4;
+  static constexpr int states_total = (2 * DK + 128) * kTokLd * 2, states_bytes = states_total + (512 + DK) * 4;   // k^T, v^T, totals alone
 };
 
 // A work-group takes one span of one (row, head) and up to 128 value columns; wave w keeps the state's columns
@@ -202,17 +203,17 @@ struct GateLds {
 // Thread (group, pair) owns DK / 16 neighbouring tokens of two channels.
 // STATES: only the span's own contribution to the state and its decays are formed (into ws).
 template <int KT, bool STATES, typename TY>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, KT <= 2 ? 2 : 1))) void gated_chunk_kernel(const GateArgs a, const RowSrc<TY> src, const RowSrc<float> fs) {
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(KT <= 2 || (STATES && KT <= 4) ? 2 : 1, KT <= 2 || STATES ? 2 : 1))) void gated_chunk_kernel(const GateArgs a, const RowSrc<TY> src, const RowSrc<float> fs) {
   constexpr int DK = KT * 32, LD = GateLds<DK>::LD, PAIRS = DK / 2, NG = 256 / PAIRS, TG = kTok / NG;
   static_assert(TG >= 2 && TG <= 16, "tokens of a thread");
   typedef GateLds<DK> Lds;
-  extern __shared__ __align__(16) unsigned char smem[];
+  extern __shared__ __align__(16) uint8_t smem[];
   uint16_t* kth = reinterpret_cast<uint16_t*>(smem + (STATES ? 0 : Lds::kt));
   uint16_t* ktl = kth + DK * kTokLd;
-  uint16_t* vt = reinterpret_cast<uint16_t*>(smem + Lds::vt);
+  uint16_t* vt = reinterpret_cast<uint16_t*>(smem + (STATES ? 2 * DK * kTokLd * 2 : Lds::vt));
   uint16_t* sch = reinterpret_cast<uint16_t*>(smem + Lds::score);
   uint16_t* scl = sch + kTok * kTokLd;
-  float* tot = reinterpret_cast<float*>(smem + Lds::total);
+  float* tot = reinterpret_cast<float*>(smem + (STATES ? Lds::states_total : Lds::total));
   float* all = tot + 512;
   const int tid = threadIdx.x, lane = tid & 63, l32 = lane & 31, lh = lane >> 5, l16 = lane & 15, lq = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -255,39 +256,58 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, KT <= 2 
   }
   f32x2 decay = f32x2{1.f, 1.f};   // of the span so far (STATES)
 
-  f32x2 qr[TG], zr[TG];
+  // the next chunk's rows, as they come (a conversion would wait for the loads)
+  constexpr bool RAW = sizeof(TY) == 2;
+  f32x2 qr[RAW ? 1 : TG], zr[TG];
+  uint32_t qw[RAW ? TG : 1];
+  u32x4 vw[2];
   float v0[8], v1[8];
   const int vp = tid >> 4, vd = dv0 + (tid & 15) * 8;      // this thread's pair of tokens and eight value columns
   auto live = [&](int t) { return t < t_end && col0 + t >= start; };
+  const int chc = ch_ok ? ch : 0, vdc = vd < a.dv ? vd : 0;
+  const TY* yb = src.y + b * a.T * src.ld;
+  const float* fb = fs.y + b * a.T * fs.ld + a.f_off + hk + chc;
   auto fetch = [&](int t0) {
+    if constexpr (RAW) {   // finished rows: loads of tokens that are not there go to the last one, and are dropped later
 #pragma unroll
-    for (int u = 0; u < TG; ++u) {
-      const int t = t0 + grp * TG + u;
-      qr[u] = zr[u] = f32x2{0.f, 0.f};
-      if (ch_ok && live(t)) {
-        if (!STATES) qr[u] = get2(src, b * a.T + t, a.q_off + hk + ch);
-        zr[u] = get2(fs, b * a.T + t, a.f_off + hk + ch);
+      for (int u = 0; u < TG; ++u) {
+        const int t = min(t0 + grp * TG + u, (int)a.T - 1);
+        if constexpr (!STATES) qw[u] = *reinterpret_cast<const uint32_t*>(yb + t * (int)src.ld + a.q_off + hk + chc);
+        zr[u] = *reinterpret_cast<const f32x2*>(fb + t * (int)fs.ld);
+      }
+      const TY* vb = yb + a.v_off + hv + vdc;
+#pragma unroll
+      for (int e = 0; e < 2; ++e) vw[e] = *reinterpret_cast<const u32x4*>(vb + min(t0 + 2 * vp + e, (int)a.T - 1) * (int)src.ld);
+    } else {
+#pragma unroll
+      for (int u = 0; u < TG; ++u) {
+        const int t = t0 + grp * TG + u;
+        qr[u] = zr[u] = f32x2{0.f, 0.f};
+        if (ch_ok && live(t)) {
+          if (!STATES) qr[u] = get2(src, b * a.T + t, a.q_off + hk + ch);
+          zr[u] = get2(fs, b * a.T + t, a.f_off + hk + ch);
+        }
+      }
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v0[j] = v1[j] = 0.f;
+      if (vd < a.dv) {
+        if (live(t0 + 2 * vp)) get8(src, b * a.T + t0 + 2 * vp, a.v_off + hv + vd, v0);
+        if (live(t0 + 2 * vp + 1)) get8(src, b * a.T + t0 + 2 * vp + 1, a.v_off + hv + vd, v1);
       }
     }
-#pragma unroll
-    for (int j = 0; j < 8; ++j) v0[j] = v1[j] = 0.f;
-    if (vd < a.dv) {
-      if (live(t0 + 2 * vp)) get8(src, b * a.T + t0 + 2 * vp, a.v_off + hv + vd, v0);
-      if (live(t0 + 2 * vp + 1)) get8(src, b * a.T + t0 + 2 * vp + 1, a.v_off + hv + vd, v1);
-    }
   };
-  // a level's operands: place of a token's row in the set, and the rows themselves
-  auto put_q = [&](int set, int row, f32x2 v) {
-    *reinterpret_cast<uint32_t*>(smem + set * Lds::set + (row * LD + ch) * 2) = cvt_pk_bf16(v[0], v[1]);
-  };
-  auto put_k = [&](int set, int row, f32x2 v) {
+  // a level's operands.  Row of token i in the set: i / 2s * s + i % s, for s below a thread's tokens grp * TG / 2 and a
+  // number that depends on the place in the thread alone
+  uint8_t* const row0 = smem + (grp * (TG / 2) * LD + ch) * 2;
+  auto put_q = [&](uint8_t* at, f32x2 v) { *reinterpret_cast<uint32_t*>(at) = cvt_pk_bf16(v[0], v[1]); };
+  auto put_k = [&](uint8_t* at, f32x2 v) {
     uint32_t hi, lo;
     split2(v[0], v[1], hi, lo);
-    *reinterpret_cast<uint32_t*>(smem + set * Lds::set + ((16 + row) * LD + ch) * 2) = hi;
-    *reinterpret_cast<uint32_t*>(smem + set * Lds::set + ((32 + row) * LD + ch) * 2) = lo;
+    *reinterpret_cast<uint32_t*>(at + 16 * LD * 2) = hi;
+    *reinterpret_cast<uint32_t*>(at + 32 * LD * 2) = lo;
   };
-  // a set's 16 x 16 product into the scores: `level` tokens per block, 0: the diagonal of odd tokens, -1: of even ones
-  auto score = [&](int set, int level) {
+  // a set's 16 x 16 product into the scores: blocks of 2^shift tokens, -1: the diagonal of odd tokens, -2: of even ones
+  auto score = [&](int set, int shift) {
     f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
     const uint16_t* p = reinterpret_cast<const uint16_t*>(smem + set * Lds::set) + l16 * LD + lq * 8;
 #pragma unroll
@@ -302,13 +322,14 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, KT <= 2 
       const int qi = 4 * lq + e, kj = l16;
       int i, j;
       bool ok;
-      if (level > 0) {
-        ok = qi / level == kj / level;
-        i = qi / level * 2 * level + level + qi % level;
-        j = kj / level * 2 * level + kj % level;
+      if (shift >= 0) {
+        const int s = 1 << shift;
+        ok = qi >> shift == kj >> shift;
+        i = qi + (qi & -s) + s;
+        j = kj + (kj & -s);
       } else {
         ok = qi == kj;
-        i = j = 2 * qi + (level == 0 ? 1 : 0);
+        i = j = 2 * qi + 2 + shift;
       }
       if (!ok) continue;
       uint32_t hi, lo;
@@ -337,7 +358,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, KT <= 2 
         forget<true>(zr[u][c] + bias[c], lower[c], f, k);
         tt[u][c] = on ? f : 1.f;
         kq[u][c] = on ? k : 0.f;
-        qp[u][c] = STATES ? 0.f : silu_fast(qr[u][c]);
+        if constexpr (STATES) qp[u][c] = 0.f;
+        else if constexpr (RAW) qp[u][c] = on ? silu_fast(c ? bfhi(qw[u]) : bflo(qw[u])) : 0.f;
+        else qp[u][c] = on ? silu_fast(qr[u][c]) : 0.f;
       }
     }
     f32x2 mine = tt[0];
@@ -347,9 +370,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, KT <= 2 
       // first phase: the diagonal and levels 1 and 2
 #pragma unroll
       for (int u = 0; u < TG; ++u) {
-        const int i = grp * TG + u;
-        put_q(u & 1 ? 0 : 1, i >> 1, qp[u]);
-        put_k(u & 1 ? 0 : 1, i >> 1, kq[u]);
+        uint8_t* at = row0 + (u & 1 ? 0 : Lds::set) + u / 2 * LD * 2;
+        put_q(at, qp[u]);
+        put_k(at, kq[u]);
         qp[u] *= tt[u];
       }
     }
@@ -361,9 +384,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, KT <= 2 
         if (s <= 2)
 #pragma unroll
           for (int u = 0; u < TG; ++u) {
-            const int i = grp * TG + u, at = i / (2 * s) * s + i % s;
-            if ((u / s) & 1) put_q(s + 1, at, qp[u]);
-            else put_k(s + 1, at, kq[u]);
+            uint8_t* at = row0 + (s + 1) * Lds::set + (u / (2 * s) * s + u % s) * LD * 2;
+            if ((u / s) & 1) put_q(at, qp[u]);
+            else put_k(at, kq[u]);
           }
       if (!STATES && s >= 4) continue;   // (formed behind the barrier)
 #pragma unroll
@@ -377,23 +400,23 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, KT <= 2 
     if constexpr (!STATES && TG == 2) {   // level 2 lies across threads: a thread's two tokens are one block
 #pragma unroll
       for (int u = 0; u < TG; ++u) {
-        const int at = grp / 2 * 2 + u;
-        if (grp & 1) put_q(3, at, qp[u]);
-        else put_k(3, at, kq[u]);
+        uint8_t* at = smem + 3 * Lds::set + ((grp / 2 * 2 + u) * LD + ch) * 2;
+        if (grp & 1) put_q(at, qp[u]);
+        else put_k(at, kq[u]);
       }
     }
     __syncthreads();
     if constexpr (!STATES) {
-      score(wave, wave == 0 ? 0 : wave == 1 ? -1 : wave - 1);
+      score(wave, wave < 2 ? -1 - wave : wave - 2);
       __syncthreads();   // the first phase's operands are read
       // second phase: levels 4, 8 and 16
 #pragma unroll
       for (int s = 4; s < TG; s *= 2) {
 #pragma unroll
         for (int u = 0; u < TG; ++u) {
-          const int i = grp * TG + u, at = i / (2 * s) * s + i % s;
-          if ((u / s) & 1) put_q(s / 8, at, qp[u]);
-          else put_k(s / 8, at, kq[u]);
+          uint8_t* at = row0 + s / 8 * Lds::set + (u / (2 * s) * s + u % s) * LD * 2;
+          if ((u / s) & 1) put_q(at, qp[u]);
+          else put_k(at, kq[u]);
         }
 #pragma unroll
         for (int u = 0; u < TG; ++u) {
@@ -410,13 +433,15 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, KT <= 2 
       const int blk = grp * TG / s, per = s / TG;
       const bool second = blk & 1;
       if constexpr (!STATES)
-        if (s >= 4)
+        if (s >= 4) {
+          uint8_t* at = smem + s / 8 * Lds::set + ((blk / 2 * s + grp % per * TG) * LD + ch) * 2;
+          if (second)
 #pragma unroll
-          for (int u = 0; u < TG; ++u) {
-            const int i = grp * TG + u, at = i / (2 * s) * s + i % s;
-            if (second) put_q(s / 8, at, qp[u]);
-            else put_k(s / 8, at, kq[u]);
-          }
+            for (int u = 0; u < TG; ++u) put_q(at + u * LD * 2, qp[u]);
+          else
+#pragma unroll
+            for (int u = 0; u < TG; ++u) put_k(at + u * LD * 2, kq[u]);
+        }
       f32x2 other = *reinterpret_cast<const f32x2*>(tot + (blk ^ 1) * per * DK + ch);
 #pragma unroll
       for (int g = 1; g < per; ++g) other *= *reinterpret_cast<const f32x2*>(tot + ((blk ^ 1) * per + g) * DK + ch);
@@ -443,8 +468,18 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, KT <= 2 
         *reinterpret_cast<uint32_t*>(&ktl[(ch + c) * kTokLd + grp * TG + u]) = lo;
       }
     }
+    if constexpr (RAW)
 #pragma unroll
-    for (int j = 0; j < 8; ++j) *reinterpret_cast<uint32_t*>(&vt[((tid & 15) * 8 + j) * kTokLd + 2 * vp]) = cvt_pk_bf16(v0[j], v1[j]);
+      for (int j = 0; j < 4; ++j) {
+        v0[2 * j] = bflo(vw[0][j]);
+        v0[2 * j + 1] = bfhi(vw[0][j]);
+        v1[2 * j] = bflo(vw[1][j]);
+        v1[2 * j + 1] = bfhi(vw[1][j]);
+      }
+#pragma unroll
+    for (int j = 0; j < 8; ++j)   // (a row that is not there may hold anything: nought times it must stay nought)
+      *reinterpret_cast<uint32_t*>(&vt[((tid & 15) * 8 + j) * kTokLd + 2 * vp]) =
+          cvt_pk_bf16(live(t0 + 2 * vp) ? v0[j] : 0.f, live(t0 + 2 * vp + 1) ? v1[j] : 0.f);
     if (t0 + kTok < t_end) fetch(t0 + kTok);
     __syncthreads();
     f32x16 O;
@@ -453,7 +488,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, KT <= 2 
 #pragma unroll
       for (int s = 0; s < 2; ++s) bv[s] = *reinterpret_cast<const u32x4*>(&vt[(wave * 32 + l32) * kTokLd + 16 * s + 8 * lh]);
     if constexpr (!STATES) {
-      if (wave < 3) score(wave, 4 << wave);
+      if (wave < 3) score(wave, 2 + wave);
       if (active) {
 #pragma unroll
         for (int i = 0; i < 16; ++i) O[i] = 0.f;
@@ -548,11 +583,11 @@ template <int KT, typename TY>
 int launch_chunk(hipStream_t st, const GateArgs& a, const RowSrc<TY>& src, const RowSrc<float>& fs) {
   static std::once_flag once;
   static hipError_t e = hipSuccess;
-  constexpr size_t kSmem = GateLds<KT * 32>::bytes;
+  constexpr size_t kSmem = GateLds<KT * 32>::bytes, kStates = GateLds<KT * 32>::states_bytes;
   std::call_once(once, [] {
     e = hipFuncSetAttribute(reinterpret_cast<const void*>(&gated_chunk_kernel<KT, false, TY>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)kSmem);
     if (e == hipSuccess)
-      e = hipFuncSetAttribute(reinterpret_cast<const void*>(&gated_chunk_kernel<KT, true, TY>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)kSmem);
+      e = hipFuncSetAttribute(reinterpret_cast<const void*>(&gated_chunk_kernel<KT, true, TY>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)kStates);
   });
   if (e != hipSuccess) {
     tnx_set_error("gated_state: cannot raise the dynamic LDS limit: %s", hipGetErrorString(e));
@@ -560,7 +595,7 @@ int launch_chunk(hipStream_t st, const GateArgs& a, const RowSrc<TY>& src, const
   }
   const dim3 grid((unsigned)(a.n_spans * cdiv(a.dv, 128)), (unsigned)a.H, (unsigned)a.B);
   if (a.n_spans > 1) {
-    hipLaunchKernelGGL((gated_chunk_kernel<KT, true, TY>), grid, dim3(256), kSmem, st, a, src, fs);
+    hipLaunchKernelGGL((gated_chunk_kernel<KT, true, TY>), grid, dim3(256), kStates, st, a, src, fs);
     hipLaunchKernelGGL(gated_scan_kernel, dim3((unsigned)cdiv((int64_t)a.dk * a.dv, 256), (unsigned)a.H, (unsigned)a.B), dim3(256), 0, st, a);
   }
   hipLaunchKernelGGL((gated_chunk_kernel<KT, false, TY>), grid, dim3(256), kSmem, st, a, src, fs);
@@ -628,13 +663,15 @@ extern "C" int tnx_gated_state(void* stream, const tnx_gated_state_desc* d) {
     return TNX_OK;
   }
   TNX_REQUIRE(!d->norm_w, "gated_state: output rows must be multiples of four");
-  const bool aligned = (d->y.ld | d->y.plane | d->f.ld | d->f.plane | d->q_off | d->v_off | d->f_off) % 8 == 0;
+  // finished bf16 rows beside finished gates, or fp32 rows throughout
+  const bool plain = y16 && ys <= 1 && fsp <= 1 && d->T * (d->y.ld > d->f.ld ? d->y.ld : d->f.ld) < ((int64_t)1 << 31);
+  const bool aligned = (plain || !y16 || ys > 1) && (d->y.ld | d->y.plane | d->f.ld | d->f.plane | d->q_off | d->v_off | d->f_off) % 8 == 0;
   if (bf && d->T > 1 && aligned && d->dk % 8 == 0 && d->dk <= 256 && d->dv % 8 == 0 && d->T < (1 << 30)) {
     a.span = span_tokens(d->B, d->T, d->H);
     a.n_spans = (int)cdiv(d->T, a.span);
     a.ws = d->ws;
     TNX_REQUIRE(a.n_spans == 1 || d->ws, "gated_state: a long prompt needs the workspace of tnx_gated_state_ws_bytes");
-    return y16 ? launch_chunk_any(st, a, s16, fs) : launch_chunk_any(st, a, s32, fs);
+    return plain ? launch_chunk_any(st, a, s16, fs) : launch_chunk_any(st, a, s32, fs);
   }
   const size_t lds = (size_t)3 * d->dk * 4;
   if (y16) hipLaunchKernelGGL(gated_any_kernel<uint16_t>, per, dim3(256), lds, st, a, s16, fs);

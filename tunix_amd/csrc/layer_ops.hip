@@ -444,7 +444,11 @@ int launch_poly(hipStream_t st, int64_t M, const RowSrc<T>& src, int64_t F, cons
   const dim3 grid((unsigned)M);
   const bool vec = F % 8 == 0 && F <= 32768 && src.ld % 8 == 0 && src.plane % 8 == 0 && out_ld % 8 == 0;
   if (!vec) hipLaunchKernelGGL((poly_norm_any_kernel<T>), grid, dim3(256), 0, st, src, F, coef, eps, out, out_ld, out_frag);
-  else if (F <= 2048) hipLaunchKernelGGL((poly_norm_kernel<256, 1, T>), grid, dim3(256), 0, st, src, F, coef, eps, out, out_ld, out_frag);
+  else if (M >= 1024 && F > 2048 && F <= 16384) {   // many rows fill the device: fewer waves meet per row
+    if (F <= 4096) hipLaunchKernelGGL((poly_norm_kernel<256, 2, T>), grid, dim3(256), 0, st, src, F, coef, eps, out, out_ld, out_frag);
+    else if (F <= 8192) hipLaunchKernelGGL((poly_norm_kernel<256, 4, T>), grid, dim3(256), 0, st, src, F, coef, eps, out, out_ld, out_frag);
+    else hipLaunchKernelGGL((poly_norm_kernel<512, 4, T>), grid, dim3(512), 0, st, src, F, coef, eps, out, out_ld, out_frag);
+  } else if (F <= 2048) hipLaunchKernelGGL((poly_norm_kernel<256, 1, T>), grid, dim3(256), 0, st, src, F, coef, eps, out, out_ld, out_frag);
   else if (F <= 4096) hipLaunchKernelGGL((poly_norm_kernel<512, 1, T>), grid, dim3(512), 0, st, src, F, coef, eps, out, out_ld, out_frag);
   else if (F <= 8192) hipLaunchKernelGGL((poly_norm_kernel<1024, 1, T>), grid, dim3(1024), 0, st, src, F, coef, eps, out, out_ld, out_frag);
   else if (F <= 16384) hipLaunchKernelGGL((poly_norm_kernel<1024, 2, T>), grid, dim3(1024), 0, st, src, F, coef, eps, out, out_ld, out_frag);
@@ -458,7 +462,7 @@ int launch_poly(hipStream_t st, int64_t M, const RowSrc<T>& src, int64_t F, cons
 // logits hold, k distinct experts are found; a row with a NaN leaves NaN weights.
 constexpr int kRankedExperts = 256;   // up to here every expert counts the ones ahead of it
 __global__ __launch_bounds__(64) void route_scores_kernel(const RowSrc<float> src, int E, int k, const float* correction, float scale, int64_t gate_off,
-                                                          float* topk_w, int32_t* topk_id, float* gate_w) {
+                                                          int ld, float* topk_w, int32_t* topk_id, float* gate_w) {
   extern __shared__ __align__(16) float lds[];   // choice scores [E rounded up to 4], scores [E], chosen scores [k]
   float *choice = lds, *score = lds + (E + 3) / 4 * 4, *sel = score + E;
   const int64_t m = blockIdx.x;
@@ -473,7 +477,14 @@ __global__ __launch_bounds__(64) void route_scores_kernel(const RowSrc<float> sr
     score[e] = z;
     top = fmaxf(top, z);
   }
-  if (gate_w && lane == 0) gate_w[m] = sigmoid_f32(src.get(m, gate_off));
+  if ((gate_w || ld > k) && lane == 0) {
+    const float g = sigmoid_f32(src.get(m, gate_off));
+    if (gate_w) gate_w[m] = g;
+    if (ld > k) {
+      topk_w[m * ld + k] = g;
+      topk_id[m * ld + k] = E;
+    }
+  }
   bad = __any(bad);
   top = wave_max(top);
   float sum = 0.f;
@@ -503,7 +514,7 @@ __global__ __launch_bounds__(64) void route_scores_kernel(const RowSrc<float> sr
       for (; o < E; ++o) ahead += choice[o] > v || (choice[o] == v && o < e);
       if (ahead < k) {
         sel[ahead] = score[e];
-        topk_id[m * k + ahead] = e;
+        topk_id[m * ld + ahead] = e;
       }
     }
     __syncthreads();
@@ -527,7 +538,7 @@ __global__ __launch_bounds__(64) void route_scores_kernel(const RowSrc<float> sr
     }
     if (lane == 0) {
       sel[j] = score[bi];
-      topk_id[m * k + j] = bi;
+      topk_id[m * ld + j] = bi;
       choice[bi] = ninf;
     }
     __syncthreads();
@@ -535,7 +546,7 @@ __global__ __launch_bounds__(64) void route_scores_kernel(const RowSrc<float> sr
   float total = 0.f;
   for (int j = lane; j < k; j += 64) total += sel[j];
   total = wave_sum(total) + 1e-20f;
-  for (int j = lane; j < k; j += 64) topk_w[m * k + j] = bad ? __builtin_nanf("") : sel[j] / total * scale;
+  for (int j = lane; j < k; j += 64) topk_w[m * ld + j] = bad ? __builtin_nanf("") : sel[j] / total * scale;
 }
 
 }  // namespace
@@ -593,12 +604,13 @@ extern "C" int tnx_poly_norm(void* stream, int dtype, const tnx_rows_src* y, int
 }
 
 extern "C" int tnx_route_scores(void* stream, const tnx_rows_src* z, int64_t M, int E, int k, const float* correction, float scale, int64_t gate_off,
-                                float* topk_w, int32_t* topk_id, float* gate_w) {
+                                int ld, float* topk_w, int32_t* topk_id, float* gate_w) {
   TNX_REQUIRE(z && src_given(*z) && topk_w && topk_id, "route_scores: null pointer");
   TNX_REQUIRE(M > 0 && M < ((int64_t)1 << 31) && E > 0 && E <= 4096 && k > 0 && k <= E && z->ld >= E, "route_scores: bad shape E=%d k=%d", E, k);
-  TNX_REQUIRE(!gate_w || (gate_off >= 0 && gate_off < z->ld), "route_scores: the gate lies outside the row");
+  TNX_REQUIRE(ld == k || ld == k + 1, "route_scores: %d entries per row for %d experts", ld, k);
+  TNX_REQUIRE((!gate_w && ld == k) || (gate_off >= 0 && gate_off < z->ld), "route_scores: the gate lies outside the row");
   hipLaunchKernelGGL(route_scores_kernel, dim3((unsigned)M), dim3(64), (size_t)((E + 3) / 4 * 4 + E + k) * 4, as_stream(stream), row_src<float>(*z), E, k,
-                     correction, scale, gate_off, topk_w, topk_id, gate_w);
+                     correction, scale, gate_off, ld, topk_w, topk_id, gate_w);
   TNX_CHECK_LAUNCH("route_scores");
   return TNX_OK;
 }

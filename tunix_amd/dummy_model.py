@@ -82,7 +82,9 @@ def create_stack_weights(cfg: StackConfig, seed: int = 0, device="cpu", scale: f
     elif name.endswith(".dwa"):
       t = 0.1 * t
       t[-1] += 1.0
-    elif name.endswith(("mlp.act", "mlp.correction")):
+    elif name.endswith("mlp.correction"):
+      t = (0.1 / shape[0]) * t
+    elif name.endswith("mlp.act"):
       t = 0.3 * t
     elif name.endswith(".talk"):
       t = torch.eye(shape[0], device=dev) + t * (0.3 * shape[0] ** -0.5)

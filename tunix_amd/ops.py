@@ -389,8 +389,8 @@ def route_softmax(src: L.RowsSrc, M, E, k, topk_w, topk_id):
   L.check(L.lib().tnx_route_softmax(_stream(), C.byref(src), M, E, k, _ptr(topk_w), _ptr(topk_id)), "tnx_route_softmax")
 
 
-def route_scores(src: L.RowsSrc, M, E, k, correction, scale, topk_w, topk_id, gate_off=0, gate_w=None):
-  L.check(L.lib().tnx_route_scores(_stream(), C.byref(src), M, E, k, _ptr(correction), float(scale), gate_off, _ptr(topk_w), _ptr(topk_id),
+def route_scores(src: L.RowsSrc, M, E, k, correction, scale, topk_w, topk_id, gate_off=0, gate_w=None, ld=None):
+  L.check(L.lib().tnx_route_scores(_stream(), C.byref(src), M, E, k, _ptr(correction), float(scale), gate_off, k if ld is None else ld, _ptr(topk_w), _ptr(topk_id),
                                    _ptr(gate_w)), "tnx_route_scores")
 
 

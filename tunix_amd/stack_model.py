@@ -208,13 +208,13 @@ class StackModel:
       if spec.mlp is not None and not cfg.parallel:
         ly["norm2"], ly["post2"] = vector(p + "norm2") if cfg.pre_norm else None, vector(p + cfg.post_norm(2))
       if isinstance(spec.mlp, ExpertsMlp):
-        e = [p + f"mlp.e{j}." for j in range(spec.mlp.experts)]
+        e = [p + f"mlp.e{j}." for j in range(spec.mlp.experts)] + ([p + "mlp.shared."] if spec.mlp.shared_routed else [])
         ly["router"] = linear([p + "mlp.router"] + ([p + "mlp.shared.sg"] if spec.mlp.shared_ff else []))
         ly["gu"] = LinearBank([linear([n + "gate", n + "up"], paired=True) if spec.mlp.gated else linear([n + "up"]) for n in e])
         ly["down"] = LinearBank([linear([n + "down"]) for n in e])
         if spec.mlp.corrected:
           ly["correction"] = vector(p + "mlp.correction")
-        if spec.mlp.shared_ff:
+        if spec.mlp.shared_ff and not spec.mlp.shared_routed:
           ly["shared_up"], ly["shared_down"] = linear([p + "mlp.shared.up"]), linear([p + "mlp.shared.down"])
       elif isinstance(spec.mlp, PolyNormMlp):
         ly["gu"], ly["down"], ly["act"] = linear([p + "mlp.up"]), linear([p + "mlp.down"]), vector(p + "mlp.act")
@@ -371,9 +371,9 @@ class StackRunner(HeadRunner):
         n_ws[0] = max(n_ws[0], self._split(model.loop_in) * M * model.loop_in.N)
       if isinstance(ly["spec"].mlp, ExpertsMlp):
         e = ly["spec"].mlp
-        n_routes, n_experts = max(n_routes, M * e.top), max(n_experts, e.experts)
+        n_routes, n_experts = max(n_routes, M * e.routes), max(n_experts, len(ly["gu"]))
         if self.dtype == torch.float32:
-          n_y[0] = max(n_y[0], M * e.top * ly["gu"].N)
+          n_y[0] = max(n_y[0], M * e.routes * ly["gu"].N)
       if isinstance(m, LightningMixer):   # (a call may bring fewer rows, and cut them into more spans)
         n_light = max([n_light] + [ops.lightning_ws_bytes(b, T, m.heads, m.dim, m.vdim) // 4 for b in range(1, B + 1)])
       elif isinstance(m, GatedStateMixer):
@@ -605,23 +605,23 @@ class StackRunner(HeadRunner):
       return src, 1, src, f.offsets[2]
     return self.linear(f, h, M, cols=(0, f.offsets[2])), 0, self.fp32_rows(f, h, M, slot=0, cols=(f.offsets[2], f.N)), 0
 
-  def gated_state(self, ly, rows, entry, col_ptr, starts, B, T) -> torch.Tensor:
-    """The recurrence and its heads' norms: what the output projection reads."""
-    m, f, M = ly["spec"].mixer, ly["in"], B * T
-    out = self._buf("gated", ly["out"].Kp)
+  def gated_state(self, ly, rows, entry, col_ptr, starts, B, T) -> tuple:
+    """The recurrence: (what the output projection reads, True), heads normed, or (fp32 [rows, heads * vdim], False)."""
+    m, f = ly["spec"].mixer, ly["in"]
     d = L.GatedStateDesc()
     d.B, d.T, d.H, d.dk, d.dv, d.dtype = B, T, m.heads, m.dim, m.vdim, self.code
     d.y, d.y_f32, d.f, d.f_off = rows
     d.q_off, d.v_off, d.bias, d.lower = f.offsets[0], f.offsets[1], ly["bias"].data_ptr(), ly["lower"].data_ptr()
     d.starts, d.col_ptr, d.state, d.ws = starts.data_ptr(), col_ptr.data_ptr(), entry.s.data_ptr(), self.light_ws.data_ptr()
     if T == 1 and ops.gated_state_step_ok(m.dim, m.vdim):
+      out = self._buf("gated", ly["out"].Kp)
       d.norm_w, d.eps, d.out, d.out_ld, d.out_frag = ly["norm"].data_ptr(), self.cfg.norm_eps, out.data_ptr(), out.shape[1], 1 if self.frag else 0
       ops.gated_state(d)
-      return out
+      return out, True
     o = self._buf("state_out", m.heads * m.vdim, torch.float32)
     d.o, d.o_ld = o.data_ptr(), o.shape[1]
     ops.gated_state(d)
-    return self.head_norm(ly, o, M)
+    return o, False
 
   def head_norm(self, ly, o, M: int) -> torch.Tensor:
     """Heads of o normed on their own, with shared weights."""
@@ -867,7 +867,8 @@ class StackRunner(HeadRunner):
     m, M = ly["spec"].mixer, B * T
     at = (entry, col_ptr, starts, B, T)
     if isinstance(m, GatedStateMixer):
-      return self.linear(ly["out"], self.gated_state(ly, self.gated_in(ly["in"], h, M), *at), M)
+      out, normed = self.gated_state(ly, self.gated_in(ly["in"], h, M), *at)
+      return self.linear(ly["out"], out if normed else self.head_norm(ly, out, M), M)
     src = self.linear(ly["in"], h, M)
     if isinstance(m, AttentionMixer):
       out = self.attend(ly, self.norm_kv(ly, src, *at) if m.row_norm else self.rotate(ly, src, *at), *at)
@@ -888,14 +889,13 @@ class StackRunner(HeadRunner):
     """Chooses every row's experts and sorts the routes by expert."""
     e = ly["spec"].mlp
     src = self.fp32_rows(ly["router"], h, M, slot=0)
-    ids = self.topk_id[:M * e.top].view(M, e.top)
+    ids = self.topk_id[:M * e.routes].view(M, e.routes)
     if e.corrected:
-      shared = e.shared_ff > 0
-      ops.route_scores(src, M, e.experts, e.top, ly["correction"], e.scale, self.topk_w, ids, ly["router"].offsets[1] if shared else 0,
-                       self.gate_w if shared else None)
+      ops.route_scores(src, M, e.experts, e.top, ly["correction"], e.scale, self.topk_w, ids, ly["router"].offsets[1] if e.shared_ff else 0,
+                       self.gate_w if "shared_up" in ly else None, ld=e.routes)
     else:
       ops.route_softmax(src, M, e.experts, e.top, self.topk_w, ids)
-    ops.moe_sort_routes(ids, e.experts, self.counts, self.offsets, self.sorted_route)
+    ops.moe_sort_routes(ids, len(ly["gu"]), self.counts, self.offsets, self.sorted_route)
 
   def experts_linear(self, f: LinearBank, x, x_frag: bool, x_div: int, routes: int, epilogue: int, y, ldy: int):
     d = L.DenseDesc()
@@ -907,22 +907,22 @@ class StackRunner(HeadRunner):
 
   def experts_gate_up(self, ly, h, M: int) -> torch.Tensor:
     e, f = ly["spec"].mlp, ly["gu"]
-    act = self._buf("act", ly["down"].Kp, rows=self.M * e.top)
+    act = self._buf("act", ly["down"].Kp, rows=self.M * e.routes)
     if not e.gated:
-      self.experts_linear(f, h, self.frag, e.top, M * e.top, L.TNX_EPI_RELU2, act, act.shape[1])
+      self.experts_linear(f, h, self.frag, e.routes, M * e.routes, L.TNX_EPI_RELU2, act, act.shape[1])
     elif self.dtype == torch.float32:
-      y = self.y[0][:M * e.top * f.N].view(M * e.top, f.N)
-      self.experts_linear(f, h, False, e.top, M * e.top, L.TNX_EPI_STORE, y, f.N)
-      ops.silu_mul(y, f.offsets[1], M * e.top, e.ff, act)
+      y = self.y[0][:M * e.routes * f.N].view(M * e.routes, f.N)
+      self.experts_linear(f, h, False, e.routes, M * e.routes, L.TNX_EPI_STORE, y, f.N)
+      ops.silu_mul(y, f.offsets[1], M * e.routes, e.ff, act)
     else:
-      self.experts_linear(f, h, self.frag, e.top, M * e.top, L.TNX_EPI_SILU_MUL, act, act.shape[1])
+      self.experts_linear(f, h, self.frag, e.routes, M * e.routes, L.TNX_EPI_SILU_MUL, act, act.shape[1])
     return act
 
   def experts_down(self, ly, act, M: int):
     """The routes' results, to be summed with their weights by the residual step."""
     e, f = ly["spec"].mlp, ly["down"]
-    y = self._buf("routes", f.N, rows=self.M * e.top)
-    self.experts_linear(f, act, False, 1, M * e.top, L.TNX_EPI_STORE, y, f.N)
+    y = self._buf("routes", f.N, rows=self.M * e.routes)
+    self.experts_linear(f, act, False, 1, M * e.routes, L.TNX_EPI_STORE, y, f.N)
     return ops.rows_src(y=y, ld=f.N)
 
   def _mlp(self, ly, h, M: int):
@@ -930,8 +930,8 @@ class StackRunner(HeadRunner):
     e = ly["spec"].mlp
     if isinstance(e, ExpertsMlp):
       self.route(ly, h, M)
-      routes = ("routes", self.experts_down(ly, self.experts_gate_up(ly, h, M), M), ly["post2"], self.topk_w, e.top)
-      if e.shared_ff:
+      routes = ("routes", self.experts_down(ly, self.experts_gate_up(ly, h, M), M), ly["post2"], self.topk_w, e.routes)
+      if "shared_up" in ly:
         routes += (self.linear(ly["shared_down"], self.shared_up(ly, h, M), M), self.gate_w)
       return routes
     if isinstance(e, PolyNormMlp):
