@@ -813,8 +813,8 @@ int tnx_silu_mul(void* stream, int dtype, const void* y, int64_t ld, int64_t up_
 int tnx_route_softmax(void* stream, const tnx_rows_src* z, int64_t M, int E, int k, float* topk_w, int32_t* topk_id);
 /* The same with scores s = softmax over all E logits: the k experts with the largest s + correction (correction [E], null:
  * none) are chosen; topk_w = s / (sum of the chosen s + 1e-20) * scale.  gate_w (null: none) fp32 [M] = sigmoid of z's column
- * gate_off.  ld: entries of a row of topk_w and topk_id, k, or k + 1: then every row's last one is expert E with that sigmoid
- * as its weight (an expert that all rows use). */
+ * gate_off.  ld: entries of a row of topk_w and topk_id; those from k on are the experts E, E + 1, .. with that sigmoid as
+ * their weight (experts that all rows use). */
 int tnx_route_scores(void* stream, const tnx_rows_src* z, int64_t M, int E, int k, const float* correction, float scale, int64_t gate_off,
                      int ld, float* topk_w, int32_t* topk_id, float* gate_w);
 

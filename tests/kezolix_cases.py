@@ -38,10 +38,10 @@ CONFIGS = {
                                attention(6, 2, 32, 48, 33, None, 0.3), attention(6, 2, 32, 48, 50, moe(64, 4, 1, 64, 0.6), 0.25, kv_from=1),
                                attention(6, 2, 32, 48, 17, dense(96), kv_from=1)]),
     # every expert of every token: nothing hangs on a close call of a router
-    "all": config(320, 128, [attention(4, 1, 64, 24, 40, moe(48, 6, 6, 64, 2.5)), state(5, 16, 32, moe(80, 2, 2, 80)), attention(4, 1, 64, 24, 9, dense(200), kv_from=0),
+    "all": config(320, 128, [attention(4, 1, 64, 24, 40, moe(48, 6, 6, 96, 2.5)), state(5, 16, 32, moe(80, 2, 2, 80)), attention(4, 1, 64, 24, 9, dense(200), kv_from=0),
                              state(2, 128, 64, moe(32, 1, 1, 40, 0.4))], mult=0.5),
     # nothing a multiple of eight
-    "odd": config(211, 100, [attention(3, 3, 21, 13, 7, moe(33, 5, 2, 21, 3.0)), state(3, 11, 9, dense(70)), attention(3, 3, 21, 13, 1000, kv_from=0, scale=0.31),
+    "odd": config(211, 100, [attention(3, 3, 21, 13, 7, moe(33, 5, 2, 99, 3.0)), state(3, 11, 9, dense(70)), attention(3, 3, 21, 13, 1000, kv_from=0, scale=0.31),
                              state(1, 20, 30, moe(20, 6, 1, 20)), attention(10, 5, 12, 45, 1)], eps=1e-3, mult=1.0, positions=200),
     # wide heads and many of them
     "wide": config(512, 192, [state(1, 200, 136, dense(256)), attention(16, 2, 136, 200, 64, moe(128, 3, 3, 128)), state(2, 256, 264),

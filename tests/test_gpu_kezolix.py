@@ -529,10 +529,12 @@ def test_choice_by_corrected_scores(gpu, E, k):
     ok = (ti.cpu() == ids).all(1)
     assert rel(tw.cpu()[ok], w[ok]) < 2e-6
     torch.testing.assert_close(gw.cpu(), torch.sigmoid(both[:, -1]), rtol=2e-6, atol=1e-7)
-    # beside an expert that every row uses: the same, one entry longer
-    tw2, ti2 = torch.empty(M, k + 1, device=gpu), torch.empty(M, k + 1, dtype=torch.int32, device=gpu)
-    ops.route_scores(src, M, E, k, cg, scale, tw2, ti2, up(E, 16), ld=k + 1)
-    assert torch.equal(ti2[:, :k], ti) and torch.equal(tw2[:, :k], tw) and bool((ti2[:, k] == E).all()) and torch.equal(tw2[:, k], gw)
+    # beside experts that every row uses: the same, and longer rows
+    for n in (1, 3):
+      tw2, ti2 = torch.empty(M, k + n, device=gpu), torch.empty(M, k + n, dtype=torch.int32, device=gpu)
+      ops.route_scores(src, M, E, k, cg, scale, tw2, ti2, up(E, 16), ld=k + n)
+      assert torch.equal(ti2[:, :k], ti) and torch.equal(tw2[:, :k], tw)
+      assert torch.equal(ti2[:, k:].cpu(), torch.arange(E, E + n, dtype=torch.int32).expand(M, n)) and torch.equal(tw2[:, k:], gw[:, None].expand(M, n))
   plain = torch.empty(M, k, device=gpu)
   ops.route_scores(src, M, E, k, None, 1.0, plain, ti)
   assert torch.equal(ti.cpu().long().sort(1).values[:1], R.route(z.double(), torch.zeros(E), k, 1.0)[0].sort(1).values[:1])

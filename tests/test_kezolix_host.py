@@ -65,6 +65,12 @@ def test_new_parts_do_not_mix_with_what_they_exclude():
     config.ExpertsMlp(8, 4, 2, shared_ff=8)
 
 
+def test_a_shared_expert_among_the_others():
+  """As large as others together it is as many routes of a token; otherwise it runs apart."""
+  make = lambda ff, shared: config.ExpertsMlp(ff, 8, 2, gated=False, corrected=True, shared_ff=shared)
+  assert [make(*a).routes for a in ((16, 16), (16, 48), (16, 24), (16, 8), (16, 0), (16, 80))] == [3, 5, 2, 2, 2, 2]
+
+
 def test_registry_and_benchmark_shapes(tmp_path):
   C.write_model(tmp_path, "odd", seed=1)
   arch, cfg = registry.read_config(str(tmp_path))

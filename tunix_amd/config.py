@@ -354,14 +354,16 @@ class ExpertsMlp:
       raise ValueError("a shared expert and a scale go with corrected scores")
 
   @property
-  def shared_routed(self) -> bool:
-    """A shared expert of the others' size is one more expert, to which every token is routed."""
-    return self.shared_ff == self.ff
+  def shared_routes(self) -> int:
+    """A shared expert of up to four times the others' size is as many more experts, to which every token is routed (0: it
+    runs apart): the square is taken element by element."""
+    n = self.shared_ff // self.ff
+    return n if n * self.ff == self.shared_ff and n <= 4 else 0
 
   @property
   def routes(self) -> int:
     """Experts that a token is routed to."""
-    return self.top + (1 if self.shared_routed else 0)
+    return self.top + self.shared_routes
 
   def weight_shapes(self, D: int) -> dict[str, tuple]:
     out = {"router": (self.experts, D)}

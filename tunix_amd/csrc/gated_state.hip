@@ -344,9 +344,11 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(KT <= 2 || 
   if (start > col0 + t_begin) t0 = t_begin + (start - col0 - t_begin) / kTok * kTok;
   if (!STATES && active && dok)
     for (int t = t_begin + lh; t < min(t0, t_end); t += 2) a.o[(b * a.T + t) * a.o_ld + hv + dcol] = 0.f;
-  if (t0 < t_end) fetch(t0);
+  constexpr bool AHEAD = KT < 8 || STATES;   // (wide heads leave no registers for the next chunk's rows)
+  if (AHEAD && t0 < t_end) fetch(t0);
   for (; t0 < t_end; t0 += kTok) {
     const int n = min(kTok, t_end - t0);
+    if (!AHEAD) fetch(t0);
     // gates; tokens that are not there keep everything and write nothing
     f32x2 qp[TG], kq[TG], tt[TG];
 #pragma unroll
@@ -480,7 +482,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(KT <= 2 || 
     for (int j = 0; j < 8; ++j)   // (a row that is not there may hold anything: nought times it must stay nought)
       *reinterpret_cast<uint32_t*>(&vt[((tid & 15) * 8 + j) * kTokLd + 2 * vp]) =
           cvt_pk_bf16(live(t0 + 2 * vp) ? v0[j] : 0.f, live(t0 + 2 * vp + 1) ? v1[j] : 0.f);
-    if (t0 + kTok < t_end) fetch(t0 + kTok);
+    if (AHEAD && t0 + kTok < t_end) fetch(t0 + kTok);
     __syncthreads();
     f32x16 O;
     u32x4 bv[2];

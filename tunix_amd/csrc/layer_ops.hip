@@ -480,9 +480,9 @@ __global__ __launch_bounds__(64) void route_scores_kernel(const RowSrc<float> sr
   if ((gate_w || ld > k) && lane == 0) {
     const float g = sigmoid_f32(src.get(m, gate_off));
     if (gate_w) gate_w[m] = g;
-    if (ld > k) {
-      topk_w[m * ld + k] = g;
-      topk_id[m * ld + k] = E;
+    for (int j = k; j < ld; ++j) {
+      topk_w[m * ld + j] = g;
+      topk_id[m * ld + j] = E + j - k;
     }
   }
   bad = __any(bad);
@@ -607,7 +607,7 @@ extern "C" int tnx_route_scores(void* stream, const tnx_rows_src* z, int64_t M, 
                                 int ld, float* topk_w, int32_t* topk_id, float* gate_w) {
   TNX_REQUIRE(z && src_given(*z) && topk_w && topk_id, "route_scores: null pointer");
   TNX_REQUIRE(M > 0 && M < ((int64_t)1 << 31) && E > 0 && E <= 4096 && k > 0 && k <= E && z->ld >= E, "route_scores: bad shape E=%d k=%d", E, k);
-  TNX_REQUIRE(ld == k || ld == k + 1, "route_scores: %d entries per row for %d experts", ld, k);
+  TNX_REQUIRE(ld >= k, "route_scores: %d entries per row for %d experts", ld, k);
   TNX_REQUIRE((!gate_w && ld == k) || (gate_off >= 0 && gate_off < z->ld), "route_scores: the gate lies outside the row");
   hipLaunchKernelGGL(route_scores_kernel, dim3((unsigned)M), dim3(64), (size_t)((E + 3) / 4 * 4 + E + k) * 4, as_stream(stream), row_src<float>(*z), E, k,
                      correction, scale, gate_off, ld, topk_w, topk_id, gate_w);

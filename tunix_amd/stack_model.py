@@ -33,15 +33,17 @@ class DenseLinear:
   (name, first row, end row) for some rows of a weight.  Every member starts at a multiple of `align` (16) output
   columns (`offsets`), K is zero-padded to a multiple of 128.  Runs of 256 columns lie behind each other in memory: at an
   offset that is a multiple of 256 a call may begin or end.
+  inputs: columns [first, end) of the members that take part, all by default.
   paired: two members of one shape whose rows alternate in blocks of 16 (gate | up), so that the
   kernel's epilogue finds both in one wave (bf16).  transpose: the members' transposes."""
 
-  def __init__(self, members: list, weights: dict, dtype, device, paired: bool = False, transpose: bool = False, align: int = 16):
+  def __init__(self, members: list, weights: dict, dtype, device, paired: bool = False, transpose: bool = False, align: int = 16, inputs: tuple | None = None):
     self.members = [m if isinstance(m, tuple) else (m, 0, weights[m].shape[0]) for m in members]
     self.names, self.dtype, self.device, self.paired = [m[0] for m in self.members], dtype, device, paired
     self.transpose = transpose
     self.full_shapes = [tuple(weights[n].shape) for n in self.names]
-    self.shapes = [(r1 - r0, s[1])[::-1 if transpose else 1] for (_, r0, r1), s in zip(self.members, self.full_shapes)]
+    self.inputs = inputs or (0, self.full_shapes[0][1])
+    self.shapes = [(r1 - r0, self.inputs[1] - self.inputs[0])[::-1 if transpose else 1] for (_, r0, r1), s in zip(self.members, self.full_shapes)]
     self.K = self.shapes[0][1]
     self.Kp = _up(self.K, 128)
     widths = [_up(s[0], align) for s in self.shapes]
@@ -61,7 +63,7 @@ class DenseLinear:
     self.check(weights)
     w = torch.zeros(self.N, self.Kp, dtype=self.dtype, device=self.device)
     for (n, r0, r1), off in zip(self.members, self.offsets):
-      src = weights[n][r0:r1].to(self.device, self.dtype)
+      src = weights[n][r0:r1, self.inputs[0]:self.inputs[1]].to(self.device, self.dtype)
       src = src.T if self.transpose else src
       w[off:off + src.shape[0], :self.K] = src
     if self.dtype == torch.bfloat16:
@@ -122,8 +124,8 @@ class StackModel:
     self.transposed: set[str] = set()                  # vectors kept as [taps, channels]
     self.vectors: dict[str, torch.Tensor] = {"final.norm": self.final_norm}
 
-    def linear(members, paired=False, transpose=False, align=16):
-      f = DenseLinear(members, weights, dtype, dev, paired, transpose, align)
+    def linear(members, paired=False, transpose=False, align=16, inputs=None):
+      f = DenseLinear(members, weights, dtype, dev, paired, transpose, align, inputs)
       for n in dict.fromkeys(f.names):
         self.linears.setdefault(n, []).append(f)
       return f
@@ -208,13 +210,15 @@ class StackModel:
       if spec.mlp is not None and not cfg.parallel:
         ly["norm2"], ly["post2"] = vector(p + "norm2") if cfg.pre_norm else None, vector(p + cfg.post_norm(2))
       if isinstance(spec.mlp, ExpertsMlp):
-        e = [p + f"mlp.e{j}." for j in range(spec.mlp.experts)] + ([p + "mlp.shared."] if spec.mlp.shared_routed else [])
+        e = [p + f"mlp.e{j}." for j in range(spec.mlp.experts)]
+        parts = [(j * spec.mlp.ff, (j + 1) * spec.mlp.ff) for j in range(spec.mlp.shared_routes)]   # of the shared expert
         ly["router"] = linear([p + "mlp.router"] + ([p + "mlp.shared.sg"] if spec.mlp.shared_ff else []))
-        ly["gu"] = LinearBank([linear([n + "gate", n + "up"], paired=True) if spec.mlp.gated else linear([n + "up"]) for n in e])
-        ly["down"] = LinearBank([linear([n + "down"]) for n in e])
+        ly["gu"] = LinearBank([linear([n + "gate", n + "up"], paired=True) if spec.mlp.gated else linear([n + "up"]) for n in e] +
+                              [linear([(p + "mlp.shared.up", *r)]) for r in parts])
+        ly["down"] = LinearBank([linear([n + "down"]) for n in e] + [linear([p + "mlp.shared.down"], inputs=r) for r in parts])
         if spec.mlp.corrected:
           ly["correction"] = vector(p + "mlp.correction")
-        if spec.mlp.shared_ff and not spec.mlp.shared_routed:
+        if spec.mlp.shared_ff and not parts:
           ly["shared_up"], ly["shared_down"] = linear([p + "mlp.shared.up"]), linear([p + "mlp.shared.down"])
       elif isinstance(spec.mlp, PolyNormMlp):
         ly["gu"], ly["down"], ly["act"] = linear([p + "mlp.up"]), linear([p + "mlp.down"]), vector(p + "mlp.act")
