@@ -44,7 +44,7 @@ def test_learned_positions(gpu, dtype, D):
 
 # ---- linears with a squared positive part -----------------------------------------------------------
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("M,K,N", [(1, 100, 48), (33, 128, 208), (65, 320, 96), (129, 1000, 272), (700, 256, 528), (1100, 128, 32)])
+@pytest.mark.parametrize("M,K,N", [(1, 100, 48), (33, 128, 208), (65, 320, 96), (129, 1000, 272), (700, 256, 528), (1100, 128, 32), (2500, 136, 112)])
 def test_square_relu_linear(gpu, dtype, M, K, N):
   w, x = rnd(N, K, seed=1, scale=K ** -0.5).to(BF).float(), rnd(M, K, seed=2).to(BF).float()
   f = DenseLinear(["w"], {"w": w}, dtype, gpu)

@@ -32,6 +32,7 @@ struct DenseArgs {
   int n_experts, x_div;
   const int32_t* offsets;
   const int32_t* sorted_route;
+  int row_xcd;             // grid x counts eight row blocks times the column blocks: a row block's stay on one XCD, whose L2 holds its rows
 };
 constexpr int kPlain = 0, kBatch = 1, kExperts = 2;
 
@@ -89,7 +90,13 @@ void dense_rows_kernel(const DenseArgs a) {
   __shared__ __align__(16) float red[4][CG * 16 * 64];
   const int tid = threadIdx.x, lane = tid & 63, l32 = lane & 31, lh = lane >> 5;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  int c64 = blockIdx.x;
   int64_t m0 = (int64_t)blockIdx.y * (32 * RT), m_end = a.M;
+  if (MODE == kPlain && a.row_xcd) {
+    c64 = blockIdx.x >> 3;
+    m0 = ((int64_t)blockIdx.y * 8 + (blockIdx.x & 7)) * (32 * RT);
+    if (m0 >= m_end) return;
+  }
   int64_t x_at = 0, w_at = 0, y_at = 0;
   if constexpr (MODE == kBatch) {
     x_at = blockIdx.z * a.x_stride;
@@ -103,7 +110,7 @@ void dense_rows_kernel(const DenseArgs a) {
     m_end = end_row;
     w_at = expert * a.w_stride;
   }
-  const int c64 = blockIdx.x, z = MODE == kBatch ? 0 : blockIdx.z;
+  const int z = MODE == kBatch ? 0 : blockIdx.z;
   const int ktiles = (int)(a.K / kDenseKT);
   const int per = (ktiles + a.split_k - 1) / a.split_k;
   const int kt0 = z * per, kt1 = min(ktiles, kt0 + per);
@@ -379,7 +386,11 @@ extern "C" int tnx_dense_linear(void* stream, const tnx_dense_desc* d) {
   int rt = d->M <= 32 || narrow ? 1 : d->M <= 64 ? 2 : 4;
   while (batch && rt > 1 && cdiv(d->N, 64) * cdiv(d->M, 32 * rt) * d->batch < 512) rt /= 2;
   TNX_REQUIRE(cdiv(d->M, 32 * rt) <= 65535 && split <= 65535, "dense_linear: too many rows or splits in one call");
-  const dim3 grid((unsigned)cdiv(d->N, 64), (unsigned)cdiv(d->M, 32 * rt), batch ? (unsigned)d->batch : (unsigned)split);
+  dim3 grid((unsigned)cdiv(d->N, 64), (unsigned)cdiv(d->M, 32 * rt), batch ? (unsigned)d->batch : (unsigned)split);
+  if (!batch && narrow && grid.x > 1 && grid.y >= 64) {
+    a.row_xcd = 1;
+    grid = dim3(grid.x * 8, (unsigned)cdiv((int64_t)grid.y, 8), grid.z);
+  }
   if (batch) launch_rows<kBatch>(st, a, rt, grid);
   else launch_rows<kPlain>(st, a, rt, grid);
   TNX_CHECK_LAUNCH("dense_rows");
